@@ -267,7 +267,7 @@ int qie_batch_debug_step(qie_batch* b, const qie_sampling* smp, int32_t* next_id
  * normed after it is computed, its input is the raw stream); the next layer's input is the depth-weighted sum over the embedding
  * output and every layer result so far. */
 enum { QIE_MIXER_LATENT_ATTENTION = 1, QIE_MIXER_GQA = 2, QIE_MIXER_GQA_RECURRENT = 3, QIE_MIXER_MINGRU = 4,
-       QIE_MIXER_CHANNEL_DELTA = 5 };
+       QIE_MIXER_CHANNEL_DELTA = 5, QIE_MIXER_STATE_SPACE = 6 };
 enum { QIE_FF_NONE = 0, QIE_FF_DENSE = 1, QIE_FF_MOE = 2 };
 /* Which keys j <= i a query at position i sees: all of them; the last `size`; those of its own
  * block of `size` positions (blocks counted from position 0 of the sequence). */
@@ -283,8 +283,9 @@ enum { QIE_ROT_HALVES = 0, QIE_ROT_INTERLEAVED = 1 };
  * vectors 'l<i>.norm1|norm2', 'final.norm'; norm_offset 0: plain weights, 1: stored around zero), one
  * norm before every branch and none after.  Options of block 2 (qie_arch_desc): several residual
  * streams with learned mixing (streams), a causal convolution on the mixer's normed input
- * (canon_taps), a norm of the embedding rows (embed_norm). */
-enum { QIE_BLOCK_POSTNORM_GAIN = 0, QIE_BLOCK_SANDWICH = 1, QIE_BLOCK_PRENORM = 2 };
+ * (canon_taps), a norm of the embedding rows (embed_norm).
+ * 3 = x += mixer(N1(x)) + ff(N2(x)), both branches of the same x, plain weight vectors 'l<i>.norm1|norm2'. */
+enum { QIE_BLOCK_POSTNORM_GAIN = 0, QIE_BLOCK_SANDWICH = 1, QIE_BLOCK_PRENORM = 2, QIE_BLOCK_PARALLEL = 3 };
 /* Router: 0 = sigmoid scores, the `top` largest scale the experts' input; 1 = logits with a
  * bias, the `top` largest weighted by the softmax over those alone scale the experts' output. */
 enum { QIE_ROUTER_SIGMOID_IN = 0, QIE_ROUTER_SOFTMAX_OUT = 1, QIE_ROUTER_SOFTMAX_ALL = 2 };
@@ -297,7 +298,10 @@ enum { QIE_ROUTER_SIGMOID_IN = 0, QIE_ROUTER_SOFTMAX_OUT = 1, QIE_ROUTER_SOFTMAX
  * numbers p, q of 'l<i>.mlp.act': xielu(z) = softplus(p) z^2 + z / 2 for z > 0, else
  * (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2.  Experts are always of form 0. */
 /* 2 = W_down (gelu_tanh(W_gate h) * W_up h), gelu_tanh(z) = z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))). */
-enum { QIE_ACT_SILU_GATED = 0, QIE_ACT_XIELU = 1, QIE_ACT_GELU_TANH_GATED = 2 };
+/* 3 = W_down (g sigmoid(1.702 g) (u + 1)), g = min(W_gate h, ff_limit), u = W_up h clamped to +-ff_limit. */
+enum { QIE_ACT_SILU_GATED = 0, QIE_ACT_XIELU = 1, QIE_ACT_GELU_TANH_GATED = 2, QIE_ACT_CLAMPED_GATED = 3 };
+/* Gates of the recurrence beside an attention (qie_recurrent_desc.kind). */
+enum { QIE_REC_LOWER_BOUND = 0, QIE_REC_KEY_DECAY = 1 };
 /* Attention weights of the visible keys: softmax of the scores, or sigmoid(score + pb_h) with a
  * number per head ('mix.pb'); a row's weights are used as they are. */
 enum { QIE_WEIGHTS_SOFTMAX = 0, QIE_WEIGHTS_SIGMOID = 1 };
@@ -341,7 +345,8 @@ typedef struct qie_gqa_desc {
     float q_temp_coef;        /*   1 + coef * ln(floor((pos + 1) / every) + 1)               */
     int32_t out_gate;         /* 1: the concatenated head outputs times sigmoid(W_g x), element by element
                                  ('mix.g' [heads * vdim, width])                             */
-    int32_t reserved2[2];
+    int32_t v_bias;           /* 1: v gets a bias vector after its projection ('mix.v.b')   */
+    int32_t mask_keep;        /* QIE_MASK_WINDOW: the keys j < mask_keep stay visible beyond the window (at their true positions) */
     qie_rot_scaling rot_scaling;
 } qie_gqa_desc;
 
@@ -350,11 +355,29 @@ typedef struct qie_gqa_desc {
  * o_t = S_t^T q_t with q = silu(W_q h), v = W_v h and the forget gate
  * f = lower + (1 - lower) * sigmoid(W_f h + b); o is RMS-normed per head over vdim with a weight
  * vector.  A slot that starts at position 0 starts from S = 0.  The mixer's result is
- * gqa_scale * attention + rec_scale * recurrence (each after its own output projection). */
+ * gqa_scale * attention + rec_scale * recurrence (each after its own output projection).
+ * kind QIE_REC_KEY_DECAY: q = W_q h * dim^(-1/2), k = W_k h (heads x dim), v = W_v h; a decay per head and key
+ * channel a = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau); S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; the
+ * normed heads times silu(W_g h) element by element.  Tensors 'mix.right.q|k|v|g|a1|a2|a2.b|norm|o'; rank: rows of
+ * W_a1 (0: taken from the tensor). */
 typedef struct qie_recurrent_desc {
     int32_t heads, dim, vdim;
-    int32_t reserved;
+    int32_t kind;             /* QIE_REC_* */
+    int32_t rank;
+    float tau;
 } qie_recurrent_desc;
+
+/* Mixer QIE_MIXER_STATE_SPACE (Mamba-2 form): inner = heads * vdim; W_in h = [z (inner) | x (inner) | B (groups *
+ * state) | C (groups * state) | dt (heads)]; x, B and C pass a causal convolution over time per channel ('mix.conv'
+ * [channels, conv], last column = the current token, bias 'mix.conv.b') and silu; dt = softplus(dt + dt_bias).  Per
+ * head (group head / (heads / groups)), S [state][vdim] fp32 in the slot, zero at position 0:
+ * S_t = exp(-exp(A_log) dt) S_(t-1) + dt B_t x_t^T; y_t = S_t^T C_t + D x_t.  y times silu(z), RMS-normed in
+ * norm_groups equal parts, times 'mix.norm', then W_o.  The last conv - 1 rows of [x | B | C] before their
+ * convolution belong to the slot's state.  Tensors 'l<i>.mix.in|conv|conv.b|dt_bias|A_log|D|norm|o'. */
+typedef struct qie_state_space_desc {
+    int32_t heads, vdim, state, groups, conv, norm_groups;
+    int32_t reserved[2];
+} qie_state_space_desc;
 
 /* Mixer QIE_MIXER_MINGRU: a recurrence per channel whose update gate and candidate depend on the current input alone.  With x the
  * mixer's input: z = sigmoid(W_z x + b_z), u = W_x x + b_x (`width` channels each), candidate
@@ -407,6 +430,9 @@ typedef struct qie_layer_desc {
     int32_t reserved3[3];
     qie_delta_desc delta;     /* QIE_MIXER_CHANNEL_DELTA                               */
     qie_rot_scaling rot_scaling;   /* latent attention                                 */
+    qie_state_space_desc ssm; /* QIE_MIXER_STATE_SPACE                                 */
+    float ff_limit;           /* QIE_ACT_CLAMPED_GATED                                 */
+    int32_t reserved4;
 } qie_layer_desc;
 
 typedef struct qie_arch_desc {
@@ -432,6 +458,7 @@ typedef struct qie_arch_desc {
      * the slot's state.  embed_norm 1: the embedding rows pass N with 'embed.norm' first. */
     int32_t streams, canon_taps, embed_norm;
     float norm_offset;
+    float logit_scale;        /* the logits are multiplied by it (0 is read as 1) */
 } qie_arch_desc;
 
 int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* opts, qie_engine** out);
@@ -442,7 +469,7 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
  * recurrence runs beside it, whose tensors are 'l<i>.mix.right.q|f|f.b|lower|v|norm|o'),
  * 'l<i>.mix.pb|g' (sigmoid weights, head gate), 'l<i>.mix.z|z.b|x|x.b|g|o' (QIE_MIXER_MINGRU),
  * 'l<i>.mix.q.b|k.b|sink' (biased, sink attention), 'l<i>.mix.dq|dq.norm|uq' (latent queries), the
- * QIE_MIXER_CHANNEL_DELTA tensors, 'embed.norm', 'l<i>.hc1|hc2.in|out|mix', 'l<i>.canon1',
+ * QIE_MIXER_CHANNEL_DELTA and QIE_MIXER_STATE_SPACE tensors, 'mix.v.b', 'embed.norm', 'l<i>.hc1|hc2.in|out|mix', 'l<i>.canon1',
  * 'l<i>.mlp.gate|up|down|act|router|router.b|correction', 'l<i>.mlp.e<j>.gate|up|down'.
  * qie_engine_finalize_weights checks every tensor the architecture needs against its shape,
  * builds the device layouts (fused projection rows, per-head transposed W_uk, experts end to
@@ -477,7 +504,7 @@ int qie_batch_step_layers(qie_batch* b, float* host_out, int64_t n);
 /* Time `iters` runs of one stage of the last step's shape (hipEvents on the engine stream):
  * which 0 = the whole layer stack, 1 = attention of `layer`, 2 = its projections (input, absorb,
  * value expansion, output), 3 = its feed-forward, 4 = its recurrence (gated scan + head norm, the
- * minGRU scan, or the delta rule's gates, scan and output norm; the slots' states of that layer run are advanced by it, so time it last).  The cache is read, not
+ * minGRU scan, the delta rule's or the state space's convolution, gates, scan and output norm; the slots' states of that layer run are advanced by it, so time it last).  The cache is read, not
  * advanced. */
 int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t iters, double* avg_us);
 

@@ -91,6 +91,16 @@ struct LayerDev {
     void *w_a2 = nullptr, *w_g2 = nullptr;
     float *dl_conv = nullptr, *dl_exp_a = nullptr, *dl_dt_bias = nullptr, *dl_norm = nullptr;
     int col_b = 0, col_a1 = 0, col_g1 = 0, rank_a = 0, rank_g = 0;
+    // attention: bias vector of v; the recurrence with a decay per key channel: w_in rows [.. ; rec q ; rec k ; rec v ;
+    // rec g ; rec a1], W_a2 in w_a2, the decay's bias, the rank in rank_a
+    float *v_bias = nullptr, *rec_a2b = nullptr;
+    int col_rk = 0, col_rg = 0;
+    // QIE_MIXER_STATE_SPACE: w_in as stored ([z ; x ; B ; C ; dt] rows), the convolution's taps and bias, dt_bias,
+    // exp(A_log), the skip, the norm's weight
+    float *ss_conv = nullptr, *ss_conv_b = nullptr, *ss_dt_bias = nullptr, *ss_a = nullptr, *ss_d = nullptr, *ss_norm = nullptr;
+    int col_dt = 0;
+    // parallel blocks: wo also holds W_down, and the feed-forward's activations follow the mixer's columns (-1: no)
+    int cat_ff = -1;
 };
 
 // One execution of a layer: layers of a repeated group run several times, each run with its
@@ -120,6 +130,16 @@ struct LayeredModel {
     size_t esz() const { return f32 ? 4 : 2; }
 };
 
+// Pieces of a step's long entries for the recurrent mixers' scans: chunks {first packed row, rows, piece index, 0} in
+// entry order, spans one {first piece, pieces, slot, first position} per entry.
+struct PieceList {
+    int4 *d_chunks = nullptr, *d_spans = nullptr;
+    int64_t cap = 0, span_cap = 0;
+    int n = 0;
+    int rows = 0;      // rows per piece
+    std::vector<int4> h_chunks, h_spans;
+};
+
 struct LayeredBatch {
     std::vector<int64_t> layer_off;   // per layer run: element offset of its (K) rows inside a page
     std::vector<int64_t> v_off;       // per layer run: its V rows (grouped-query attention)
@@ -140,13 +160,17 @@ struct LayeredBatch {
     int64_t qgroups_cap = 0;
     int n_qgroups = 0;
     std::vector<int4> h_qgroups;
-    // recurrent mixers, long entries: pieces of kScanPiece rows scanned side by side (lay::gated_carry)
-    int4 *d_chunks = nullptr, *d_spans = nullptr;
-    int64_t chunks_cap = 0;
-    int n_chunks = 0, max_count = 0;
-    std::vector<int4> h_chunks, h_spans;
+    // recurrent mixers, long entries: pieces of kScanPiece rows scanned side by side (lay::gated_carry); pieces of
+    // lin_rows rows for the mixers of lay::linrec_walk
+    PieceList pieces, lin;
+    int max_count = 0;
+    bool has_scan = false, has_lin = false;   // layer runs of either kind
+    int64_t lin_units = 0;                    // fewest (head, column tile) blocks of a linear recurrence of the model
     float *s_loc = nullptr, *s_in = nullptr, *s_decay = nullptr;
     int64_t scan_cap = 0;             // pieces the three buffers hold
+    // parallel blocks: the feed-forward's normed rows
+    float* y2 = nullptr;
+    uint16_t* y2_bf = nullptr;
     int64_t m_state = 0, m_hd = 0;    // largest state / gate row count of a layer run
     // bf16 K / V caches on the matrix-core attention: V rows stored [kv_heads][vdim][page_tokens].  Per layer run
     // (vt_of): a grouped-query mixer whose sizes fit that kernel; v_transposed: any run does.
@@ -328,6 +352,58 @@ static int lm_vector(LayeredModel* m, float** dev, const std::string& name, int6
     return lm_floats(m, dev, *t);
 }
 
+// [rows][n_i] tensors side by side in a device matrix: one product over the concatenated inputs
+static int lm_upload_columns(LayeredModel* m, void* dev, int64_t rows, std::initializer_list<const HostTensor*> parts) {
+    HostTensor cat;
+    int64_t n = 0;
+    for (const HostTensor* t : parts) n += t ? t->shape[1] : 0;
+    cat.dtype = 2;
+    cat.shape = {rows, n};
+    cat.data.resize((size_t)rows * n * 4);
+    float* c = (float*)cat.data.data();
+    int64_t at = 0;
+    for (const HostTensor* t : parts) {
+        if (!t) continue;
+        const int64_t k = t->shape[1];
+        for (int64_t r = 0; r < rows; r++)
+            for (int64_t i = 0; i < k; i++) c[r * n + at + i] = host_elem(*t, r * k + i);
+        at += k;
+    }
+    return lm_upload_rows(m, dev, 0, n, cat);
+}
+
+// Output matrix of layer i: the mixer's W_o (and its recurrence's) and, in parallel blocks with a gated dense
+// feed-forward, W_down behind them.  n_cat is the mixer's width on entry, the whole width on return.
+static int finalize_out(LayeredModel* m, int i, const HostTensor* o1, const HostTensor* o2 = nullptr) {
+    LayerDev& L = m->L[i];
+    const qie_layer_desc& d = L.d;
+    const int64_t W = m->a.width;
+    const HostTensor* wd = nullptr;
+    if (m->a.block == QIE_BLOCK_PARALLEL && d.ff_kind == QIE_FF_DENSE && d.ff_act != QIE_ACT_XIELU) {
+        wd = lm_find(m, "l" + std::to_string(i) + ".mlp.down", {W, (int64_t)d.ff});
+        if (!wd) return -22;
+        L.cat_ff = L.n_cat;
+        L.n_cat += d.ff;
+    }
+    QIE_TRY(lm_alloc(m, &L.wo, (size_t)W * L.n_cat * m->esz()));
+    return lm_upload_columns(m, L.wo, W, {o1, o2, wd});
+}
+
+static int lm_exp_vector(LayeredModel* m, float** dev, const HostTensor& t) {
+    HostTensor e;
+    e.dtype = 2;
+    e.shape = t.shape;
+    e.data.resize((size_t)t.numel() * 4);
+    for (int64_t k = 0; k < t.numel(); k++) ((float*)e.data.data())[k] = (float)std::exp((double)host_elem(t, k));
+    return lm_floats(m, dev, e);
+}
+
+// rows of a two-dimensional tensor, 0 when it is missing
+static int64_t lm_rows_of(LayeredModel* m, const std::string& name) {
+    auto it = m->host.find(name);
+    return it != m->host.end() && it->second.shape.size() == 2 ? it->second.shape[0] : 0;
+}
+
 // Fused input rows and output columns of a grouped-query attention, alone ('mix.') or beside a
 // gated recurrence ('mix.left.' / 'mix.right.').
 static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
@@ -339,14 +415,23 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
     const std::string pl = "l" + std::to_string(i) + ".", pa = pl + (rec ? "mix.left." : "mix."), pr = pl + "mix.right.";
     const int64_t nq = (int64_t)a.heads * a.dim, nk = (int64_t)a.kv_heads * a.dim, nv = a.values_are_keys ? 0 : (int64_t)a.kv_heads * a.vdim;
     const int64_t rq = rec ? (int64_t)d.rec.heads * d.rec.dim : 0, rv = rec ? (int64_t)d.rec.heads * d.rec.vdim : 0;
+    const bool key_decay = rec && d.rec.kind == QIE_REC_KEY_DECAY;
     L.col_k = (int)nq;
     L.col_v = a.values_are_keys ? -1 : (int)(nq + nk);
     const int64_t ng = a.out_gate ? (int64_t)a.heads * a.vdim : a.head_gate ? a.heads : 0;
     L.col_gate = ng ? (int)(nq + nk + nv) : -1;
     L.col_rq = (int)(nq + nk + nv + ng);
     L.col_rf = (int)(L.col_rq + rq);
+    L.col_rk = L.col_rf;   // a recurrence holds gates or keys here, by its kind
     L.col_rv = (int)(L.col_rf + rq);
     L.n_in = (int)(L.col_rv + rv);
+    if (key_decay) {
+        L.rank_a = d.rec.rank > 0 ? d.rec.rank : (int)lm_rows_of(m, pr + "a1");
+        QIE_REQUIRE(L.rank_a > 0, "layered weights: layer %d: tensor '%sa1' gives no rank", i, pr.c_str());
+        L.col_rg = L.n_in;
+        L.col_a1 = (int)(L.col_rg + rv);
+        L.n_in = L.col_a1 + L.rank_a;
+    }
     QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
     LM_GET(tq, pa + "q", nq, W);
     LM_GET(tk, pa + "k", nk, W);
@@ -372,6 +457,7 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
         QIE_TRY(lm_vector(m, &L.q_bias, pa + "q.b", nq));
         QIE_TRY(lm_vector(m, &L.k_bias, pa + "k.b", nk));
     }
+    if (a.v_bias) QIE_TRY(lm_vector(m, &L.v_bias, pa + "v.b", nv));
     if (a.sink) QIE_TRY(lm_vector(m, &L.sink, pa + "sink", a.heads));
     if (a.weights == QIE_WEIGHTS_SIGMOID) QIE_TRY(lm_vector(m, &L.pb, pa + "pb", a.heads));
     if (a.slope_bias) {
@@ -387,35 +473,54 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
     const int64_t ca = (int64_t)a.heads * a.vdim;
     L.cat_rec = (int)ca;
     L.n_cat = (int)(ca + rv);
-    QIE_TRY(lm_alloc(m, &L.wo, (size_t)W * L.n_cat * m->esz()));
     LM_GET(to, pa + "o", W, ca);
-    if (!rec) {
-        QIE_TRY(lm_upload_rows(m, L.wo, 0, ca, *to));
-        return 0;
-    }
+    if (!rec) return finalize_out(m, i, to);
     LM_GET(trq, pr + "q", rq, W);
-    LM_GET(trf, pr + "f", rq, W);
+    LM_GET(trf, pr + (key_decay ? "k" : "f"), rq, W);
     LM_GET(trv, pr + "v", rv, W);
     QIE_TRY(lm_upload_rows(m, L.w_in, L.col_rq, W, *trq));
     QIE_TRY(lm_upload_rows(m, L.w_in, L.col_rf, W, *trf));
     QIE_TRY(lm_upload_rows(m, L.w_in, L.col_rv, W, *trv));
-    QIE_TRY(lm_vector(m, &L.rec_fb, pr + "f.b", rq));
-    QIE_TRY(lm_vector(m, &L.rec_lower, pr + "lower", rq));
+    if (key_decay) {
+        LM_GET(trg, pr + "g", rv, W);
+        LM_GET(ta1, pr + "a1", (int64_t)L.rank_a, W);
+        LM_GET(ta2, pr + "a2", rq, (int64_t)L.rank_a);
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_rg, W, *trg));
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_a1, W, *ta1));
+        QIE_TRY(lm_alloc(m, &L.w_a2, (size_t)ta2->numel() * m->esz()));
+        QIE_TRY(lm_upload_rows(m, L.w_a2, 0, L.rank_a, *ta2));
+        QIE_TRY(lm_vector(m, &L.rec_a2b, pr + "a2.b", rq));
+    } else {
+        QIE_TRY(lm_vector(m, &L.rec_fb, pr + "f.b", rq));
+        QIE_TRY(lm_vector(m, &L.rec_lower, pr + "lower", rq));
+    }
     QIE_TRY(lm_vector(m, &L.rec_norm, pr + "norm", d.rec.vdim));
     LM_GET(tro, pr + "o", W, rv);
-    {   // [W][ca] and [W][rv] side by side: one product over the concatenated head outputs
-        HostTensor cat;
-        cat.dtype = 2;
-        cat.shape = {W, (int64_t)L.n_cat};
-        cat.data.resize((size_t)W * L.n_cat * 4);
-        float* c = (float*)cat.data.data();
-        for (int64_t r = 0; r < W; r++) {
-            for (int64_t k = 0; k < ca; k++) c[r * L.n_cat + k] = host_elem(*to, r * ca + k);
-            for (int64_t k = 0; k < rv; k++) c[r * L.n_cat + ca + k] = host_elem(*tro, r * rv + k);
-        }
-        QIE_TRY(lm_upload_rows(m, L.wo, 0, L.n_cat, cat));
-    }
-    return 0;
+    return finalize_out(m, i, to, tro);
+}
+
+// State space: the projection as stored, the convolution, per-head vectors (exp(A_log) in double)
+static int finalize_state_space(LayeredModel* m, int i) {
+    LayerDev& L = m->L[i];
+    const qie_state_space_desc& c = L.d.ssm;
+    const int64_t W = m->a.width, inner = (int64_t)c.heads * c.vdim, C = inner + 2 * (int64_t)c.groups * c.state;
+    const std::string px = "l" + std::to_string(i) + ".mix.";
+    L.col_dt = (int)(inner + C);
+    L.n_in = L.col_dt + c.heads;
+    L.n_cat = (int)inner;
+    LM_GET(ti, px + "in", (int64_t)L.n_in, W);
+    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
+    QIE_TRY(lm_upload_rows(m, L.w_in, 0, W, *ti));
+    LM_GET(tc, px + "conv", C, (int64_t)c.conv);
+    QIE_TRY(lm_floats(m, &L.ss_conv, *tc));
+    QIE_TRY(lm_vector(m, &L.ss_conv_b, px + "conv.b", C));
+    QIE_TRY(lm_vector(m, &L.ss_dt_bias, px + "dt_bias", c.heads));
+    LM_GET(ta, px + "A_log", (int64_t)c.heads);
+    QIE_TRY(lm_exp_vector(m, &L.ss_a, *ta));
+    QIE_TRY(lm_vector(m, &L.ss_d, px + "D", c.heads));
+    QIE_TRY(lm_vector(m, &L.ss_norm, px + "norm", inner));
+    LM_GET(to, px + "o", W, inner);
+    return finalize_out(m, i, to);
 }
 
 static int finalize_ff(LayeredModel* m, int i);
@@ -437,9 +542,7 @@ static int finalize_mingru(LayeredModel* m, int i) {
     QIE_TRY(lm_vector(m, &L.mg_zb, px + "z.b", n));
     QIE_TRY(lm_vector(m, &L.mg_xb, px + "x.b", n));
     LM_GET(to, px + "o", W, n);
-    QIE_TRY(lm_alloc(m, &L.wo, (size_t)W * n * m->esz()));
-    QIE_TRY(lm_upload_rows(m, L.wo, 0, n, *to));
-    return 0;
+    return finalize_out(m, i, to);
 }
 
 // Gated delta rule: fused input rows [q ; k ; v ; b ; a1 ; g1], the second-stage matrices, the three
@@ -449,12 +552,8 @@ static int finalize_delta(LayeredModel* m, int i) {
     const qie_delta_desc& c = L.d.delta;
     const int64_t W = m->a.width, nk = (int64_t)c.kv_heads * c.dim, nv = (int64_t)c.heads * c.vdim, C = 2 * nk + nv;
     const std::string px = "l" + std::to_string(i) + ".mix.";
-    auto rows_of = [&](const std::string& name) -> int64_t {
-        auto it = m->host.find(name);
-        return it != m->host.end() && it->second.shape.size() == 2 ? it->second.shape[0] : 0;
-    };
-    L.rank_a = c.rank_a > 0 ? c.rank_a : (int)rows_of(px + "a1");
-    L.rank_g = c.rank_g > 0 ? c.rank_g : (int)rows_of(px + "g1");
+    L.rank_a = c.rank_a > 0 ? c.rank_a : (int)lm_rows_of(m, px + "a1");
+    L.rank_g = c.rank_g > 0 ? c.rank_g : (int)lm_rows_of(m, px + "g1");
     QIE_REQUIRE(L.rank_a > 0 && L.rank_g > 0, "layered weights: layer %d: tensors '%sa1' / '%sg1' give no rank", i, px.c_str(), px.c_str());
     L.col_k = (int)nk;
     L.col_v = (int)(2 * nk);
@@ -497,20 +596,11 @@ static int finalize_delta(LayeredModel* m, int i) {
         QIE_TRY(lm_floats(m, &L.dl_conv, cat));
     }
     LM_GET(tal, px + "A_log", (int64_t)c.heads);
-    {
-        HostTensor ea;
-        ea.dtype = 2;
-        ea.shape = {(int64_t)c.heads};
-        ea.data.resize((size_t)c.heads * 4);
-        for (int h = 0; h < c.heads; h++) ((float*)ea.data.data())[h] = (float)std::exp((double)host_elem(*tal, h));
-        QIE_TRY(lm_floats(m, &L.dl_exp_a, ea));
-    }
+    QIE_TRY(lm_exp_vector(m, &L.dl_exp_a, *tal));
     QIE_TRY(lm_vector(m, &L.dl_dt_bias, px + "dt_bias", (int64_t)c.heads * c.dim));
     QIE_TRY(lm_vector(m, &L.dl_norm, px + "norm", (int64_t)c.vdim));
     LM_GET(to, px + "o", W, nv);
-    QIE_TRY(lm_alloc(m, &L.wo, (size_t)W * nv * m->esz()));
-    QIE_TRY(lm_upload_rows(m, L.wo, 0, nv, *to));
-    return 0;
+    return finalize_out(m, i, to);
 }
 
 static int finalize_layer(qie_engine* e, LayeredModel* m, int i) {
@@ -540,7 +630,7 @@ static int finalize_layer(qie_engine* e, LayeredModel* m, int i) {
             QIE_TRY(lm_vector(m, &L.n2b, pl + "norm2b", Wn));
         }
     }
-    if (m->a.block == QIE_BLOCK_PRENORM) {
+    if (m->a.block == QIE_BLOCK_PRENORM || m->a.block == QIE_BLOCK_PARALLEL) {
         QIE_TRY(lm_vector(m, &L.n1, pl + "norm1", m->a.width));
         if (d.ff_kind != QIE_FF_NONE) QIE_TRY(lm_vector(m, &L.n2, pl + "norm2", m->a.width));
     }
@@ -550,6 +640,10 @@ static int finalize_layer(qie_engine* e, LayeredModel* m, int i) {
     }
     if (d.mixer == QIE_MIXER_CHANNEL_DELTA) {
         QIE_TRY(finalize_delta(m, i));
+        return finalize_ff(m, i);
+    }
+    if (d.mixer == QIE_MIXER_STATE_SPACE) {
+        QIE_TRY(finalize_state_space(m, i));
         return finalize_ff(m, i);
     }
     if (d.mixer != QIE_MIXER_LATENT_ATTENTION) {
@@ -652,6 +746,7 @@ static int finalize_ff(LayeredModel* m, int i) {
         QIE_TRY(lm_alloc(m, &L.w_gu, (size_t)2 * ff * W * m->esz()));
         QIE_TRY(lm_upload_rows(m, L.w_gu, 0, W, *wg));
         QIE_TRY(lm_upload_rows(m, L.w_gu, ff, W, *wu));
+        if (L.cat_ff >= 0) return 0;   // W_down sits beside W_o
         QIE_TRY(lm_alloc(m, &L.w_down, (size_t)W * ff * m->esz()));
         QIE_TRY(lm_upload_rows(m, L.w_down, 0, ff, *wd));
     } else if (d.ff_kind == QIE_FF_MOE) {
@@ -885,7 +980,8 @@ static int enq_mixer_out(qie_batch* b, int i, int T) {
     return dense(b, s->ov, HV, L.wo, s->mix, m->a.width, T, m->a.width, (int)HV, s->ov_bf);
 }
 
-// feed-forward of layer i on rows y -> ffo
+// feed-forward of layer i on its normed rows (s->y, in parallel blocks s->y2) -> ffo; where the layer's output product
+// takes the activations as well (cat_ff), they go beside the mixer's columns and the product is left to it
 static int enq_ff(qie_batch* b, int i, int T) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
@@ -894,14 +990,20 @@ static int enq_ff(qie_batch* b, int i, int T) {
     LayeredBatch* s = b->lb;
     const int W = m->a.width, ff = d.ff;
     hipStream_t st = e->stream;
+    const bool par = m->a.block == QIE_BLOCK_PARALLEL;
+    const float* y = par ? s->y2 : s->y;
+    const uint16_t* y_bf = par ? s->y2_bf : s->y_bf;
     if (d.ff_kind == QIE_FF_DENSE && d.ff_act == QIE_ACT_XIELU) {
-        QIE_TRY(dense(b, s->y, W, L.w_gu, s->gu, ff, T, ff, W, s->y_bf));
+        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, ff, T, ff, W, y_bf));
         QIE_TRY(lay::xielu(s->gu, s->act, s->act_bf, (int64_t)T * ff, L.act_p, L.act_q, st));
         return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf);
     }
     if (d.ff_kind == QIE_FF_DENSE) {
-        QIE_TRY(dense(b, s->y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, s->y_bf));
-        QIE_TRY(lay::silu_mul(s->gu, s->act, s->act_bf, T, ff, st, d.ff_act == QIE_ACT_GELU_TANH_GATED ? 1 : 0));
+        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, y_bf));
+        const int act = d.ff_act == QIE_ACT_GELU_TANH_GATED ? 1 : d.ff_act == QIE_ACT_CLAMPED_GATED ? 2 : 0;
+        if (L.cat_ff >= 0)
+            return lay::silu_mul(s->gu, s->ov + L.cat_ff, s->ov_bf ? s->ov_bf + L.cat_ff : nullptr, T, ff, st, act, d.ff_limit, L.n_cat);
+        QIE_TRY(lay::silu_mul(s->gu, s->act, s->act_bf, T, ff, st, act, d.ff_limit));
         return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf);
     }
     const int E = d.experts, top = d.top, n = T * top;
@@ -913,13 +1015,13 @@ static int enq_ff(qie_batch* b, int i, int T) {
     const int ER = E + (d.router == QIE_ROUTER_SOFTMAX_ALL ? d.identity : 0);
     const int32_t* id_sel = ER > E ? s->sel : nullptr;
     if (d.router == QIE_ROUTER_SOFTMAX_ALL)
-        QIE_TRY(lay::route_grouped(s->y, L.w_router, L.correction, m->f32, T, W, ER, top, d.groups, d.groups_keep, d.route_scale,
+        QIE_TRY(lay::route_grouped(y, L.w_router, L.correction, m->f32, T, W, ER, top, d.groups, d.groups_keep, d.route_scale,
                                    s->sel, s->score, st));
     else
-        QIE_TRY(lay::route_topk(s->y, L.w_router, L.router_b, m->f32, T, W, E, top, out_w ? 1 : 0, s->sel, s->score, st));
+        QIE_TRY(lay::route_topk(y, L.w_router, L.router_b, m->f32, T, W, E, top, out_w ? 1 : 0, s->sel, s->score, st));
     QIE_TRY(lay::moe_group(s->sel, n, ER, s->cnt, s->off, s->slot_of, st));
     const bool per_expert = !m->f32 && n >= kMoeSyncRows && W % 8 == 0 && ff % 8 == 0;
-    QIE_TRY(lay::moe_gather(s->y, in_score, s->slot_of, T, top, W, s->xg, per_expert ? s->xg_bf : nullptr, st));
+    QIE_TRY(lay::moe_gather(y, in_score, s->slot_of, T, top, W, s->xg, per_expert ? s->xg_bf : nullptr, st));
     if (per_expert) {
         // prompt-sized steps: the expert row ranges come to the host and every expert's rows go
         // through the MFMA kernels; the products are the grouped kernel's, in another order
@@ -997,6 +1099,7 @@ static lay::GqaAttnP gqa_attn_params(qie_batch* b, int r) {
     p.gate_col = (a.head_gate || a.out_gate) ? L.col_gate : -1;
     p.gate_elem = a.out_gate ? 1 : 0;
     p.sink = a.sink ? L.sink : nullptr;
+    p.mask_keep = a.mask_keep;
     return p;
 }
 
@@ -1036,6 +1139,7 @@ static int enq_gqa_post(qie_batch* b, int r, int T) {
     p.q_temp_coef = a.q_temp_coef;
     p.q_bias = a.qk_bias ? L.q_bias : nullptr;
     p.k_bias = a.qk_bias ? L.k_bias : nullptr;
+    p.v_bias = a.v_bias ? L.v_bias : nullptr;
     return lay::gqa_post(p, m->f32, T, e->stream);
 }
 
@@ -1047,7 +1151,7 @@ static int enq_gqa_attention(qie_batch* b, int r, int T) {
         // enough key splits to fill the chip when the step has few rows (decoding)
         const int tiles = (p.heads + 3) / 4 * 4;
         const int64_t waves = (int64_t)s->n_qgroups * p.heads;
-        const int max_blocks = (p.mask == QIE_MASK_CAUSAL ? b->max_ctx : std::min(b->max_ctx, p.mask_size)) / 32 + 2;
+        const int max_blocks = (p.mask == QIE_MASK_CAUSAL ? b->max_ctx : std::min(b->max_ctx, p.mask_size + p.mask_keep)) / 32 + 2;
         // (a wave walks its key blocks one after the other, each a trip to memory: prompts of a
         // few thousand rows leave too few waves to hide them, so their keys are split as well)
         static const int split_waves = dev_env("QIE_GQA_SPLIT_WAVES", 6144);   // dev A/B knob: waves a launch aims for
@@ -1077,12 +1181,97 @@ static int enq_gqa_attention(qie_batch* b, int r, int T) {
 // Rows of an entry above which the recurrence runs in pieces; rows per piece.
 constexpr int kScanLong = 128, kScanPiece = 64;
 
+// Rows of an entry up to which a linear recurrence takes them in order on the vector units
+constexpr int kLinStep = 8;
+
+// The linear recurrence p of layer run r (its state and outputs are filled in here).  Entries of more rows than a
+// piece: end states and decays of the pieces from zero, a carry over each entry's pieces, then the outputs from the
+// states that enter them.
+static int enq_linrec(qie_batch* b, int r, lay::LinRecP p) {
+    const qie_engine* e = b->e;
+    LayeredBatch* s = b->lb;
+    p.entries = s->d_ent; p.n_entries = s->n_ent;
+    p.init = p.end = s->state;
+    p.init_stride = p.end_stride = s->slot_state;
+    p.init_off = p.end_off = s->state_off[r];
+    p.init_if_pos = 1;
+    p.out = s->olat;
+    if (s->max_count <= kLinStep || !lay::linrec_walk_fits(p.dim, p.vdim)) return lay::linrec_step(p, e->stream);
+    if (s->max_count <= s->lin.rows || !s->s_loc) return lay::linrec_walk(p, e->stream);
+    const int64_t n = (int64_t)p.heads * p.dim * p.vdim;
+    lay::LinRecP a = p;
+    a.entries = s->lin.d_chunks; a.n_entries = s->lin.n;
+    a.init = nullptr;
+    a.end = s->s_loc; a.end_stride = n; a.end_off = 0;
+    a.decay = s->s_decay;
+    a.out = nullptr;
+    QIE_TRY(lay::linrec_walk(a, e->stream));
+    lay::LinRecCarryP k{s->lin.d_spans, s->n_ent, p.heads, p.dim, p.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
+                        s->state_off[r]};
+    QIE_TRY(lay::linrec_carry(k, e->stream));
+    a.init = s->s_in; a.init_stride = n; a.init_off = 0; a.init_if_pos = 0;
+    a.end = nullptr; a.decay = nullptr;
+    a.out = p.out;
+    return lay::linrec_walk(a, e->stream);
+}
+
+// Gated linear attention of layer run r: log decays through the low-rank projection, the recurrence, head norm and gate
+static int enq_key_decay(qie_batch* b, int r, int T) {
+    const qie_engine* e = b->e;
+    const LayeredModel* m = e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    const qie_recurrent_desc& c = L.d.rec;
+    LayeredBatch* s = b->lb;
+    QIE_TRY(lay::low_rank_log_sigmoid(s->proj + L.col_a1, L.n_in, L.rank_a, L.w_a2, m->f32, L.rec_a2b, c.tau, c.heads * c.dim, T, s->qabs,
+                                      e->stream));
+    lay::LinRecP p{};
+    p.q = s->proj + L.col_rq; p.k = s->proj + L.col_rk; p.v = s->proj + L.col_rv;
+    p.ldq = p.ldk = p.ldv = L.n_in;
+    p.rep = 1;
+    p.q_scale = 1.0f / sqrtf((float)c.dim);
+    p.log_decay = s->qabs;
+    p.heads = c.heads; p.dim = c.dim; p.vdim = c.vdim;
+    QIE_TRY(enq_linrec(b, r, p));
+    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, s->ov, s->ov_bf, L.n_cat,
+                               L.cat_rec, e->stream, s->proj + L.col_rg, L.n_in, 1);
+}
+
+// State space of layer run r on its projection rows: convolution, recurrence, gate and norm in parts
+static int enq_state_space(qie_batch* b, int r, int T) {
+    const qie_engine* e = b->e;
+    const LayeredModel* m = e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    const qie_state_space_desc& c = L.d.ssm;
+    LayeredBatch* s = b->lb;
+    const int inner = c.heads * c.vdim, C = inner + 2 * c.groups * c.state;
+    lay::CausalConvP cv{};
+    cv.in = s->proj; cv.ld_in = L.n_in; cv.col = inner; cv.C = C; cv.taps = c.conv; cv.w = L.ss_conv; cv.bias = L.ss_conv_b;
+    cv.row_slot = s->row_slot; cv.row_pos = s->row_pos; cv.row_k = s->row_k;
+    cv.state = s->state; cv.slot_stride = s->slot_state; cv.state_off = s->conv_off[r];
+    cv.residual = 0; cv.silu = 1;
+    cv.out = s->pre; cv.ld_out = C; cv.out_bf = nullptr;
+    cv.entries = s->d_ent; cv.n_entries = s->n_ent;
+    QIE_TRY(lay::causal_conv_advance(cv, T, e->stream));
+    lay::LinRecP p{};
+    p.v = s->pre; p.k = s->pre + inner; p.q = p.k + c.groups * c.state;
+    p.ldq = p.ldk = p.ldv = C;
+    p.rep = c.heads / c.groups;
+    p.q_scale = 1.0f;
+    p.dt = s->proj + L.col_dt; p.ld_dt = L.n_in;
+    p.dt_bias = L.ss_dt_bias; p.a_h = L.ss_a; p.skip = L.ss_d;
+    p.heads = c.heads; p.dim = c.state; p.vdim = c.vdim;
+    QIE_TRY(enq_linrec(b, r, p));
+    return lay::gated_norm_parts(s->olat, s->proj, L.n_in, L.ss_norm, m->a.norm_eps, inner, c.norm_groups, T, s->ov, s->ov_bf, L.n_cat,
+                                 e->stream);
+}
+
 static int enq_recurrence(qie_batch* b, int r, int T) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     const qie_recurrent_desc& c = L.d.rec;
     LayeredBatch* s = b->lb;
+    if (c.kind == QIE_REC_KEY_DECAY) return enq_key_decay(b, r, T);
     lay::GatedScanP p{};
     p.proj = s->proj; p.ld = L.n_in; p.q_col = L.col_rq; p.f_col = L.col_rf; p.v_col = L.col_rv;
     p.entries = s->d_ent; p.n_entries = s->n_ent;
@@ -1093,11 +1282,11 @@ static int enq_recurrence(qie_batch* b, int r, int T) {
     if (s->max_count > kScanLong && s->s_loc) {
         const int64_t n = (int64_t)c.heads * c.dim * c.vdim;
         lay::GatedScanP a = p;       // pieces from zero states: local outputs, end states, gate products
-        a.entries = s->d_chunks; a.n_entries = s->n_chunks;
+        a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
         a.state = s->s_loc; a.slot_stride = n; a.state_off = 0;
         a.decay = s->s_decay;
         QIE_TRY(lay::gated_scan(a, e->stream));
-        lay::GatedCarryP k{s->d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
+        lay::GatedCarryP k{s->pieces.d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
                            s->state_off[r]};
         QIE_TRY(lay::gated_carry(k, e->stream));
         a.state = s->s_in;           // the incoming states' share of every row, summed in the head norm
@@ -1113,6 +1302,23 @@ static int enq_recurrence(qie_batch* b, int r, int T) {
                                L.cat_rec, e->stream);
 }
 
+// the layer's output product over the mixer's columns (parallel blocks: and the feed-forward's) -> s->mix
+static int enq_out(qie_batch* b, int r, int T) {
+    const LayeredModel* m = b->e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    LayeredBatch* s = b->lb;
+    return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
+}
+
+static int enq_state_space_mixer(qie_batch* b, int r, int T) {
+    const LayeredModel* m = b->e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    LayeredBatch* s = b->lb;
+    QIE_TRY(dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf));
+    QIE_TRY(enq_state_space(b, r, T));
+    return enq_out(b, r, T);
+}
+
 static int enq_gqa_mixer(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
@@ -1121,7 +1327,7 @@ static int enq_gqa_mixer(qie_batch* b, int r, int T) {
     QIE_TRY(enq_gqa_post(b, r, T));
     QIE_TRY(enq_gqa_attention(b, r, T));
     if (L.d.mixer == QIE_MIXER_GQA_RECURRENT) QIE_TRY(enq_recurrence(b, r, T));
-    return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
+    return enq_out(b, r, T);
 }
 
 // minGRU of layer run r: the scan over the fused projection rows -> s->ov (gated, with its bf16 image).
@@ -1138,17 +1344,17 @@ static int enq_mingru(qie_batch* b, int r, int T) {
     p.proj = s->proj; p.ld = L.n_in; p.z_col = 0; p.x_col = n; p.g_col = 2 * n;
     p.z_b = L.mg_zb; p.x_b = L.mg_xb;
     p.n = n;
-    p.out = s->ov; p.out_bf = s->ov_bf; p.ld_out = n;
+    p.out = s->ov; p.out_bf = s->ov_bf; p.ld_out = L.n_cat;
     if (s->max_count > kScanLong && s->s_loc) {
         lay::MinGruScanP a = p;
-        a.entries = s->d_chunks; a.n_entries = s->n_chunks;
+        a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
         a.out = nullptr; a.out_bf = nullptr;
         a.end = s->s_loc; a.decay = s->s_decay; a.end_stride = n; a.end_off = 0;
         QIE_TRY(lay::mingru_scan(a, e->stream));
-        lay::MinGruCarryP k{s->d_spans, s->n_ent, n, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state, s->state_off[r]};
+        lay::MinGruCarryP k{s->pieces.d_spans, s->n_ent, n, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state, s->state_off[r]};
         QIE_TRY(lay::mingru_carry(k, e->stream));
         a = p;
-        a.entries = s->d_chunks; a.n_entries = s->n_chunks;
+        a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
         a.init = s->s_in; a.init_stride = n; a.init_off = 0; a.init_if_pos = 0;
         return lay::mingru_scan(a, e->stream);
     }
@@ -1235,15 +1441,15 @@ static int enq_delta_scan(qie_batch* b, int r, int T, bool advance) {
         // queries), a carry over each entry's pieces, then the incoming states' share of every row
         const int64_t n = (int64_t)c.heads * c.dim * c.vdim;
         lay::DeltaScanP a = sp;
-        a.entries = s->d_chunks; a.n_entries = s->n_chunks;
+        a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
         a.state = s->s_loc; a.slot_stride = n; a.state_off = 0;
         a.read_state = 0; a.write_state = 1;
         a.trans = s->s_decay; a.w_out = s->dw;
         QIE_TRY(lay::delta_scan(a, e->stream));
-        lay::DeltaCarryP k{s->d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
+        lay::DeltaCarryP k{s->pieces.d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
                            s->state_off[r], advance ? 1 : 0};
         QIE_TRY(lay::delta_carry(k, e->stream));
-        lay::DeltaApplyP ap{s->d_chunks, s->n_chunks, kScanPiece, c.heads, c.dim, c.vdim, s->s_in, s->dw, s->olat};
+        lay::DeltaApplyP ap{s->pieces.d_chunks, s->pieces.n, kScanPiece, c.heads, c.dim, c.vdim, s->s_in, s->dw, s->olat};
         QIE_TRY(lay::delta_apply(ap, e->stream));
     } else {
         QIE_TRY(lay::delta_scan(sp, e->stream));
@@ -1305,6 +1511,7 @@ static int enq_run_prenorm(qie_batch* b, int r, int T, bool h_ready, bool* next_
         case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
         case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
         case QIE_MIXER_CHANNEL_DELTA: QIE_TRY(enq_delta_mixer(b, r, T)); break;
+        case QIE_MIXER_STATE_SPACE: QIE_TRY(enq_state_space_mixer(b, r, T)); break;
         default: QIE_TRY(enq_gqa_mixer(b, r, T)); break;
     }
     const bool has_ff = L.d.ff_kind != QIE_FF_NONE;
@@ -1366,6 +1573,41 @@ static int enq_run_sandwich(qie_batch* b, int r, int T, bool h_ready, bool* next
     return 0;
 }
 
+// Parallel blocks: x += mixer(N1(x)) + ff(N2(x)).  The stream x lives in plane 1 of the stack, the embedding rows stay in
+// plane 0 when a group repeats.  Both normed rows come from one kernel, which also takes the residual add before them
+// (and the embedding rows ahead of a repeated pass); gated dense feed-forwards share the mixer's output product.
+static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next_ready) {
+    const qie_engine* e = b->e;
+    const LayeredModel* m = e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    LayeredBatch* s = b->lb;
+    const int W = m->a.width;
+    const int64_t plane = s->cap * W;
+    float* x0 = s->stack;
+    float* x = s->stack + plane;
+    auto norms = [&](const float* xin, const float* v, const float* v2, const float* add, const LayerDev* N) -> int {
+        lay::NormPairP p{x, xin, v, v2, add, N ? N->n1 : nullptr, N ? N->n2 : nullptr, s->y, s->y2, s->y_bf, s->y2_bf, T, W, m->a.norm_eps};
+        return lay::norm_pair(p, e->stream);
+    };
+    if (!h_ready) QIE_TRY(norms(r == 0 && m->loops ? x0 : x, nullptr, nullptr, m->runs[r].add_embed ? x0 : nullptr, &L));
+    const bool has_ff = L.d.ff_kind != QIE_FF_NONE;
+    if (has_ff) QIE_TRY(enq_ff(b, m->runs[r].layer, T));
+    switch (L.d.mixer) {
+        case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
+        case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
+        case QIE_MIXER_CHANNEL_DELTA: QIE_TRY(enq_delta_mixer(b, r, T)); break;
+        case QIE_MIXER_STATE_SPACE: QIE_TRY(enq_state_space_mixer(b, r, T)); break;
+        default: QIE_TRY(enq_gqa_mixer(b, r, T)); break;
+    }
+    const bool last = r + 1 == (int)m->runs.size(), fuse_next = !last && !s->keep_on;
+    const LayerDev* N = fuse_next ? &m->L[m->runs[r + 1].layer] : nullptr;
+    QIE_TRY(norms(x, s->mix, has_ff && L.cat_ff < 0 ? s->ffo : nullptr, fuse_next && m->runs[r + 1].add_embed ? x0 : nullptr, N));
+    *next_ready = fuse_next;
+    if (s->keep_on && s->keep)
+        QIE_HIP(hipMemcpyAsync(s->keep + (int64_t)r * plane, x, (size_t)T * W * 4, hipMemcpyDeviceToDevice, e->stream));
+    return 0;
+}
+
 static int enq_layer(qie_batch* b, int i, const float* xin, const uint16_t* xin_bf, int T, const float** xout,
                      const uint16_t** xout_bf) {
     const qie_engine* e = b->e;
@@ -1406,7 +1648,7 @@ static int enq_forward(qie_batch* b, int T, int n_want) {
     LayeredBatch* s = b->lb;
     const int W = m->a.width;
     const float* x = s->stack;
-    const float w_one = m->a.block == QIE_BLOCK_PRENORM ? m->a.norm_offset : 1.f;
+    const float w_one = m->a.block == QIE_BLOCK_PRENORM ? m->a.norm_offset : m->a.block == QIE_BLOCK_PARALLEL ? 0.f : 1.f;
     if (m->a.block == QIE_BLOCK_PRENORM) {
         // one residual row: plane 1; several: planes 0 .. streams - 1, all equal to the embedding output
         const int n = m->a.streams;
@@ -1424,6 +1666,13 @@ static int enq_forward(qie_batch* b, int T, int n_want) {
         bool ready = false;
         for (int r = 0; r < (int)m->runs.size(); r++) QIE_TRY(enq_run_prenorm(b, r, T, ready, &ready));
         x = n > 0 ? s->x : xs;
+    } else if (m->a.block == QIE_BLOCK_PARALLEL) {
+        float* xs = s->stack + s->cap * W;
+        QIE_TRY(lay::embed_rows(m->embed, m->f32, s->tok, m->loops ? s->stack : xs, nullptr, T, W, m->a.vocab, e->stream, m->a.embed_scale,
+                                m->a.pos_embed == QIE_POS_SINUSOID ? s->row_pos : nullptr, m->pos_freq));
+        bool ready = false;
+        for (int r = 0; r < (int)m->runs.size(); r++) QIE_TRY(enq_run_parallel(b, r, T, ready, &ready));
+        x = xs;
     } else if (m->a.block == QIE_BLOCK_SANDWICH) {
         // the embedding rows stay in plane 0 only when a repeated group adds them again
         float* xs = s->stack + s->cap * W;
@@ -1456,14 +1705,15 @@ static void lb_free(LayeredBatch* s) {
     drop_graphs(s);   // captured launches hold these buffers' addresses
     void* ps[] = {s->stack, s->x, s->proj, s->qabs, s->olat, s->ov, s->mix, s->y, s->gu, s->act, s->ffo, s->xg, s->yd, s->score,
                   s->row_slot, s->row_pos, s->tok, s->sel, s->cnt, s->off, s->slot_of, s->keep, s->abf,
-                  s->x_bf, s->y_bf, s->ov_bf, s->act_bf, s->xg_bf, s->pre, s->aux, s->row_k, s->dw};
+                  s->x_bf, s->y_bf, s->ov_bf, s->act_bf, s->xg_bf, s->pre, s->aux, s->row_k, s->dw, s->y2, s->y2_bf};
     for (void* p : ps)
         if (p) hipFree(p);
     s->stack = s->x = s->proj = s->qabs = s->olat = s->ov = s->mix = s->y = s->gu = s->act = s->ffo = s->xg = s->yd = s->score =
         s->keep = nullptr;
     s->abf = s->x_bf = s->y_bf = s->ov_bf = s->act_bf = s->xg_bf = nullptr;
     s->row_slot = s->row_pos = s->tok = s->sel = s->cnt = s->off = s->slot_of = s->row_k = nullptr;
-    s->pre = s->aux = s->dw = nullptr;
+    s->pre = s->aux = s->dw = s->y2 = nullptr;
+    s->y2_bf = nullptr;
     s->cap = 0;
 }
 
@@ -1478,7 +1728,7 @@ static int run_forward(qie_batch* b, int T, int n_want) {
     for (const LayerDev& L : m->L)
         if (L.d.ff_kind == QIE_FF_MOE && (int64_t)T * L.d.top >= kMoeSyncRows) can = false;   // host round trip inside
     if (!can) return enq_forward(b, T, n_want);
-    std::vector<int> key{T, n_want, s->n_ent, s->n_qgroups};
+    std::vector<int> key{T, n_want, s->n_ent, s->n_qgroups, s->max_count > kLinStep};
     for (const auto& g : s->groups) {
         key.push_back(g.first);
         key.push_back(g.second.first);
@@ -1538,6 +1788,7 @@ static int ensure_rows(qie_batch* b, int64_t T) {
         A((void**)&s->ov, cap * s->m_hv);
         A((void**)&s->mix, cap * W);
         A((void**)&s->y, cap * W);
+        if (m->a.block == QIE_BLOCK_PARALLEL) A((void**)&s->y2, cap * W);
         A((void**)&s->gu, cap * std::max<int64_t>(s->m_gu, 1));
         A((void**)&s->act, cap * std::max<int64_t>(s->m_act, 1));
         A((void**)&s->ffo, cap * W);
@@ -1555,6 +1806,7 @@ static int ensure_rows(qie_batch* b, int64_t T) {
             A((void**)&s->abf, cap * s->m_abf + 64, 2);
             A((void**)&s->x_bf, cap * W, 2);
             A((void**)&s->y_bf, cap * W, 2);
+            if (m->a.block == QIE_BLOCK_PARALLEL) A((void**)&s->y2_bf, cap * W, 2);
             A((void**)&s->ov_bf, cap * s->m_hv, 2);
             A((void**)&s->act_bf, cap * std::max<int64_t>(s->m_act, 1), 2);
             A((void**)&s->xg_bf, cap * std::max<int64_t>(s->m_top, 1) * W, 2);
@@ -1599,6 +1851,49 @@ static int ensure_want(qie_batch* b, int64_t n) {
     b->samp_ws = nullptr;
     QIE_TRY(dmalloc(&b->samp_ws, (size_t)qie_sample_workspace_bytes(cap, V)));
     s->want_cap = cap;
+    return 0;
+}
+
+// Cuts the step's entries into pieces of `rows` rows, uploads the list and makes room for the pieces' states
+static int build_pieces(qie_batch* b, PieceList& L, int rows) {
+    LayeredBatch* s = b->lb;
+    hipStream_t st = b->e->stream;
+    L.rows = rows;
+    L.h_chunks.clear();
+    L.h_spans.clear();
+    for (const int4& en : s->h_ent) {
+        const int c0 = (int)L.h_chunks.size();
+        for (int k = 0; k < en.y; k += rows) L.h_chunks.push_back(int4{en.x + k, std::min(rows, en.y - k), (int)L.h_chunks.size(), 0});
+        L.h_spans.push_back(int4{c0, (int)L.h_chunks.size() - c0, en.z, en.w});
+    }
+    const int64_t nc = (int64_t)L.h_chunks.size(), ns = (int64_t)L.h_spans.size();
+    if (nc > L.cap || ns > L.span_cap || nc > s->scan_cap) {
+        QIE_HIP(hipStreamSynchronize(st));
+        const int64_t cap = (nc + 63) / 64 * 64, scap = std::max<int64_t>(b->B, ns);
+        void* ps[] = {L.d_chunks, L.d_spans};
+        for (void* q : ps)
+            if (q) hipFree(q);
+        L.d_chunks = L.d_spans = nullptr;
+        L.cap = L.span_cap = 0;
+        QIE_TRY(dmalloc((void**)&L.d_chunks, (size_t)cap * sizeof(int4)));
+        QIE_TRY(dmalloc((void**)&L.d_spans, (size_t)scap * sizeof(int4)));
+        L.cap = cap;
+        L.span_cap = scap;
+        if (nc > s->scan_cap) {
+            void* qs[] = {s->s_loc, s->s_in, s->s_decay};
+            for (void* q : qs)
+                if (q) hipFree(q);
+            s->s_loc = s->s_in = s->s_decay = nullptr;
+            s->scan_cap = 0;
+            QIE_TRY(dmalloc((void**)&s->s_loc, (size_t)cap * s->m_state * 4));
+            QIE_TRY(dmalloc((void**)&s->s_in, (size_t)cap * s->m_state * 4));
+            QIE_TRY(dmalloc((void**)&s->s_decay, (size_t)cap * s->m_hd * 4));
+            s->scan_cap = cap;
+        }
+    }
+    QIE_HIP(hipMemcpyAsync(L.d_chunks, L.h_chunks.data(), L.h_chunks.size() * sizeof(int4), hipMemcpyHostToDevice, st));
+    QIE_HIP(hipMemcpyAsync(L.d_spans, L.h_spans.data(), L.h_spans.size() * sizeof(int4), hipMemcpyHostToDevice, st));
+    L.n = (int)nc;
     return 0;
 }
 
@@ -1648,6 +1943,13 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
         s->m_vd = std::max<int64_t>(s->m_vd, d.gqa.vdim);
     }
     int64_t off = 0;
+    auto lin = [&](int64_t heads, int64_t dim, int64_t vdim) {   // a run on lay::linrec_*
+        const int64_t units = heads * ((vdim + 63) / 64);
+        s->lin_units = s->has_lin ? std::min(s->lin_units, units) : units;
+        s->has_lin = true;
+        s->m_state = std::max<int64_t>(s->m_state, heads * dim * vdim);
+        s->m_hd = std::max<int64_t>(s->m_hd, heads * dim);
+    };
     for (int r = 0; r < n_runs; r++) {
         const int i = m->runs[r].layer;
         const qie_layer_desc& d = m->L[i].d;
@@ -1670,9 +1972,25 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
             s->m_dw = std::max<int64_t>(s->m_dw, (int64_t)c.heads * c.dim);
             s->m_state = std::max<int64_t>(s->m_state, (int64_t)c.heads * c.dim * c.vdim);
             s->m_hd = std::max<int64_t>(s->m_hd, (int64_t)c.heads * c.dim * c.dim);
-            s->m_hv = std::max<int64_t>(s->m_hv, (int64_t)c.heads * c.vdim);
-            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)c.heads * c.vdim});
+            s->m_hv = std::max<int64_t>(s->m_hv, m->L[i].n_cat);
+            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)m->L[i].n_cat});
+            s->has_scan = true;
+        } else if (d.mixer == QIE_MIXER_STATE_SPACE) {
+            // no cache rows; per slot the heads' states and the convolution's last inputs
+            const qie_state_space_desc& c = d.ssm;
+            const int64_t inner = (int64_t)c.heads * c.vdim, C = inner + 2 * (int64_t)c.groups * c.state;
+            s->state_off[r] = s->slot_state;
+            s->slot_state += (int64_t)c.heads * c.state * c.vdim;
+            s->conv_off[r] = s->slot_state;
+            s->slot_state += (int64_t)(c.conv - 1) * C;
+            s->m_in = std::max<int64_t>(s->m_in, m->L[i].n_in);
+            s->m_pre = std::max<int64_t>(s->m_pre, C);
+            s->m_hr = std::max<int64_t>(s->m_hr, inner);
+            s->m_hv = std::max<int64_t>(s->m_hv, m->L[i].n_cat);
+            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)m->L[i].n_cat});
+            lin(c.heads, c.state, c.vdim);
         } else if (d.mixer == QIE_MIXER_MINGRU) {
+            s->has_scan = true;
             // no cache rows; `width` state elements per slot
             const int64_t n = d.mingru.width;
             s->state_off[r] = s->slot_state;
@@ -1680,8 +1998,8 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
             s->m_state = std::max<int64_t>(s->m_state, n);
             s->m_hd = std::max<int64_t>(s->m_hd, n);
             s->m_in = std::max<int64_t>(s->m_in, m->L[i].n_in);
-            s->m_hv = std::max<int64_t>(s->m_hv, n);
-            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, n});
+            s->m_hv = std::max<int64_t>(s->m_hv, m->L[i].n_cat);
+            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)m->L[i].n_cat});
         } else if (d.mixer != QIE_MIXER_LATENT_ATTENTION) {
             // K rows, then V rows of this run; one state per slot for the recurrence
             const qie_gqa_desc& a = d.gqa;
@@ -1693,6 +2011,12 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
             if (rv) {
                 s->state_off[r] = s->slot_state;
                 s->slot_state += (int64_t)d.rec.heads * d.rec.dim * d.rec.vdim;
+                if (d.rec.kind == QIE_REC_KEY_DECAY) {
+                    lin(d.rec.heads, d.rec.dim, d.rec.vdim);
+                    s->m_hr = std::max<int64_t>(s->m_hr, (int64_t)d.rec.heads * d.rec.dim);
+                } else {
+                    s->has_scan = true;
+                }
                 s->m_state = std::max<int64_t>(s->m_state, (int64_t)d.rec.heads * d.rec.dim * d.rec.vdim);
                 s->m_hd = std::max<int64_t>(s->m_hd, (int64_t)d.rec.heads * d.rec.dim);
             }
@@ -1778,7 +2102,8 @@ void layered_batch_destroy(qie_batch* b) {
     if (!s) return;
     lb_free(s);
     void* ps[] = {s->want, s->xn, s->logits, s->logits_bf, s->d_ids, s->d_step, s->d_groups, s->part_o, s->part_ml, s->xn_bf,
-                  s->state, s->d_ent, s->d_qgroups, s->gpart_o, s->gpart_ml, s->d_chunks, s->d_spans, s->s_loc, s->s_in, s->s_decay};
+                  s->state, s->d_ent, s->d_qgroups, s->gpart_o, s->gpart_ml, s->pieces.d_chunks, s->pieces.d_spans, s->lin.d_chunks, s->lin.d_spans, s->s_loc, s->s_in,
+                  s->s_decay};
     for (void* p : ps)
         if (p) hipFree(p);
     if (s->h_stage) hipHostFree(s->h_stage);
@@ -1804,20 +2129,21 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
                 "qie_engine_create_layered: invalid sizes");
     QIE_REQUIRE(!opts || !opts->tp_comm, "qie_engine_create_layered: layered engines run on one device");
     QIE_REQUIRE(!opts || (!opts->weight_fp8 && !opts->prefill_fp8), "qie_engine_create_layered: fp8 weights are not covered");
-    QIE_REQUIRE(arch->block >= QIE_BLOCK_POSTNORM_GAIN && arch->block <= QIE_BLOCK_PRENORM, "qie_engine_create_layered: block %d",
+    QIE_REQUIRE(arch->block >= QIE_BLOCK_POSTNORM_GAIN && arch->block <= QIE_BLOCK_PARALLEL, "qie_engine_create_layered: block %d",
                 arch->block);
     QIE_REQUIRE(arch->pos_embed == QIE_POS_NONE || arch->pos_embed == QIE_POS_SINUSOID, "qie_engine_create_layered: positions %d",
                 arch->pos_embed);
     QIE_REQUIRE((arch->pos_embed == QIE_POS_NONE && (arch->embed_scale == 0.f || arch->embed_scale == 1.f)) ||
-                    arch->block == QIE_BLOCK_PRENORM,
-                "qie_engine_create_layered: scaled embeddings and position vectors go with the pre-norm block");
+                    arch->block == QIE_BLOCK_PRENORM || arch->block == QIE_BLOCK_PARALLEL,
+                "qie_engine_create_layered: scaled embeddings and position vectors go with the pre-norm and parallel blocks");
     QIE_REQUIRE(arch->block == QIE_BLOCK_POSTNORM_GAIN || !arch->depth_mix,
                 "qie_engine_create_layered: depth-weighted residuals go with the post-norm block");
     const bool loops = arch->loop_times > 1 && arch->loop_stop > arch->loop_start;
     QIE_REQUIRE(!loops || (arch->loop_start >= 0 && arch->loop_stop <= arch->n_layers && arch->loop_times <= 64),
                 "qie_engine_create_layered: repeated group [%d, %d) x %d of %d layers", arch->loop_start, arch->loop_stop,
                 arch->loop_times, arch->n_layers);
-    QIE_REQUIRE(!loops || arch->block == QIE_BLOCK_SANDWICH, "qie_engine_create_layered: repeated groups go with the sandwich block");
+    QIE_REQUIRE(!loops || arch->block == QIE_BLOCK_SANDWICH || arch->block == QIE_BLOCK_PARALLEL,
+                "qie_engine_create_layered: repeated groups go with the sandwich and parallel blocks");
     QIE_REQUIRE(arch->streams >= 0 && arch->streams <= 32 && arch->canon_taps >= 0 && arch->canon_taps <= 64,
                 "qie_engine_create_layered: %d residual streams (at most 32), %d input taps (at most 64)", arch->streams, arch->canon_taps);
     QIE_REQUIRE(arch->block == QIE_BLOCK_PRENORM || (arch->streams == 0 && arch->canon_taps == 0 && !arch->embed_norm &&
@@ -1831,7 +2157,8 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
         QIE_REQUIRE(d.ff_kind != QIE_FF_MOE || (d.experts > 0 && d.top > 0 && d.top <= d.experts + std::max(d.identity, 0)),
                     "layer %d: %d of %d experts", i, d.top, d.experts + std::max(d.identity, 0));
         QIE_REQUIRE(d.router >= QIE_ROUTER_SIGMOID_IN && d.router <= QIE_ROUTER_SOFTMAX_ALL, "layer %d: router %d", i, d.router);
-        QIE_REQUIRE(d.ff_act >= QIE_ACT_SILU_GATED && d.ff_act <= QIE_ACT_GELU_TANH_GATED, "layer %d: activation %d", i, d.ff_act);
+        QIE_REQUIRE(d.ff_act >= QIE_ACT_SILU_GATED && d.ff_act <= QIE_ACT_CLAMPED_GATED, "layer %d: activation %d", i, d.ff_act);
+        const bool pre = arch->block == QIE_BLOCK_PRENORM || arch->block == QIE_BLOCK_PARALLEL;
         if (d.ff_kind == QIE_FF_MOE && d.router == QIE_ROUTER_SOFTMAX_ALL) {
             const int n = d.experts + d.identity;
             QIE_REQUIRE(d.identity >= 0 && d.groups >= 1 && n % d.groups == 0 && d.groups_keep >= 1 && d.groups_keep <= d.groups &&
@@ -1842,13 +2169,22 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
             QIE_REQUIRE(d.identity == 0, "layer %d: identity experts go with the grouped softmax router", i);
         }
         if (d.mixer == QIE_MIXER_MINGRU) {
-            QIE_REQUIRE(arch->block == QIE_BLOCK_PRENORM, "layer %d: this mixer is wired to the pre-norm block", i);
+            QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
             QIE_REQUIRE(d.mingru.width > 0, "layer %d: minGRU width", i);
+            continue;
+        }
+        if (d.mixer == QIE_MIXER_STATE_SPACE) {
+            const qie_state_space_desc& c = d.ssm;
+            QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
+            QIE_REQUIRE(c.heads > 0 && c.vdim > 0 && c.state > 0 && c.state <= 512 && c.groups > 0 && c.heads % c.groups == 0 &&
+                            c.norm_groups > 0 && (c.heads * c.vdim) % c.norm_groups == 0 && c.conv >= 1 && c.conv <= 64,
+                        "layer %d: state space with %d heads of %d in %d groups, state %d (at most 512), %d taps, a norm in %d parts", i,
+                        c.heads, c.vdim, c.groups, c.state, c.conv, c.norm_groups);
             continue;
         }
         if (d.mixer == QIE_MIXER_CHANNEL_DELTA) {
             const qie_delta_desc& c = d.delta;
-            QIE_REQUIRE(arch->block == QIE_BLOCK_PRENORM, "layer %d: this mixer is wired to the pre-norm block", i);
+            QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
             QIE_REQUIRE(c.heads > 0 && c.kv_heads > 0 && c.heads % c.kv_heads == 0 && c.dim > 0 && c.dim <= 512 && c.vdim > 0 &&
                             c.conv >= 1 && c.conv <= 64 && c.rank_a >= 0 && c.rank_g >= 0,
                         "layer %d: delta rule with %d heads over %d key heads of %d (at most 512) / %d, %d taps", i, c.heads, c.kv_heads,
@@ -1857,8 +2193,12 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
         }
         if (d.mixer == QIE_MIXER_GQA || d.mixer == QIE_MIXER_GQA_RECURRENT) {
             const qie_gqa_desc& a = d.gqa;
-            QIE_REQUIRE(arch->block == QIE_BLOCK_SANDWICH || (arch->block == QIE_BLOCK_PRENORM && d.mixer == QIE_MIXER_GQA),
-                        "layer %d: this mixer is wired to the sandwich block (alone: also the pre-norm block)", i);
+            QIE_REQUIRE(arch->block == QIE_BLOCK_SANDWICH || arch->block == QIE_BLOCK_PARALLEL ||
+                            (arch->block == QIE_BLOCK_PRENORM && d.mixer == QIE_MIXER_GQA),
+                        "layer %d: this mixer is wired to the sandwich and parallel blocks (alone: also the pre-norm block)", i);
+            QIE_REQUIRE(a.mask_keep >= 0 && (a.mask_keep == 0 || a.mask == QIE_MASK_WINDOW), "layer %d: %d kept first keys go with the window mask",
+                        i, a.mask_keep);
+            QIE_REQUIRE(!a.v_bias || !a.values_are_keys, "layer %d: keys as values carry the key's bias", i);
             QIE_REQUIRE(a.weights == QIE_WEIGHTS_SOFTMAX || a.weights == QIE_WEIGHTS_SIGMOID, "layer %d: attention weights %d", i,
                         a.weights);
             QIE_REQUIRE(a.q_temp_every >= 0, "layer %d: query temperature every %d", i, a.q_temp_every);
@@ -1880,12 +2220,15 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
                                                         a.rot_scaling.low >= 0.f && a.rot_scaling.original > 0.f),
                         "layer %d: rotary scaling", i);
             if (d.mixer == QIE_MIXER_GQA_RECURRENT)
-                QIE_REQUIRE(d.rec.heads > 0 && d.rec.dim > 0 && d.rec.dim <= 512 && d.rec.vdim > 0, "layer %d: recurrence sizes", i);
+                QIE_REQUIRE(d.rec.heads > 0 && d.rec.dim > 0 && d.rec.dim <= 512 && d.rec.vdim > 0 &&
+                                (d.rec.kind == QIE_REC_LOWER_BOUND || (d.rec.kind == QIE_REC_KEY_DECAY && d.rec.tau > 0.f && d.rec.rank >= 0)),
+                            "layer %d: recurrence sizes", i);
             continue;
         }
         QIE_REQUIRE(d.mixer == QIE_MIXER_LATENT_ATTENTION, "layer %d: unknown mixer %d", i, d.mixer);
-        QIE_REQUIRE(arch->block == QIE_BLOCK_POSTNORM_GAIN || arch->block == QIE_BLOCK_PRENORM,
-                    "layer %d: latent attention is wired to the post-norm and pre-norm blocks", i);
+        QIE_REQUIRE(arch->block == QIE_BLOCK_POSTNORM_GAIN || pre,
+                    "layer %d: latent attention is wired to the post-norm, pre-norm and parallel blocks", i);
+        QIE_REQUIRE(!loops, "layer %d: latent attention in a model with a repeated group", i);
         QIE_REQUIRE(d.heads > 0 && d.dim > 0 && d.rot_dim >= 0 && d.vdim > 0 && d.kv_rank > 0 && d.window >= 0 && d.q_rank >= 0,
                     "layer %d: invalid mixer sizes", i);
         QIE_REQUIRE(d.rot_layout == QIE_ROT_HALVES || d.rot_layout == QIE_ROT_INTERLEAVED, "layer %d: rotary layout %d", i, d.rot_layout);
@@ -1984,12 +2327,13 @@ int qie_engine_finalize_weights(qie_engine* e) {
         QIE_HIP(hipMemcpy(m->pos_freq, fr.data(), fr.size() * 8, hipMemcpyHostToDevice));
     }
     if (m->a.embed_norm) QIE_TRY(lm_vector(m, &m->w_embed, "embed.norm", W));
-    if (m->a.block == QIE_BLOCK_SANDWICH || m->a.block == QIE_BLOCK_PRENORM) {
+    if (m->a.block != QIE_BLOCK_POSTNORM_GAIN) {
         QIE_TRY(lm_vector(m, &m->w_final, "final.norm", W));
     } else {
         LM_GET(tn, "final.norm");
         m->g_final = host_elem(*tn, 0);
     }
+    if (m->a.logit_scale != 0.f) m->g_final *= m->a.logit_scale;   // the head is linear: its input carries the scale
     for (int i = 0; i < m->a.n_layers; i++) QIE_TRY(finalize_layer(e, m, i));
     m->host.clear();
     m->final = true;
@@ -2074,35 +2418,12 @@ int qie_batch_step(qie_batch* b, int32_t n_entries, const int32_t* slots, const 
         s->n_qgroups = (int)s->h_qgroups.size();
         s->max_count = 0;
         for (int i = 0; i < n_entries; i++) s->max_count = std::max(s->max_count, (int)counts[i]);
-        if (s->slot_state > 0 && s->max_count > kScanLong) {
-            s->h_chunks.clear();
-            s->h_spans.clear();
-            for (const int4& en : s->h_ent) {
-                const int c0 = (int)s->h_chunks.size();
-                for (int k = 0; k < en.y; k += kScanPiece)
-                    s->h_chunks.push_back(int4{en.x + k, std::min(kScanPiece, en.y - k), (int)s->h_chunks.size(), 0});
-                s->h_spans.push_back(int4{c0, (int)s->h_chunks.size() - c0, en.z, en.w});
-            }
-            const int64_t nc = (int64_t)s->h_chunks.size();
-            if (nc > s->chunks_cap || nc > s->scan_cap) {
-                QIE_HIP(hipStreamSynchronize(st));
-                void* ps[] = {s->d_chunks, s->d_spans, s->s_loc, s->s_in, s->s_decay};
-                for (void* q : ps)
-                    if (q) hipFree(q);
-                s->d_chunks = s->d_spans = nullptr;
-                s->s_loc = s->s_in = s->s_decay = nullptr;
-                s->chunks_cap = s->scan_cap = 0;
-                const int64_t cap = (nc + 63) / 64 * 64;
-                QIE_TRY(dmalloc((void**)&s->d_chunks, (size_t)cap * sizeof(int4)));
-                QIE_TRY(dmalloc((void**)&s->d_spans, (size_t)std::max<int64_t>(b->B, n_entries) * sizeof(int4)));
-                QIE_TRY(dmalloc((void**)&s->s_loc, (size_t)cap * s->m_state * 4));
-                QIE_TRY(dmalloc((void**)&s->s_in, (size_t)cap * s->m_state * 4));
-                QIE_TRY(dmalloc((void**)&s->s_decay, (size_t)cap * s->m_hd * 4));
-                s->chunks_cap = s->scan_cap = cap;
-            }
-            QIE_HIP(hipMemcpyAsync(s->d_chunks, s->h_chunks.data(), s->h_chunks.size() * sizeof(int4), hipMemcpyHostToDevice, st));
-            QIE_HIP(hipMemcpyAsync(s->d_spans, s->h_spans.data(), s->h_spans.size() * sizeof(int4), hipMemcpyHostToDevice, st));
-            s->n_chunks = (int)nc;
+        if (s->has_scan && s->max_count > kScanLong) QIE_TRY(build_pieces(b, s->pieces, kScanPiece));
+        if (s->has_lin) {
+            // linear recurrences: long pieces (less state traffic) as long as two blocks a CU remain
+            const int64_t want = T * s->lin_units / 512;
+            s->lin.rows = want >= 512 ? 512 : want >= 256 ? 256 : 128;
+            if (s->max_count > s->lin.rows) QIE_TRY(build_pieces(b, s->lin, s->lin.rows));
         }
     }
     QIE_HIP(hipMemcpyAsync(s->row_slot, hs, (size_t)T * 4, hipMemcpyHostToDevice, st));
@@ -2189,9 +2510,10 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
     int rc = 0;
     const bool gqa = which != 0 && m->L[layer].d.mixer != QIE_MIXER_LATENT_ATTENTION;
     QIE_REQUIRE(which != 4 || m->L[layer].d.mixer == QIE_MIXER_GQA_RECURRENT || m->L[layer].d.mixer == QIE_MIXER_MINGRU ||
-                    m->L[layer].d.mixer == QIE_MIXER_CHANNEL_DELTA,
+                    m->L[layer].d.mixer == QIE_MIXER_CHANNEL_DELTA || m->L[layer].d.mixer == QIE_MIXER_STATE_SPACE,
                 "qie_batch_time_stage: layer %d has no recurrence", layer);
-    QIE_REQUIRE(which != 1 || (m->L[layer].d.mixer != QIE_MIXER_MINGRU && m->L[layer].d.mixer != QIE_MIXER_CHANNEL_DELTA),
+    QIE_REQUIRE(which != 1 || (m->L[layer].d.mixer != QIE_MIXER_MINGRU && m->L[layer].d.mixer != QIE_MIXER_CHANNEL_DELTA &&
+                               m->L[layer].d.mixer != QIE_MIXER_STATE_SPACE),
                 "qie_batch_time_stage: layer %d has no attention", layer);
     int run = 0;   // the layer's first run
     while (which != 0 && m->runs[run].layer != layer) run++;
@@ -2207,7 +2529,7 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
                 default: return enq_delta_scan(b, run, T, false);
             }
         }
-        if (!gqa && which != 0 && m->a.block == QIE_BLOCK_PRENORM) {   // latent attention on the branch input s->y
+        if (!gqa && which != 0 && m->a.block != QIE_BLOCK_POSTNORM_GAIN) {   // latent attention on the branch input s->y
             switch (which) {
                 case 1: return enq_attention(b, layer, T);
                 case 2:
@@ -2225,7 +2547,10 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
                     QIE_TRY(enq_gqa_proj(b, run, T));
                     return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
                 case 3: return enq_ff(b, layer, T);
-                default: return L.d.mixer == QIE_MIXER_MINGRU ? enq_mingru(b, run, T) : enq_recurrence(b, run, T);
+                default:
+                    return L.d.mixer == QIE_MIXER_MINGRU        ? enq_mingru(b, run, T)
+                           : L.d.mixer == QIE_MIXER_STATE_SPACE ? enq_state_space(b, run, T)
+                                                                : enq_recurrence(b, run, T);
             }
         }
         switch (which) {

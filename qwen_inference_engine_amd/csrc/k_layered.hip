@@ -559,21 +559,32 @@ int depth_mix(const float* stack, int64_t stride, const float* a, int n, float* 
 
 // ------------------------------------------------------------------ gated activation
 // a[m, j] = silu(gu[m, j]) * gu[m, ff + j]
-// (act 1: the tanh form of gelu instead of silu, gelu(g) = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))))
-__global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a, uint16_t* a_bf, int ff, int64_t n, int act) {
+// (act 1: the tanh form of gelu instead of silu, gelu(g) = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)));
+// act 2: g sigmoid(1.702 g) (u + 1) with the gate cut at limit and u clamped to +-limit)
+__global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a, uint16_t* a_bf, int ff, int64_t n, int act, float limit,
+                                                       int64_t ld_a) {
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= n) return;
     const int64_t m = i / ff;
     const int j = (int)(i % ff);
     const float g = gu[m * 2 * ff + j], u = gu[m * 2 * ff + ff + j];
+    const int64_t oi = m * ld_a + j;
+    if (act == 2) {
+        const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit);
+        const float oc = gc / (1.0f + expf(-1.702f * gc)) * (uc + 1.0f);
+        a[oi] = oc;
+        if (a_bf) a_bf[oi] = f2bf(oc);
+        return;
+    }
     const float o = (act == 1 ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g))) * u;
-    a[i] = o;
-    if (a_bf) a_bf[i] = f2bf(o);
+    a[oi] = o;
+    if (a_bf) a_bf[oi] = f2bf(o);
 }
-int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act) {
+int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act, float limit, int64_t ld_a) {
     const int64_t n = M * ff;
     if (n == 0) return 0;
-    hipLaunchKernelGGL(silu_mul_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, gu, a, a_bf, ff, n, act);
+    hipLaunchKernelGGL(silu_mul_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, gu, a, a_bf, ff, n, act,
+                       limit, ld_a ? ld_a : (int64_t)ff);
     QIE_LAUNCH_CHECK();
     return 0;
 }

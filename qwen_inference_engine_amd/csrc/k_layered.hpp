@@ -135,11 +135,13 @@ struct GqaPostP {
     float q_temp_coef;
     const float* q_bias;      // [heads * dim] / [kv_heads * dim] or null: added to q / k as they leave the projection
     const float* k_bias;      //   (a key cached as the value carries its bias)
+    const float* v_bias;      // [kv_heads * vdim] or null: added to v as it leaves the projection
 };
 int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st);
 
 // Softmax attention of every (row, head) over the keys its mask lets it see (mask 0: all j <= i;
-// 1: the last mask_size; 2: those with j / mask_size == i / mask_size); score = q.k * scale
+// 1: the last mask_size and, of the earlier ones, the first mask_keep of the sequence; 2: those with
+// j / mask_size == i / mask_size); score = q.k * scale
 // - r1[h] * ln(1 + r2[h] * (i - j)) when r1 is set.  rot_values: the weighted sum is turned back
 // by the row's position.  The result times out_scale goes to out[t * ld_out + out_col + h * vdim
 // ...] (and its bf16 image).
@@ -171,6 +173,7 @@ struct GqaAttnP {
     int gate_col;             // >= 0: head h's result times sigmoid(proj[t * ld + gate_col + h])
     int gate_elem;            // with gate_col: one gate per coordinate, proj[t * ld + gate_col + h * vdim + c]
     const float* sink;        // [heads] or null: exp(sink[h]) joins the softmax denominator (no key, no value)
+    int mask_keep;            // mask 1 only, else 0
 };
 int gqa_attention(const GqaAttnP& p, bool cache_f32, int T, hipStream_t st);
 // The matrix-core form for bf16 caches whose V rows are stored transposed (v_transposed: inside a
@@ -283,9 +286,27 @@ struct MinGruCarryP {
 };
 int mingru_carry(const MinGruCarryP& p, hipStream_t st);
 
-// gate (optional, [T][heads * vdim]): the result is also multiplied by sigmoid(gate[t, h * vdim + c])
+// gate (optional): the result is also multiplied by sigmoid(gate[t * ld_gate + h * vdim + c]), or silu of it
+// (gate_silu); ld_gate 0: heads * vdim
 int head_norm_rows(const float* o, const float* o2, const float* w, float eps, float scale, int heads, int vdim, int T, float* out,
-                   uint16_t* out_bf, int64_t ld_out, int out_col, hipStream_t st, const float* gate = nullptr);
+                   uint16_t* out_bf, int64_t ld_out, int out_col, hipStream_t st, const float* gate = nullptr, int64_t ld_gate = 0,
+                   int gate_silu = 0);
+// out[t, c] = y[t, c] * silu(z[t * ld_z + c]), then every one of `parts` equal parts of the n columns divided by its
+// root mean square and multiplied by w[c] (with its bf16 image)
+int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* w, float eps, int n, int parts, int T, float* out,
+                     uint16_t* out_bf, int64_t ld_out, hipStream_t st);
+// Rows of W, two norms of one row: x = xin + v (when v) + v2 (when v2) + add (when add); h1 = rms(x) w1, h2 = rms(x) w2
+// (each with its bf16 image; null w1: neither norm is made, null w2: only the first)
+struct NormPairP {
+    float* x;
+    const float *xin, *v, *v2, *add;
+    const float *w1, *w2;
+    float *h1, *h2;
+    uint16_t *h1_bf, *h2_bf;
+    int T, W;
+    float eps;
+};
+int norm_pair(const NormPairP& p, hipStream_t st);
 
 // ------------------------------------------------------------------ residual streams (k_streams.hip)
 // n residual rows per token, X + s * plane (rows of W).  With y (a sublayer's result, [T][W]) the rows
@@ -309,7 +330,7 @@ struct StreamStepP {
 };
 int stream_step(const StreamStepP& p, hipStream_t st);
 
-// Causal convolution over time per channel on the packed rows of a step: out[t, c] =
+// Causal convolution over time per channel on the packed rows of a step: out[t, c] = (bias ? bias[c] : 0) +
 // (residual ? in[t, c] : 0) + sum_j w[c * taps + j] in[t - (taps - 1 - j), c], then silu when asked.
 // Rows before an entry's first come from the slot's state ([taps - 1][C] floats at state + slot *
 // slot_stride + state_off: the inputs at the taps - 1 positions before the entry, oldest first), rows
@@ -332,6 +353,7 @@ struct CausalConvP {
     uint16_t* out_bf;
     const int4* entries;
     int n_entries;
+    const float* bias;    // [C] or null
 };
 int causal_conv(const CausalConvP& p, int T, hipStream_t st);
 int causal_conv_state(const CausalConvP& p, hipStream_t st);
@@ -408,6 +430,56 @@ struct DeltaApplyP {
     float* out;
 };
 int delta_apply(const DeltaApplyP& p, hipStream_t st);
+// ------------------------------------------------------------------ decayed linear recurrences (k_linrec.hip)
+// Per entry {first packed row, rows, slot (or piece), first position} and head h, the fp32 state S [dim][vdim] at
+// state + index * stride + off + h * dim * vdim walks the rows in order:
+//   S = diag(a) S + m k v^T,  o = q_scale S^T q (+ skip[h] v)  ->  out[t * heads * vdim + h * vdim + c]
+// q(t, h) = q + t ldq + (h / rep) dim, k alike (rep heads share a q / k row), v(t, h) = v + t ldv + h vdim.
+// log_decay set: a = exp(log_decay[t * heads * dim + h dim + d]), m = 1.  dt set: one decay per head,
+// dt_h = softplus(dt[t ld_dt + h] + dt_bias[h]), a = exp(-a_h[h] dt_h), m = dt_h.
+// An entry whose first position is 0 starts from S = 0 (init_if_pos), else from the state at init.
+struct LinRecP {
+    const float *q, *k, *v;
+    int64_t ldq, ldk, ldv;
+    int rep;
+    float q_scale;
+    const float* log_decay;
+    const float* dt;
+    int64_t ld_dt;
+    const float *dt_bias, *a_h, *skip;
+    int heads, dim, vdim;
+    const int4* entries;
+    int n_entries;
+    const float* init;        // null: every entry starts from zero
+    int64_t init_stride, init_off;
+    int init_if_pos;
+    float* end;               // null: the state after the last row is not kept
+    int64_t end_stride, end_off;
+    float* decay;             // optional [entries][heads * dim]: the product of the entry's decays
+    float* out;               // null: only end and decay are wanted
+};
+// Rows in order on the vector units: entries of few rows (any dim up to 512)
+int linrec_step(const LinRecP& p, hipStream_t st);
+// 16 rows at a time on the fp32 matrix cores, the state in registers (dim up to 256)
+bool linrec_walk_fits(int dim, int vdim);
+int linrec_walk(const LinRecP& p, hipStream_t st);
+// Walks every entry's pieces (spans {first piece, pieces, slot, first position}): s_in[c] = the state entering piece
+// c, from the slot's state (zero at position 0) through s <- decay[c] s + s_loc[c]; the slot's state = what leaves
+// the last piece.
+struct LinRecCarryP {
+    const int4* spans;
+    int n_spans;
+    int heads, dim, vdim;
+    const float *s_loc, *decay;
+    float* s_in;
+    float* state;
+    int64_t slot_stride, state_off;
+};
+int linrec_carry(const LinRecCarryP& p, hipStream_t st);
+// out[t, c] = log(sigmoid(z)) / tau, z = sum_r w[c * rank + r] in[t * ld_in + r] + bias[c]; c < n
+int low_rank_log_sigmoid(const float* in, int64_t ld_in, int rank, const void* w, bool w_f32, const float* bias, float tau, int n, int T,
+                         float* out, hipStream_t st);
+
 // Rows of W: x = xin + (wb ? rms(v) * (w_one + wb) : v) (when v) + add (when add); then (when wn)
 // h = rms(x) * (w_one + wn) with its bf16 image.  xin may be x.  w_one = 1: weight vectors stored
 // around zero; 0: plain weights.
@@ -428,8 +500,10 @@ int postnorm_add(const float* x, const float* v, float* y, uint16_t* y_bf, int T
 int final_rows(const float* x, const int32_t* rows, float* out, uint16_t* out_bf, int n, int W, float gain, const float* w1p,
                float eps, hipStream_t st, float w_one = 1.0f);
 int depth_mix(const float* stack, int64_t stride, const float* a, int n, float* x, uint16_t* x_bf, int64_t count, hipStream_t st);
-// a[m, j] = act(gu[m, j]) * gu[m, ff + j]; act 0: silu, 1: the tanh form of gelu
-int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act = 0);
+// a[m * ld_a + j] = act(gu[m, j]) * gu[m, ff + j]; act 0: silu, 1: the tanh form of gelu, 2: g sigmoid(1.702 g) (u + 1)
+// with g = min(gu[m, j], limit), u = gu[m, ff + j] clamped to +-limit; ld_a 0: ff
+int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act = 0, float limit = 0.f,
+             int64_t ld_a = 0);
 // a = ap u^2 + u / 2 where u > 0, else aq (exp(u) - 1 - u) + u / 2; n elements
 int xielu(const float* u, float* a, uint16_t* a_bf, int64_t n, float ap, float aq, hipStream_t st);
 // mode 0: score = sigmoid(z) of the `top` largest z = W_r y; mode 1: z = W_r y + bias, score = the

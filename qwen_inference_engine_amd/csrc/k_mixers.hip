@@ -148,7 +148,7 @@ __global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p) {
         const int g = g0 + wave;
         const bool on = g < G;
         if (on)
-            for (int i = lane; i < vdim; i += 64) buf[i] = row[p.v_col + g * vdim + i];
+            for (int i = lane; i < vdim; i += 64) buf[i] = row[p.v_col + g * vdim + i] + (p.v_bias ? p.v_bias[g * vdim + i] : 0.f);
         __syncthreads();
         if (on)
             for (int i = lane; i < vdim; i += 64)
@@ -206,10 +206,13 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
     // a sink is a score without key or value: the running maximum and sum start from it
     float m_run = p.sink ? p.sink[h] : -INFINITY, l_run = p.sink ? 1.f : 0.f;
     float acc[GA_MAXV] = {};
-    for (int j0 = lo; j0 <= pos; j0 += GA_CHUNK) {
-        const int nk = min(GA_CHUNK, pos + 1 - j0);
+    // the visible keys in order: the kept first ones that lie before the window, then the window's
+    const int kept = min(p.mask_keep, lo), n_vis = kept + pos + 1 - lo;
+    auto key_of = [&](int i) { return i < kept ? i : lo + i - kept; };
+    for (int j0 = 0; j0 < n_vis; j0 += GA_CHUNK) {
+        const int nk = min(GA_CHUNK, n_vis - j0);
         for (int jj = wave; jj < nk; jj += 4) {
-            const int j = j0 + jj;
+            const int j = key_of(j0 + jj);
             const TC* k = (const TC*)p.cache.pool + page_base(p.cache, slot, j) + p.k_off +
                           ((int64_t)(j % p.cache.page_tokens) * G + g) * dim;
             float s = 0.f;
@@ -225,7 +228,7 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
         __syncthreads();
         if (sig) {   // the weights are final: no running maximum, no normalisation
             for (int jj = 0; jj < nk; jj++) {
-                const int j = j0 + jj;
+                const int j = key_of(j0 + jj);
                 const int pt = j % p.cache.page_tokens;
                 const TC* v = (const TC*)p.cache.pool + page_base(p.cache, slot, j) + p.v_off;
                 const float w = sc[jj];
@@ -261,7 +264,7 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
 #pragma unroll
         for (int i = 0; i < GA_MAXV; i++) acc[i] *= alpha;
         for (int jj = 0; jj < nk; jj++) {
-            const int j = j0 + jj;
+            const int j = key_of(j0 + jj);
             const int pt = j % p.cache.page_tokens;
             const TC* v = (const TC*)p.cache.pool + page_base(p.cache, slot, j) + p.v_off;
             const float w = sc[jj];
@@ -300,6 +303,7 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
 int gqa_attention(const GqaAttnP& p, bool cache_f32, int T, hipStream_t st) {
     QIE_REQUIRE(p.vdim <= 256 * GA_MAXV, "gqa attention: vdim %d above %d", p.vdim, 256 * GA_MAXV);
     QIE_REQUIRE(p.mask == 0 || p.mask_size >= 1, "gqa attention: mask size %d", p.mask_size);
+    QIE_REQUIRE(p.mask_keep >= 0 && (p.mask_keep == 0 || p.mask == 1), "gqa attention: kept first keys go with the window mask");
     QIE_REQUIRE(p.heads % p.kv_heads == 0, "gqa attention: %d query heads over %d key heads", p.heads, p.kv_heads);
     const size_t shm = (size_t)(p.dim + GA_CHUNK + p.vdim) * 4;
     QIE_REQUIRE(shm <= 48 * 1024, "gqa attention: head size above the kernel's staging");
@@ -445,9 +449,11 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
     }
     const int lo_q = first_visible(a.mask, a.mask_size, qpos);
     const int kmin = first_visible(a.mask, a.mask_size, pos0), kmax = pos0 + n_tok - 1;
-    const int b0 = kmin >> 5, nb = (kmax >> 5) - b0 + 1;
+    // 32-key blocks: those of the kept first keys that lie before the window's first block, then the window's
+    const int b0 = kmin >> 5, nk0 = min((a.mask_keep + 31) >> 5, b0), nb = nk0 + (kmax >> 5) - b0 + 1;
     const int S = P.S, z = blockIdx.z;
-    const int bs = b0 + (int)((int64_t)nb * z / S), be = b0 + (int)((int64_t)nb * (z + 1) / S);
+    const int bs = (int)((int64_t)nb * z / S), be = (int)((int64_t)nb * (z + 1) / S);
+    auto block_of = [&](int i) { return i < nk0 ? i : b0 + i - nk0; };
     const float b1 = a.r1 ? a.r1[hh] : 0.f, b2 = a.r1 ? a.r2[hh] : 0.f;
     const float slope = a.slopes ? a.slopes[hh] : 0.f;
     const bool sig = a.pb != nullptr;   // sigmoid weights: final as computed, no running maximum or sum
@@ -504,11 +510,11 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
         }
     };
     if (bs < be) {
-        if (SHARE) fetch_tiles(bs);
-        else load_k(bs, kf);
+        if (SHARE) fetch_tiles(block_of(bs));
+        else load_k(block_of(bs), kf);
     }
     for (int kb = bs; kb < be; kb++) {
-        const int key0 = kb << 5;
+        const int key0 = block_of(kb) << 5;
         const int64_t pb = (int64_t)tab[key0 / PT] * a.cache.page_stride;
         const int tok0 = key0 % PT;
         uint2 vf[DV][2];
@@ -516,7 +522,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
             __syncthreads();   // the previous tiles have been read
             store_tiles();
             __syncthreads();
-            if (kb + 1 < be) fetch_tiles(kb + 1);
+            if (kb + 1 < be) fetch_tiles(block_of(kb + 1));
 #pragma unroll
             for (int tt = 0; tt < 2; tt++)
 #pragma unroll
@@ -533,7 +539,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
                 vf[dv][0] = *reinterpret_cast<const uint2*>(vr + (int64_t)16 * dv * PT);
                 vf[dv][1] = *reinterpret_cast<const uint2*>(vr + (int64_t)16 * dv * PT + 16);
             }
-            if (kb + 1 < be) load_k(kb + 1, kn);
+            if (kb + 1 < be) load_k(block_of(kb + 1), kn);
         }
         gf32x4_t sacc[2];
 #pragma unroll
@@ -549,7 +555,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
 #pragma unroll
         for (int e = 0; e < 8; e++) {
             const int kj = key0 + 16 * (e >> 2) + 4 * g + (e & 3);
-            vis[e] = valid && kj >= lo_q && kj <= qpos;
+            vis[e] = valid && kj <= qpos && (kj >= lo_q || kj < a.mask_keep);
             float x = sacc[e >> 2][e & 3] * a.scale;
             if (a.r1) x -= b1 * __logf(1.0f + b2 * (float)max(qpos - kj, 0));
             x -= slope * (float)max(qpos - kj, 0);
@@ -688,6 +694,7 @@ int gqa_attention_mfma(const GqaAttnMfmaP& p, hipStream_t st) {
                 "gqa attention: sizes %d / %d, pages of %d tokens do not fit the matrix-core form", a.dim, a.vdim, a.cache.page_tokens);
     QIE_REQUIRE(p.n_groups > 0 && p.S >= 1 && (p.S == 1 || (p.part_o && p.part_ml)), "gqa attention: bad launch");
     QIE_REQUIRE(a.heads % a.kv_heads == 0, "gqa attention: %d query heads over %d key heads", a.heads, a.kv_heads);
+    QIE_REQUIRE(a.mask_keep >= 0 && (a.mask_keep == 0 || a.mask == 1), "gqa attention: kept first keys go with the window mask");
     QIE_REQUIRE(p.pack == ((a.heads / a.kv_heads) % 4 != 0), "gqa attention: packing goes with head ratios that are no multiple of 4");
     dim3 grid((unsigned)p.n_groups, (unsigned)((a.heads + 3) / 4), (unsigned)p.S);
     switch (a.dim / 32) {
@@ -950,7 +957,7 @@ int mingru_carry(const MinGruCarryP& p, hipStream_t st) {
 // ------------------------------------------------------------------ per-head norm
 __global__ __launch_bounds__(256) void head_norm_rows_kernel(const float* o, const float* o2, const float* w, float eps, float scale,
                                                              int heads, int vdim, float* out, uint16_t* out_bf, int64_t ld_out,
-                                                             int out_col, const float* gate) {
+                                                             int out_col, const float* gate, int64_t ld_gate, int gate_silu) {
     const int64_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     for (int h = blockIdx.y * 4 + wave; h < heads; h += 4 * gridDim.y) {
@@ -966,17 +973,126 @@ __global__ __launch_bounds__(256) void head_norm_rows_kernel(const float* o, con
         const int64_t o0 = t * ld_out + out_col + (int64_t)h * vdim;
         for (int i = lane; i < vdim; i += 64) {
             float y = (x2 ? x[i] + x2[i] : x[i]) * inv * w[i];
-            if (gate) y *= 1.0f / (1.0f + expf(-gate[(t * heads + h) * vdim + i]));
+            if (gate) {
+                const float gz = gate[t * ld_gate + h * vdim + i], sg = 1.0f / (1.0f + expf(-gz));
+                y *= gate_silu ? gz * sg : sg;
+            }
             out[o0 + i] = y;
             if (out_bf) out_bf[o0 + i] = f2bf(y);
         }
     }
 }
 int head_norm_rows(const float* o, const float* o2, const float* w, float eps, float scale, int heads, int vdim, int T, float* out,
-                   uint16_t* out_bf, int64_t ld_out, int out_col, hipStream_t st, const float* gate) {
+                   uint16_t* out_bf, int64_t ld_out, int out_col, hipStream_t st, const float* gate, int64_t ld_gate, int gate_silu) {
     const int ny = T <= 64 ? std::min(8, (heads + 3) / 4) : 1;   // few rows: a row's heads over several blocks
     hipLaunchKernelGGL(head_norm_rows_kernel, dim3(T, ny), dim3(256), 0, st, o, o2, w, eps, scale, heads, vdim, out, out_bf, ld_out,
-                       out_col, gate);
+                       out_col, gate, ld_gate ? ld_gate : (int64_t)heads * vdim, gate_silu);
+    QIE_LAUNCH_CHECK();
+    return 0;
+}
+
+// ------------------------------------------------------------------ gate, then a norm in equal parts
+// One block per (row, part); the gated values stay in LDS between the two passes when they fit.
+__global__ __launch_bounds__(256) void gated_norm_parts_kernel(const float* y, const float* z, int64_t ld_z, const float* w, float eps,
+                                                               int n, int len, float* out, uint16_t* out_bf, int64_t ld_out, int stage) {
+    extern __shared__ float sm[];
+    __shared__ float red[4];
+    const int64_t t = blockIdx.x;
+    const int c0 = blockIdx.y * len;
+    auto gated = [&](int i) {
+        const float g = z[t * ld_z + c0 + i];
+        return y[t * n + c0 + i] * (g / (1.0f + expf(-g)));
+    };
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < len; i += 256) {
+        const float a = gated(i);
+        if (stage) sm[i] = a;   // read back by the same thread
+        ss += a * a;
+    }
+    ss = bsum256(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)len + eps);
+    for (int i = threadIdx.x; i < len; i += 256) {
+        const float o = (stage ? sm[i] : gated(i)) * inv * w[c0 + i];
+        out[t * ld_out + c0 + i] = o;
+        if (out_bf) out_bf[t * ld_out + c0 + i] = f2bf(o);
+    }
+}
+int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* w, float eps, int n, int parts, int T, float* out,
+                     uint16_t* out_bf, int64_t ld_out, hipStream_t st) {
+    QIE_REQUIRE(y && z && w && out && n > 0 && parts > 0 && n % parts == 0, "gated norm: %d columns in %d parts", n, parts);
+    const int len = n / parts, stage = (size_t)len * 4 <= 48 * 1024 ? 1 : 0;
+    hipLaunchKernelGGL(gated_norm_parts_kernel, dim3((unsigned)T, (unsigned)parts), dim3(256), stage ? (size_t)len * 4 : 0, st, y, z, ld_z,
+                       w, eps, n, len, out, out_bf, ld_out, stage);
+    QIE_LAUNCH_CHECK();
+    return 0;
+}
+
+// ------------------------------------------------------------------ two norms of one row
+// One block per row; a thread's coordinates stay in registers between the sum and the two scaled copies (rows of up
+// to 256 * NR coordinates; NR = 0: re-read).
+template <int NR>
+__global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
+    __shared__ float red[4];
+    const int64_t r0 = (int64_t)blockIdx.x * p.W;
+    float keep[NR > 0 ? NR : 1];
+    auto sum_at = [&](int i) {
+        float a = p.xin[r0 + i];
+        if (p.v) a += p.v2 ? p.v[r0 + i] + p.v2[r0 + i] : p.v[r0 + i];
+        if (p.add) a += p.add[r0 + i];
+        return a;
+    };
+    const bool moved = p.v || p.add || p.xin != p.x;
+    float ss = 0.f;
+    if (NR > 0) {
+#pragma unroll
+        for (int k = 0; k < NR; k++) {
+            const int i = threadIdx.x + 256 * k;
+            keep[k] = i < p.W ? sum_at(i) : 0.f;
+            ss += keep[k] * keep[k];
+        }
+#pragma unroll
+        for (int k = 0; k < NR; k++) {
+            const int i = threadIdx.x + 256 * k;
+            if (moved && i < p.W) p.x[r0 + i] = keep[k];
+        }
+    } else {
+        for (int i = threadIdx.x; i < p.W; i += 256) {
+            const float a = sum_at(i);
+            if (moved) p.x[r0 + i] = a;
+            ss += a * a;
+        }
+    }
+    if (!p.w1) return;
+    ss = bsum256(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
+    auto emit = [&](int i, float a) {
+        const float o1 = a * inv * p.w1[i];
+        p.h1[r0 + i] = o1;
+        if (p.h1_bf) p.h1_bf[r0 + i] = f2bf(o1);
+        if (p.w2) {
+            const float o2 = a * inv * p.w2[i];
+            p.h2[r0 + i] = o2;
+            if (p.h2_bf) p.h2_bf[r0 + i] = f2bf(o2);
+        }
+    };
+    if (NR > 0) {
+#pragma unroll
+        for (int k = 0; k < NR; k++) {
+            const int i = threadIdx.x + 256 * k;
+            if (i < p.W) emit(i, keep[k]);
+        }
+    } else {
+        for (int i = threadIdx.x; i < p.W; i += 256) emit(i, p.x[r0 + i]);   // the thread's own store above (or the row as it was)
+    }
+}
+int norm_pair(const NormPairP& p, hipStream_t st) {
+    QIE_REQUIRE(p.x && p.xin && p.T > 0 && p.W > 0 && (!p.w1 || p.h1) && (!p.w2 || (p.w1 && p.h2)) && (!p.v2 || p.v), "norm_pair: bad arguments");
+    if (p.W <= 1024)
+        hipLaunchKernelGGL(norm_pair_kernel<4>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+    else if (p.W <= 4096)
+        hipLaunchKernelGGL(norm_pair_kernel<16>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+    else
+        hipLaunchKernelGGL(norm_pair_kernel<0>, dim3((unsigned)p.T), dim3(256), 0, st, p);
     QIE_LAUNCH_CHECK();
     return 0;
 }

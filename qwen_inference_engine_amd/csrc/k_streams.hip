@@ -150,7 +150,7 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(CausalConvP p, int T) 
     const float* w = p.w + (int64_t)c * p.taps;
     const float* sb = p.state + (int64_t)slot * p.slot_stride + p.state_off;
     const float cur = p.in[(int64_t)t * p.ld_in + p.col + c];
-    float a = 0.f;
+    float a = p.bias ? p.bias[c] : 0.f;
     for (int j = 0; j < p.taps; j++) {
         const int back = p.taps - 1 - j;
         float x;
@@ -204,7 +204,7 @@ __global__ __launch_bounds__(256) void causal_conv_fused_kernel(CausalConvP p) {
     for (int k = 0; k < en.y; k++) {
         const int t = en.x + k, pos = en.w + k;
         const float cur = p.in[(int64_t)t * p.ld_in + p.col + c];
-        float a = 0.f;
+        float a = p.bias ? p.bias[c] : 0.f;
         for (int j = 0; j < p.taps; j++) {
             const int back = p.taps - 1 - j;
             float x;

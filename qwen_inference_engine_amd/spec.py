@@ -217,6 +217,8 @@ class GqaAttention:
     sink: bool = False           # exp(a number per head) joins the softmax denominator
     out_gate: bool = False       # the concatenated head outputs times sigmoid(W_g x), element by element
     rot_scaling: Optional[Tuple[float, float, float, float]] = None   # (factor, low, high, original) wavelengths
+    v_bias: bool = False         # a bias vector on the v projection
+    mask_keep: int = 0           # mask "window": the keys j < mask_keep stay visible beyond the window
 
 
 @dataclasses.dataclass(frozen=True)
@@ -228,11 +230,22 @@ class GatedRecurrence:
 
 
 @dataclasses.dataclass(frozen=True)
+class KeyDecayRecurrence:
+    """Gated linear attention: separate q and k, one decay per head and key channel through a low-rank projection
+    (sigmoid(.)^(1 / tau)), a silu output gate; a [dim, vdim] fp32 state per head and slot."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    rank: int = 0     # rows of W_a1 (0: only the tensor gives it)
+
+
+@dataclasses.dataclass(frozen=True)
 class AttentionWithRecurrence:
-    """Mixer: a GqaAttention and a GatedRecurrence read the same input; their results are added
-    with fixed scales."""
+    """Mixer: a GqaAttention and a recurrence (GatedRecurrence or KeyDecayRecurrence) read the same input; their
+    results are added with fixed scales."""
     attn: GqaAttention
-    rec: GatedRecurrence
+    rec: object
     attn_scale: float
     rec_scale: float
 
@@ -262,6 +275,27 @@ class ChannelDelta:
 
 
 @dataclasses.dataclass(frozen=True)
+class StateSpace:
+    """Mixer: Mamba-2 (state-space duality): a scalar decay per head and token, input and output vectors shared by the
+    heads of a group, a short convolution in front, the gate before a norm in equal parts; a [state, vdim] fp32 state
+    per head and slot plus the convolution's last inputs."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int         # taps of the short convolution
+    norm_groups: int
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+@dataclasses.dataclass(frozen=True)
 class FeedForward:
     kind: str         # "dense" or "moe"
     ff: int           # hidden size (of one expert for "moe")
@@ -271,16 +305,18 @@ class FeedForward:
                                  # biased logits, softmax over the chosen ones weights the output;
                                  # "softmax_all": softmax over all router outputs, chosen by score +
                                  # correction inside the best groups, renormalised, times route_scale
-    act: str = "silu_gated"      # dense: "silu_gated" | "gelu_tanh_gated" (gate, up, down) | "xielu" (up, down, two numbers)
+    act: str = "silu_gated"      # dense: "silu_gated" | "gelu_tanh_gated" | "clamped_gated" (gate, up, down) |
+                                 # "xielu" (up, down, two numbers)
     identity: int = 0            # "softmax_all": identity experts after the `experts` real ones
     groups: int = 1
     groups_keep: int = 1
     route_scale: float = 1.0
+    limit: float = 0.0           # "clamped_gated": the gate is cut at limit, the up value to +-limit
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: object     # LatentAttention | GqaAttention | AttentionWithRecurrence | MinGru | ChannelDelta
+    mixer: object     # LatentAttention | GqaAttention | AttentionWithRecurrence | MinGru | ChannelDelta | StateSpace
     mlp: Optional[FeedForward]
 
 
@@ -294,6 +330,7 @@ class LayeredSpec:
     depth_mix: bool = True
     block: str = "postnorm_gain"     # "postnorm_gain" | "sandwich" (weight-vector norms around every branch)
                                      # | "prenorm" (one plain-weight norm before every branch)
+                                     # | "parallel" (both branches of the same row, each behind its own norm)
     tied_head: bool = False
     embed_scale: float = 1.0
     pos_embed: str = "none"          # "none" | "sinusoid" (added to the scaled embedding row)
@@ -303,6 +340,7 @@ class LayeredSpec:
     streams: int = 0                 # >= 1: that many residual rows mixed by 'l<i>.hc<q>.in|out|mix' (hyper-connections)
     canon_taps: int = 0              # >= 1: the mixer reads h + causal conv(h) over time ('l<i>.canon1' [width, taps])
     embed_norm: bool = False         # the embedding rows are normed with 'embed.norm'
+    logit_scale: float = 1.0
 
     @property
     def n_layers(self) -> int:
@@ -339,6 +377,7 @@ class LayeredSpec:
             g.slope_bias, g.head_gate = int(m.slope_bias), int(m.head_gate)
             g.q_temp_coef, g.q_temp_every = m.q_temp_coef, m.q_temp_every
             g.qk_bias, g.sink, g.out_gate = int(m.qk_bias), int(m.sink), int(m.out_gate)
+            g.v_bias, g.mask_keep = int(m.v_bias), m.mask_keep
             if m.rot_scaling:
                 g.rot_scaling.factor, g.rot_scaling.low, g.rot_scaling.high, g.rot_scaling.original = m.rot_scaling
 
@@ -351,6 +390,8 @@ class LayeredSpec:
                 d.mixer = _lib.QIE_MIXER_GQA_RECURRENT
                 gqa(d.gqa, m.attn)
                 d.rec.heads, d.rec.dim, d.rec.vdim = m.rec.heads, m.rec.dim, m.rec.vdim
+                if isinstance(m.rec, KeyDecayRecurrence):
+                    d.rec.kind, d.rec.rank, d.rec.tau = _lib.QIE_REC_KEY_DECAY, m.rec.rank, m.rec.tau
                 d.gqa_scale, d.rec_scale = m.attn_scale, m.rec_scale
             elif isinstance(m, MinGru):
                 d.mixer = _lib.QIE_MIXER_MINGRU
@@ -359,6 +400,10 @@ class LayeredSpec:
                 d.mixer = _lib.QIE_MIXER_CHANNEL_DELTA
                 x = d.delta
                 x.heads, x.kv_heads, x.dim, x.vdim, x.conv, x.rank_a, x.rank_g = m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.rank_a, m.rank_g
+            elif isinstance(m, StateSpace):
+                d.mixer = _lib.QIE_MIXER_STATE_SPACE
+                x = d.ssm
+                x.heads, x.vdim, x.state, x.groups, x.conv, x.norm_groups = m.heads, m.vdim, m.state, m.groups, m.conv, m.norm_groups
             else:
                 d.mixer = _lib.QIE_MIXER_LATENT_ATTENTION
                 d.heads, d.dim, d.rot_dim, d.vdim, d.kv_rank = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
@@ -373,7 +418,8 @@ class LayeredSpec:
             elif L.mlp.kind == "dense":
                 d.ff_kind, d.ff = _lib.QIE_FF_DENSE, L.mlp.ff
                 d.ff_act = {"silu_gated": _lib.QIE_ACT_SILU_GATED, "xielu": _lib.QIE_ACT_XIELU,
-                            "gelu_tanh_gated": _lib.QIE_ACT_GELU_TANH_GATED}[L.mlp.act]
+                            "gelu_tanh_gated": _lib.QIE_ACT_GELU_TANH_GATED, "clamped_gated": _lib.QIE_ACT_CLAMPED_GATED}[L.mlp.act]
+                d.ff_limit = L.mlp.limit
             else:
                 d.ff_kind, d.ff, d.experts, d.top = _lib.QIE_FF_MOE, L.mlp.ff, L.mlp.experts, L.mlp.top
                 d.router = {"sigmoid_in": _lib.QIE_ROUTER_SIGMOID_IN, "softmax_out": _lib.QIE_ROUTER_SOFTMAX_OUT,
@@ -383,7 +429,7 @@ class LayeredSpec:
         a.n_layers, a.width, a.vocab, a.norm_eps = len(self.layers), self.width, self.vocab, self.norm_eps
         a.depth_mix = int(self.depth_mix)
         a.block = {"postnorm_gain": _lib.QIE_BLOCK_POSTNORM_GAIN, "sandwich": _lib.QIE_BLOCK_SANDWICH,
-                   "prenorm": _lib.QIE_BLOCK_PRENORM}[self.block]
+                   "prenorm": _lib.QIE_BLOCK_PRENORM, "parallel": _lib.QIE_BLOCK_PARALLEL}[self.block]
         a.tied_head = int(self.tied_head)
         a.embed_scale = self.embed_scale
         a.pos_embed = _lib.QIE_POS_SINUSOID if self.pos_embed == "sinusoid" else _lib.QIE_POS_NONE
@@ -391,13 +437,14 @@ class LayeredSpec:
             a.loop_start, a.loop_stop, a.loop_times = self.loop
         a.layers = arr
         a.streams, a.canon_taps, a.embed_norm, a.norm_offset = self.streams, self.canon_taps, int(self.embed_norm), self.norm_offset
+        a.logit_scale = self.logit_scale
         return a, arr
 
     def tensor_shapes(self) -> "dict[str, List[int]]":
         """Checkpoint tensor names and shapes of this architecture."""
         W, out = self.width, {"embed": [self.vocab, self.width]}
         sandwich = self.block == "sandwich"
-        nshape = [W] if self.block in ("sandwich", "prenorm") else []
+        nshape = [W] if self.block in ("sandwich", "prenorm", "parallel") else []
 
         def gqa(q, m):
             out[q + "q"], out[q + "k"] = [m.heads * m.dim, W], [m.kv_heads * m.dim, W]
@@ -413,6 +460,8 @@ class LayeredSpec:
                 out[q + "g"] = [m.heads, W]
             if m.qk_bias:
                 out[q + "q.b"], out[q + "k.b"] = [m.heads * m.dim], [m.kv_heads * m.dim]
+            if m.v_bias:
+                out[q + "v.b"] = [m.kv_heads * m.vdim]
             if m.sink:
                 out[q + "sink"] = [m.heads]
             if m.out_gate:
@@ -439,9 +488,19 @@ class LayeredSpec:
             elif isinstance(m, AttentionWithRecurrence):
                 gqa(p + "mix.left.", m.attn)
                 r, c = p + "mix.right.", m.rec
-                out[r + "q"], out[r + "f"], out[r + "v"] = [c.heads * c.dim, W], [c.heads * c.dim, W], [c.heads * c.vdim, W]
-                out[r + "f.b"], out[r + "lower"], out[r + "norm"] = [c.heads * c.dim], [c.heads * c.dim], [c.vdim]
-                out[r + "o"] = [W, c.heads * c.vdim]
+                nk, nv = c.heads * c.dim, c.heads * c.vdim
+                if isinstance(c, KeyDecayRecurrence):
+                    out.update({r + "q": [nk, W], r + "k": [nk, W], r + "v": [nv, W], r + "g": [nv, W], r + "norm": [c.vdim],
+                                r + "a1": [c.rank, W], r + "a2": [nk, c.rank], r + "a2.b": [nk]})
+                else:
+                    out[r + "q"], out[r + "f"], out[r + "v"] = [nk, W], [nk, W], [nv, W]
+                    out[r + "f.b"], out[r + "lower"], out[r + "norm"] = [nk], [nk], [c.vdim]
+                out[r + "o"] = [W, nv]
+            elif isinstance(m, StateSpace):
+                q = p + "mix."
+                out.update({q + "in": [m.inner + m.conv_channels + m.heads, W], q + "conv": [m.conv_channels, m.conv],
+                            q + "conv.b": [m.conv_channels], q + "dt_bias": [m.heads], q + "A_log": [m.heads], q + "D": [m.heads],
+                            q + "norm": [m.inner], q + "o": [W, m.inner]})
             elif isinstance(m, MinGru):
                 q = p + "mix."
                 out.update({q + "z": [m.width, W], q + "z.b": [m.width], q + "x": [m.width, W], q + "x.b": [m.width],
@@ -494,7 +553,7 @@ class LayeredSpec:
             m = self.layers[i].mixer
             if isinstance(m, LatentAttention):
                 n += m.kv_rank + m.rot_dim if m.kv_from is None else 0
-            elif isinstance(m, (MinGru, ChannelDelta)):
+            elif isinstance(m, (MinGru, ChannelDelta, StateSpace)):
                 pass
             else:
                 a = m.attn if isinstance(m, AttentionWithRecurrence) else m
@@ -512,6 +571,8 @@ class LayeredSpec:
                 n += m.width
             elif isinstance(m, ChannelDelta):
                 n += m.heads * m.dim * m.vdim + (m.conv - 1) * m.conv_channels
+            elif isinstance(m, StateSpace):
+                n += m.heads * m.state * m.vdim + (m.conv - 1) * m.conv_channels
             if self.canon_taps > 1:
                 n += (self.canon_taps - 1) * self.width
         return n
@@ -529,6 +590,10 @@ class LayeredSpec:
                 if L.mlp is not None:
                     f += 2.0 * rows * 3 * W * L.mlp.ff
                 continue
+            if isinstance(m, StateSpace):
+                f += 2.0 * rows * W * (2 * m.inner + m.conv_channels + m.heads) + 2.0 * rows * m.heads * m.state * m.vdim * 2
+                f += 2.0 * rows * 3 * W * L.mlp.ff if L.mlp is not None else 0.0
+                continue
             if isinstance(m, MinGru):
                 f += 2.0 * rows * W * 4 * m.width
                 if L.mlp is not None:
@@ -539,11 +604,14 @@ class LayeredSpec:
                 n_in = a.heads * a.dim + a.kv_heads * (a.dim + (0 if a.values_are_keys else a.vdim)) + (a.heads if a.head_gate else 0) \
                     + (a.heads * a.vdim if a.out_gate else 0)
                 n_cat = a.heads * a.vdim
-                keys = ctx if a.mask == "causal" else min(ctx, a.mask_size if a.mask == "window" else (a.mask_size + 1) // 2)
+                keys = ctx if a.mask == "causal" else min(ctx, a.mask_size + a.mask_keep if a.mask == "window" else (a.mask_size + 1) // 2)
                 f += 2.0 * rows * a.heads * keys * (a.dim + a.vdim)
                 if isinstance(m, AttentionWithRecurrence):
                     c = m.rec
                     n_in += c.heads * (2 * c.dim + c.vdim)
+                    if isinstance(c, KeyDecayRecurrence):
+                        n_in += c.heads * c.vdim + c.rank
+                        f += 2.0 * rows * c.rank * c.heads * c.dim
                     n_cat += c.heads * c.vdim
                     f += 2.0 * rows * c.heads * c.dim * c.vdim * 2
                 f += 2.0 * rows * W * (n_in + n_cat)
@@ -726,8 +794,52 @@ def _verelorn_from_config(cfg: dict, name: str) -> LayeredSpec:
                        block="prenorm", tied_head=False, norm_offset=1.0, streams=streams, canon_taps=taps, embed_norm=True)
 
 
+def _sefelorn_from_config(cfg: dict, name: str) -> LayeredSpec:
+    """Sefelorn: blocks whose mixer and feed-forward read the same row through two norms, over a scaled embedding; a
+    repeated group of layers; tied head with a logit scale.  Mixers: a Mamba-2 state space, or a grouped-query attention
+    (biased q, k and v, partial rotate-half rotary, a sliding window that keeps the sequence's first tokens) beside a
+    gated linear attention with a decay per key channel.  Feed-forward: dense, clamped gate and up values, or none."""
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        m = L["mixer"]
+        if L["type"] == "parallel":
+            a, c = m["left"], m["right"]
+            rot, mask = a.get("rot") or {}, a["mask"]
+            attn = GqaAttention(
+                heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]), scale=float(a["scale"]),
+                rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)), rot_layout="halves", mask="window",
+                mask_size=int(mask["size"]), mask_keep=int(mask.get("keep_first", 0)), qk_bias=True, v_bias=True)
+            # the rank of the decay projection is a size only the tensors give (0: taken from them)
+            rec = KeyDecayRecurrence(heads=int(c["heads"]), dim=int(c["dim"]), vdim=int(c["vdim"]), tau=float(c["tau"]),
+                                     rank=int(c.get("rank", 0)))
+            mixer = AttentionWithRecurrence(attn, rec, float(m["left_scale"]), float(m["right_scale"]))
+        elif L["type"] == "mamba2":
+            mixer = StateSpace(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                               conv=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+            if mixer.heads % mixer.groups or mixer.inner % mixer.norm_groups:
+                raise ValueError(f"layer {i}: {mixer.heads} heads in {mixer.groups} groups, a norm of {mixer.inner} in "
+                                 f"{mixer.norm_groups} parts")
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {L['type']!r}")
+        f = L.get("mlp")
+        if f is None:
+            mlp = None
+        elif f["kind"] == "dense":
+            mlp = FeedForward("dense", int(f["ff"]), act="clamped_gated", limit=float(f["limit"]))
+        else:
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+        layers.append(LayerSpec(mixer, mlp))
+    lp = cfg.get("loop")
+    loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"])) if lp else None
+    if loop and not (0 <= loop[0] <= loop[1] <= len(layers) and loop[2] >= 1):
+        raise ValueError(f"loop {loop} does not fit {len(layers)} layers")
+    return LayeredSpec(name, int(cfg["width"]), int(cfg["vocab"]), float(cfg["norm"]["eps"]), tuple(layers), depth_mix=False,
+                       block="parallel", tied_head=True, embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), loop=loop,
+                       logit_scale=float(cfg.get("logit_scale", 1.0)))
+
+
 ARCHITECTURES = {"Tivazen": _tivazen_from_config, "Nodutar": _nodutar_from_config, "Lugipel": _lugipel_from_config,
-                 "Verelorn": _verelorn_from_config}
+                 "Verelorn": _verelorn_from_config, "Sefelorn": _sefelorn_from_config}
 
 
 def spec_from_config(cfg: dict, name: str = "model", numerics: str = "hf"):
@@ -741,9 +853,15 @@ def spec_from_config(cfg: dict, name: str = "model", numerics: str = "hf"):
     return ModelSpec.from_hf_config(cfg, name=name, numerics=numerics)
 
 
+def _needs_tensor_sizes(m) -> bool:
+    if isinstance(m, ChannelDelta):
+        return 0 in (m.rank_a, m.rank_g)
+    return isinstance(m, AttentionWithRecurrence) and isinstance(m.rec, KeyDecayRecurrence) and m.rec.rank == 0
+
+
 def with_tensor_sizes(spec, shapes: "dict[str, List[int]]"):
-    """Sizes a config leaves to the checkpoint's tensors (the ranks of a ChannelDelta's decay and gate
-    projections), filled in from a name -> shape table."""
+    """Sizes a config leaves to the checkpoint's tensors (the ranks of a ChannelDelta's decay and gate projections, of a
+    KeyDecayRecurrence's decay projection), filled in from a name -> shape table."""
     if not isinstance(spec, LayeredSpec):
         return spec
     layers = list(spec.layers)
@@ -754,6 +872,11 @@ def with_tensor_sizes(spec, shapes: "dict[str, List[int]]"):
             if a1 is None or g1 is None:
                 raise ValueError(f"layer {i}: tensors 'l{i}.mix.a1' / 'l{i}.mix.g1' are missing")
             layers[i] = LayerSpec(dataclasses.replace(m, rank_a=m.rank_a or int(a1[0]), rank_g=m.rank_g or int(g1[0])), L.mlp)
+        if isinstance(m, AttentionWithRecurrence) and isinstance(m.rec, KeyDecayRecurrence) and m.rec.rank == 0:
+            a1 = shapes.get(f"l{i}.mix.right.a1")
+            if a1 is None:
+                raise ValueError(f"layer {i}: tensor 'l{i}.mix.right.a1' is missing")
+            layers[i] = LayerSpec(dataclasses.replace(m, rec=dataclasses.replace(m.rec, rank=int(a1[0]))), L.mlp)
     return dataclasses.replace(spec, layers=tuple(layers))
 
 
@@ -763,7 +886,7 @@ def spec_from_dir(path: str, numerics: str = "hf"):
         spec = spec_from_config(json.load(f), name=os.path.basename(os.path.normpath(path)), numerics=numerics)
     st = os.path.join(path, "model.safetensors")
     if isinstance(spec, LayeredSpec) and os.path.exists(st) and any(
-            isinstance(L.mixer, ChannelDelta) and 0 in (L.mixer.rank_a, L.mixer.rank_g) for L in spec.layers):
+            _needs_tensor_sizes(L.mixer) for L in spec.layers):
         import struct
         with open(st, "rb") as f:
             n = struct.unpack("<Q", f.read(8))[0]

@@ -1,0 +1,183 @@
+"""The Sefelorn design restated in numpy float64, one function per mechanism.
+
+Slow and plain on purpose: whole sequences at once, explicit loops over positions where a recurrence runs, no cache
+and no batching.  Shares no code with the engine.  ``cfg`` is a config dictionary in the layout of a Sefelorn
+config.json, ``W`` maps tensor names to arrays.
+
+Notation: T tokens, h the input of a mixer or feed-forward (a normed residual row).
+"""
+from __future__ import annotations
+
+import math
+
+import numpy as np
+
+
+def f64(a):
+    return np.asarray(a, dtype=np.float64)
+
+
+def rms_unit(x, eps):
+    """x over its root mean square, eps inside the root."""
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
+
+
+def norm(x, w, eps):
+    return rms_unit(x, eps) * f64(w)
+
+
+def sigmoid(z):
+    return np.exp(-np.logaddexp(0.0, -f64(z)))
+
+
+def silu(z):
+    return z * sigmoid(z)
+
+
+def softplus(z):
+    return np.logaddexp(0.0, z)
+
+
+def causal_conv(x, w, b):
+    """x [T, C], w [C, taps], b [C]: out_t = b + sum_j w[:, j] x_(t - taps + 1 + j); zeros before the start."""
+    x, w = f64(x), f64(w)
+    T, taps = x.shape[0], w.shape[1]
+    out = np.tile(f64(b), (T, 1))
+    for t in range(T):
+        for j in range(taps):
+            s = t - (taps - 1) + j
+            if s >= 0:
+                out[t] += w[:, j] * x[s]
+    return out
+
+
+def rotate_halves(x, dims, base):
+    """x [T, heads, D]: coordinate i < dims / 2 pairs with i + dims / 2, turned by t * base^(-2i / dims)."""
+    if dims == 0:
+        return x
+    T, half = x.shape[0], dims // 2
+    f = np.array([base ** (-2.0 * i / dims) for i in range(half)])
+    ang = np.arange(T)[:, None] * f[None, :]
+    c, s = np.cos(ang)[:, None, :], np.sin(ang)[:, None, :]
+    out = x.copy()
+    u, v = x[..., :half], x[..., half:dims]
+    out[..., :half] = u * c - v * s
+    out[..., half:dims] = v * c + u * s
+    return out
+
+
+def visible(T, size, keep):
+    """[T, T] mask: row i sees column j <= i within the last `size` positions or among the first `keep`."""
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    return (j <= i) & ((i - j < size) | (j < keep))
+
+
+def softmax_rows(scores, mask):
+    s = np.where(mask[None], scores, -np.inf)
+    e = np.exp(s - s.max(axis=-1, keepdims=True))
+    return e / e.sum(axis=-1, keepdims=True)
+
+
+def window_attention(m, W, p, h):
+    """Grouped-query softmax attention with biased projections, a partial rotary and a sliding window that keeps the
+    first tokens of the sequence."""
+    H, G, D, Dv = int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"])
+    T = h.shape[0]
+    q = (h @ f64(W[p + "q"]).T + f64(W[p + "q.b"])).reshape(T, H, D)
+    k = (h @ f64(W[p + "k"]).T + f64(W[p + "k.b"])).reshape(T, G, D)
+    v = (h @ f64(W[p + "v"]).T + f64(W[p + "v.b"])).reshape(T, G, Dv)
+    rot = m.get("rot") or {"dims": 0, "base": 1.0}
+    q = rotate_halves(q, int(rot["dims"]), float(rot["base"]))
+    k = rotate_halves(k, int(rot["dims"]), float(rot["base"]))
+    rep = H // G
+    scores = np.stack([q[:, a] @ k[:, a // rep].T for a in range(H)]) * float(m["scale"])
+    wts = softmax_rows(scores, visible(T, int(m["mask"]["size"]), int(m["mask"]["keep_first"])))
+    o = np.stack([wts[a] @ v[:, a // rep] for a in range(H)], axis=1)
+    return o.reshape(T, H * Dv) @ f64(W[p + "o"]).T
+
+
+def key_decay_attention(m, W, p, h, eps):
+    """Gated linear attention: S <- diag(alpha) S + k v^T, o = S^T q; alpha per head and key channel."""
+    H, D, Dv, tau = int(m["heads"]), int(m["dim"]), int(m["vdim"]), float(m["tau"])
+    T = h.shape[0]
+    q = (h @ f64(W[p + "q"]).T).reshape(T, H, D) * D ** -0.5
+    k = (h @ f64(W[p + "k"]).T).reshape(T, H, D)
+    v = (h @ f64(W[p + "v"]).T).reshape(T, H, Dv)
+    z = (h @ f64(W[p + "a1"]).T) @ f64(W[p + "a2"]).T + f64(W[p + "a2.b"])
+    alpha = (sigmoid(z) ** (1.0 / tau)).reshape(T, H, D)
+    o = np.zeros((T, H, Dv))
+    for a in range(H):
+        S = np.zeros((D, Dv))
+        for t in range(T):
+            S = alpha[t, a][:, None] * S + np.outer(k[t, a], v[t, a])
+            o[t, a] = S.T @ q[t, a]
+    o = (rms_unit(o, eps) * f64(W[p + "norm"])).reshape(T, H * Dv)
+    return (o * silu(h @ f64(W[p + "g"]).T)) @ f64(W[p + "o"]).T
+
+
+def state_space(m, W, p, h, eps):
+    """Mamba-2: a scalar decay per head and token, input and output vectors shared by groups of heads, a skip per
+    head, the gate before a norm in equal parts."""
+    H, Dv, N, G, parts = (int(m[k]) for k in ("heads", "vdim", "state", "groups", "norm_groups"))
+    inner, T = H * Dv, h.shape[0]
+    proj = h @ f64(W[p + "in"]).T
+    z, xbc, dt = proj[:, :inner], proj[:, inner:2 * inner + 2 * G * N], proj[:, 2 * inner + 2 * G * N:]
+    xbc = silu(causal_conv(xbc, W[p + "conv"], W[p + "conv.b"]))
+    x = xbc[:, :inner].reshape(T, H, Dv)
+    B = xbc[:, inner:inner + G * N].reshape(T, G, N)
+    C = xbc[:, inner + G * N:].reshape(T, G, N)
+    dt = softplus(dt + f64(W[p + "dt_bias"]))
+    a, D = np.exp(f64(W[p + "A_log"])), f64(W[p + "D"])
+    y = np.zeros((T, H, Dv))
+    for hh in range(H):
+        S, g = np.zeros((N, Dv)), hh // (H // G)
+        for t in range(T):
+            S = np.exp(-a[hh] * dt[t, hh]) * S + dt[t, hh] * np.outer(B[t, g], x[t, hh])
+            y[t, hh] = S.T @ C[t, g] + D[hh] * x[t, hh]
+    y = y.reshape(T, inner) * silu(z)
+    y = rms_unit(y.reshape(T, parts, inner // parts), eps).reshape(T, inner) * f64(W[p + "norm"])
+    return y @ f64(W[p + "o"]).T
+
+
+def clamped_ff(mlp, W, p, h):
+    lim = float(mlp["limit"])
+    g = np.minimum(h @ f64(W[p + "gate"]).T, lim)
+    u = np.clip(h @ f64(W[p + "up"]).T, -lim, lim)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ f64(W[p + "down"]).T
+
+
+def layer_runs(cfg):
+    """(layer, embedding added first?) of every layer run in order."""
+    n, lp = len(cfg["layers"]), cfg.get("loop")
+    if not lp:
+        return [(i, False) for i in range(n)]
+    a, b, t = int(lp["start"]), int(lp["stop"]), int(lp["times"])
+    out = [(i, False) for i in range(a)]
+    for k in range(t):
+        out += [(i, k > 0 and i == a) for i in range(a, b)]
+    return out + [(i, False) for i in range(b, n)]
+
+
+def forward(cfg, W, tokens, layers_out=None):
+    """Logits [T, vocab] of one sequence.  layers_out (a list) receives the stream after every layer run."""
+    eps = float(cfg["norm"]["eps"])
+    x0 = f64(W["embed"])[np.asarray(tokens)] * float(cfg["embedding"]["scale"])
+    x = x0.copy()
+    for i, again in layer_runs(cfg):
+        L, p = cfg["layers"][i], f"l{i}."
+        if again:
+            x = x + x0
+        m, h = L["mixer"], norm(x, W[p + "norm1"], eps)
+        if L["type"] == "mamba2":
+            y = state_space(m, W, p + "mix.", h, eps)
+        elif L["type"] == "parallel":
+            y = float(m["left_scale"]) * window_attention(m["left"], W, p + "mix.left.", h) \
+                + float(m["right_scale"]) * key_decay_attention(m["right"], W, p + "mix.right.", h, eps)
+        else:
+            raise ValueError(L["type"])
+        if L.get("mlp") is not None:
+            y = y + clamped_ff(L["mlp"], W, p + "mlp.", norm(x, W[p + "norm2"], eps))
+        x = x + y
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return norm(x, W["final.norm"], eps) @ f64(W["embed"]).T * float(cfg["logit_scale"])
