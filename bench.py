@@ -84,6 +84,15 @@ VERELORN_SIZES = {
 }
 
 
+# Sizes of `--sefelorn`: (width, attention heads, kv heads, head dim, rotated dims, window, first tokens kept, recurrence
+# heads, recurrence dim, recurrence vdim, decay rank, state-space heads, vdim, state, groups, taps, norm parts, ff, vocab).
+# Four layers, each with its feed-forward: state space, attention beside gated linear attention, the same two again.
+SEFELORN_SIZES = {
+    "1k": (1024, 16, 4, 64, 32, 512, 4, 8, 64, 128, 16, 32, 64, 128, 1, 4, 1, 2816, 32000),
+    "2k": (2048, 16, 4, 128, 64, 1024, 4, 16, 64, 128, 16, 64, 64, 128, 8, 4, 8, 5632, 32000),
+}
+
+
 def parse(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -134,6 +143,10 @@ def parse(argv=None):
                          "layers beside it (one JSON line of its own)")
     ap.add_argument("--verelorn", choices=sorted(VERELORN_SIZES), default=None,
                     help="instead of the default workload: prefill and decode throughput of a Verelorn model at this "
+                         "size with random weights, per-stage times, and the Qwen decoder at equal width / heads / "
+                         "layers beside it (one JSON line of its own)")
+    ap.add_argument("--sefelorn", choices=sorted(SEFELORN_SIZES), default=None,
+                    help="instead of the default workload: prefill and decode throughput of a Sefelorn model at this "
                          "size with random weights, per-stage times, and the Qwen decoder at equal width / heads / "
                          "layers beside it (one JSON line of its own)")
     ap.add_argument("--dry-run", action="store_true",
@@ -197,6 +210,8 @@ def main(argv=None):
         return run_lugipel(a)
     if a.verelorn:
         return run_verelorn(a)
+    if a.sefelorn:
+        return run_sefelorn(a)
     return run(a)
 
 
@@ -591,6 +606,124 @@ def run_verelorn(a):
     b.close()
     eng.close()
     out["qwen_equal_size"] = qwen_twin(Q, S, Wt, a.verelorn, W, H, G, hd, ff, V, P, B, steps, prompts, a.prefill_iters, max_ctx)
+    print(json.dumps(out), flush=True)
+    return 0
+
+
+def sefelorn_model(S, size):
+    """(LayeredSpec, {name: bf16 words}) at one of SEFELORN_SIZES, random weights from one pool."""
+    W, H, G, hd, rot, win, keep, RH, rd, rv, rank, SH, sv, N, SG, taps, parts, ff, V = SEFELORN_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    ssm = {"type": "mamba2", "mlp": mlp, "mixer": {"heads": SH, "vdim": sv, "state": N, "groups": SG, "conv": taps, "norm_groups": parts}}
+    par = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "mask": {"size": win, "keep_first": keep}, "scale": hd ** -0.5,
+                 "rot": {"base": 10000.0, "dims": rot}},
+        "right": {"heads": RH, "dim": rd, "vdim": rv, "tau": 8.0}, "left_scale": 1.0, "right_scale": 0.75}}
+    cfg = {"architecture": "Sefelorn", "layers": [ssm, par, ssm, par], "norm": {"eps": 1e-6}, "embedding": {"scale": 4.0},
+           "logit_scale": 0.25, "vocab": V, "width": W}
+    spec = S.spec_from_config(cfg, name=f"sefelorn-{size}")
+    spec = S.with_tensor_sizes(spec, {f"l{i}.mix.right.a1": [rank, W] for i in (1, 3)})
+    pool = np.random.default_rng(0).standard_normal(1 << 22).astype(np.float32)
+    tensors = {}
+    for k, (name, shape) in enumerate(spec.tensor_shapes().items()):
+        n = int(np.prod(shape))
+        if name.endswith(("norm", "norm1", "norm2", ".D")):
+            v = np.ones(shape, np.float32)
+        elif name.endswith(("q.b", "k.b", "v.b", "conv.b")):
+            v = np.zeros(shape, np.float32)
+        elif name.endswith("a2.b"):
+            v = np.full(shape, 2.0, np.float32)
+        elif name.endswith("dt_bias"):
+            v = np.full(shape, -3.0, np.float32)
+        elif name.endswith("A_log"):
+            v = np.linspace(0.0, 2.5, n, dtype=np.float32).reshape(shape)
+        else:
+            fan = shape[-1] if name != "embed" else 1
+            v = (np.resize(np.roll(pool, 7919 * k), n) * fan ** -0.5).reshape(shape)
+        tensors[name] = (np.ascontiguousarray(v, np.float32).view(np.uint32) >> 16).astype(np.uint16).reshape(shape)
+    return spec, tensors
+
+
+def run_sefelorn(a):
+    """Prefill (one step of P tokens) and decode (B single-token entries a step at context ~P) of a Sefelorn model,
+    per-stage hipEvent times at both shapes, and the Qwen decoder at equal sizes."""
+    import qwen_inference_engine_amd as Q
+    from qwen_inference_engine_amd import spec as S, weights as Wt
+    W, H, G, hd, rot, win, keep, RH, rd, rv, rank, SH, sv, N, SG, taps, parts, ff, V = SEFELORN_SIZES[a.sefelorn]
+    P, B, steps = a.prompt, max(a.batch, 8), min(a.steps, 128)
+    max_ctx = P + steps + 80
+    spec, tensors = sefelorn_model(S, a.sefelorn)
+    names = ("width", "heads", "kv_heads", "head_dim", "rot_dims", "window", "keep_first", "rec_heads", "rec_dim", "rec_vdim",
+             "rec_rank", "ssm_heads", "ssm_vdim", "ssm_state", "ssm_groups", "ssm_taps", "ssm_norm_parts", "ff", "vocab")
+    out = {"metric": "sefelorn_decode_tokens_per_sec", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
+           "data": "synthetic (random weights, random token ids)", "higher_is_better": True,
+           "config": {"model": spec.name, "sizes": dict(zip(names, SEFELORN_SIZES[a.sefelorn])), "layers": 4, "prompt": P,
+                      "decode_batch": B, "decode_steps": steps}}
+    eng = Q.Engine(spec, max_ctx=max_ctx).load_tensors(tensors)
+    del tensors
+    b = eng.batch(B, max_ctx, page_tokens=64)
+    rng = np.random.default_rng(1)
+    prompts = rng.integers(0, V, size=(B, P), dtype=np.int32)
+    ts = []
+    for it in range(1 + a.prefill_iters):
+        t0 = time.perf_counter()
+        b.step([(0, prompts[0])], [P - 1], fetch=False)
+        ts.append(time.perf_counter() - t0)
+        if it < a.prefill_iters:
+            b.release(0)
+    t_pf = float(np.median(ts[1:]))
+    stages = {"prefill": {}, "decode": {}}
+    # stage 2 of a layer: its input product and its output product, which also takes the feed-forward's activations;
+    # stage 3: the gate / up product and the activation
+    ssm_in, ssm_out = 2 * SH * sv + 2 * SG * N + SH, SH * sv + ff
+    par_in = H * hd + 2 * G * hd + RH * (2 * rd + 2 * rv) + rank
+    par_out = H * hd + RH * rv + ff
+
+    def stage_times(tag, rows, ctx):
+        st = stages[tag]
+        st["window_attention_us"] = round(b.time_stage(1, 1, 10), 2)
+        st["parallel_products_us"] = round(b.time_stage(2, 1, 10), 2)
+        st["ssm_products_us"] = round(b.time_stage(2, 0, 10), 2)
+        st["gate_up_us"] = round(b.time_stage(3, 0, 10), 2)
+        st["linear_attention_us"] = round(b.time_stage(4, 1, 10), 2)
+        st["ssm_scan_us"] = round(b.time_stage(4, 0, 10), 2)
+        # keys a row sees: the window (short of it at the start of a prompt)
+        keys = min(ctx, win + keep) if tag == "decode" else (win + keep) * (1.0 - win / (2.0 * ctx)) if ctx > win else ctx / 2.0
+        st["window_attention_tflops"] = round(4.0 * rows * H * keys * hd / st["window_attention_us"] / 1e6, 2)
+        st["parallel_products_tflops"] = round(2.0 * rows * W * (par_in + par_out) / st["parallel_products_us"] / 1e6, 2)
+        st["ssm_products_tflops"] = round(2.0 * rows * W * (ssm_in + ssm_out) / st["ssm_products_us"] / 1e6, 2)
+        st["gate_up_tflops"] = round(2.0 * rows * W * 2 * ff / st["gate_up_us"] / 1e6, 2)
+        # per row and head: the state's update and its product with the query, 4 flops per state element (fp32)
+        st["linear_attention_tflops_fp32"] = round(rows * RH * rd * rv * 4.0 / st["linear_attention_us"] / 1e6, 3)
+        st["ssm_scan_tflops_fp32"] = round(rows * SH * N * sv * 4.0 / st["ssm_scan_us"] / 1e6, 3)
+        if tag == "decode":
+            st["window_attention_GBps"] = round(rows * keys * 2 * G * hd * 2 / st["window_attention_us"] / 1e3, 1)
+            st["parallel_products_GBps"] = round(W * (par_in + par_out) * 2 / st["parallel_products_us"] / 1e3, 1)
+            st["ssm_products_GBps"] = round(W * (ssm_in + ssm_out) * 2 / st["ssm_products_us"] / 1e3, 1)
+            st["gate_up_GBps"] = round(2 * W * ff * 2 / st["gate_up_us"] / 1e3, 1)
+            st["linear_attention_state_GBps"] = round(rows * RH * rd * rv * 8 / st["linear_attention_us"] / 1e3, 1)
+            st["ssm_scan_state_GBps"] = round(rows * SH * N * sv * 8 / st["ssm_scan_us"] / 1e3, 1)
+        st["layer_stack_us"] = round(b.time_stage(0, 0, 5), 2)
+    stage_times("prefill", P, P)
+    b.release(0)
+    for s_ in range(B):
+        for c0 in range(0, P, 512):
+            b.step([(s_, prompts[s_][c0:c0 + 512])], [], fetch=False)
+    toks = rng.integers(0, V, size=(steps + 8, B), dtype=np.int32)
+    for i in range(8):
+        b.step([(s_, [toks[i][s_]]) for s_ in range(B)], range(B), fetch=False)
+    t0 = time.perf_counter()
+    for i in range(8, 8 + steps):
+        b.step([(s_, [toks[i][s_]]) for s_ in range(B)], range(B), fetch=False)
+        b.step_sample()
+    dt = time.perf_counter() - t0
+    stage_times("decode", B, P)
+    out.update(value=round(B * steps / dt, 1), steps=steps, warmup=8, ms_per_step=round(dt * 1e3 / steps, 4),
+               prefill_tok_s=round(P / t_pf, 1), prefill_ms=round(t_pf * 1e3, 3),
+               prefill_tflops=round(spec.step_flops(P, P // 2) / t_pf / 1e12, 2), stages=stages, vs_baseline=None)
+    b.close()
+    eng.close()
+    out["qwen_equal_size"] = qwen_twin(Q, S, Wt, a.sefelorn, W, H, G, hd, ff, V, P, B, steps, prompts, a.prefill_iters, max_ctx)
     print(json.dumps(out), flush=True)
     return 0
 

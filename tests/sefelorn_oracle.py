@@ -181,3 +181,81 @@ def forward(cfg, W, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return norm(x, W["final.norm"], eps) @ f64(W["embed"]).T * float(cfg["logit_scale"])
+
+
+# ---------------------------------------------------------------- small configurations and random weights
+def dense(ff=40, limit=1.25):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def ssm(heads=4, vdim=12, state=10, groups=2, conv=3, norm_groups=2, mlp="dense"):
+    return {"type": "mamba2", "mixer": {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv,
+                                        "norm_groups": norm_groups}, "mlp": dense() if mlp == "dense" else mlp}
+
+
+def par(heads=4, kv_heads=2, dim=16, vdim=12, size=11, keep=3, rot_dims=8, base=10000.0, scale=None, left=0.9, rec_heads=3,
+        rec_dim=10, rec_vdim=14, tau=4.0, rank=5, right=1.15, mlp="dense"):
+    """rank: rows of a1 - a size only the tensors carry."""
+    a = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": size, "keep_first": keep},
+         "scale": scale if scale is not None else dim ** -0.5}
+    if rot_dims:
+        a["rot"] = {"base": base, "dims": rot_dims}
+    return {"type": "parallel", "mixer": {"left": a, "right": {"heads": rec_heads, "dim": rec_dim, "vdim": rec_vdim, "tau": tau},
+                                          "left_scale": left, "right_scale": right},
+            "mlp": dense() if mlp == "dense" else mlp, "_rank": rank}
+
+
+def config(layers, vocab=101, width=40, eps=1e-5, embed_scale=3.0, logit_scale=0.7, loop=None):
+    cfg = {"architecture": "Sefelorn", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": {"scale": embed_scale},
+           "logit_scale": logit_scale, "layers": [{k: v for k, v in L.items() if k != "_rank"} for L in layers]}
+    if loop:
+        cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
+    cfg["_ranks"] = [L.get("_rank") for L in layers]
+    return cfg
+
+
+def to_bf16_exact(a):
+    """float32 values rounded to the nearest bf16 (kept as float32)."""
+    u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
+    u = (u + 0x7FFF + ((u >> 16) & 1)) & np.uint32(0xFFFF0000)
+    return u.view(np.float32).reshape(np.shape(a))
+
+
+def random_weights(cfg, seed=0, qk_gain=2.0):
+    """{name: float32 array of exact bf16 values} for a config made by config().  The branches' output projections are
+    small beside the residual rows, so that a rounding error shrinks from layer to layer.  qk_gain: how sharp the
+    softmaxes are."""
+    rng = np.random.default_rng(seed)
+    W, V, T = cfg["width"], cfg["vocab"], {}
+
+    def lin(o, i, gain=1.0):
+        return rng.normal(0.0, gain / math.sqrt(i), (o, i))
+
+    def vec(n, sd=0.2, mean=0.0):
+        return mean + rng.normal(0.0, sd, n)
+
+    T["embed"], T["final.norm"] = rng.normal(0, 0.4, (V, W)), vec(W, 0.2, 1.0)
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        T[p + "norm1"] = vec(W, 0.25, 1.0)
+        if L["type"] == "mamba2":
+            x, inner = p + "mix.", m["heads"] * m["vdim"]
+            C = inner + 2 * m["groups"] * m["state"]
+            T[x + "in"], T[x + "conv"], T[x + "conv.b"] = lin(inner + C + m["heads"], W, 1.5), rng.normal(0, 0.6, (C, m["conv"])), vec(C)
+            T[x + "dt_bias"], T[x + "A_log"], T[x + "D"] = vec(m["heads"], 1.0, -1.0), vec(m["heads"], 0.7), vec(m["heads"], 0.4, 0.8)
+            T[x + "norm"], T[x + "o"] = vec(inner, 0.2, 1.0), lin(W, inner, 0.5)
+        else:
+            a, c = m["left"], m["right"]
+            x, H, G = p + "mix.left.", a["heads"], a["kv_heads"]
+            T[x + "q"], T[x + "k"], T[x + "v"] = lin(H * a["dim"], W, qk_gain), lin(G * a["dim"], W, qk_gain), lin(G * a["vdim"], W)
+            T[x + "q.b"], T[x + "k.b"], T[x + "v.b"] = vec(H * a["dim"], 0.5), vec(G * a["dim"], 0.5), vec(G * a["vdim"], 0.5)
+            T[x + "o"] = lin(W, H * a["vdim"], 0.5)
+            x, nk, nv, r = p + "mix.right.", c["heads"] * c["dim"], c["heads"] * c["vdim"], cfg["_ranks"][i]
+            T[x + "q"], T[x + "k"], T[x + "v"], T[x + "g"] = lin(nk, W, 1.5), lin(nk, W, 1.5), lin(nv, W), lin(nv, W)
+            T[x + "a1"], T[x + "a2"], T[x + "a2.b"], T[x + "norm"] = lin(r, W), lin(nk, r, 2.0), vec(nk, 1.0, 1.0), vec(c["vdim"], 0.2, 1.0)
+            T[x + "o"] = lin(W, nv, 0.5)
+        if L.get("mlp") is not None:
+            ff = L["mlp"]["ff"]
+            T[p + "norm2"] = vec(W, 0.25, 1.0)
+            T[p + "mlp.gate"], T[p + "mlp.up"], T[p + "mlp.down"] = lin(ff, W, 1.5), lin(ff, W), lin(W, ff, 0.4)
+    return {k: to_bf16_exact(v) for k, v in T.items()}
