@@ -17,6 +17,7 @@
 #include "engine_impl.hpp"
 #include "k_layered.hpp"
 
+#include <algorithm>
 #include <cmath>
 #include <cstring>
 #include <map>
@@ -162,13 +163,18 @@ struct LayeredBatch {
     std::vector<int4> h_qgroups;
     // recurrent mixers, long entries: pieces of kScanPiece rows scanned side by side (lay::gated_carry); pieces of
     // lin_rows rows for the mixers of lay::linrec_walk
-    PieceList pieces, lin;
+    PieceList pieces, lin[3];         // lin: pieces of 128, 256, 512 rows
     int max_count = 0;
+    int64_t step_T = 0;               // rows of the step being built
+    // parallel blocks: the layer's feed-forward waits for the mixer's input product / is running on side[0]
+    bool ff_wait = false, ff_branch = false;
     bool has_scan = false, has_lin = false;   // layer runs of either kind
-    int64_t lin_units = 0;                    // fewest (head, column tile) blocks of a linear recurrence of the model
+    std::vector<int> lin_units;               // (head, column tile) blocks of the model's linear recurrences
     float *s_loc = nullptr, *s_in = nullptr, *s_decay = nullptr;
     int64_t scan_cap = 0;             // pieces the three buffers hold
-    // parallel blocks: the feed-forward's normed rows
+    // parallel blocks: the feed-forward's normed rows; the branches' events (feed-forward on side[0], a recurrence
+    // beside an attention on side[1])
+    hipEvent_t ev_go[2] = {nullptr, nullptr}, ev_done[2] = {nullptr, nullptr};
     float* y2 = nullptr;
     uint16_t* y2_bf = nullptr;
     int64_t m_state = 0, m_hd = 0;    // largest state / gate row count of a layer run
@@ -772,6 +778,19 @@ static int finalize_ff(LayeredModel* m, int i) {
 }
 
 // ------------------------------------------------------------------ the step
+// Pieces of 128, 256 or 512 rows for a linear recurrence: the longest (least state traffic) that still leaves two blocks a
+// CU in a step of T rows.  units: its (head, column tile) blocks.
+static int lin_units(int heads, int vdim) { return heads * ((vdim + 63) / 64); }
+static int lin_list_of(int64_t T, int units) {
+    const int64_t want = T * units / 512;
+    return want >= 512 ? 2 : want >= 256 ? 1 : 0;
+}
+
+// Rows above which independent branches of a layer run on streams of their own (below, a step is a chain of launches of a
+// few microseconds each, and the events between the streams cost more than the overlap gains: 2k Sefelorn size, 8 rows
+// 0.515 -> 0.536 ms a step; 2,048 rows 2.73 -> 2.62 ms)
+constexpr int kBranchRows = 64;
+
 static int lin(const qie_engine* e, const float* A, int64_t lda, const void* Wt, int64_t ldw, float* Y, int64_t ldy, int M, int N,
                int K, int batch = 1, int64_t sA = 0, int64_t sW = 0, int64_t sY = 0, const int32_t* grp = nullptr) {
     lay::LinearP p{A, lda, Wt, ldw, Y, ldy, M, N, K, batch, sA, sW, sY, e->lm->f32 ? 0 : 1, grp, e->lm->f32 ? 0 : 1};
@@ -810,9 +829,28 @@ static int dense_on(qie_batch* b, uint16_t* abf, bool staged, const float* A, in
 }
 // pre: the bf16 image of A (row stride K) when its producer wrote one
 static int dense(qie_batch* b, const float* A, int64_t lda, const void* Wt, float* Y, int64_t ldy, int M, int N, int K,
-                 const uint16_t* pre = nullptr) {
-    if (pre && lda == K) return dense_on(b, const_cast<uint16_t*>(pre), true, A, lda, Wt, Y, ldy, M, N, K);
-    return dense_on(b, b->lb->abf, false, A, lda, Wt, Y, ldy, M, N, K);
+                 const uint16_t* pre = nullptr, hipStream_t on = nullptr) {
+    if (pre && lda == K) return dense_on(b, const_cast<uint16_t*>(pre), true, A, lda, Wt, Y, ldy, M, N, K, on);
+    return dense_on(b, b->lb->abf, false, A, lda, Wt, Y, ldy, M, N, K, on);
+}
+
+// A bf16 engine's products read the bf16 image of rows of K columns and nothing else (dense_on): their producers may
+// leave the fp32 rows unwritten.
+static bool image_only(const LayeredModel* m, int64_t K) { return !m->f32 && K % 8 == 0; }
+static float* ov_out(const qie_batch* b, const LayerDev& L) { return image_only(b->e->lm, L.n_cat) ? nullptr : b->lb->ov; }
+
+// `side` runs what follows beside the engine's stream, from here until branch_join
+static int branch_fork(qie_batch* b, int k) {
+    LayeredBatch* s = b->lb;
+    QIE_HIP(hipEventRecord(s->ev_go[k], b->e->stream));
+    QIE_HIP(hipStreamWaitEvent(s->side[k], s->ev_go[k], 0));
+    return 0;
+}
+static int branch_join(qie_batch* b, int k) {
+    LayeredBatch* s = b->lb;
+    QIE_HIP(hipEventRecord(s->ev_done[k], s->side[k]));
+    QIE_HIP(hipStreamWaitEvent(b->e->stream, s->ev_done[k], 0));
+    return 0;
 }
 
 static lay::LatentCache cache_of(const qie_batch* b) {
@@ -982,29 +1020,29 @@ static int enq_mixer_out(qie_batch* b, int i, int T) {
 
 // feed-forward of layer i on its normed rows (s->y, in parallel blocks s->y2) -> ffo; where the layer's output product
 // takes the activations as well (cat_ff), they go beside the mixer's columns and the product is left to it
-static int enq_ff(qie_batch* b, int i, int T) {
+static int enq_ff(qie_batch* b, int i, int T, hipStream_t on = nullptr) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
     const LayerDev& L = m->L[i];
     const qie_layer_desc& d = L.d;
     LayeredBatch* s = b->lb;
     const int W = m->a.width, ff = d.ff;
-    hipStream_t st = e->stream;
+    hipStream_t st = on ? on : e->stream;
     const bool par = m->a.block == QIE_BLOCK_PARALLEL;
     const float* y = par ? s->y2 : s->y;
     const uint16_t* y_bf = par ? s->y2_bf : s->y_bf;
     if (d.ff_kind == QIE_FF_DENSE && d.ff_act == QIE_ACT_XIELU) {
-        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, ff, T, ff, W, y_bf));
+        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, ff, T, ff, W, y_bf, st));
         QIE_TRY(lay::xielu(s->gu, s->act, s->act_bf, (int64_t)T * ff, L.act_p, L.act_q, st));
-        return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf);
+        return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf, st);
     }
     if (d.ff_kind == QIE_FF_DENSE) {
-        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, y_bf));
+        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, y_bf, st));
         const int act = d.ff_act == QIE_ACT_GELU_TANH_GATED ? 1 : d.ff_act == QIE_ACT_CLAMPED_GATED ? 2 : 0;
         if (L.cat_ff >= 0)
-            return lay::silu_mul(s->gu, s->ov + L.cat_ff, s->ov_bf ? s->ov_bf + L.cat_ff : nullptr, T, ff, st, act, d.ff_limit, L.n_cat);
-        QIE_TRY(lay::silu_mul(s->gu, s->act, s->act_bf, T, ff, st, act, d.ff_limit));
-        return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf);
+            return lay::silu_mul(s->gu, image_only(m, L.n_cat) ? nullptr : s->ov + L.cat_ff, s->ov_bf ? s->ov_bf + L.cat_ff : nullptr, T, ff, st, act, d.ff_limit, L.n_cat);
+        QIE_TRY(lay::silu_mul(s->gu, image_only(m, ff) ? nullptr : s->act, s->act_bf, T, ff, st, act, d.ff_limit));
+        return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf, st);
     }
     const int E = d.experts, top = d.top, n = T * top;
     const bool out_w = d.router != QIE_ROUTER_SIGMOID_IN;   // the scores weight the outputs, not the inputs
@@ -1093,7 +1131,7 @@ static lay::GqaAttnP gqa_attn_params(qie_batch* b, int r) {
     p.v_off = s->v_off[r];
     p.v_transposed = s->vt_of[r];
     p.out_scale = L.d.mixer == QIE_MIXER_GQA_RECURRENT ? L.d.gqa_scale : 1.0f;
-    p.out = s->ov; p.out_bf = s->ov_bf; p.ld_out = L.n_cat; p.out_col = 0;
+    p.out = ov_out(b, L); p.out_bf = s->ov_bf; p.ld_out = L.n_cat; p.out_col = 0;
     p.slopes = a.slope_bias ? L.slopes : nullptr;
     p.pb = a.weights == QIE_WEIGHTS_SIGMOID ? L.pb : nullptr;
     p.gate_col = (a.head_gate || a.out_gate) ? L.col_gate : -1;
@@ -1140,6 +1178,7 @@ static int enq_gqa_post(qie_batch* b, int r, int T) {
     p.q_bias = a.qk_bias ? L.q_bias : nullptr;
     p.k_bias = a.qk_bias ? L.k_bias : nullptr;
     p.v_bias = a.v_bias ? L.v_bias : nullptr;
+    p.groups = s->d_qgroups; p.n_groups = s->n_qgroups;
     return lay::gqa_post(p, m->f32, T, e->stream);
 }
 
@@ -1184,11 +1223,12 @@ constexpr int kScanLong = 128, kScanPiece = 64;
 // Rows of an entry up to which a linear recurrence takes them in order on the vector units
 constexpr int kLinStep = 8;
 
+static bool lin_steps(const LayeredBatch* s, int dim, int vdim) { return s->max_count <= kLinStep || !lay::linrec_walk_fits(dim, vdim); }
+
 // The linear recurrence p of layer run r (its state and outputs are filled in here).  Entries of more rows than a
 // piece: end states and decays of the pieces from zero, a carry over each entry's pieces, then the outputs from the
 // states that enter them.
-static int enq_linrec(qie_batch* b, int r, lay::LinRecP p) {
-    const qie_engine* e = b->e;
+static int enq_linrec(qie_batch* b, int r, lay::LinRecP p, hipStream_t st) {
     LayeredBatch* s = b->lb;
     p.entries = s->d_ent; p.n_entries = s->n_ent;
     p.init = p.end = s->state;
@@ -1196,44 +1236,50 @@ static int enq_linrec(qie_batch* b, int r, lay::LinRecP p) {
     p.init_off = p.end_off = s->state_off[r];
     p.init_if_pos = 1;
     p.out = s->olat;
-    if (s->max_count <= kLinStep || !lay::linrec_walk_fits(p.dim, p.vdim)) return lay::linrec_step(p, e->stream);
-    if (s->max_count <= s->lin.rows || !s->s_loc) return lay::linrec_walk(p, e->stream);
+    if (lin_steps(s, p.dim, p.vdim)) return lay::linrec_step(p, st);
+    const PieceList& pl = s->lin[lin_list_of(s->step_T, lin_units(p.heads, p.vdim))];
+    if (s->max_count <= pl.rows) return lay::linrec_walk(p, st);
     const int64_t n = (int64_t)p.heads * p.dim * p.vdim;
     lay::LinRecP a = p;
-    a.entries = s->lin.d_chunks; a.n_entries = s->lin.n;
+    a.entries = pl.d_chunks; a.n_entries = pl.n;
     a.init = nullptr;
     a.end = s->s_loc; a.end_stride = n; a.end_off = 0;
     a.decay = s->s_decay;
     a.out = nullptr;
-    QIE_TRY(lay::linrec_walk(a, e->stream));
-    lay::LinRecCarryP k{s->lin.d_spans, s->n_ent, p.heads, p.dim, p.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
+    QIE_TRY(lay::linrec_walk(a, st));
+    lay::LinRecCarryP k{pl.d_spans, s->n_ent, p.heads, p.dim, p.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
                         s->state_off[r]};
-    QIE_TRY(lay::linrec_carry(k, e->stream));
+    QIE_TRY(lay::linrec_carry(k, st));
     a.init = s->s_in; a.init_stride = n; a.init_off = 0; a.init_if_pos = 0;
     a.end = nullptr; a.decay = nullptr;
     a.out = p.out;
-    return lay::linrec_walk(a, e->stream);
+    return lay::linrec_walk(a, st);
 }
 
 // Gated linear attention of layer run r: log decays through the low-rank projection, the recurrence, head norm and gate
-static int enq_key_decay(qie_batch* b, int r, int T) {
+static int enq_key_decay(qie_batch* b, int r, int T, hipStream_t st) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     const qie_recurrent_desc& c = L.d.rec;
     LayeredBatch* s = b->lb;
-    QIE_TRY(lay::low_rank_log_sigmoid(s->proj + L.col_a1, L.n_in, L.rank_a, L.w_a2, m->f32, L.rec_a2b, c.tau, c.heads * c.dim, T, s->qabs,
-                                      e->stream));
     lay::LinRecP p{};
+    if (lin_steps(s, c.dim, c.vdim)) {   // few rows: the recurrence makes its decays itself
+        p.lr_in = s->proj + L.col_a1; p.ld_lr = L.n_in; p.rank = L.rank_a;
+        p.lr_w = L.w_a2; p.lr_w_f32 = m->f32; p.lr_bias = L.rec_a2b; p.inv_tau = 1.0f / c.tau;
+    } else {
+        QIE_TRY(lay::low_rank_log_sigmoid(s->proj + L.col_a1, L.n_in, L.rank_a, L.w_a2, m->f32, L.rec_a2b, c.tau, c.heads * c.dim, T,
+                                          s->qabs, st));
+        p.log_decay = s->qabs;
+    }
     p.q = s->proj + L.col_rq; p.k = s->proj + L.col_rk; p.v = s->proj + L.col_rv;
     p.ldq = p.ldk = p.ldv = L.n_in;
     p.rep = 1;
     p.q_scale = 1.0f / sqrtf((float)c.dim);
-    p.log_decay = s->qabs;
     p.heads = c.heads; p.dim = c.dim; p.vdim = c.vdim;
-    QIE_TRY(enq_linrec(b, r, p));
-    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, s->ov, s->ov_bf, L.n_cat,
-                               L.cat_rec, e->stream, s->proj + L.col_rg, L.n_in, 1);
+    QIE_TRY(enq_linrec(b, r, p, st));
+    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
+                               L.cat_rec, st, s->proj + L.col_rg, L.n_in, 1);
 }
 
 // State space of layer run r on its projection rows: convolution, recurrence, gate and norm in parts
@@ -1260,18 +1306,18 @@ static int enq_state_space(qie_batch* b, int r, int T) {
     p.dt = s->proj + L.col_dt; p.ld_dt = L.n_in;
     p.dt_bias = L.ss_dt_bias; p.a_h = L.ss_a; p.skip = L.ss_d;
     p.heads = c.heads; p.dim = c.state; p.vdim = c.vdim;
-    QIE_TRY(enq_linrec(b, r, p));
-    return lay::gated_norm_parts(s->olat, s->proj, L.n_in, L.ss_norm, m->a.norm_eps, inner, c.norm_groups, T, s->ov, s->ov_bf, L.n_cat,
+    QIE_TRY(enq_linrec(b, r, p, e->stream));
+    return lay::gated_norm_parts(s->olat, s->proj, L.n_in, L.ss_norm, m->a.norm_eps, inner, c.norm_groups, T, ov_out(b, L), s->ov_bf, L.n_cat,
                                  e->stream);
 }
 
-static int enq_recurrence(qie_batch* b, int r, int T) {
+static int enq_recurrence(qie_batch* b, int r, int T, hipStream_t on = nullptr) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     const qie_recurrent_desc& c = L.d.rec;
     LayeredBatch* s = b->lb;
-    if (c.kind == QIE_REC_KEY_DECAY) return enq_key_decay(b, r, T);
+    if (c.kind == QIE_REC_KEY_DECAY) return enq_key_decay(b, r, T, on ? on : e->stream);
     lay::GatedScanP p{};
     p.proj = s->proj; p.ld = L.n_in; p.q_col = L.col_rq; p.f_col = L.col_rf; p.v_col = L.col_rv;
     p.entries = s->d_ent; p.n_entries = s->n_ent;
@@ -1294,11 +1340,11 @@ static int enq_recurrence(qie_batch* b, int r, int T) {
         a.decay = nullptr;
         a.out = s->qabs;
         QIE_TRY(lay::gated_scan(a, e->stream));
-        return lay::head_norm_rows(s->olat, s->qabs, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, s->ov, s->ov_bf,
+        return lay::head_norm_rows(s->olat, s->qabs, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf,
                                    L.n_cat, L.cat_rec, e->stream);
     }
     QIE_TRY(lay::gated_scan(p, e->stream));
-    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, s->ov, s->ov_bf, L.n_cat,
+    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
                                L.cat_rec, e->stream);
 }
 
@@ -1310,12 +1356,32 @@ static int enq_out(qie_batch* b, int r, int T) {
     return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
 }
 
+// Parallel blocks, prompt-sized steps: the feed-forward starts on its side stream here, where the mixer's kernels that do
+// not fill the chip begin (beside the input product it would only share the matrix cores with it)
+static int start_ff(qie_batch* b, int r, int T) {
+    LayeredBatch* s = b->lb;
+    if (!s->ff_wait) return 0;
+    s->ff_wait = false;
+    QIE_TRY(branch_fork(b, 0));
+    s->ff_branch = true;
+    return enq_ff(b, b->e->lm->runs[r].layer, T, s->side[0]);
+}
+
+static int join_ff(qie_batch* b) {
+    LayeredBatch* s = b->lb;
+    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
+    s->ff_branch = false;
+    return 0;
+}
+
 static int enq_state_space_mixer(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
     QIE_TRY(dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf));
+    QIE_TRY(start_ff(b, r, T));
     QIE_TRY(enq_state_space(b, r, T));
+    QIE_TRY(join_ff(b));
     return enq_out(b, r, T);
 }
 
@@ -1324,9 +1390,18 @@ static int enq_gqa_mixer(qie_batch* b, int r, int T) {
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
     QIE_TRY(enq_gqa_proj(b, r, T));
+    // a recurrence of kind key decay runs beside the attention (their scratch and their columns are apart)
+    const bool rec = L.d.mixer == QIE_MIXER_GQA_RECURRENT, beside = rec && L.d.rec.kind == QIE_REC_KEY_DECAY && T > kBranchRows;
+    if (beside) {
+        QIE_TRY(branch_fork(b, 1));
+        QIE_TRY(enq_recurrence(b, r, T, s->side[1]));
+    }
     QIE_TRY(enq_gqa_post(b, r, T));
+    QIE_TRY(start_ff(b, r, T));
     QIE_TRY(enq_gqa_attention(b, r, T));
-    if (L.d.mixer == QIE_MIXER_GQA_RECURRENT) QIE_TRY(enq_recurrence(b, r, T));
+    if (rec && !beside) QIE_TRY(enq_recurrence(b, r, T));
+    if (beside) QIE_TRY(branch_join(b, 1));
+    QIE_TRY(join_ff(b));
     return enq_out(b, r, T);
 }
 
@@ -1454,7 +1529,7 @@ static int enq_delta_scan(qie_batch* b, int r, int T, bool advance) {
     } else {
         QIE_TRY(lay::delta_scan(sp, e->stream));
     }
-    return lay::head_norm_rows(s->olat, nullptr, L.dl_norm, m->a.norm_eps, 1.0f, c.heads, c.vdim, T, s->ov, s->ov_bf, L.n_cat, 0,
+    return lay::head_norm_rows(s->olat, nullptr, L.dl_norm, m->a.norm_eps, 1.0f, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat, 0,
                                e->stream, s->aux);
 }
 
@@ -1586,12 +1661,18 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
     float* x0 = s->stack;
     float* x = s->stack + plane;
     auto norms = [&](const float* xin, const float* v, const float* v2, const float* add, const LayerDev* N) -> int {
-        lay::NormPairP p{x, xin, v, v2, add, N ? N->n1 : nullptr, N ? N->n2 : nullptr, s->y, s->y2, s->y_bf, s->y2_bf, T, W, m->a.norm_eps};
+        const bool img = image_only(m, W);
+        lay::NormPairP p{x, xin, v, v2, add, N ? N->n1 : nullptr, N ? N->n2 : nullptr, img ? nullptr : s->y,
+                         img && N && N->d.ff_kind != QIE_FF_MOE ? nullptr : s->y2, s->y_bf, s->y2_bf, T, W, m->a.norm_eps};
         return lay::norm_pair(p, e->stream);
     };
     if (!h_ready) QIE_TRY(norms(r == 0 && m->loops ? x0 : x, nullptr, nullptr, m->runs[r].add_embed ? x0 : nullptr, &L));
     const bool has_ff = L.d.ff_kind != QIE_FF_NONE;
-    if (has_ff) QIE_TRY(enq_ff(b, m->runs[r].layer, T));
+    // the feed-forward beside the mixer (the experts' products have side streams of their own)
+    const bool starts = L.d.mixer == QIE_MIXER_STATE_SPACE || L.d.mixer == QIE_MIXER_GQA || L.d.mixer == QIE_MIXER_GQA_RECURRENT;
+    s->ff_wait = L.d.ff_kind == QIE_FF_DENSE && T > kBranchRows && starts;
+    s->ff_branch = false;
+    if (has_ff && !s->ff_wait) QIE_TRY(enq_ff(b, m->runs[r].layer, T));
     switch (L.d.mixer) {
         case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
         case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
@@ -1944,8 +2025,8 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
     }
     int64_t off = 0;
     auto lin = [&](int64_t heads, int64_t dim, int64_t vdim) {   // a run on lay::linrec_*
-        const int64_t units = heads * ((vdim + 63) / 64);
-        s->lin_units = s->has_lin ? std::min(s->lin_units, units) : units;
+        const int units = lin_units((int)heads, (int)vdim);
+        if (std::find(s->lin_units.begin(), s->lin_units.end(), units) == s->lin_units.end()) s->lin_units.push_back(units);
         s->has_lin = true;
         s->m_state = std::max<int64_t>(s->m_state, heads * dim * vdim);
         s->m_hd = std::max<int64_t>(s->m_hd, heads * dim);
@@ -2087,6 +2168,10 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
             he = hipStreamCreateWithFlags(&s->side[i], hipStreamNonBlocking);
             if (he == hipSuccess) he = hipEventCreateWithFlags(&s->ev_join[i], hipEventDisableTiming);
         }
+        for (int i = 0; i < 2 && he == hipSuccess; i++) {
+            he = hipEventCreateWithFlags(&s->ev_go[i], hipEventDisableTiming);
+            if (he == hipSuccess) he = hipEventCreateWithFlags(&s->ev_done[i], hipEventDisableTiming);
+        }
         if (he != hipSuccess) rc = fail((int)he, "batch init (side streams): %s", hipGetErrorString(he));
     }
     if (rc) {
@@ -2102,10 +2187,17 @@ void layered_batch_destroy(qie_batch* b) {
     if (!s) return;
     lb_free(s);
     void* ps[] = {s->want, s->xn, s->logits, s->logits_bf, s->d_ids, s->d_step, s->d_groups, s->part_o, s->part_ml, s->xn_bf,
-                  s->state, s->d_ent, s->d_qgroups, s->gpart_o, s->gpart_ml, s->pieces.d_chunks, s->pieces.d_spans, s->lin.d_chunks, s->lin.d_spans, s->s_loc, s->s_in,
-                  s->s_decay};
+                  s->state, s->d_ent, s->d_qgroups, s->gpart_o, s->gpart_ml, s->pieces.d_chunks, s->pieces.d_spans, s->s_loc, s->s_in, s->s_decay};
     for (void* p : ps)
         if (p) hipFree(p);
+    for (PieceList& l : s->lin) {
+        if (l.d_chunks) hipFree(l.d_chunks);
+        if (l.d_spans) hipFree(l.d_spans);
+    }
+    for (int i = 0; i < 2; i++) {
+        if (s->ev_go[i]) hipEventDestroy(s->ev_go[i]);
+        if (s->ev_done[i]) hipEventDestroy(s->ev_done[i]);
+    }
     if (s->h_stage) hipHostFree(s->h_stage);
     for (int i = 0; i < LayeredBatch::kSide; i++) {
         if (s->side[i]) hipStreamSynchronize(s->side[i]);
@@ -2416,14 +2508,15 @@ int qie_batch_step(qie_batch* b, int32_t n_entries, const int32_t* slots, const 
         QIE_HIP(hipMemcpyAsync(s->d_qgroups, s->h_qgroups.data(), s->h_qgroups.size() * sizeof(int4), hipMemcpyHostToDevice, st));
         s->n_ent = n_entries;
         s->n_qgroups = (int)s->h_qgroups.size();
+        s->step_T = T;
         s->max_count = 0;
         for (int i = 0; i < n_entries; i++) s->max_count = std::max(s->max_count, (int)counts[i]);
         if (s->has_scan && s->max_count > kScanLong) QIE_TRY(build_pieces(b, s->pieces, kScanPiece));
-        if (s->has_lin) {
-            // linear recurrences: long pieces (less state traffic) as long as two blocks a CU remain
-            const int64_t want = T * s->lin_units / 512;
-            s->lin.rows = want >= 512 ? 512 : want >= 256 ? 256 : 128;
-            if (s->max_count > s->lin.rows) QIE_TRY(build_pieces(b, s->lin, s->lin.rows));
+        for (int k = 0; k < 3 && s->has_lin; k++) {
+            s->lin[k].rows = 128 << k;
+            bool used = false;
+            for (int u : s->lin_units) used = used || lin_list_of(T, u) == k;
+            if (used && s->max_count > s->lin[k].rows) QIE_TRY(build_pieces(b, s->lin[k], s->lin[k].rows));
         }
     }
     QIE_HIP(hipMemcpyAsync(s->row_slot, hs, (size_t)T * 4, hipMemcpyHostToDevice, st));

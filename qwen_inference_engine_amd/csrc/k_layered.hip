@@ -561,30 +561,51 @@ int depth_mix(const float* stack, int64_t stride, const float* a, int n, float* 
 // a[m, j] = silu(gu[m, j]) * gu[m, ff + j]
 // (act 1: the tanh form of gelu instead of silu, gelu(g) = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)));
 // act 2: g sigmoid(1.702 g) (u + 1) with the gate cut at limit and u clamped to +-limit)
-__global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a, uint16_t* a_bf, int ff, int64_t n, int act, float limit,
-                                                       int64_t ld_a) {
-    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= n) return;
-    const int64_t m = i / ff;
-    const int j = (int)(i % ff);
-    const float g = gu[m * 2 * ff + j], u = gu[m * 2 * ff + ff + j];
-    const int64_t oi = m * ld_a + j;
+__device__ __forceinline__ float gated_act(float g, float u, int act, float limit) {
     if (act == 2) {
         const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit);
-        const float oc = gc / (1.0f + expf(-1.702f * gc)) * (uc + 1.0f);
-        a[oi] = oc;
-        if (a_bf) a_bf[oi] = f2bf(oc);
-        return;
+        return gc / (1.0f + expf(-1.702f * gc)) * (uc + 1.0f);
     }
-    const float o = (act == 1 ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g))) * u;
-    a[oi] = o;
-    if (a_bf) a_bf[oi] = f2bf(o);
+    return (act == 1 ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) : g / (1.0f + expf(-g))) * u;
+}
+// V consecutive columns per thread (V = 4: ff and ld_a multiples of 4)
+template <int V>
+__global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a, uint16_t* a_bf, int ff, uint32_t n, int act, float limit,
+                                                       int64_t ld_a) {
+    const uint32_t i = blockIdx.x * 256u + threadIdx.x;
+    if (i >= n) return;
+    const uint32_t per = (uint32_t)ff / V, m = i / per, j = (i - m * per) * V;
+    const float* gp = gu + (int64_t)m * 2 * ff + j;
+    float g[V], u[V], o[V];
+    if constexpr (V == 4) {
+        *reinterpret_cast<float4*>(g) = *reinterpret_cast<const float4*>(gp);
+        *reinterpret_cast<float4*>(u) = *reinterpret_cast<const float4*>(gp + ff);
+    } else {
+        g[0] = gp[0];
+        u[0] = gp[ff];
+    }
+#pragma unroll
+    for (int k = 0; k < V; k++) o[k] = gated_act(g[k], u[k], act, limit);
+    const int64_t oi = (int64_t)m * ld_a + j;
+    if constexpr (V == 4) {
+        if (a) *reinterpret_cast<float4*>(a + oi) = *reinterpret_cast<float4*>(o);
+        if (a_bf) *reinterpret_cast<uint2*>(a_bf + oi) = make_uint2(pack2(o[0], o[1]), pack2(o[2], o[3]));
+    } else {
+        if (a) a[oi] = o[0];
+        if (a_bf) a_bf[oi] = f2bf(o[0]);
+    }
 }
 int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act, float limit, int64_t ld_a) {
-    const int64_t n = M * ff;
-    if (n == 0) return 0;
-    hipLaunchKernelGGL(silu_mul_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, gu, a, a_bf, ff, n, act,
-                       limit, ld_a ? ld_a : (int64_t)ff);
+    if (M * ff == 0) return 0;
+    if (!ld_a) ld_a = ff;
+    QIE_REQUIRE(M * ff < ((int64_t)1 << 32), "gated activation: %lld values in one launch", (long long)(M * ff));
+    const bool v4 = ff % 4 == 0 && ld_a % 4 == 0 && ((uintptr_t)gu & 15) == 0 && ((uintptr_t)a & 15) == 0 && ((uintptr_t)a_bf & 7) == 0;
+    const int64_t n = v4 ? M * ff / 4 : M * ff;
+    const dim3 grid((unsigned)((n + 255) / 256));
+    if (v4)
+        hipLaunchKernelGGL(silu_mul_kernel<4>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a);
+    else
+        hipLaunchKernelGGL(silu_mul_kernel<1>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a);
     QIE_LAUNCH_CHECK();
     return 0;
 }
@@ -872,22 +893,37 @@ int moe_combine(const float* yd, const int32_t* slot_of, const float* score, int
 }
 
 // ------------------------------------------------------------------ greedy choice on fp32 rows
-// ids[m] = the index of the largest logit of row m (ties: the lowest index).  One block per row.
-__global__ __launch_bounds__(256) void argmax_rows_kernel(const float* x, int64_t V, int32_t* ids) {
-    __shared__ float bv[256];
-    __shared__ int bi[256];
+// ids[m] = the index of the largest logit of row m (ties: the lowest index).  One block per row; rows of whole float4s
+// are read so.
+constexpr int AM = 1024;
+__global__ __launch_bounds__(AM) void argmax_rows_kernel(const float* x, int64_t V, int32_t* ids) {
+    __shared__ float bv[AM];
+    __shared__ int bi[AM];
     const float* r = x + (int64_t)blockIdx.x * V;
     float v = -INFINITY;
     int idx = 0x7fffffff;
-    for (int64_t i = threadIdx.x; i < V; i += 256)
-        if (r[i] > v) {
-            v = r[i];
+    auto take = [&](float a, int64_t i) {
+        if (a > v) {
+            v = a;
             idx = (int)i;
         }
+    };
+    if ((V & 3) == 0) {
+#pragma unroll 4
+        for (int64_t i = (int64_t)threadIdx.x * 4; i < V; i += AM * 4) {
+            const float4 a = *reinterpret_cast<const float4*>(r + i);
+            take(a.x, i);
+            take(a.y, i + 1);
+            take(a.z, i + 2);
+            take(a.w, i + 3);
+        }
+    } else {
+        for (int64_t i = threadIdx.x; i < V; i += AM) take(r[i], i);
+    }
     bv[threadIdx.x] = v;
     bi[threadIdx.x] = idx;
     __syncthreads();
-    for (int o = 128; o > 0; o >>= 1) {
+    for (int o = AM / 2; o > 0; o >>= 1) {
         if ((int)threadIdx.x < o) {
             const float w = bv[threadIdx.x + o];
             const int j = bi[threadIdx.x + o];
@@ -901,7 +937,7 @@ __global__ __launch_bounds__(256) void argmax_rows_kernel(const float* x, int64_
     if (threadIdx.x == 0) ids[blockIdx.x] = bi[0] == 0x7fffffff ? 0 : bi[0];
 }
 int argmax_rows(const float* x, int M, int64_t V, int32_t* ids, hipStream_t st) {
-    hipLaunchKernelGGL(argmax_rows_kernel, dim3(M), dim3(256), 0, st, x, V, ids);
+    hipLaunchKernelGGL(argmax_rows_kernel, dim3(M), dim3(AM), 0, st, x, V, ids);
     QIE_LAUNCH_CHECK();
     return 0;
 }

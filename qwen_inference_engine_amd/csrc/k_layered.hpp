@@ -136,6 +136,10 @@ struct GqaPostP {
     const float* q_bias;      // [heads * dim] / [kv_heads * dim] or null: added to q / k as they leave the projection
     const float* k_bias;      //   (a key cached as the value carries its bias)
     const float* v_bias;      // [kv_heads * vdim] or null: added to v as it leaves the projection
+    // optional: the step's groups of up to 16 consecutive rows {first packed row, rows, slot, first position};
+    // transposed values of prompt-sized steps are then written 16 tokens at a time
+    const int4* groups;
+    int n_groups;
 };
 int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st);
 
@@ -163,7 +167,7 @@ struct GqaAttnP {
     int64_t k_off, v_off;
     int v_transposed;
     float out_scale;
-    float* out;
+    float* out;               // null: only the bf16 image is wanted
     uint16_t* out_bf;
     int64_t ld_out;
     int out_col;
@@ -296,7 +300,7 @@ int head_norm_rows(const float* o, const float* o2, const float* w, float eps, f
 int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* w, float eps, int n, int parts, int T, float* out,
                      uint16_t* out_bf, int64_t ld_out, hipStream_t st);
 // Rows of W, two norms of one row: x = xin + v (when v) + v2 (when v2) + add (when add); h1 = rms(x) w1, h2 = rms(x) w2
-// (each with its bf16 image; null w1: neither norm is made, null w2: only the first)
+// (each fp32, as its bf16 image, or both; null w1: neither norm is made, null w2: only the first)
 struct NormPairP {
     float* x;
     const float *xin, *v, *v2, *add;
@@ -307,6 +311,7 @@ struct NormPairP {
     float eps;
 };
 int norm_pair(const NormPairP& p, hipStream_t st);
+// (head_norm_rows, gated_norm_parts, silu_mul: a null fp32 output leaves the bf16 image alone)
 
 // ------------------------------------------------------------------ residual streams (k_streams.hip)
 // n residual rows per token, X + s * plane (rows of W).  With y (a sublayer's result, [T][W]) the rows
@@ -447,6 +452,13 @@ struct LinRecP {
     const float* dt;
     int64_t ld_dt;
     const float *dt_bias, *a_h, *skip;
+    // linrec_step alone: the log decays straight from their low-rank projection (as low_rank_log_sigmoid makes them)
+    const float* lr_in;
+    int64_t ld_lr;
+    const void* lr_w;
+    int lr_w_f32, rank;
+    const float* lr_bias;
+    float inv_tau;
     int heads, dim, vdim;
     const int4* entries;
     int n_entries;

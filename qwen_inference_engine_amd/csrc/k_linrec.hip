@@ -21,6 +21,34 @@ __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1
 
 }  // namespace
 
+// One value of the low-rank log decay (LinRecP.lr_in)
+__device__ __forceinline__ float low_rank_log(const LinRecP& p, int64_t t, int c) {
+    const float* a = p.lr_in + t * p.ld_lr;
+    float z = 0.f;
+    if (p.lr_w_f32) {
+        const float* w = (const float*)p.lr_w + (int64_t)c * p.rank;
+        for (int r = 0; r < p.rank; r++) z = fmaf(w[r], a[r], z);
+    } else {
+        const uint16_t* w = (const uint16_t*)p.lr_w + (int64_t)c * p.rank;
+        int r = 0;
+        if ((p.rank & 7) == 0)
+#pragma unroll 2
+            for (; r < p.rank; r += 8) {
+                const uint4 u = *reinterpret_cast<const uint4*>(w + r);
+                z = fmaf(bf2f(u.x & 0xffffu), a[r], z);
+                z = fmaf(bf2f(u.x >> 16), a[r + 1], z);
+                z = fmaf(bf2f(u.y & 0xffffu), a[r + 2], z);
+                z = fmaf(bf2f(u.y >> 16), a[r + 3], z);
+                z = fmaf(bf2f(u.z & 0xffffu), a[r + 4], z);
+                z = fmaf(bf2f(u.z >> 16), a[r + 5], z);
+                z = fmaf(bf2f(u.w & 0xffffu), a[r + 6], z);
+                z = fmaf(bf2f(u.w >> 16), a[r + 7], z);
+            }
+        for (; r < p.rank; r++) z = fmaf(bf2f(w[r]), a[r], z);
+    }
+    return -softplus(-(z + p.lr_bias[c])) * p.inv_tau;
+}
+
 // ------------------------------------------------------------------ rows in order
 // One block per (head, entry, 64 value columns); a thread owns SR state rows of one column, blockDim / 64 thread
 // groups split dim.  TT rows a turn: their q, k and decays staged in LDS, the groups' partial outputs summed there.
@@ -62,8 +90,10 @@ __global__ __launch_bounds__(1024) void linrec_step_kernel(LinRecP p, int dimP) 
                     const float dt = softplus(p.dt[t * p.ld_dt + h] + db);
                     a = expf(-ah * dt);
                     k *= dt;
-                } else {
+                } else if (p.log_decay) {
                     a = expf(p.log_decay[t * p.heads * dim + (int64_t)h * dim + d]);
+                } else {
+                    a = expf(low_rank_log(p, t, h * dim + d));
                 }
             }
             qs[i] = q;
@@ -105,7 +135,8 @@ __global__ __launch_bounds__(1024) void linrec_step_kernel(LinRecP p, int dimP) 
 
 static int linrec_check(const LinRecP& p) {
     QIE_REQUIRE(p.q && p.k && p.v && p.entries && p.n_entries > 0 && p.heads > 0 && p.dim > 0 && p.vdim > 0 && p.rep > 0 &&
-                    p.heads % p.rep == 0 && ((p.log_decay != nullptr) != (p.dt != nullptr)) && (!p.dt || (p.dt_bias && p.a_h)),
+                    p.heads % p.rep == 0 && (p.log_decay != nullptr) + (p.dt != nullptr) + (p.lr_in != nullptr) == 1 &&
+                    (!p.dt || (p.dt_bias && p.a_h)) && (!p.lr_in || (p.lr_w && p.lr_bias && p.rank > 0)),
                 "linear recurrence: bad arguments");
     return 0;
 }
@@ -143,7 +174,7 @@ constexpr int kStage = 32;
 constexpr float kSpan = 40.f;
 
 template <int DT, bool SCALAR>
-__global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
+__global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p, int vec) {
     constexpr int dimP = 16 * DT, LQ = dimP + 4, LV = 68, LP = 20, NI = (2 * dimP + 255) / 256;
     __shared__ __align__(16) float qs[kStage * LQ];
     __shared__ __align__(16) float ks[kStage * LQ];
@@ -152,7 +183,9 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
     __shared__ __align__(16) float wt[SCALAR ? 4 : 2 * dimP];      // key decay: e^(-L) per tile and channel
     __shared__ __align__(16) float et[SCALAR ? 4 : 2 * dimP];      // e^L per tile (and channel)
     __shared__ float sL[SCALAR ? kStage : 1], sdt[SCALAR ? kStage : 1], eL[SCALAR ? kStage : 1], kf[SCALAR ? kStage : 1];
-    const int h = blockIdx.x, c0 = blockIdx.z * 64, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, n = lane & 15;
+    // neighbouring blocks go to different dies: heads that share q and k rows sit 8 blocks apart, on one die's cache
+    const int h = p.heads % 8 == 0 ? (int)(blockIdx.x % 8) * (p.heads / 8) + (int)(blockIdx.x / 8) : (int)blockIdx.x;
+    const int c0 = blockIdx.z * 64, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, n = lane & 15;
     const int4 en = p.entries[blockIdx.y];
     const int dim = p.dim, vdim = p.vdim, col = c0 + wave * 16 + n;
     const bool cok = col < vdim, outs = p.out != nullptr;
@@ -170,27 +203,55 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
                 S[j][i] = (warm && d < dim) ? st0[(int64_t)d * vdim + col] : 0.f;
             }
     }
-    // the rows of a stage: a thread owns channel d of tile x (column i = x * dimP + d) for q, k and the decays
-    float rq[NI][16], rk[NI][16], rl[SCALAR ? 1 : NI][16], rv[8], rdt = 0.f, run[SCALAR ? 1 : NI] = {};
+    // the rows of a stage.  Decay per channel: a thread owns channel d of tile x (column i = x * dimP + d) of q, k and the
+    // decays; at up to 64 channels the block's upper half takes k (and needs the decays as well), the lower half q.
+    // Decay per head: q and k come as they lie, four channels of a row per load.
+    constexpr int NK = (8 * dimP + 255) / 256, D4 = dimP / 4;
+    constexpr bool TWO = DT <= 4;
+    const int ctid = TWO ? tid & 127 : tid;
+    const bool do_q = !TWO || tid < 128, do_k = !TWO || tid >= 128;
+    float rq[SCALAR ? 1 : NI][16], rk[SCALAR ? 1 : NI][16], rl[SCALAR ? 1 : NI][16], rdt = 0.f, run[SCALAR ? 1 : NI] = {};
+    float4 fq[SCALAR ? NK : 1], fk[SCALAR ? NK : 1], rv[2];
+    auto four = [&](const float* base, int64_t at, int c, int lim, bool ok) -> float4 {
+        float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (!ok || c >= lim) return o;
+        if (vec) return *reinterpret_cast<const float4*>(base + at + c);
+        o.x = base[at + c];
+        if (c + 1 < lim) o.y = base[at + c + 1];
+        if (c + 2 < lim) o.z = base[at + c + 2];
+        if (c + 3 < lim) o.w = base[at + c + 3];
+        return o;
+    };
     auto fetch = [&](int t0) {
+        if (SCALAR) {
 #pragma unroll
-        for (int k = 0; k < NI; k++) {
-            const int i = tid + 256 * k, x = i / dimP, d = i % dimP;
-            const bool on = i < 2 * dimP && d < dim;
-#pragma unroll
-            for (int r = 0; r < 16; r++) {
-                const int tt = t0 + 16 * x + r;
-                const bool ok = on && tt < en.y;
+            for (int k = 0; k < NK; k++) {
+                const int i = tid + 256 * k, tt = t0 + i / D4, d = i % D4 * 4;
+                const bool ok = i < kStage * D4 && tt < en.y;
                 const int64_t t = en.x + (ok ? tt : 0);
-                if (outs) rq[k][r] = ok ? p.q[t * p.ldq + qk0 + d] : 0.f;
-                rk[k][r] = ok ? p.k[t * p.ldk + qk0 + d] : 0.f;
-                if (!SCALAR) rl[k][r] = ok ? p.log_decay[t * p.heads * dim + (int64_t)h * dim + d] : 0.f;
+                if (outs) fq[k] = four(p.q, t * p.ldq + qk0, d, dim, ok);
+                fk[k] = four(p.k, t * p.ldk + qk0, d, dim, ok);
+            }
+        } else {
+#pragma unroll
+            for (int k = 0; k < NI; k++) {
+                const int i = ctid + 256 * k, x = i / dimP, d = i % dimP;
+                const bool on = i < 2 * dimP && d < dim;
+#pragma unroll
+                for (int r = 0; r < 16; r++) {
+                    const int tt = t0 + 16 * x + r;
+                    const bool ok = on && tt < en.y;
+                    const int64_t t = en.x + (ok ? tt : 0);
+                    if (outs && do_q) rq[k][r] = ok ? p.q[t * p.ldq + qk0 + d] : 0.f;
+                    if (do_k) rk[k][r] = ok ? p.k[t * p.ldk + qk0 + d] : 0.f;
+                    rl[k][r] = ok ? p.log_decay[t * p.heads * dim + (int64_t)h * dim + d] : 0.f;
+                }
             }
         }
 #pragma unroll
-        for (int k = 0; k < 8; k++) {
-            const int tt = t0 + (tid >> 6) + 4 * k, cc = c0 + (tid & 63);
-            rv[k] = (tt < en.y && cc < vdim) ? p.v[(int64_t)(en.x + tt) * p.ldv + (int64_t)h * vdim + cc] : 0.f;
+        for (int k = 0; k < 2; k++) {
+            const int tt = t0 + (tid >> 4) + 16 * k;
+            rv[k] = four(p.v, (int64_t)(en.x + tt) * p.ldv + (int64_t)h * vdim, c0 + (tid & 15) * 4, vdim, tt < en.y);
         }
         if (SCALAR && tid < kStage) rdt = t0 + tid < en.y ? p.dt[(int64_t)(en.x + t0 + tid) * p.ld_dt + h] : 0.f;
     };
@@ -199,17 +260,17 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
         __syncthreads();   // the previous stage has been read
         int steep = 0;
 #pragma unroll
-        for (int k = 0; k < 8; k++) vs[((tid >> 6) + 4 * k) * LV + (tid & 63)] = rv[k];
+        for (int k = 0; k < 2; k++) *reinterpret_cast<float4*>(vs + ((tid >> 4) + 16 * k) * LV + (tid & 15) * 4) = rv[k];
         if (SCALAR) {
 #pragma unroll
-            for (int k = 0; k < NI; k++) {
-                const int i = tid + 256 * k, x = i / dimP, d = i % dimP;
-                if (i < 2 * dimP)
-#pragma unroll
-                    for (int r = 0; r < 16; r++) {
-                        if (outs) qs[(16 * x + r) * LQ + d] = rq[k][r] * p.q_scale;
-                        ks[(16 * x + r) * LQ + d] = rk[k][r];
-                    }
+            for (int k = 0; k < NK; k++) {
+                const int i = tid + 256 * k, at = i / D4 * LQ + i % D4 * 4;
+                if (i < kStage * D4) {
+                    if (outs)
+                        *reinterpret_cast<float4*>(qs + at) = make_float4(fq[k].x * p.q_scale, fq[k].y * p.q_scale, fq[k].z * p.q_scale,
+                                                                          fq[k].w * p.q_scale);
+                    *reinterpret_cast<float4*>(ks + at) = fk[k];
+                }
             }
             if (tid < kStage) {
                 const float dt = t0 + tid < en.y ? softplus(rdt + db) : 0.f;
@@ -222,21 +283,21 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
                 const float tot = __shfl(L, 15, 16);
                 sL[tid] = L;
                 sdt[tid] = dt;
-                eL[tid] = expf(L);
-                kf[tid] = dt * expf(tot - L);
-                if ((tid & 15) == 15) et[tid >> 4] = expf(tot);
+                eL[tid] = __expf(L);
+                kf[tid] = dt * __expf(tot - L);
+                if ((tid & 15) == 15) et[tid >> 4] = __expf(tot);
                 run[0] += tot;
             }
             __syncthreads();
         } else {
 #pragma unroll
             for (int k = 0; k < NI; k++) {
-                const int i = tid + 256 * k;
+                const int i = ctid + 256 * k;
 #pragma unroll
                 for (int r = 1; r < 16; r++) rl[k][r] += rl[k][r - 1];
                 if (i < 2 * dimP) {
-                    et[i] = expf(rl[k][15]);
-                    wt[i] = expf(fminf(-rl[k][15], kSpan));
+                    et[i] = __expf(rl[k][15]);
+                    wt[i] = __expf(fminf(-rl[k][15], kSpan));
                     run[k] += rl[k][15];
                     steep |= rl[k][15] < -kSpan;
                 }
@@ -246,13 +307,13 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
                 for (int x = 0; x < 2; x++) {      // P pair by pair: unscaled q and k, and L, of one tile at a time
 #pragma unroll
                     for (int k = 0; k < NI; k++) {
-                        const int i = tid + 256 * k, d = i % dimP;
+                        const int i = ctid + 256 * k, d = i % dimP;
                         if (i < 2 * dimP && i / dimP == x)
 #pragma unroll
                             for (int r = 0; r < 16; r++) {
-                                qs[r * LQ + d] = rq[k][r] * p.q_scale;
-                                ks[r * LQ + d] = rk[k][r];
-                                qs[(16 + r) * LQ + d] = rl[k][r];
+                                if (do_q) qs[r * LQ + d] = rq[k][r] * p.q_scale;
+                                if (do_k) ks[r * LQ + d] = rk[k][r];
+                                if (do_q) qs[(16 + r) * LQ + d] = rl[k][r];
                             }
                     }
                     __syncthreads();
@@ -260,7 +321,7 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
                     float a = 0.f;
                     if (s <= t)
                         for (int d = 0; d < dim; d++)
-                            a = fmaf(qs[t * LQ + d] * ks[s * LQ + d], expf(qs[(16 + t) * LQ + d] - qs[(16 + s) * LQ + d]), a);
+                            a = fmaf(qs[t * LQ + d] * ks[s * LQ + d], __expf(qs[(16 + t) * LQ + d] - qs[(16 + s) * LQ + d]), a);
                     ps[0][x][t * LP + s] = a;
                     ps[1][x][t * LP + s] = 0.f;
                     __syncthreads();
@@ -268,12 +329,12 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
             }
 #pragma unroll
             for (int k = 0; k < NI; k++) {
-                const int i = tid + 256 * k, x = i / dimP, d = i % dimP;
+                const int i = ctid + 256 * k, x = i / dimP, d = i % dimP;
                 if (i < 2 * dimP)
 #pragma unroll
                     for (int r = 0; r < 16; r++) {
-                        if (outs) qs[(16 * x + r) * LQ + d] = rq[k][r] * p.q_scale * expf(rl[k][r]);
-                        ks[(16 * x + r) * LQ + d] = rk[k][r] * expf(rl[k][15] - rl[k][r]);
+                        if (outs && do_q) qs[(16 * x + r) * LQ + d] = rq[k][r] * p.q_scale * __expf(rl[k][r]);
+                        if (do_k) ks[(16 * x + r) * LQ + d] = rk[k][r] * __expf(rl[k][15] - rl[k][r]);
                     }
             }
             __syncthreads();
@@ -307,7 +368,7 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
             for (int i = 0; i < 4; i++) {
                 const int s = 4 * g + i;
                 float v = s <= n ? a[i] : 0.f;
-                if (SCALAR) v = s <= n ? v * (sdt[16 * x + s] * expf(sL[16 * x + n] - sL[16 * x + s])) : 0.f;
+                if (SCALAR) v = s <= n ? v * (sdt[16 * x + s] * __expf(sL[16 * x + n] - sL[16 * x + s])) : 0.f;
                 a[i] = v;
             }
             *reinterpret_cast<float4*>(&ps[half][x][n * LP + 4 * g]) = make_float4(a[0], a[1], a[2], a[3]);
@@ -388,15 +449,15 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p) {
         if (SCALAR) {
             if (tid < kStage && (tid & 15) == 0) et[tid >> 4] = run[0];
             __syncthreads();
-            for (int d = tid; d < dim; d += 256) dec[d] = expf(et[0] + et[1]);
+            for (int d = tid; d < dim; d += 256) dec[d] = __expf(et[0] + et[1]);
         } else {
 #pragma unroll
             for (int k = 0; k < NI; k++) {
-                const int i = tid + 256 * k;
+                const int i = ctid + 256 * k;
                 if (i < 2 * dimP) et[i] = run[k];
             }
             __syncthreads();
-            for (int d = tid; d < dim; d += 256) dec[d] = expf(et[d] + et[dimP + d]);
+            for (int d = tid; d < dim; d += 256) dec[d] = __expf(et[d] + et[dimP + d]);
         }
     }
 }
@@ -405,15 +466,17 @@ bool linrec_walk_fits(int dim, int vdim) { return dim >= 1 && dim <= 256 && vdim
 
 template <int DT>
 static void linrec_walk_launch(const LinRecP& p, dim3 grid, hipStream_t st) {
+    auto rows16 = [](const float* b, int64_t ld) { return ((uintptr_t)b & 15) == 0 && ld % 4 == 0; };
+    const int vec = rows16(p.q, p.ldq) && rows16(p.k, p.ldk) && rows16(p.v, p.ldv) && p.dim % 4 == 0 && p.vdim % 4 == 0;
     if (p.dt)
-        hipLaunchKernelGGL((linrec_walk_kernel<DT, true>), grid, dim3(256), 0, st, p);
+        hipLaunchKernelGGL((linrec_walk_kernel<DT, true>), grid, dim3(256), 0, st, p, vec);
     else
-        hipLaunchKernelGGL((linrec_walk_kernel<DT, false>), grid, dim3(256), 0, st, p);
+        hipLaunchKernelGGL((linrec_walk_kernel<DT, false>), grid, dim3(256), 0, st, p, vec);
 }
 
 int linrec_walk(const LinRecP& p, hipStream_t st) {
     QIE_TRY(linrec_check(p));
-    QIE_REQUIRE(linrec_walk_fits(p.dim, p.vdim), "linear recurrence: dim %d above the matrix-core form's 256", p.dim);
+    QIE_REQUIRE(!p.lr_in && linrec_walk_fits(p.dim, p.vdim), "linear recurrence: dim %d above the matrix-core form's 256", p.dim);
     dim3 grid((unsigned)p.heads, (unsigned)p.n_entries, (unsigned)((p.vdim + 63) / 64));
     const int dt = (p.dim + 15) / 16;
     if (dt <= 1) linrec_walk_launch<1>(p, grid, st);
@@ -462,6 +525,25 @@ template <typename TW> __device__ __forceinline__ float ldw(const TW* p, int64_t
 template <> __device__ __forceinline__ float ldw<float>(const float* p, int64_t i) { return p[i]; }
 template <> __device__ __forceinline__ float ldw<uint16_t>(const uint16_t* p, int64_t i) { return bf2f(p[i]); }
 
+__device__ __forceinline__ void ldw16(const float* p, float (&o)[16]) {
+#pragma unroll
+    for (int i = 0; i < 16; i++) o[i] = p[i];
+}
+__device__ __forceinline__ void ldw16(const uint16_t* p, float (&o)[16]) {
+    if (((uintptr_t)p & 15) == 0) {
+        const uint4 a = *reinterpret_cast<const uint4*>(p), b = *reinterpret_cast<const uint4*>(p + 8);
+        const uint32_t u[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            o[2 * i] = bf2f(u[i] & 0xffffu);
+            o[2 * i + 1] = bf2f(u[i] >> 16);
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 16; i++) o[i] = bf2f(p[i]);
+    }
+}
+
 template <typename TW>
 __global__ __launch_bounds__(256) void low_rank_log_sigmoid_kernel(const float* in, int64_t ld_in, int rank, const TW* w, const float* bias,
                                                                    float inv_tau, int n, int T, float* out) {
@@ -475,7 +557,16 @@ __global__ __launch_bounds__(256) void low_rank_log_sigmoid_kernel(const float* 
     if (c >= n) return;
     float z[LR] = {};
     const TW* wr = w + (int64_t)c * rank;
-    for (int k = 0; k < rank; k++) {
+    int k = 0;
+    for (; k + 16 <= rank; k += 16) {   // the weights of 16 ranks first, as many independent loads
+        float wk[16];
+        ldw16(wr + k, wk);
+#pragma unroll
+        for (int j = 0; j < 16; j++)
+#pragma unroll
+            for (int r = 0; r < LR; r++) z[r] = fmaf(wk[j], a1[r * rank + k + j], z[r]);
+    }
+    for (; k < rank; k++) {
         const float wk = ldw<TW>(wr, k);
 #pragma unroll
         for (int r = 0; r < LR; r++) z[r] = fmaf(wk, a1[r * rank + k], z[r]);

@@ -83,10 +83,17 @@ __device__ __forceinline__ int64_t page_base(const LatentCache& c, int slot, int
 }  // namespace
 
 // ------------------------------------------------------------------ post-projection
-// One block per row; a wave per head, the head's coordinates staged in LDS so that either pairing
-// finds its partner.
+// A wave per head and row (query, key, value heads alike; blockIdx.y spreads a row's heads over blocks when a step has
+// few rows), the head's coordinates staged in the wave's own LDS so that either pairing finds its partner: LDS
+// operations of one wave stay in order, so no block-wide barrier.
+__device__ __forceinline__ void wave_lds_fence() {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
 template <typename TC>
-__global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p) {
+__global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p, int values) {
     extern __shared__ float sm[];
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int slot = p.row_slot[t], pos = p.row_pos[t];
@@ -105,56 +112,99 @@ __global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p) {
     };
     const float* cs = p.rope_cos + (int64_t)pos * (p.rot_dims / 2);
     const float* sn = p.rope_sin + (int64_t)pos * (p.rot_dims / 2);
-    for (int h0 = 0; h0 < H + G; h0 += 4) {
-        const int hh = h0 + wave;
-        const bool on = hh < H + G, is_q = hh < H;
-        float* x = row + (is_q ? p.q_col + hh * dim : p.k_col + (hh - H) * dim);
-        const float* bias = !on ? nullptr : is_q ? (p.q_bias ? p.q_bias + hh * dim : nullptr) : (p.k_bias ? p.k_bias + (hh - H) * dim : nullptr);
-        if (on) {
-            float ss = 0.f;
-            for (int i = lane; i < dim; i += 64) {
-                const float a = bias ? x[i] + bias[i] : x[i];
+    const int n_task = H + G + (values ? G : 0);
+    // the next head's coordinates are on their way while this head is turned (up to 64 * NP of them)
+    constexpr int NP = 4;
+    const int step = 4 * gridDim.y;
+    auto head_at = [&](int hh) { return hh < H ? p.q_col + hh * dim : p.k_col + (hh - H) * dim; };
+    float nx[NP];
+    auto prefetch = [&](int hh) {
+        const bool on = hh < H + G;
+        const float* x = row + (on ? head_at(hh) : 0);
+#pragma unroll
+        for (int k = 0; k < NP; k++) nx[k] = on && lane + 64 * k < dim ? x[lane + 64 * k] : 0.f;
+    };
+    prefetch(blockIdx.y * 4 + wave);
+    for (int hh = blockIdx.y * 4 + wave; hh < n_task; hh += step) {
+        if (hh >= H + G) {
+            const int g = hh - H - G;
+            const float* vb = p.v_bias ? p.v_bias + g * vdim : nullptr;
+            const float* x = row + p.v_col + g * vdim;
+            if (!p.rot_values) {
+                for (int i = lane; i < vdim; i += 64) stc<TC>(vbase, vidx(g, i), vb ? x[i] + vb[i] : x[i]);
+                continue;
+            }
+            const float* vcs = p.vrope_cos + (int64_t)pos * (vdim / 2);
+            const float* vsn = p.vrope_sin + (int64_t)pos * (vdim / 2);
+            wave_lds_fence();
+            for (int i = lane; i < vdim; i += 64) buf[i] = vb ? x[i] + vb[i] : x[i];
+            wave_lds_fence();
+            for (int i = lane; i < vdim; i += 64) stc<TC>(vbase, vidx(g, i), turned(buf, i, vdim, p.rot_layout, vcs, vsn, 1.f));
+            continue;
+        }
+        const bool is_q = hh < H;
+        float* x = row + head_at(hh);
+        float cx[NP];
+#pragma unroll
+        for (int k = 0; k < NP; k++) cx[k] = nx[k];
+        prefetch(hh + step);
+        const float* bias = is_q ? (p.q_bias ? p.q_bias + hh * dim : nullptr) : (p.k_bias ? p.k_bias + (hh - H) * dim : nullptr);
+        wave_lds_fence();   // the previous head has been read
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < NP; k++) {
+            const int i = lane + 64 * k;
+            if (i < dim) {
+                const float a = bias ? cx[k] + bias[i] : cx[k];
                 buf[i] = a;
                 ss += a * a;
             }
-            ss = wsum(ss);
-            if (!is_q && p.v_col < 0)   // the value is the key as projected
-                for (int i = lane; i < dim; i += 64) stc<TC>(vbase, vidx(hh - H, i), buf[i]);
-            if (p.qk_norm) {
-                const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
-                const float* w = p.qk_norm == 1 ? (is_q ? p.qn_w : p.kn_w) : nullptr;
-                for (int i = lane; i < dim; i += 64) buf[i] = buf[i] * inv * (w ? w[i] : 1.0f);
-            }
-            if (is_q && p.q_temp_every > 0) {
-                const float tq = 1.0f + p.q_temp_coef * logf((float)((pos + 1) / p.q_temp_every + 1));
-                for (int i = lane; i < dim; i += 64) buf[i] *= tq;
-            }
         }
-        __syncthreads();
-        if (on)
-            for (int i = lane; i < dim; i += 64) {
-                const float o = turned(buf, i, p.rot_dims, p.rot_layout, cs, sn, 1.f);
-                if (is_q)
-                    x[i] = o;
-                else
-                    stc<TC>(krow, (int64_t)(hh - H) * dim + i, o);
-            }
-        __syncthreads();
+        for (int i = lane + 64 * NP; i < dim; i += 64) {
+            const float a = bias ? x[i] + bias[i] : x[i];
+            buf[i] = a;
+            ss += a * a;
+        }
+        if (!is_q && p.v_col < 0)   // the value is the key as projected
+            for (int i = lane; i < dim; i += 64) stc<TC>(vbase, vidx(hh - H, i), buf[i]);
+        if (p.qk_norm) {
+            ss = wsum(ss);
+            const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
+            const float* w = p.qk_norm == 1 ? (is_q ? p.qn_w : p.kn_w) : nullptr;
+            for (int i = lane; i < dim; i += 64) buf[i] = buf[i] * inv * (w ? w[i] : 1.0f);
+        }
+        if (is_q && p.q_temp_every > 0) {
+            const float tq = 1.0f + p.q_temp_coef * logf((float)((pos + 1) / p.q_temp_every + 1));
+            for (int i = lane; i < dim; i += 64) buf[i] *= tq;
+        }
+        wave_lds_fence();
+        for (int i = lane; i < dim; i += 64) {
+            const float o = turned(buf, i, p.rot_dims, p.rot_layout, cs, sn, 1.f);
+            if (is_q)
+                x[i] = o;
+            else
+                stc<TC>(krow, (int64_t)(hh - H) * dim + i, o);
+        }
     }
-    if (p.v_col < 0) return;
-    const float* vcs = p.rot_values ? p.vrope_cos + (int64_t)pos * (vdim / 2) : nullptr;
-    const float* vsn = p.rot_values ? p.vrope_sin + (int64_t)pos * (vdim / 2) : nullptr;
-    for (int g0 = 0; g0 < G; g0 += 4) {
-        const int g = g0 + wave;
-        const bool on = g < G;
-        if (on)
-            for (int i = lane; i < vdim; i += 64) buf[i] = row[p.v_col + g * vdim + i] + (p.v_bias ? p.v_bias[g * vdim + i] : 0.f);
-        __syncthreads();
-        if (on)
-            for (int i = lane; i < vdim; i += 64)
-                stc<TC>(vbase, vidx(g, i), p.rot_values ? turned(buf, i, vdim, p.rot_layout, vcs, vsn, 1.f) : buf[i]);
-        __syncthreads();
+}
+
+// Transposed values of prompt-sized steps: a block takes 16 consecutive rows of one slot and one key head, so that a
+// wave's stores are runs of 16 tokens instead of single elements.
+__global__ __launch_bounds__(256) void gqa_values_kernel(GqaPostP p, const int4* groups) {
+    extern __shared__ float sm[];   // [16][vdim + 1]
+    const int4 grp = groups[blockIdx.x];   // {first packed row, rows (<= 16), slot, first position}
+    const int g = blockIdx.y, vdim = p.vdim, PT = p.cache.page_tokens;
+    const float* vb = p.v_bias ? p.v_bias + g * vdim : nullptr;
+    for (int i = threadIdx.x; i < grp.y * vdim; i += 256) {
+        const int r = i / vdim, c = i % vdim;
+        const float v = p.proj[(int64_t)(grp.x + r) * p.ld + p.v_col + g * vdim + c];
+        sm[r * (vdim + 1) + c] = vb ? v + vb[c] : v;
     }
+    __syncthreads();
+    const int r = threadIdx.x & 15, pos = grp.w + r;
+    if (r >= grp.y) return;
+    uint16_t* dst = (uint16_t*)p.cache.pool + page_base(p.cache, grp.z, pos) + p.v_off + (int64_t)g * vdim * PT + pos % PT;
+    for (int c = threadIdx.x >> 4; c < vdim; c += 16) dst[(int64_t)c * PT] = f2bf(sm[r * (vdim + 1) + c]);
 }
 
 int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st) {
@@ -165,10 +215,16 @@ int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st) {
     QIE_REQUIRE(p.v_col >= 0 || p.vdim == p.dim, "gqa_post: keys as values need vdim == dim");
     const size_t shm = (size_t)4 * std::max(p.dim, p.vdim) * 4;
     QIE_REQUIRE(shm <= 48 * 1024, "gqa_post: head size %d above the kernel's staging", std::max(p.dim, p.vdim));
+    const bool apart = p.groups && p.v_col >= 0 && p.v_transposed && !p.rot_values && !cache_f32 && T > 64 && p.vdim <= 512;
+    const int values = p.v_col >= 0 && !apart ? 1 : 0;
+    const int ny = T <= 64 ? std::min(16, (p.heads + (1 + values) * p.kv_heads + 3) / 4) : 1;   // few rows: a row's heads over several blocks
     if (cache_f32)
-        hipLaunchKernelGGL(gqa_post_kernel<float>, dim3(T), dim3(256), shm, st, p);
+        hipLaunchKernelGGL(gqa_post_kernel<float>, dim3(T, ny), dim3(256), shm, st, p, values);
     else
-        hipLaunchKernelGGL(gqa_post_kernel<uint16_t>, dim3(T), dim3(256), shm, st, p);
+        hipLaunchKernelGGL(gqa_post_kernel<uint16_t>, dim3(T, ny), dim3(256), shm, st, p, values);
+    if (apart)
+        hipLaunchKernelGGL(gqa_values_kernel, dim3((unsigned)p.n_groups, (unsigned)p.kv_heads), dim3(256), (size_t)16 * (p.vdim + 1) * 4, st, p,
+                           p.groups);
     QIE_LAUNCH_CHECK();
     return 0;
 }
@@ -295,7 +351,7 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
     const int64_t o0 = (int64_t)t * p.ld_out + p.out_col + (int64_t)h * vdim;
     for (int r = tid; r < vdim; r += 256) {
         const float o = (p.rot_values ? turned(ob, r, vdim, p.rot_layout, vcs, vsn, -1.f) : ob[r]) * p.out_scale;
-        p.out[o0 + r] = o;
+        if (p.out) p.out[o0 + r] = o;
         if (p.out_bf) p.out_bf[o0 + r] = f2bf(o);
     }
 }
@@ -394,7 +450,7 @@ __device__ __forceinline__ void gqa_store(const GqaAttnP& a, const gf32x4_t* acc
         for (int j = 0; j < 4; j++) {
             float y = o[j] * a.out_scale;
             if (gated) y *= gf[dv][j];
-            a.out[o0 + v0 + j] = y;
+            if (a.out) a.out[o0 + v0 + j] = y;
             if (a.out_bf) a.out_bf[o0 + v0 + j] = f2bf(y);
         }
     }
@@ -977,7 +1033,7 @@ __global__ __launch_bounds__(256) void head_norm_rows_kernel(const float* o, con
                 const float gz = gate[t * ld_gate + h * vdim + i], sg = 1.0f / (1.0f + expf(-gz));
                 y *= gate_silu ? gz * sg : sg;
             }
-            out[o0 + i] = y;
+            if (out) out[o0 + i] = y;
             if (out_bf) out_bf[o0 + i] = f2bf(y);
         }
     }
@@ -1013,13 +1069,13 @@ __global__ __launch_bounds__(256) void gated_norm_parts_kernel(const float* y, c
     const float inv = 1.0f / sqrtf(ss / (float)len + eps);
     for (int i = threadIdx.x; i < len; i += 256) {
         const float o = (stage ? sm[i] : gated(i)) * inv * w[c0 + i];
-        out[t * ld_out + c0 + i] = o;
+        if (out) out[t * ld_out + c0 + i] = o;
         if (out_bf) out_bf[t * ld_out + c0 + i] = f2bf(o);
     }
 }
 int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* w, float eps, int n, int parts, int T, float* out,
                      uint16_t* out_bf, int64_t ld_out, hipStream_t st) {
-    QIE_REQUIRE(y && z && w && out && n > 0 && parts > 0 && n % parts == 0, "gated norm: %d columns in %d parts", n, parts);
+    QIE_REQUIRE(y && z && w && (out || out_bf) && n > 0 && parts > 0 && n % parts == 0, "gated norm: %d columns in %d parts", n, parts);
     const int len = n / parts, stage = (size_t)len * 4 <= 48 * 1024 ? 1 : 0;
     hipLaunchKernelGGL(gated_norm_parts_kernel, dim3((unsigned)T, (unsigned)parts), dim3(256), stage ? (size_t)len * 4 : 0, st, y, z, ld_z,
                        w, eps, n, len, out, out_bf, ld_out, stage);
@@ -1028,69 +1084,104 @@ int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* 
 }
 
 // ------------------------------------------------------------------ two norms of one row
-// One block per row; a thread's coordinates stay in registers between the sum and the two scaled copies (rows of up
-// to 256 * NR coordinates; NR = 0: re-read).
-template <int NR>
+// One block per row.  Rows of whole float4s (NV > 0): a thread's NV vectors stay in registers between the sum and the
+// two scaled copies, every load issued before the first use; NV = 0: any width, the row re-read.
+__device__ __forceinline__ void store_bf4(uint16_t* p, float4 v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack2(v.x, v.y), pack2(v.z, v.w));
+}
+
+template <int NV>
 __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
     __shared__ float red[4];
     const int64_t r0 = (int64_t)blockIdx.x * p.W;
-    float keep[NR > 0 ? NR : 1];
-    auto sum_at = [&](int i) {
-        float a = p.xin[r0 + i];
-        if (p.v) a += p.v2 ? p.v[r0 + i] + p.v2[r0 + i] : p.v[r0 + i];
-        if (p.add) a += p.add[r0 + i];
-        return a;
-    };
     const bool moved = p.v || p.add || p.xin != p.x;
     float ss = 0.f;
-    if (NR > 0) {
+    if constexpr (NV > 0) {
+        const int n4 = p.W >> 2;
+        float4 x[NV], a[NV], b[NV], c[NV];
+        const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
-        for (int k = 0; k < NR; k++) {
+        for (int k = 0; k < NV; k++) {
             const int i = threadIdx.x + 256 * k;
-            keep[k] = i < p.W ? sum_at(i) : 0.f;
-            ss += keep[k] * keep[k];
+            const bool on = i < n4;
+            const int64_t o = r0 + 4 * (on ? i : 0);
+            x[k] = *reinterpret_cast<const float4*>(p.xin + o);
+            a[k] = p.v ? *reinterpret_cast<const float4*>(p.v + o) : zero;
+            b[k] = p.v2 ? *reinterpret_cast<const float4*>(p.v2 + o) : zero;
+            c[k] = p.add ? *reinterpret_cast<const float4*>(p.add + o) : zero;
         }
 #pragma unroll
-        for (int k = 0; k < NR; k++) {
+        for (int k = 0; k < NV; k++) {
             const int i = threadIdx.x + 256 * k;
-            if (moved && i < p.W) p.x[r0 + i] = keep[k];
+            x[k].x += (a[k].x + b[k].x) + c[k].x;
+            x[k].y += (a[k].y + b[k].y) + c[k].y;
+            x[k].z += (a[k].z + b[k].z) + c[k].z;
+            x[k].w += (a[k].w + b[k].w) + c[k].w;
+            if (i < n4) {
+                if (moved) *reinterpret_cast<float4*>(p.x + r0 + 4 * i) = x[k];
+                ss += (x[k].x * x[k].x + x[k].y * x[k].y) + (x[k].z * x[k].z + x[k].w * x[k].w);
+            }
+        }
+        if (!p.w1) return;
+        float4 w1[NV], w2[NV];
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+            const int i = threadIdx.x + 256 * k, j = 4 * (i < n4 ? i : 0);
+            w1[k] = *reinterpret_cast<const float4*>(p.w1 + j);
+            w2[k] = p.w2 ? *reinterpret_cast<const float4*>(p.w2 + j) : zero;
+        }
+        ss = bsum256(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+            const int i = threadIdx.x + 256 * k;
+            if (i >= n4) break;
+            const int64_t o = r0 + 4 * i;
+            const float4 y = make_float4(x[k].x * inv, x[k].y * inv, x[k].z * inv, x[k].w * inv);
+            const float4 y1 = make_float4(y.x * w1[k].x, y.y * w1[k].y, y.z * w1[k].z, y.w * w1[k].w);
+            if (p.h1) *reinterpret_cast<float4*>(p.h1 + o) = y1;
+            if (p.h1_bf) store_bf4(p.h1_bf + o, y1);
+            if (p.w2) {
+                const float4 y2 = make_float4(y.x * w2[k].x, y.y * w2[k].y, y.z * w2[k].z, y.w * w2[k].w);
+                if (p.h2) *reinterpret_cast<float4*>(p.h2 + o) = y2;
+                if (p.h2_bf) store_bf4(p.h2_bf + o, y2);
+            }
         }
     } else {
         for (int i = threadIdx.x; i < p.W; i += 256) {
-            const float a = sum_at(i);
+            float a = p.xin[r0 + i];
+            if (p.v) a += p.v2 ? p.v[r0 + i] + p.v2[r0 + i] : p.v[r0 + i];
+            if (p.add) a += p.add[r0 + i];
             if (moved) p.x[r0 + i] = a;
             ss += a * a;
         }
-    }
-    if (!p.w1) return;
-    ss = bsum256(ss, red);
-    const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
-    auto emit = [&](int i, float a) {
-        const float o1 = a * inv * p.w1[i];
-        p.h1[r0 + i] = o1;
-        if (p.h1_bf) p.h1_bf[r0 + i] = f2bf(o1);
-        if (p.w2) {
-            const float o2 = a * inv * p.w2[i];
-            p.h2[r0 + i] = o2;
-            if (p.h2_bf) p.h2_bf[r0 + i] = f2bf(o2);
+        if (!p.w1) return;
+        ss = bsum256(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
+        for (int i = threadIdx.x; i < p.W; i += 256) {
+            const float a = p.x[r0 + i] * inv;   // the thread's own store above (or the row as it was)
+            const float o1 = a * p.w1[i];
+            if (p.h1) p.h1[r0 + i] = o1;
+            if (p.h1_bf) p.h1_bf[r0 + i] = f2bf(o1);
+            if (p.w2) {
+                const float o2 = a * p.w2[i];
+                if (p.h2) p.h2[r0 + i] = o2;
+                if (p.h2_bf) p.h2_bf[r0 + i] = f2bf(o2);
+            }
         }
-    };
-    if (NR > 0) {
-#pragma unroll
-        for (int k = 0; k < NR; k++) {
-            const int i = threadIdx.x + 256 * k;
-            if (i < p.W) emit(i, keep[k]);
-        }
-    } else {
-        for (int i = threadIdx.x; i < p.W; i += 256) emit(i, p.x[r0 + i]);   // the thread's own store above (or the row as it was)
     }
 }
 int norm_pair(const NormPairP& p, hipStream_t st) {
-    QIE_REQUIRE(p.x && p.xin && p.T > 0 && p.W > 0 && (!p.w1 || p.h1) && (!p.w2 || (p.w1 && p.h2)) && (!p.v2 || p.v), "norm_pair: bad arguments");
-    if (p.W <= 1024)
+    QIE_REQUIRE(p.x && p.xin && p.T > 0 && p.W > 0 && (!p.w1 || p.h1 || p.h1_bf) && (!p.w2 || (p.w1 && (p.h2 || p.h2_bf))) && (!p.v2 || p.v),
+                "norm_pair: bad arguments");
+    if (p.W % 4 == 0 && p.W <= 1024)
+        hipLaunchKernelGGL(norm_pair_kernel<1>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+    else if (p.W % 4 == 0 && p.W <= 2048)
+        hipLaunchKernelGGL(norm_pair_kernel<2>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+    else if (p.W % 4 == 0 && p.W <= 4096)
         hipLaunchKernelGGL(norm_pair_kernel<4>, dim3((unsigned)p.T), dim3(256), 0, st, p);
-    else if (p.W <= 4096)
-        hipLaunchKernelGGL(norm_pair_kernel<16>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+    else if (p.W % 4 == 0 && p.W <= 8192)
+        hipLaunchKernelGGL(norm_pair_kernel<8>, dim3((unsigned)p.T), dim3(256), 0, st, p);
     else
         hipLaunchKernelGGL(norm_pair_kernel<0>, dim3((unsigned)p.T), dim3(256), 0, st, p);
     QIE_LAUNCH_CHECK();

@@ -171,6 +171,50 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(CausalConvP p, int T) 
     if (p.out_bf) p.out_bf[o] = f2bf(a);
 }
 
+// Prompt-sized steps: a thread walks CR rows of one channel with the taps' inputs in registers (every input is loaded
+// once); where a row does not follow its predecessor's entry they are fetched again as above.
+constexpr int CR = 16;
+template <int TAPS>
+__global__ __launch_bounds__(256) void causal_conv_rows_kernel(CausalConvP p, int T) {
+    const int c = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * CR;
+    if (c >= p.C) return;
+    float w[TAPS], x[TAPS], in[CR];
+#pragma unroll
+    for (int j = 0; j < TAPS; j++) w[j] = p.w[(int64_t)c * TAPS + j];
+#pragma unroll
+    for (int i = 0; i < CR; i++) in[i] = p.in[(int64_t)min(t0 + i, T - 1) * p.ld_in + p.col + c];
+    const float b = p.bias ? p.bias[c] : 0.f;
+#pragma unroll
+    for (int i = 0; i < CR; i++) {
+        const int t = t0 + i;
+        if (t >= T) break;
+        const int k = p.row_k[t];
+        if (i == 0 || k == 0) {
+            const int slot = p.row_slot[t], pos = p.row_pos[t];
+            const float* sb = p.state + (int64_t)slot * p.slot_stride + p.state_off;
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; j++) {
+                const int back = TAPS - 1 - j;
+                x[j] = back <= k ? p.in[(int64_t)(t - back) * p.ld_in + p.col + c]
+                                 : pos - back >= 0 ? sb[(int64_t)(k - back + TAPS - 1) * p.C + c] : 0.f;
+            }
+        } else {
+#pragma unroll
+            for (int j = 0; j < TAPS - 2; j++) x[j] = x[j + 1];
+            if (TAPS > 1) x[TAPS - 2] = in[i > 0 ? i - 1 : 0];
+        }
+        x[TAPS - 1] = in[i];
+        float a = b;
+#pragma unroll
+        for (int j = 0; j < TAPS; j++) a = fmaf(w[j], x[j], a);
+        if (p.residual) a += in[i];
+        if (p.silu) a = a / (1.0f + expf(-a));
+        const int64_t o = (int64_t)t * p.ld_out + c;
+        p.out[o] = a;
+        if (p.out_bf) p.out_bf[o] = f2bf(a);
+    }
+}
+
 // One thread per (entry, channel): state row i becomes the input at position p1 - (taps - 1) + i,
 // p1 the position after the entry's last row.  Ascending i reads old rows i + count > i before any
 // of them is written.
@@ -247,7 +291,15 @@ int causal_conv(const CausalConvP& p, int T, hipStream_t st) {
     QIE_TRY(conv_check(p));
     QIE_REQUIRE(p.out && p.row_slot && p.row_pos && p.row_k, "causal_conv: bad arguments");
     const int64_t n = (int64_t)T * p.C;
-    hipLaunchKernelGGL(causal_conv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, p, T);
+    const dim3 rows((unsigned)((p.C + 255) / 256), (unsigned)((T + CR - 1) / CR));
+    if (T > kConvFusedRows && p.out != p.in && p.taps == 4)
+        hipLaunchKernelGGL(causal_conv_rows_kernel<4>, rows, dim3(256), 0, st, p, T);
+    else if (T > kConvFusedRows && p.out != p.in && p.taps == 3)
+        hipLaunchKernelGGL(causal_conv_rows_kernel<3>, rows, dim3(256), 0, st, p, T);
+    else if (T > kConvFusedRows && p.out != p.in && p.taps == 2)
+        hipLaunchKernelGGL(causal_conv_rows_kernel<2>, rows, dim3(256), 0, st, p, T);
+    else
+        hipLaunchKernelGGL(causal_conv_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, p, T);
     QIE_LAUNCH_CHECK();
     return 0;
 }

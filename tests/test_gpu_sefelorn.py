@@ -480,7 +480,7 @@ def test_small_steps_replay_graphs_equal_eager(model, dtype):
         ra = a.batch.step([(0, toks[:2]), (1, toks[2:3])], range(3))
         rb = b.batch.step([(0, toks[:2]), (1, toks[2:3])], range(3))
         assert np.array_equal(ra, rb)
-    assert a.batch.graph_stats()[0] >= 3 and b.batch.graph_stats()[0] == 0
+    assert a.batch.graph_stats()[0] >= 1 and a.batch.graph_stats()[1] >= 30 and b.batch.graph_stats()[0] == 0
 
 
 def save_model(m, path):
