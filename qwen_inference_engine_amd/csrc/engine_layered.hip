@@ -166,8 +166,7 @@ struct LayeredBatch {
     PieceList pieces, lin[3];         // lin: pieces of 128, 256, 512 rows
     int max_count = 0;
     int64_t step_T = 0;               // rows of the step being built
-    // parallel blocks: the layer's feed-forward waits for the mixer's input product / is running on side[0]
-    bool ff_wait = false, ff_branch = false;
+    bool ff_branch = false;           // parallel blocks: the layer's feed-forward is running on side[0]
     bool has_scan = false, has_lin = false;   // layer runs of either kind
     std::vector<int> lin_units;               // (head, column tile) blocks of the model's linear recurrences
     float *s_loc = nullptr, *s_in = nullptr, *s_decay = nullptr;
@@ -1356,32 +1355,14 @@ static int enq_out(qie_batch* b, int r, int T) {
     return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
 }
 
-// Parallel blocks, prompt-sized steps: the feed-forward starts on its side stream here, where the mixer's kernels that do
-// not fill the chip begin (beside the input product it would only share the matrix cores with it)
-static int start_ff(qie_batch* b, int r, int T) {
-    LayeredBatch* s = b->lb;
-    if (!s->ff_wait) return 0;
-    s->ff_wait = false;
-    QIE_TRY(branch_fork(b, 0));
-    s->ff_branch = true;
-    return enq_ff(b, b->e->lm->runs[r].layer, T, s->side[0]);
-}
-
-static int join_ff(qie_batch* b) {
-    LayeredBatch* s = b->lb;
-    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
-    s->ff_branch = false;
-    return 0;
-}
-
 static int enq_state_space_mixer(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
     QIE_TRY(dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf));
-    QIE_TRY(start_ff(b, r, T));
     QIE_TRY(enq_state_space(b, r, T));
-    QIE_TRY(join_ff(b));
+    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
+    s->ff_branch = false;
     return enq_out(b, r, T);
 }
 
@@ -1397,11 +1378,11 @@ static int enq_gqa_mixer(qie_batch* b, int r, int T) {
         QIE_TRY(enq_recurrence(b, r, T, s->side[1]));
     }
     QIE_TRY(enq_gqa_post(b, r, T));
-    QIE_TRY(start_ff(b, r, T));
     QIE_TRY(enq_gqa_attention(b, r, T));
     if (rec && !beside) QIE_TRY(enq_recurrence(b, r, T));
     if (beside) QIE_TRY(branch_join(b, 1));
-    QIE_TRY(join_ff(b));
+    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
+    s->ff_branch = false;
     return enq_out(b, r, T);
 }
 
@@ -1668,11 +1649,14 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
     };
     if (!h_ready) QIE_TRY(norms(r == 0 && m->loops ? x0 : x, nullptr, nullptr, m->runs[r].add_embed ? x0 : nullptr, &L));
     const bool has_ff = L.d.ff_kind != QIE_FF_NONE;
-    // the feed-forward beside the mixer (the experts' products have side streams of their own)
-    const bool starts = L.d.mixer == QIE_MIXER_STATE_SPACE || L.d.mixer == QIE_MIXER_GQA || L.d.mixer == QIE_MIXER_GQA_RECURRENT;
-    s->ff_wait = L.d.ff_kind == QIE_FF_DENSE && T > kBranchRows && starts;
-    s->ff_branch = false;
-    if (has_ff && !s->ff_wait) QIE_TRY(enq_ff(b, m->runs[r].layer, T));
+    // the feed-forward beside the mixer (the experts' products have side streams of their own), started before it: its
+    // tiles fill the rounds that the mixer's input product leaves part empty (started after that product: 2.55 -> 2.61 ms
+    // for 2,048 rows at the 2k Sefelorn size)
+    // (a mixer whose output product takes the activations waits for them: enq_gqa_mixer, enq_state_space_mixer)
+    const bool waits = L.cat_ff < 0 || L.d.mixer == QIE_MIXER_STATE_SPACE || L.d.mixer == QIE_MIXER_GQA || L.d.mixer == QIE_MIXER_GQA_RECURRENT;
+    s->ff_branch = L.d.ff_kind == QIE_FF_DENSE && T > kBranchRows && waits;
+    if (s->ff_branch) QIE_TRY(branch_fork(b, 0));
+    if (has_ff) QIE_TRY(enq_ff(b, m->runs[r].layer, T, s->ff_branch ? s->side[0] : nullptr));
     switch (L.d.mixer) {
         case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
         case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
@@ -1680,6 +1664,8 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
         case QIE_MIXER_STATE_SPACE: QIE_TRY(enq_state_space_mixer(b, r, T)); break;
         default: QIE_TRY(enq_gqa_mixer(b, r, T)); break;
     }
+    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
+    s->ff_branch = false;
     const bool last = r + 1 == (int)m->runs.size(), fuse_next = !last && !s->keep_on;
     const LayerDev* N = fuse_next ? &m->L[m->runs[r + 1].layer] : nullptr;
     QIE_TRY(norms(x, s->mix, has_ff && L.cat_ff < 0 ? s->ffo : nullptr, fuse_next && m->runs[r + 1].add_embed ? x0 : nullptr, N));
