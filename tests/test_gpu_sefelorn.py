@@ -147,9 +147,9 @@ def test_each_mechanism_alone(model, name, times):
     assert rel(feed(m, 1, toks, [20, 2, 9]), want) < m.tol
 
 
-@pytest.mark.parametrize("loop", [None, (0, 5, 2), (1, 4, 2), (4, 5, 4), (0, 1, 3), (2, 2, 3)])
-def test_repeated_groups(model, loop):
-    m = model(MIXED, seed=5, loop=loop)
+@pytest.mark.parametrize("loop,width", [(None, 40), ((0, 5, 2), 40), ((1, 4, 2), 39), ((4, 5, 4), 44), ((0, 1, 3), 40), ((2, 2, 3), 40)])
+def test_repeated_groups(model, loop, width):
+    m = model(MIXED, seed=5, loop=loop, width=width)
     toks = m.tokens(45)
     lay = []
     want = m.ref(toks, lay)
@@ -163,8 +163,9 @@ def test_repeated_groups(model, loop):
     assert rel(feed(m, 1, toks, [11, 2, 20]), want) < m.tol
 
 
-def test_bf16_layers(model):
-    m = model(MIXED, seed=5, dtype="bfloat16", loop=LOOP)
+@pytest.mark.parametrize("width", [40, 42])      # rows of whole 16-byte vectors, and rows that are not
+def test_bf16_layers(model, width):
+    m = model(MIXED, seed=5, dtype="bfloat16", loop=LOOP, width=width)
     toks = m.tokens(70)
     lay = []
     want = m.ref(toks, lay)
@@ -525,3 +526,91 @@ def test_trace_replay_and_generation_command_lines(model, tmp_path, dtype):
         got = {ln.split(":")[0]: [int(t) for t in ln.split(":")[1].split()] for ln in r.stdout.splitlines() if ln.startswith("tokens[")}
         assert got["tokens[0]"] == oracle_greedy(m, b, 5)
         assert got["tokens[1]"] == oracle_greedy(m, a[:7], 5)
+
+
+# ------------------------------------------------------------------ the new pieces beside other designs' pieces
+@pytest.mark.parametrize("block", ["parallel", "prenorm"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_blocks_and_mixers_combine(block, dtype):
+    """The parallel block around every mixer and a routed feed-forward, the state space inside the pre-norm block: a
+    model no reader makes, restated with the designs' oracles; portions above and below the branch threshold."""
+    import lugipel_oracle as LO
+    import nodutar_oracle as NO
+    import qwen_inference_engine_amd as q
+    import verelorn_oracle as VO
+    from qwen_inference_engine_amd import spec as S
+    W, V, eps, n = 48, 83, 1e-5, 150
+    ff = lambda act, **k: S.FeedForward("dense", 32, act=act, **k)
+    layers = [S.LayerSpec(S.StateSpace(4, 8, 12, 2, 3, 2), ff("clamped_gated", limit=1.0)),
+              S.LayerSpec(S.MinGru(40), ff("gelu_tanh_gated")),
+              S.LayerSpec(S.ChannelDelta(2, 1, 8, 16, 3, 4, 4), ff("silu_gated")),
+              S.LayerSpec(S.LatentAttention(2, 8, 4, 8, 16, 0, 4, 100.0, 0.3, None, 8, "interleaved", False), ff("clamped_gated", limit=0.5)),
+              S.LayerSpec(S.StateSpace(2, 24, 16, 1, 4, 1), S.FeedForward("moe", 16, 4, 2, "softmax_out"))]
+    if block == "parallel":
+        layers.append(S.LayerSpec(S.AttentionWithRecurrence(
+            S.GqaAttention(4, 2, 8, 8, 0.3, qk_norm="weight", rot_dims=4, rot_base=100.0, rot_layout="interleaved", rot_values=True,
+                           mask="chunk", mask_size=9), S.GatedRecurrence(2, 8, 8), 0.8, 1.1), None))
+    spec = S.LayeredSpec("mix", W, V, eps, tuple(layers), False, block=block, tied_head=True, embed_scale=2.0, logit_scale=0.5)
+    rng = np.random.default_rng(3)
+    T = {}
+    for name, shape in spec.tensor_shapes().items():
+        if name.endswith(("norm", "norm1", "norm2", ".D")):
+            v = 1.0 + 0.2 * rng.standard_normal(shape)
+        elif name.endswith("lower"):
+            v = rng.uniform(0.1, 0.9, shape)
+        elif len(shape) == 1:
+            v = 0.3 * rng.standard_normal(shape)
+        else:
+            v = rng.standard_normal(shape) * (0.4 if name.endswith((".o", "down")) else 0.5 if name == "embed" else 1.0) / \
+                (np.sqrt(shape[-1]) if name != "embed" else 1.0)
+        T[name] = O.to_bf16_exact(v)
+    D = {k: v.astype(np.float64) for k, v in T.items()}
+
+    def mixer(i, h):
+        m, p = layers[i].mixer, f"l{i}.mix."
+        if isinstance(m, S.StateSpace):
+            return O.state_space({k: getattr(m, k) for k in ("heads", "vdim", "state", "groups", "norm_groups")}, D, p, h, eps)
+        if isinstance(m, S.MinGru):
+            return LO.min_gru(h, D, p)[0]
+        if isinstance(m, S.ChannelDelta):
+            return VO.channel_delta({k: getattr(m, k) for k in ("heads", "kv_heads", "dim", "vdim")}, D, p, h, eps)
+        if isinstance(m, S.LatentAttention):
+            c = {"heads": m.heads, "dim": m.dim, "rot_dim": m.rot_dim, "vdim": m.vdim, "kv_rank": m.kv_rank, "scale": m.scale,
+                 "rot": {"base": 100.0, "dims": 4}}
+            return VO.latent_attention(c, D, p, h, eps, VO.latent_kv(c, D, p, h, eps))
+        a, c = m.attn, m.rec
+        cfg = {"left_scale": 0.8, "right_scale": 1.1, "right": {"heads": c.heads, "dim": c.dim, "vdim": c.vdim},
+               "left": {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim, "vdim": a.vdim, "scale": a.scale,
+                        "mask": {"size": 9}, "rot": {"base": 100.0, "dims": 4}}}
+        return NO.parallel_mixer(h, cfg, D, p, eps)
+
+    def feed_forward(i, h):
+        f, p = layers[i].mlp, f"l{i}.mlp."
+        if f.kind == "moe":
+            return NO.moe_ff(h, {"router": {"experts": 4, "top": 2}}, D, p)
+        if f.act == "clamped_gated":
+            return O.clamped_ff({"limit": f.limit}, D, p, h)
+        if f.act == "gelu_tanh_gated":
+            return VO.dense_ff(D, p, h)
+        return (O.silu(h @ D[p + "gate"].T) * (h @ D[p + "up"].T)) @ D[p + "down"].T
+
+    toks = [int(t) for t in rng.integers(0, V, n)]
+    x = D["embed"][toks] * 2.0
+    for i, L in enumerate(layers):
+        y = mixer(i, O.norm(x, D[f"l{i}.norm1"], eps))
+        z = x if block == "parallel" else x + y
+        f = feed_forward(i, O.norm(z, D[f"l{i}.norm2"], eps)) if L.mlp is not None else 0.0
+        x = x + y + f
+    want = O.norm(x, D["final.norm"], eps) @ D["embed"].T * 0.5
+    eng = q.Engine(spec, max_ctx=256, dtype=dtype).load_tensors({k: words(v) for k, v in T.items()})
+    b = eng.batch(2, 256, page_tokens=32)
+    rel.rows = dtype != "float32"
+    for slot, cuts in ((0, [n]), (1, [70, 2, 66, 3])):
+        got, pos = [], 0
+        while pos < n:
+            c = min(cuts.pop(0) if cuts else 1, n - pos)
+            got.append(b.step([(slot, toks[pos:pos + c])], range(c)))
+            pos += c
+        assert rel(np.concatenate(got), want) < (REL32 if dtype == "float32" else REL16)
+    b.close()
+    eng.close()
