@@ -247,7 +247,6 @@ struct GatedCarryP {
     int64_t slot_stride, state_off;
 };
 int gated_carry(const GatedCarryP& p, hipStream_t st);
-// out[t, out_col + h * vdim + c] = scale * o[t, h, c] / sqrt(mean_c o^2 + eps) * w[c], o = o1 + o2 when o2
 // ------------------------------------------------------------------ minGRU
 // Per entry {first packed row, rows, index, first position} and channel c < n: with
 // z = sigmoid(proj[z_col + c] + z_b[c]), u = proj[x_col + c] + x_b[c], cand = u >= 0 ? u + 1/2 :
@@ -290,6 +289,7 @@ struct MinGruCarryP {
 };
 int mingru_carry(const MinGruCarryP& p, hipStream_t st);
 
+// out[t, out_col + h * vdim + c] = scale * o[t, h, c] / sqrt(mean_c o^2 + eps) * w[c], o = o1 + o2 when o2
 // gate (optional): the result is also multiplied by sigmoid(gate[t * ld_gate + h * vdim + c]), or silu of it
 // (gate_silu); ld_gate 0: heads * vdim
 int head_norm_rows(const float* o, const float* o2, const float* w, float eps, float scale, int heads, int vdim, int T, float* out,
@@ -311,7 +311,7 @@ struct NormPairP {
     float eps;
 };
 int norm_pair(const NormPairP& p, hipStream_t st);
-// (head_norm_rows, gated_norm_parts, silu_mul: a null fp32 output leaves the bf16 image alone)
+// (head_norm_rows, gated_norm_parts, silu_mul: with a null fp32 output only the bf16 image is written)
 
 // ------------------------------------------------------------------ residual streams (k_streams.hip)
 // n residual rows per token, X + s * plane (rows of W).  With y (a sublayer's result, [T][W]) the rows

@@ -426,9 +426,9 @@ __global__ __launch_bounds__(256) void linrec_walk_kernel(LinRecP p, int vec) {
                 }
             }
 #pragma unroll
-            for (int j = 0; j < DT; j++)
+            for (int i = 0; i < 4; i++)   // the tiles' products are independent, a tile's four are not
 #pragma unroll
-                for (int i = 0; i < 4; i++)
+                for (int j = 0; j < DT; j++)
                     S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(ks[(16 * x + 4 * g + i) * LQ + 16 * j + n], vb[i], S[j], 0, 0, 0);
         }
     }

@@ -8,10 +8,12 @@
 //                        and / or a linear one with a slope per head; softmax weights (optionally with a
 //                        sink: one more term exp(sink_h) in the denominator, no key, no value), or sigmoid
 //                        weights with a bias per head; an optional sigmoid gate per head or per coordinate;
-//                        bias vectors on q and k (gqa_post)
+//                        bias vectors on q, k and v (gqa_post); a window that keeps the first tokens visible
 //   lay::gated_scan      gated linear recurrence with an fp32 state per slot and head
 //   lay::mingru_scan     minGRU: a recurrence per channel, update gate and candidate from the current input alone
 //   lay::head_norm_rows  per-head RMS norm with a weight
+//   lay::gated_norm_parts   silu gate, then an RMS norm in equal parts
+//   lay::norm_pair       residual add of parallel branches fused with two norms of the result
 //   lay::add_norm        residual add of a normed branch fused with the next branch's input norm
 //
 // Scores, softmax statistics, norms, gates and the recurrent state are fp32; cache rows are
