@@ -267,14 +267,15 @@ int qie_batch_debug_step(qie_batch* b, const qie_sampling* smp, int32_t* next_id
  * normed after it is computed, its input is the raw stream); the next layer's input is the depth-weighted sum over the embedding
  * output and every layer result so far. */
 enum { QIE_MIXER_LATENT_ATTENTION = 1, QIE_MIXER_GQA = 2, QIE_MIXER_GQA_RECURRENT = 3, QIE_MIXER_MINGRU = 4,
-       QIE_MIXER_CHANNEL_DELTA = 5, QIE_MIXER_STATE_SPACE = 6 };
+       QIE_MIXER_CHANNEL_DELTA = 5, QIE_MIXER_STATE_SPACE = 6, QIE_MIXER_RGLRU = 7 };
 enum { QIE_FF_NONE = 0, QIE_FF_DENSE = 1, QIE_FF_MOE = 2 };
 /* Which keys j <= i a query at position i sees: all of them; the last `size`; those of its own
  * block of `size` positions (blocks counted from position 0 of the sequence). */
 enum { QIE_MASK_CAUSAL = 0, QIE_MASK_WINDOW = 1, QIE_MASK_CHUNK = 2 };
 /* RMS norm of every query / key head over dim before rotation: none, with a weight vector
- * shared by the heads, or without one. */
-enum { QIE_QKNORM_NONE = 0, QIE_QKNORM_WEIGHT = 1, QIE_QKNORM_PLAIN = 2 };
+ * shared by the heads, or without one.  QIE_QKNORM_ROW: one norm over all query heads at once and one over all
+ * key heads, with weight vectors of those sizes ('mix.q.norm' [heads * dim], 'mix.k.norm' [kv_heads * dim]). */
+enum { QIE_QKNORM_NONE = 0, QIE_QKNORM_WEIGHT = 1, QIE_QKNORM_PLAIN = 2, QIE_QKNORM_ROW = 3 };
 /* Rotary pairs inside the rotated coordinates: i with i + dims / 2, or 2i with 2i + 1. */
 enum { QIE_ROT_HALVES = 0, QIE_ROT_INTERLEAVED = 1 };
 /* Block: 0 = y = x + g * rms(branch(x)) with scalar gains (branches read the raw stream);
@@ -284,7 +285,8 @@ enum { QIE_ROT_HALVES = 0, QIE_ROT_INTERLEAVED = 1 };
  * norm before every branch and none after.  Options of block 2 (qie_arch_desc): several residual
  * streams with learned mixing (streams), a causal convolution on the mixer's normed input
  * (canon_taps), a norm of the embedding rows (embed_norm).
- * 3 = x += mixer(N1(x)) + ff(N2(x)), both branches of the same x, plain weight vectors 'l<i>.norm1|norm2'. */
+ * 3 = x += mixer(N1(x)) + ff(N2(x)), both branches of the same x, plain weight vectors 'l<i>.norm1|norm2';
+ * with qie_arch_desc.shared_norm both read N1(x) and there is no 'norm2'. */
 enum { QIE_BLOCK_POSTNORM_GAIN = 0, QIE_BLOCK_SANDWICH = 1, QIE_BLOCK_PRENORM = 2, QIE_BLOCK_PARALLEL = 3 };
 /* Router: 0 = sigmoid scores, the `top` largest scale the experts' input; 1 = logits with a
  * bias, the `top` largest weighted by the softmax over those alone scale the experts' output. */
@@ -299,9 +301,12 @@ enum { QIE_ROUTER_SIGMOID_IN = 0, QIE_ROUTER_SOFTMAX_OUT = 1, QIE_ROUTER_SOFTMAX
  * (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2.  Experts are always of form 0. */
 /* 2 = W_down (gelu_tanh(W_gate h) * W_up h), gelu_tanh(z) = z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))). */
 /* 3 = W_down (g sigmoid(1.702 g) (u + 1)), g = min(W_gate h, ff_limit), u = W_up h clamped to +-ff_limit. */
-enum { QIE_ACT_SILU_GATED = 0, QIE_ACT_XIELU = 1, QIE_ACT_GELU_TANH_GATED = 2, QIE_ACT_CLAMPED_GATED = 3 };
-/* Gates of the recurrence beside an attention (qie_recurrent_desc.kind). */
-enum { QIE_REC_LOWER_BOUND = 0, QIE_REC_KEY_DECAY = 1 };
+/* 4 = W_down (max(W_gate h, 0) * W_up h). */
+enum { QIE_ACT_SILU_GATED = 0, QIE_ACT_XIELU = 1, QIE_ACT_GELU_TANH_GATED = 2, QIE_ACT_CLAMPED_GATED = 3, QIE_ACT_RELU_GATED = 4 };
+/* The recurrence beside an attention (qie_recurrent_desc.kind). */
+enum { QIE_REC_LOWER_BOUND = 0, QIE_REC_KEY_DECAY = 1, QIE_REC_DELTA = 2 };
+/* Decay and output gate of a delta rule (qie_delta_desc.decay). */
+enum { QIE_DELTA_CHANNEL = 0, QIE_DELTA_HEAD = 1 };
 /* Attention weights of the visible keys: softmax of the scores, or sigmoid(score + pb_h) with a
  * number per head ('mix.pb'); a row's weights are used as they are. */
 enum { QIE_WEIGHTS_SOFTMAX = 0, QIE_WEIGHTS_SIGMOID = 1 };
@@ -319,9 +324,14 @@ enum { QIE_POS_NONE = 0, QIE_POS_SINUSOID = 1 };
  * (before its norm; vdim == dim); dist_bias: the score loses r1_h * ln(1 + r2_h * (i - j)). */
 /* Rotary frequencies scaled by their wavelength l = 2 pi / f (factor 0: no scaling): f stays where
  * l < original / high, becomes f / factor where l > original / low, and between the two, with
- * s = (original / l - low) / (high - low), (1 - s) f / factor + s f. */
+ * s = (original / l - low) / (high - low), (1 - s) f / factor + s f.
+ * kind QIE_ROT_SCALE_YARN: the same blend by pair index instead.  With dim(t) = dims ln(original / (2 pi t)) / (2 ln base),
+ * lo = max(floor(dim(high)), 0), hi = min(ceil(dim(low)), dims - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
+ * pair i turns at f_i (r_i / factor + 1 - r_i); cos and sin are multiplied by 0.1 ln(factor) + 1. */
+enum { QIE_ROT_SCALE_WAVELENGTH = 0, QIE_ROT_SCALE_YARN = 1 };
 typedef struct qie_rot_scaling {
     float factor, low, high, original;
+    int32_t kind;             /* QIE_ROT_SCALE_* */
 } qie_rot_scaling;
 
 typedef struct qie_gqa_desc {
@@ -348,6 +358,7 @@ typedef struct qie_gqa_desc {
     int32_t v_bias;           /* 1: v gets a bias vector after its projection ('mix.v.b')   */
     int32_t mask_keep;        /* QIE_MASK_WINDOW: the keys j < mask_keep stay visible beyond the window (at their true positions) */
     qie_rot_scaling rot_scaling;
+    float softcap;            /* > 0: a score s (scaled, before biases) becomes softcap * tanh(s / softcap) */
 } qie_gqa_desc;
 
 /* Gated linear recurrence (the second half of QIE_MIXER_GQA_RECURRENT): per head a state
@@ -359,7 +370,11 @@ typedef struct qie_gqa_desc {
  * kind QIE_REC_KEY_DECAY: q = W_q h * dim^(-1/2), k = W_k h (heads x dim), v = W_v h; a decay per head and key
  * channel a = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau); S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; the
  * normed heads times silu(W_g h) element by element.  Tensors 'mix.right.q|k|v|g|a1|a2|a2.b|norm|o'; rank: rows of
- * W_a1 (0: taken from the tensor). */
+ * W_a1 (0: taken from the tensor).
+ * kind QIE_REC_DELTA: a gated delta rule of qie_layer_desc.delta (decay QIE_DELTA_HEAD), its tensors under 'mix.right.';
+ * heads, dim, vdim, rank and tau here are unused.
+ * qie_layer_desc.mix_norm: the two results are RMS-normed over the width with 'mix.left.out' / 'mix.right.out' before
+ * they are scaled and added. */
 typedef struct qie_recurrent_desc {
     int32_t heads, dim, vdim;
     int32_t kind;             /* QIE_REC_* */
@@ -398,17 +413,32 @@ typedef struct qie_mingru_desc {
  * position 0: S = diag(g) S; u = beta (v - S^T k); S += k u^T; o = S^T q.  o is RMS-normed per head over
  * vdim with the weight 'mix.norm' [vdim], times sigmoid(W_g2 (W_g1 x)) (heads x vdim), then W_o.  The
  * last conv - 1 rows of q, k, v before their convolution belong to the slot's state.  rank_a / rank_g:
- * rows of W_a1 / W_g1.  Tensors 'l<i>.mix.q|q.conv|k|k.conv|v|v.conv|b|A_log|a1|a2|dt_bias|g1|g2|norm|o'. */
+ * rows of W_a1 / W_g1.  Tensors 'l<i>.mix.q|q.conv|k|k.conv|v|v.conv|b|A_log|a1|a2|dt_bias|g1|g2|norm|o'.
+ * decay QIE_DELTA_HEAD: one decay per head, g = exp(-exp(A_log_h) softplus(W_a x + dt_bias)) ('mix.a' [heads, width],
+ * 'mix.dt_bias' [heads]), and the output gate silu(W_g x) ('mix.g' [heads * vdim, width]); no a1, a2, g1, g2. */
 typedef struct qie_delta_desc {
     int32_t heads, kv_heads, dim, vdim, conv, rank_a, rank_g;
-    int32_t reserved;
+    int32_t decay;            /* QIE_DELTA_* */
 } qie_delta_desc;
+
+/* Mixer QIE_MIXER_RGLRU (real-gated linear recurrent unit behind a short convolution, times a gelu branch): with x the
+ * mixer's input and n = width, y = gelu_tanh(W_y x + b_y), u = conv(W_x x + b_x) (causal over time per channel, `conv`
+ * taps, last column = the current token, with a bias; inputs before the start are zero).  u in `blocks` equal parts of s
+ * channels: r = sigmoid(R_b u_b + r_b), i = sigmoid(I_b u_b + i_b) with square matrices per part; log a = -decay * r *
+ * softplus(lam); per channel S_t = a S_(t-1) + sqrt(1 - a^2) i u, S fp32 in the slot, zero at position 0; output
+ * W_o (S * y).  The last conv - 1 rows W_x x belong to the slot's state.  Tensors 'l<i>.mix.y|y.b|x|x.b' [n, width] / [n],
+ * 'conv' [n, conv], 'conv.b', 'ra|ri' [blocks, s, s], 'ra.b|ri.b' [blocks, s], 'lam' [n], 'o' [width, n]. */
+typedef struct qie_rglru_desc {
+    int32_t width, blocks, conv;
+    float decay;
+} qie_rglru_desc;
 
 typedef struct qie_layer_desc {
     int32_t mixer;            /* QIE_MIXER_*                                          */
     int32_t heads, dim, rot_dim, vdim, kv_rank;
     int32_t window;           /* query at position i attends keys i - window < j <= i */
-    int32_t kv_from;          /* -1: own W_dkv; else the layer whose cache rows it reads */
+    int32_t kv_from;          /* -1: own cache rows; else the earlier layer whose rows it reads (latent attention: no W_dkv;
+                                 QIE_MIXER_GQA: no W_k, W_v)                              */
     int32_t rot_dims;         /* rotated coordinates of a rotated part (even, <= rot_dim) */
     float rot_base, scale;
     int32_t ff_kind;          /* QIE_FF_*                                             */
@@ -432,7 +462,8 @@ typedef struct qie_layer_desc {
     qie_rot_scaling rot_scaling;   /* latent attention                                 */
     qie_state_space_desc ssm; /* QIE_MIXER_STATE_SPACE                                 */
     float ff_limit;           /* QIE_ACT_CLAMPED_GATED                                 */
-    int32_t reserved4;
+    int32_t mix_norm;         /* QIE_MIXER_GQA_RECURRENT: both results normed before they are scaled and added */
+    qie_rglru_desc rglru;     /* QIE_MIXER_RGLRU                                       */
 } qie_layer_desc;
 
 typedef struct qie_arch_desc {
@@ -459,6 +490,8 @@ typedef struct qie_arch_desc {
     int32_t streams, canon_taps, embed_norm;
     float norm_offset;
     float logit_scale;        /* the logits are multiplied by it (0 is read as 1) */
+    int32_t shared_norm;      /* QIE_BLOCK_PARALLEL: mixer and feed-forward read the same normed row, no 'norm2' */
+    float logit_softcap;      /* > 0: the logits z become logit_softcap * tanh(z / logit_softcap) */
 } qie_arch_desc;
 
 int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* opts, qie_engine** out);
@@ -469,7 +502,7 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
  * recurrence runs beside it, whose tensors are 'l<i>.mix.right.q|f|f.b|lower|v|norm|o'),
  * 'l<i>.mix.pb|g' (sigmoid weights, head gate), 'l<i>.mix.z|z.b|x|x.b|g|o' (QIE_MIXER_MINGRU),
  * 'l<i>.mix.q.b|k.b|sink' (biased, sink attention), 'l<i>.mix.dq|dq.norm|uq' (latent queries), the
- * QIE_MIXER_CHANNEL_DELTA and QIE_MIXER_STATE_SPACE tensors, 'mix.v.b', 'embed.norm', 'l<i>.hc1|hc2.in|out|mix', 'l<i>.canon1',
+ * QIE_MIXER_CHANNEL_DELTA, QIE_MIXER_STATE_SPACE and QIE_MIXER_RGLRU tensors, 'l<i>.mix.left.out|right.out', 'mix.v.b', 'embed.norm', 'l<i>.hc1|hc2.in|out|mix', 'l<i>.canon1',
  * 'l<i>.mlp.gate|up|down|act|router|router.b|correction', 'l<i>.mlp.e<j>.gate|up|down'.
  * qie_engine_finalize_weights checks every tensor the architecture needs against its shape,
  * builds the device layouts (fused projection rows, per-head transposed W_uk, experts end to

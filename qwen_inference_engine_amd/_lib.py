@@ -82,21 +82,23 @@ class EngineOptsC(C.Structure):
 
 
 QIE_MIXER_LATENT_ATTENTION, QIE_MIXER_GQA, QIE_MIXER_GQA_RECURRENT, QIE_MIXER_MINGRU, QIE_MIXER_CHANNEL_DELTA = 1, 2, 3, 4, 5
-QIE_MIXER_STATE_SPACE = 6
+QIE_MIXER_STATE_SPACE, QIE_MIXER_RGLRU = 6, 7
 QIE_FF_NONE, QIE_FF_DENSE, QIE_FF_MOE = 0, 1, 2
 QIE_MASK_CAUSAL, QIE_MASK_WINDOW, QIE_MASK_CHUNK = 0, 1, 2
-QIE_QKNORM_NONE, QIE_QKNORM_WEIGHT, QIE_QKNORM_PLAIN = 0, 1, 2
+QIE_QKNORM_NONE, QIE_QKNORM_WEIGHT, QIE_QKNORM_PLAIN, QIE_QKNORM_ROW = 0, 1, 2, 3
 QIE_ROT_HALVES, QIE_ROT_INTERLEAVED = 0, 1
 QIE_BLOCK_POSTNORM_GAIN, QIE_BLOCK_SANDWICH, QIE_BLOCK_PRENORM, QIE_BLOCK_PARALLEL = 0, 1, 2, 3
 QIE_ROUTER_SIGMOID_IN, QIE_ROUTER_SOFTMAX_OUT, QIE_ROUTER_SOFTMAX_ALL = 0, 1, 2
-QIE_ACT_SILU_GATED, QIE_ACT_XIELU, QIE_ACT_GELU_TANH_GATED, QIE_ACT_CLAMPED_GATED = 0, 1, 2, 3
-QIE_REC_LOWER_BOUND, QIE_REC_KEY_DECAY = 0, 1
+QIE_ACT_SILU_GATED, QIE_ACT_XIELU, QIE_ACT_GELU_TANH_GATED, QIE_ACT_CLAMPED_GATED, QIE_ACT_RELU_GATED = 0, 1, 2, 3, 4
+QIE_REC_LOWER_BOUND, QIE_REC_KEY_DECAY, QIE_REC_DELTA = 0, 1, 2
+QIE_DELTA_CHANNEL, QIE_DELTA_HEAD = 0, 1
+QIE_ROT_SCALE_WAVELENGTH, QIE_ROT_SCALE_YARN = 0, 1
 QIE_WEIGHTS_SOFTMAX, QIE_WEIGHTS_SIGMOID = 0, 1
 QIE_POS_NONE, QIE_POS_SINUSOID = 0, 1
 
 
 class RotScalingC(C.Structure):
-    _fields_ = [("factor", C.c_float), ("low", C.c_float), ("high", C.c_float), ("original", C.c_float)]
+    _fields_ = [("factor", C.c_float), ("low", C.c_float), ("high", C.c_float), ("original", C.c_float), ("kind", C.c_int32)]
 
 
 class GqaDescC(C.Structure):
@@ -105,7 +107,8 @@ class GqaDescC(C.Structure):
                 ("mask", C.c_int32), ("mask_size", C.c_int32), ("values_are_keys", C.c_int32), ("dist_bias", C.c_int32),
                 ("rot_base", C.c_float), ("scale", C.c_float), ("qk_bias", C.c_int32), ("sink", C.c_int32),
                 ("weights", C.c_int32), ("slope_bias", C.c_int32), ("head_gate", C.c_int32), ("q_temp_every", C.c_int32),
-                ("q_temp_coef", C.c_float), ("out_gate", C.c_int32), ("v_bias", C.c_int32), ("mask_keep", C.c_int32), ("rot_scaling", RotScalingC)]
+                ("q_temp_coef", C.c_float), ("out_gate", C.c_int32), ("v_bias", C.c_int32), ("mask_keep", C.c_int32), ("rot_scaling", RotScalingC),
+                ("softcap", C.c_float)]
 
 
 class RecurrentDescC(C.Structure):
@@ -123,7 +126,11 @@ class MinGruDescC(C.Structure):
 
 class DeltaDescC(C.Structure):
     _fields_ = [("heads", C.c_int32), ("kv_heads", C.c_int32), ("dim", C.c_int32), ("vdim", C.c_int32), ("conv", C.c_int32),
-                ("rank_a", C.c_int32), ("rank_g", C.c_int32), ("reserved", C.c_int32)]
+                ("rank_a", C.c_int32), ("rank_g", C.c_int32), ("decay", C.c_int32)]
+
+
+class RgLruDescC(C.Structure):
+    _fields_ = [("width", C.c_int32), ("blocks", C.c_int32), ("conv", C.c_int32), ("decay", C.c_float)]
 
 
 class LayerDescC(C.Structure):
@@ -136,7 +143,7 @@ class LayerDescC(C.Structure):
                 ("mingru", MinGruDescC), ("ff_act", C.c_int32), ("identity", C.c_int32), ("groups", C.c_int32),
                 ("groups_keep", C.c_int32), ("route_scale", C.c_float), ("reserved3", C.c_int32 * 3),
                 ("delta", DeltaDescC), ("rot_scaling", RotScalingC), ("ssm", StateSpaceDescC), ("ff_limit", C.c_float),
-                ("reserved4", C.c_int32)]
+                ("mix_norm", C.c_int32), ("rglru", RgLruDescC)]
 
 
 class ArchDescC(C.Structure):
@@ -145,7 +152,7 @@ class ArchDescC(C.Structure):
                 ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32),
                 ("pos_embed", C.c_int32), ("embed_scale", C.c_float), ("layers", C.POINTER(LayerDescC)),
                 ("streams", C.c_int32), ("canon_taps", C.c_int32), ("embed_norm", C.c_int32), ("norm_offset", C.c_float),
-                ("logit_scale", C.c_float)]
+                ("logit_scale", C.c_float), ("shared_norm", C.c_int32), ("logit_softcap", C.c_float)]
 
 
 # (name, restype, argtypes) — every symbol the public headers declare.

@@ -102,7 +102,27 @@ struct LayerDev {
     int col_dt = 0;
     // parallel blocks: wo also holds W_down, and the feed-forward's activations follow the mixer's columns (-1: no)
     int cat_ff = -1;
+    // parallel blocks with one norm: the feed-forward's gate and up rows are the last of w_in (-1: a product of their own)
+    int col_ff = -1;
+    // delta rule: its first column inside the projection (behind an attention's); decay per head: the columns of W_a, W_g
+    int col_d = 0;
+    // attention beside a recurrence, both normed before they are added: output matrices of their own (wo: the
+    // attention's), weights of the two norms
+    void* wo_r = nullptr;
+    float *out_l = nullptr, *out_r = nullptr;
+    // QIE_MIXER_RGLRU: w_in = [y ; x] rows; biases, the convolution's taps and bias, gate matrices [blocks][2 s][s] and
+    // biases, decay * softplus(lam)
+    float *lr_yb = nullptr, *lr_xb = nullptr, *lr_conv = nullptr, *lr_conv_b = nullptr, *lr_rb = nullptr, *lr_ib = nullptr, *lr_decay = nullptr;
+    void* lr_gates = nullptr;
 };
+
+// columns of the recurrence beside an attention
+static int64_t rec_cols(const qie_layer_desc& d) {
+    return d.mixer != QIE_MIXER_GQA_RECURRENT ? 0
+           : d.rec.kind == QIE_REC_DELTA      ? (int64_t)d.delta.heads * d.delta.vdim
+                                              : (int64_t)d.rec.heads * d.rec.vdim;
+}
+static bool gated_dense(const qie_layer_desc& d) { return d.ff_kind == QIE_FF_DENSE && d.ff_act != QIE_ACT_XIELU; }
 
 // One execution of a layer: layers of a repeated group run several times, each run with its
 // own cache region and recurrent state.
@@ -175,6 +195,7 @@ struct LayeredBatch {
     // beside an attention on side[1])
     hipEvent_t ev_go[2] = {nullptr, nullptr}, ev_done[2] = {nullptr, nullptr};
     float* y2 = nullptr;
+    float* mix2 = nullptr;            // the recurrence's output product where both branches are normed before they are added
     uint16_t* y2_bf = nullptr;
     int64_t m_state = 0, m_hd = 0;    // largest state / gate row count of a layer run
     // bf16 K / V caches on the matrix-core attention: V rows stored [kv_heads][vdim][page_tokens].  Per layer run
@@ -312,10 +333,21 @@ static int lm_rope(LayeredModel* m, qie_engine* e, double base, int dims, int* i
             return 0;
         }
     const int half = dims / 2, rows = e->opts.max_ctx;
+    double amp = 1.0, lo = 0.0, hi = 0.0;
+    const bool yarn = sc.factor > 0.f && sc.kind == QIE_ROT_SCALE_YARN;
+    if (yarn) {
+        auto index_of = [&](double turns) { return dims * std::log(sc.original / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
+        lo = std::max(std::floor(index_of(sc.high)), 0.0);
+        hi = std::min(std::ceil(index_of(sc.low)), (double)(dims - 1));
+        amp = 0.1 * std::log((double)sc.factor) + 1.0;
+    }
     std::vector<float> cs((size_t)rows * half), sn((size_t)rows * half);
     for (int j = 0; j < half; j++) {
         double f = std::pow(base, -2.0 * j / dims);
-        if (sc.factor > 0.f) {   // by wavelength: short ones stay, long ones slow down by the factor, a blend between
+        if (yarn) {   // by pair index: the first ones stay, the last ones slow down by the factor
+            const double ramp = std::min(std::max((j - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f = f / sc.factor * ramp + f * (1.0 - ramp);
+        } else if (sc.factor > 0.f) {   // by wavelength: short ones stay, long ones slow down by the factor, a blend between
             const double lam = 2.0 * M_PI / f, orig = sc.original;
             if (lam > orig / sc.low)
                 f = f / sc.factor;
@@ -325,8 +357,8 @@ static int lm_rope(LayeredModel* m, qie_engine* e, double base, int dims, int* i
             }
         }
         for (int p = 0; p < rows; p++) {
-            cs[(size_t)p * half + j] = (float)std::cos(p * f);
-            sn[(size_t)p * half + j] = (float)std::sin(p * f);
+            cs[(size_t)p * half + j] = (float)(amp * std::cos(p * f));
+            sn[(size_t)p * half + j] = (float)(amp * std::sin(p * f));
         }
     }
     RopeTab t{base, dims, sc, nullptr, nullptr};
@@ -384,7 +416,7 @@ static int finalize_out(LayeredModel* m, int i, const HostTensor* o1, const Host
     const qie_layer_desc& d = L.d;
     const int64_t W = m->a.width;
     const HostTensor* wd = nullptr;
-    if (m->a.block == QIE_BLOCK_PARALLEL && d.ff_kind == QIE_FF_DENSE && d.ff_act != QIE_ACT_XIELU) {
+    if (m->a.block == QIE_BLOCK_PARALLEL && gated_dense(d)) {
         wd = lm_find(m, "l" + std::to_string(i) + ".mlp.down", {W, (int64_t)d.ff});
         if (!wd) return -22;
         L.cat_ff = L.n_cat;
@@ -409,6 +441,95 @@ static int64_t lm_rows_of(LayeredModel* m, const std::string& name) {
     return it != m->host.end() && it->second.shape.size() == 2 ? it->second.shape[0] : 0;
 }
 
+// Input matrix of layer i: n_in mixer rows (filled by the caller) and, in parallel blocks with one norm, the gate and up
+// rows of a gated dense feed-forward behind them (their first column a multiple of 4, for 16-byte loads).
+static int alloc_input(LayeredModel* m, int i) {
+    LayerDev& L = m->L[i];
+    const int64_t W = m->a.width, ff = L.d.ff, rows = L.n_in;
+    if (m->a.block == QIE_BLOCK_PARALLEL && m->a.shared_norm && gated_dense(L.d)) {
+        L.col_ff = (L.n_in + 3) / 4 * 4;
+        L.n_in = (int)((L.col_ff + 2 * ff + 3) / 4 * 4);
+    }
+    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
+    if (L.col_ff < 0) return 0;
+    const std::string pl = "l" + std::to_string(i) + ".mlp.";
+    LM_GET(wg, pl + "gate", ff, W);
+    LM_GET(wu, pl + "up", ff, W);
+    // rows between the mixer's and the gate's, and behind the last: zero
+    QIE_HIP(hipMemset((char*)L.w_in + (size_t)rows * W * m->esz(), 0, (size_t)(L.n_in - rows) * W * m->esz()));
+    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_ff, W, *wg));
+    return lm_upload_rows(m, L.w_in, L.col_ff + ff, W, *wu);
+}
+
+// Columns of a delta rule inside its layer's projection rows, from col0 on: channel decay [q ; k ; v ; b ; a1 ; g1], head
+// decay [q ; k ; v ; g ; b ; a].  Returns the column behind them.
+static int delta_columns(LayerDev& L, int col0) {
+    const qie_delta_desc& c = L.d.delta;
+    const int nk = c.kv_heads * c.dim, nv = c.heads * c.vdim, C = 2 * nk + nv;
+    L.col_d = col0;
+    if (c.decay == QIE_DELTA_HEAD) {
+        L.col_g1 = col0 + C;
+        L.col_b = L.col_g1 + nv;
+        L.col_a1 = L.col_b + c.heads;
+        return L.col_a1 + c.heads;
+    }
+    L.col_b = col0 + C;
+    L.col_a1 = L.col_b + c.heads;
+    L.col_g1 = L.col_a1 + L.rank_a;
+    return L.col_g1 + L.rank_g;
+}
+
+// A delta rule's rows of w_in, second-stage matrices, convolution taps (end to end), exp(A_log) in double, head norm
+static int delta_upload(LayeredModel* m, int i, const std::string& px) {
+    LayerDev& L = m->L[i];
+    const qie_delta_desc& c = L.d.delta;
+    const int64_t W = m->a.width, nk = (int64_t)c.kv_heads * c.dim, nv = (int64_t)c.heads * c.vdim, C = 2 * nk + nv;
+    LM_GET(tq, px + "q", nk, W);
+    LM_GET(tk, px + "k", nk, W);
+    LM_GET(tv, px + "v", nv, W);
+    LM_GET(tb, px + "b", (int64_t)c.heads, W);
+    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_d, W, *tq));
+    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_d + nk, W, *tk));
+    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_d + 2 * nk, W, *tv));
+    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_b, W, *tb));
+    if (c.decay == QIE_DELTA_HEAD) {
+        LM_GET(ta, px + "a", (int64_t)c.heads, W);
+        LM_GET(tg, px + "g", nv, W);
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_a1, W, *ta));
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_g1, W, *tg));
+        QIE_TRY(lm_vector(m, &L.dl_dt_bias, px + "dt_bias", (int64_t)c.heads));
+    } else {
+        LM_GET(ta1, px + "a1", (int64_t)L.rank_a, W);
+        LM_GET(tg1, px + "g1", (int64_t)L.rank_g, W);
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_a1, W, *ta1));
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_g1, W, *tg1));
+        LM_GET(ta2, px + "a2", (int64_t)c.heads * c.dim, (int64_t)L.rank_a);
+        LM_GET(tg2, px + "g2", nv, (int64_t)L.rank_g);
+        QIE_TRY(lm_alloc(m, &L.w_a2, (size_t)ta2->numel() * m->esz()));
+        QIE_TRY(lm_upload_rows(m, L.w_a2, 0, L.rank_a, *ta2));
+        QIE_TRY(lm_alloc(m, &L.w_g2, (size_t)tg2->numel() * m->esz()));
+        QIE_TRY(lm_upload_rows(m, L.w_g2, 0, L.rank_g, *tg2));
+        QIE_TRY(lm_vector(m, &L.dl_dt_bias, px + "dt_bias", (int64_t)c.heads * c.dim));
+    }
+    LM_GET(cq, px + "q.conv", nk, (int64_t)c.conv);
+    LM_GET(ck, px + "k.conv", nk, (int64_t)c.conv);
+    LM_GET(cv, px + "v.conv", nv, (int64_t)c.conv);
+    {
+        HostTensor cat;
+        cat.dtype = 2;
+        cat.shape = {C, (int64_t)c.conv};
+        cat.data.resize((size_t)C * c.conv * 4);
+        float* f = (float*)cat.data.data();
+        int64_t o = 0;
+        for (const HostTensor* t : {cq, ck, cv})
+            for (int64_t k = 0; k < t->numel(); k++) f[o++] = host_elem(*t, k);
+        QIE_TRY(lm_floats(m, &L.dl_conv, cat));
+    }
+    LM_GET(tal, px + "A_log", (int64_t)c.heads);
+    QIE_TRY(lm_exp_vector(m, &L.dl_exp_a, *tal));
+    return lm_vector(m, &L.dl_norm, px + "norm", (int64_t)c.vdim);
+}
+
 // Fused input rows and output columns of a grouped-query attention, alone ('mix.') or beside a
 // gated recurrence ('mix.left.' / 'mix.right.').
 static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
@@ -418,8 +539,10 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
     const bool rec = d.mixer == QIE_MIXER_GQA_RECURRENT;
     const int64_t W = m->a.width;
     const std::string pl = "l" + std::to_string(i) + ".", pa = pl + (rec ? "mix.left." : "mix."), pr = pl + "mix.right.";
-    const int64_t nq = (int64_t)a.heads * a.dim, nk = (int64_t)a.kv_heads * a.dim, nv = a.values_are_keys ? 0 : (int64_t)a.kv_heads * a.vdim;
-    const int64_t rq = rec ? (int64_t)d.rec.heads * d.rec.dim : 0, rv = rec ? (int64_t)d.rec.heads * d.rec.vdim : 0;
+    const bool own = d.kv_from < 0, delta = rec && d.rec.kind == QIE_REC_DELTA;
+    const int64_t nq = (int64_t)a.heads * a.dim, nk = own ? (int64_t)a.kv_heads * a.dim : 0,
+                  nv = a.values_are_keys || !own ? 0 : (int64_t)a.kv_heads * a.vdim;
+    const int64_t rq = rec && !delta ? (int64_t)d.rec.heads * d.rec.dim : 0, rv = delta ? 0 : rec_cols(d), rec_out = rec_cols(d);
     const bool key_decay = rec && d.rec.kind == QIE_REC_KEY_DECAY;
     L.col_k = (int)nq;
     L.col_v = a.values_are_keys ? -1 : (int)(nq + nk);
@@ -437,18 +560,25 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
         L.col_a1 = (int)(L.col_rg + rv);
         L.n_in = L.col_a1 + L.rank_a;
     }
-    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
+    if (delta) L.n_in = delta_columns(L, L.n_in);
+    QIE_TRY(alloc_input(m, i));
     LM_GET(tq, pa + "q", nq, W);
-    LM_GET(tk, pa + "k", nk, W);
     QIE_TRY(lm_upload_rows(m, L.w_in, 0, W, *tq));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_k, W, *tk));
-    if (!a.values_are_keys) {
+    if (own) {
+        LM_GET(tk, pa + "k", nk, W);
+        QIE_TRY(lm_upload_rows(m, L.w_in, L.col_k, W, *tk));
+    }
+    if (own && !a.values_are_keys) {
         LM_GET(tv, pa + "v", nv, W);
         QIE_TRY(lm_upload_rows(m, L.w_in, L.col_v, W, *tv));
     }
     if (a.qk_norm == QIE_QKNORM_WEIGHT) {
         QIE_TRY(lm_vector(m, &L.qn_w, pa + "q.norm", a.dim));
-        QIE_TRY(lm_vector(m, &L.kn_w, pa + "k.norm", a.dim));
+        if (own) QIE_TRY(lm_vector(m, &L.kn_w, pa + "k.norm", a.dim));
+    }
+    if (a.qk_norm == QIE_QKNORM_ROW) {
+        QIE_TRY(lm_vector(m, &L.qn_w, pa + "q.norm", nq));
+        if (own) QIE_TRY(lm_vector(m, &L.kn_w, pa + "k.norm", nk));
     }
     if (a.dist_bias) {
         QIE_TRY(lm_vector(m, &L.r1, pa + "r1", a.heads));
@@ -460,9 +590,9 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
     }
     if (a.qk_bias) {
         QIE_TRY(lm_vector(m, &L.q_bias, pa + "q.b", nq));
-        QIE_TRY(lm_vector(m, &L.k_bias, pa + "k.b", nk));
+        if (own) QIE_TRY(lm_vector(m, &L.k_bias, pa + "k.b", nk));
     }
-    if (a.v_bias) QIE_TRY(lm_vector(m, &L.v_bias, pa + "v.b", nv));
+    if (a.v_bias && own) QIE_TRY(lm_vector(m, &L.v_bias, pa + "v.b", nv));
     if (a.sink) QIE_TRY(lm_vector(m, &L.sink, pa + "sink", a.heads));
     if (a.weights == QIE_WEIGHTS_SIGMOID) QIE_TRY(lm_vector(m, &L.pb, pa + "pb", a.heads));
     if (a.slope_bias) {
@@ -477,9 +607,26 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
     if (a.rot_values) QIE_TRY(lm_rope(m, e, (double)a.rot_base, a.vdim, &L.rope_v));
     const int64_t ca = (int64_t)a.heads * a.vdim;
     L.cat_rec = (int)ca;
-    L.n_cat = (int)(ca + rv);
+    L.n_cat = (int)(ca + rec_out);
     LM_GET(to, pa + "o", W, ca);
     if (!rec) return finalize_out(m, i, to);
+    auto outputs = [&]() -> int {
+        LM_GET(tro, pr + "o", W, rec_out);
+        if (!d.mix_norm) return finalize_out(m, i, to, tro);
+        // both branches are normed before they are added: a product for each, columns at multiples of 8 for 16-byte loads
+        L.cat_rec = (int)((ca + 7) / 8 * 8);
+        L.n_cat = (int)(L.cat_rec + (rec_out + 7) / 8 * 8);
+        QIE_TRY(lm_alloc(m, &L.wo, (size_t)to->numel() * m->esz()));
+        QIE_TRY(lm_upload_rows(m, L.wo, 0, ca, *to));
+        QIE_TRY(lm_alloc(m, &L.wo_r, (size_t)tro->numel() * m->esz()));
+        QIE_TRY(lm_upload_rows(m, L.wo_r, 0, rec_out, *tro));
+        QIE_TRY(lm_vector(m, &L.out_l, pa + "out", W));
+        return lm_vector(m, &L.out_r, pr + "out", W);
+    };
+    if (delta) {
+        QIE_TRY(delta_upload(m, i, pr));
+        return outputs();
+    }
     LM_GET(trq, pr + "q", rq, W);
     LM_GET(trf, pr + (key_decay ? "k" : "f"), rq, W);
     LM_GET(trv, pr + "v", rv, W);
@@ -500,8 +647,7 @@ static int finalize_gqa_mixer(qie_engine* e, LayeredModel* m, int i) {
         QIE_TRY(lm_vector(m, &L.rec_lower, pr + "lower", rq));
     }
     QIE_TRY(lm_vector(m, &L.rec_norm, pr + "norm", d.rec.vdim));
-    LM_GET(tro, pr + "o", W, rv);
-    return finalize_out(m, i, to, tro);
+    return outputs();
 }
 
 // State space: the projection as stored, the convolution, per-head vectors (exp(A_log) in double)
@@ -514,7 +660,7 @@ static int finalize_state_space(LayeredModel* m, int i) {
     L.n_in = L.col_dt + c.heads;
     L.n_cat = (int)inner;
     LM_GET(ti, px + "in", (int64_t)L.n_in, W);
-    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
+    QIE_TRY(alloc_input(m, i));
     QIE_TRY(lm_upload_rows(m, L.w_in, 0, W, *ti));
     LM_GET(tc, px + "conv", C, (int64_t)c.conv);
     QIE_TRY(lm_floats(m, &L.ss_conv, *tc));
@@ -537,7 +683,7 @@ static int finalize_mingru(LayeredModel* m, int i) {
     const std::string px = "l" + std::to_string(i) + ".mix.";
     L.n_in = (int)(3 * n);
     L.n_cat = (int)n;
-    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
+    QIE_TRY(alloc_input(m, i));
     LM_GET(tz, px + "z", n, W);
     LM_GET(tx, px + "x", n, W);
     LM_GET(tg, px + "g", n, W);
@@ -550,61 +696,76 @@ static int finalize_mingru(LayeredModel* m, int i) {
     return finalize_out(m, i, to);
 }
 
-// Gated delta rule: fused input rows [q ; k ; v ; b ; a1 ; g1], the second-stage matrices, the three
-// convolutions' taps end to end, exp(A_log) in double.  rank_a / rank_g 0: the rows of 'a1' / 'g1'.
+// Gated delta rule as a layer's mixer.  rank_a / rank_g 0: the rows of 'a1' / 'g1'.
 static int finalize_delta(LayeredModel* m, int i) {
     LayerDev& L = m->L[i];
     const qie_delta_desc& c = L.d.delta;
-    const int64_t W = m->a.width, nk = (int64_t)c.kv_heads * c.dim, nv = (int64_t)c.heads * c.vdim, C = 2 * nk + nv;
+    const int64_t nv = (int64_t)c.heads * c.vdim;
     const std::string px = "l" + std::to_string(i) + ".mix.";
-    L.rank_a = c.rank_a > 0 ? c.rank_a : (int)lm_rows_of(m, px + "a1");
-    L.rank_g = c.rank_g > 0 ? c.rank_g : (int)lm_rows_of(m, px + "g1");
-    QIE_REQUIRE(L.rank_a > 0 && L.rank_g > 0, "layered weights: layer %d: tensors '%sa1' / '%sg1' give no rank", i, px.c_str(), px.c_str());
-    L.col_k = (int)nk;
-    L.col_v = (int)(2 * nk);
-    L.col_b = (int)C;
-    L.col_a1 = (int)(C + c.heads);
-    L.col_g1 = L.col_a1 + L.rank_a;
-    L.n_in = L.col_g1 + L.rank_g;
+    if (c.decay == QIE_DELTA_CHANNEL) {
+        L.rank_a = c.rank_a > 0 ? c.rank_a : (int)lm_rows_of(m, px + "a1");
+        L.rank_g = c.rank_g > 0 ? c.rank_g : (int)lm_rows_of(m, px + "g1");
+        QIE_REQUIRE(L.rank_a > 0 && L.rank_g > 0, "layered weights: layer %d: tensors '%sa1' / '%sg1' give no rank", i, px.c_str(), px.c_str());
+    }
+    L.n_in = delta_columns(L, 0);
     L.n_cat = (int)nv;
-    QIE_TRY(lm_alloc(m, &L.w_in, (size_t)L.n_in * W * m->esz()));
-    LM_GET(tq, px + "q", nk, W);
-    LM_GET(tk, px + "k", nk, W);
-    LM_GET(tv, px + "v", nv, W);
-    LM_GET(tb, px + "b", (int64_t)c.heads, W);
-    LM_GET(ta1, px + "a1", (int64_t)L.rank_a, W);
-    LM_GET(tg1, px + "g1", (int64_t)L.rank_g, W);
-    QIE_TRY(lm_upload_rows(m, L.w_in, 0, W, *tq));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_k, W, *tk));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_v, W, *tv));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_b, W, *tb));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_a1, W, *ta1));
-    QIE_TRY(lm_upload_rows(m, L.w_in, L.col_g1, W, *tg1));
-    LM_GET(ta2, px + "a2", (int64_t)c.heads * c.dim, (int64_t)L.rank_a);
-    LM_GET(tg2, px + "g2", nv, (int64_t)L.rank_g);
-    QIE_TRY(lm_alloc(m, &L.w_a2, (size_t)ta2->numel() * m->esz()));
-    QIE_TRY(lm_upload_rows(m, L.w_a2, 0, L.rank_a, *ta2));
-    QIE_TRY(lm_alloc(m, &L.w_g2, (size_t)tg2->numel() * m->esz()));
-    QIE_TRY(lm_upload_rows(m, L.w_g2, 0, L.rank_g, *tg2));
-    LM_GET(cq, px + "q.conv", nk, (int64_t)c.conv);
-    LM_GET(ck, px + "k.conv", nk, (int64_t)c.conv);
-    LM_GET(cv, px + "v.conv", nv, (int64_t)c.conv);
+    QIE_TRY(alloc_input(m, i));
+    QIE_TRY(delta_upload(m, i, px));
+    LM_GET(to, px + "o", (int64_t)m->a.width, nv);
+    return finalize_out(m, i, to);
+}
+
+// Real-gated linear recurrent unit: fused input rows [y ; x], the convolution, a block's two gate matrices end to end,
+// decay * softplus(lam) in double
+static int finalize_rglru(LayeredModel* m, int i) {
+    LayerDev& L = m->L[i];
+    const qie_rglru_desc& c = L.d.rglru;
+    const int64_t W = m->a.width, n = c.width, bs = n / c.blocks;
+    const std::string px = "l" + std::to_string(i) + ".mix.";
+    L.n_in = (int)(2 * n);
+    L.n_cat = (int)n;
+    QIE_TRY(alloc_input(m, i));
+    LM_GET(ty, px + "y", n, W);
+    LM_GET(tx, px + "x", n, W);
+    QIE_TRY(lm_upload_rows(m, L.w_in, 0, W, *ty));
+    QIE_TRY(lm_upload_rows(m, L.w_in, n, W, *tx));
+    QIE_TRY(lm_vector(m, &L.lr_yb, px + "y.b", n));
+    QIE_TRY(lm_vector(m, &L.lr_xb, px + "x.b", n));
+    LM_GET(tc, px + "conv", n, (int64_t)c.conv);
+    QIE_TRY(lm_floats(m, &L.lr_conv, *tc));
+    QIE_TRY(lm_vector(m, &L.lr_conv_b, px + "conv.b", n));
+    LM_GET(tr, px + "ra", (int64_t)c.blocks, bs, bs);
+    LM_GET(ti, px + "ri", (int64_t)c.blocks, bs, bs);
+    QIE_TRY(lm_alloc(m, &L.lr_gates, (size_t)2 * n * bs * m->esz()));
     {
-        HostTensor cat;
+        HostTensor cat;   // [blocks][R rows, I rows][bs]
         cat.dtype = 2;
-        cat.shape = {C, (int64_t)c.conv};
-        cat.data.resize((size_t)C * c.conv * 4);
+        cat.shape = {2 * n, bs};
+        cat.data.resize((size_t)2 * n * bs * 4);
         float* f = (float*)cat.data.data();
         int64_t o = 0;
-        for (const HostTensor* t : {cq, ck, cv})
-            for (int64_t k = 0; k < t->numel(); k++) f[o++] = host_elem(*t, k);
-        QIE_TRY(lm_floats(m, &L.dl_conv, cat));
+        for (int64_t b = 0; b < c.blocks; b++)
+            for (const HostTensor* t : {tr, ti})
+                for (int64_t k = 0; k < bs * bs; k++) f[o++] = host_elem(*t, b * bs * bs + k);
+        QIE_TRY(lm_upload_rows(m, L.lr_gates, 0, bs, cat));
     }
-    LM_GET(tal, px + "A_log", (int64_t)c.heads);
-    QIE_TRY(lm_exp_vector(m, &L.dl_exp_a, *tal));
-    QIE_TRY(lm_vector(m, &L.dl_dt_bias, px + "dt_bias", (int64_t)c.heads * c.dim));
-    QIE_TRY(lm_vector(m, &L.dl_norm, px + "norm", (int64_t)c.vdim));
-    LM_GET(to, px + "o", W, nv);
+    LM_GET(trb, px + "ra.b", (int64_t)c.blocks, bs);
+    LM_GET(tib, px + "ri.b", (int64_t)c.blocks, bs);
+    QIE_TRY(lm_floats(m, &L.lr_rb, *trb));
+    QIE_TRY(lm_floats(m, &L.lr_ib, *tib));
+    LM_GET(tl, px + "lam", n);
+    {
+        HostTensor dc;
+        dc.dtype = 2;
+        dc.shape = {n};
+        dc.data.resize((size_t)n * 4);
+        for (int64_t k = 0; k < n; k++) {
+            const double z = host_elem(*tl, k);
+            ((float*)dc.data.data())[k] = (float)((double)c.decay * (std::log1p(std::exp(-std::fabs(z))) + std::max(z, 0.0)));
+        }
+        QIE_TRY(lm_floats(m, &L.lr_decay, dc));
+    }
+    LM_GET(to, px + "o", W, n);
     return finalize_out(m, i, to);
 }
 
@@ -637,7 +798,11 @@ static int finalize_layer(qie_engine* e, LayeredModel* m, int i) {
     }
     if (m->a.block == QIE_BLOCK_PRENORM || m->a.block == QIE_BLOCK_PARALLEL) {
         QIE_TRY(lm_vector(m, &L.n1, pl + "norm1", m->a.width));
-        if (d.ff_kind != QIE_FF_NONE) QIE_TRY(lm_vector(m, &L.n2, pl + "norm2", m->a.width));
+        if (d.ff_kind != QIE_FF_NONE && !m->a.shared_norm) QIE_TRY(lm_vector(m, &L.n2, pl + "norm2", m->a.width));
+    }
+    if (d.mixer == QIE_MIXER_RGLRU) {
+        QIE_TRY(finalize_rglru(m, i));
+        return finalize_ff(m, i);
     }
     if (d.mixer == QIE_MIXER_MINGRU) {
         QIE_TRY(finalize_mingru(m, i));
@@ -748,9 +913,11 @@ static int finalize_ff(LayeredModel* m, int i) {
         LM_GET(wg, pl + "mlp.gate", ff, W);
         LM_GET(wu, pl + "mlp.up", ff, W);
         LM_GET(wd, pl + "mlp.down", W, ff);
-        QIE_TRY(lm_alloc(m, &L.w_gu, (size_t)2 * ff * W * m->esz()));
-        QIE_TRY(lm_upload_rows(m, L.w_gu, 0, W, *wg));
-        QIE_TRY(lm_upload_rows(m, L.w_gu, ff, W, *wu));
+        if (L.col_ff < 0) {   // else they are the last rows of the input matrix
+            QIE_TRY(lm_alloc(m, &L.w_gu, (size_t)2 * ff * W * m->esz()));
+            QIE_TRY(lm_upload_rows(m, L.w_gu, 0, W, *wg));
+            QIE_TRY(lm_upload_rows(m, L.w_gu, ff, W, *wu));
+        }
         if (L.cat_ff >= 0) return 0;   // W_down sits beside W_o
         QIE_TRY(lm_alloc(m, &L.w_down, (size_t)W * ff * m->esz()));
         QIE_TRY(lm_upload_rows(m, L.w_down, 0, ff, *wd));
@@ -836,7 +1003,28 @@ static int dense(qie_batch* b, const float* A, int64_t lda, const void* Wt, floa
 // A bf16 engine's products read the bf16 image of rows of K columns and nothing else (dense_on): their producers may
 // leave the fp32 rows unwritten.
 static bool image_only(const LayeredModel* m, int64_t K) { return !m->f32 && K % 8 == 0; }
-static float* ov_out(const qie_batch* b, const LayerDev& L) { return image_only(b->e->lm, L.n_cat) ? nullptr : b->lb->ov; }
+static float* ov_out(const qie_batch* b, const LayerDev& L) {
+    const bool img = L.wo_r ? image_only(b->e->lm, (int64_t)L.d.gqa.heads * L.d.gqa.vdim) && image_only(b->e->lm, rec_cols(L.d))
+                            : image_only(b->e->lm, L.n_cat);
+    return img ? nullptr : b->lb->ov;
+}
+
+// y[M, N] = A[M, K] W^T for K columns inside rows of lda (their bf16 image A_bf laid out alike)
+static int dense_cols(qie_batch* b, const float* A, const uint16_t* A_bf, int64_t lda, const void* Wt, float* Y, int64_t ldy, int M, int N,
+                      int K, hipStream_t st) {
+    const LayeredModel* m = b->e->lm;
+    if (!m->f32 && A_bf && K % 8 == 0 && lda % 8 == 0 && al16(Wt) && al16(A_bf)) {
+        qie_linear_args a{};
+        a.x = A_bf; a.ldx = lda;
+        a.w[0] = Wt; a.seg_rows[0] = N;
+        a.M = M; a.K = K; a.N = N;
+        a.y = Y; a.ldy = ldy;
+        a.epilogue = QIE_EPI_F32;
+        return qie_linear(&a, st);
+    }
+    lay::LinearP p{A, lda, Wt, K, Y, ldy, M, N, K, 1, 0, 0, 0, m->f32 ? 0 : 1, nullptr, m->f32 ? 0 : 1};
+    return lay::linear(p, m->f32, st);
+}
 
 // `side` runs what follows beside the engine's stream, from here until branch_join
 static int branch_fork(qie_batch* b, int k) {
@@ -1027,7 +1215,7 @@ static int enq_ff(qie_batch* b, int i, int T, hipStream_t on = nullptr) {
     LayeredBatch* s = b->lb;
     const int W = m->a.width, ff = d.ff;
     hipStream_t st = on ? on : e->stream;
-    const bool par = m->a.block == QIE_BLOCK_PARALLEL;
+    const bool par = m->a.block == QIE_BLOCK_PARALLEL && !m->a.shared_norm;
     const float* y = par ? s->y2 : s->y;
     const uint16_t* y_bf = par ? s->y2_bf : s->y_bf;
     if (d.ff_kind == QIE_FF_DENSE && d.ff_act == QIE_ACT_XIELU) {
@@ -1036,11 +1224,14 @@ static int enq_ff(qie_batch* b, int i, int T, hipStream_t on = nullptr) {
         return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf, st);
     }
     if (d.ff_kind == QIE_FF_DENSE) {
-        QIE_TRY(dense(b, y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, y_bf, st));
-        const int act = d.ff_act == QIE_ACT_GELU_TANH_GATED ? 1 : d.ff_act == QIE_ACT_CLAMPED_GATED ? 2 : 0;
+        // one norm for both branches: the input product has made the gate and up columns as well
+        if (L.col_ff < 0) QIE_TRY(dense(b, y, W, L.w_gu, s->gu, 2 * ff, T, 2 * ff, W, y_bf, st));
+        const float* gu = L.col_ff < 0 ? s->gu : s->proj + L.col_ff;
+        const int64_t ld_gu = L.col_ff < 0 ? 2 * ff : L.n_in;
+        const int act = d.ff_act == QIE_ACT_GELU_TANH_GATED ? 1 : d.ff_act == QIE_ACT_CLAMPED_GATED ? 2 : d.ff_act == QIE_ACT_RELU_GATED ? 3 : 0;
         if (L.cat_ff >= 0)
-            return lay::silu_mul(s->gu, image_only(m, L.n_cat) ? nullptr : s->ov + L.cat_ff, s->ov_bf ? s->ov_bf + L.cat_ff : nullptr, T, ff, st, act, d.ff_limit, L.n_cat);
-        QIE_TRY(lay::silu_mul(s->gu, image_only(m, ff) ? nullptr : s->act, s->act_bf, T, ff, st, act, d.ff_limit));
+            return lay::silu_mul(gu, image_only(m, L.n_cat) ? nullptr : s->ov + L.cat_ff, s->ov_bf ? s->ov_bf + L.cat_ff : nullptr, T, ff, st, act, d.ff_limit, L.n_cat, ld_gu);
+        QIE_TRY(lay::silu_mul(gu, image_only(m, ff) ? nullptr : s->act, s->act_bf, T, ff, st, act, d.ff_limit, 0, ld_gu));
         return dense(b, s->act, ff, L.w_down, s->ffo, W, T, W, ff, s->act_bf, st);
     }
     const int E = d.experts, top = d.top, n = T * top;
@@ -1129,7 +1320,8 @@ static lay::GqaAttnP gqa_attn_params(qie_batch* b, int r) {
     p.k_off = s->layer_off[r];
     p.v_off = s->v_off[r];
     p.v_transposed = s->vt_of[r];
-    p.out_scale = L.d.mixer == QIE_MIXER_GQA_RECURRENT ? L.d.gqa_scale : 1.0f;
+    p.out_scale = L.d.mixer == QIE_MIXER_GQA_RECURRENT && !L.d.mix_norm ? L.d.gqa_scale : 1.0f;
+    p.softcap = a.softcap;
     p.out = ov_out(b, L); p.out_bf = s->ov_bf; p.ld_out = L.n_cat; p.out_col = 0;
     p.slopes = a.slope_bias ? L.slopes : nullptr;
     p.pb = a.weights == QIE_WEIGHTS_SIGMOID ? L.pb : nullptr;
@@ -1140,11 +1332,24 @@ static lay::GqaAttnP gqa_attn_params(qie_batch* b, int r) {
     return p;
 }
 
-static int enq_gqa_proj(qie_batch* b, int r, int T) {
+// the fused input product of layer run r on its normed rows
+static int enq_proj(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
     return dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf);
+}
+
+// ... and, where it made the feed-forward's gate and up columns too, the rest of the feed-forward (prompt steps: on side[0])
+static int enq_in(qie_batch* b, int r, int T) {
+    const LayeredModel* m = b->e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    LayeredBatch* s = b->lb;
+    QIE_TRY(enq_proj(b, r, T));
+    if (L.col_ff < 0) return 0;
+    s->ff_branch = T > kBranchRows;
+    if (s->ff_branch) QIE_TRY(branch_fork(b, 0));
+    return enq_ff(b, m->runs[r].layer, T, s->ff_branch ? s->side[0] : nullptr);
 }
 
 static int enq_gqa_post(qie_batch* b, int r, int T) {
@@ -1178,6 +1383,7 @@ static int enq_gqa_post(qie_batch* b, int r, int T) {
     p.k_bias = a.qk_bias ? L.k_bias : nullptr;
     p.v_bias = a.v_bias ? L.v_bias : nullptr;
     p.groups = s->d_qgroups; p.n_groups = s->n_qgroups;
+    p.q_only = L.d.kv_from >= 0;
     return lay::gqa_post(p, m->f32, T, e->stream);
 }
 
@@ -1255,6 +1461,9 @@ static int enq_linrec(qie_batch* b, int r, lay::LinRecP p, hipStream_t st) {
     return lay::linrec_walk(a, st);
 }
 
+// what a recurrence's columns are multiplied by (branches that are normed first take their scale with the norm)
+static float rec_out_scale(const qie_layer_desc& d) { return d.mixer == QIE_MIXER_GQA_RECURRENT && !d.mix_norm ? d.rec_scale : 1.0f; }
+
 // Gated linear attention of layer run r: log decays through the low-rank projection, the recurrence, head norm and gate
 static int enq_key_decay(qie_batch* b, int r, int T, hipStream_t st) {
     const qie_engine* e = b->e;
@@ -1277,7 +1486,7 @@ static int enq_key_decay(qie_batch* b, int r, int T, hipStream_t st) {
     p.q_scale = 1.0f / sqrtf((float)c.dim);
     p.heads = c.heads; p.dim = c.dim; p.vdim = c.vdim;
     QIE_TRY(enq_linrec(b, r, p, st));
-    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
+    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, rec_out_scale(L.d), c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
                                L.cat_rec, st, s->proj + L.col_rg, L.n_in, 1);
 }
 
@@ -1310,6 +1519,8 @@ static int enq_state_space(qie_batch* b, int r, int T) {
                                  e->stream);
 }
 
+static int enq_delta_scan(qie_batch* b, int r, int T, bool advance, hipStream_t st);
+
 static int enq_recurrence(qie_batch* b, int r, int T, hipStream_t on = nullptr) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
@@ -1317,6 +1528,7 @@ static int enq_recurrence(qie_batch* b, int r, int T, hipStream_t on = nullptr) 
     const qie_recurrent_desc& c = L.d.rec;
     LayeredBatch* s = b->lb;
     if (c.kind == QIE_REC_KEY_DECAY) return enq_key_decay(b, r, T, on ? on : e->stream);
+    if (c.kind == QIE_REC_DELTA) return enq_delta_scan(b, r, T, true, on ? on : e->stream);
     lay::GatedScanP p{};
     p.proj = s->proj; p.ld = L.n_in; p.q_col = L.col_rq; p.f_col = L.col_rf; p.v_col = L.col_rv;
     p.entries = s->d_ent; p.n_entries = s->n_ent;
@@ -1339,30 +1551,43 @@ static int enq_recurrence(qie_batch* b, int r, int T, hipStream_t on = nullptr) 
         a.decay = nullptr;
         a.out = s->qabs;
         QIE_TRY(lay::gated_scan(a, e->stream));
-        return lay::head_norm_rows(s->olat, s->qabs, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf,
+        return lay::head_norm_rows(s->olat, s->qabs, L.rec_norm, m->a.norm_eps, rec_out_scale(L.d), c.heads, c.vdim, T, ov_out(b, L), s->ov_bf,
                                    L.n_cat, L.cat_rec, e->stream);
     }
     QIE_TRY(lay::gated_scan(p, e->stream));
-    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, L.d.rec_scale, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
+    return lay::head_norm_rows(s->olat, nullptr, L.rec_norm, m->a.norm_eps, rec_out_scale(L.d), c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat,
                                L.cat_rec, e->stream);
 }
 
-// the layer's output product over the mixer's columns (parallel blocks: and the feed-forward's) -> s->mix
-static int enq_out(qie_batch* b, int r, int T) {
+// the recurrence's own output product, where both branches are normed before they are added -> s->mix2
+static int enq_out_rec(qie_batch* b, int r, int T, hipStream_t st) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
+    return dense_cols(b, s->ov + L.cat_rec, s->ov_bf ? s->ov_bf + L.cat_rec : nullptr, L.n_cat, L.wo_r, s->mix2, m->a.width, T, m->a.width,
+                      (int)rec_cols(L.d), st);
+}
+
+// the layer's output product over the mixer's columns (parallel blocks: and the feed-forward's) -> s->mix; rec: also the
+// recurrence's own
+static int enq_out(qie_batch* b, int r, int T, bool rec = true) {
+    const LayeredModel* m = b->e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    LayeredBatch* s = b->lb;
+    if (L.wo_r) {
+        if (rec) QIE_TRY(enq_out_rec(b, r, T, b->e->stream));
+        return dense_cols(b, s->ov, s->ov_bf, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.d.gqa.heads * L.d.gqa.vdim, b->e->stream);
+    }
+    if (s->ff_branch && L.cat_ff >= 0) {   // the product takes the feed-forward's activations
+        QIE_TRY(branch_join(b, 0));
+        s->ff_branch = false;
+    }
     return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
 }
 
 static int enq_state_space_mixer(qie_batch* b, int r, int T) {
-    const LayeredModel* m = b->e->lm;
-    const LayerDev& L = m->L[m->runs[r].layer];
-    LayeredBatch* s = b->lb;
-    QIE_TRY(dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf));
+    QIE_TRY(enq_in(b, r, T));
     QIE_TRY(enq_state_space(b, r, T));
-    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
-    s->ff_branch = false;
     return enq_out(b, r, T);
 }
 
@@ -1370,20 +1595,21 @@ static int enq_gqa_mixer(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     LayeredBatch* s = b->lb;
-    QIE_TRY(enq_gqa_proj(b, r, T));
-    // a recurrence of kind key decay runs beside the attention (their scratch and their columns are apart)
-    const bool rec = L.d.mixer == QIE_MIXER_GQA_RECURRENT, beside = rec && L.d.rec.kind == QIE_REC_KEY_DECAY && T > kBranchRows;
+    QIE_TRY(enq_in(b, r, T));
+    // recurrences with scratch and columns apart from the attention's run beside it
+    const bool rec = L.d.mixer == QIE_MIXER_GQA_RECURRENT, beside = rec && L.d.rec.kind != QIE_REC_LOWER_BOUND && T > kBranchRows;
     if (beside) {
         QIE_TRY(branch_fork(b, 1));
         QIE_TRY(enq_recurrence(b, r, T, s->side[1]));
+        if (L.wo_r) QIE_TRY(enq_out_rec(b, r, T, s->side[1]));
     }
     QIE_TRY(enq_gqa_post(b, r, T));
     QIE_TRY(enq_gqa_attention(b, r, T));
     if (rec && !beside) QIE_TRY(enq_recurrence(b, r, T));
-    if (beside) QIE_TRY(branch_join(b, 1));
-    if (s->ff_branch) QIE_TRY(branch_join(b, 0));
-    s->ff_branch = false;
-    return enq_out(b, r, T);
+    if (beside && !L.wo_r) QIE_TRY(branch_join(b, 1));
+    QIE_TRY(enq_out(b, r, T, !beside));
+    if (beside && L.wo_r) QIE_TRY(branch_join(b, 1));
+    return 0;
 }
 
 // minGRU of layer run r: the scan over the fused projection rows -> s->ov (gated, with its bf16 image).
@@ -1421,12 +1647,57 @@ static int enq_mingru(qie_batch* b, int r, int T) {
 }
 
 static int enq_mingru_mixer(qie_batch* b, int r, int T) {
-    const LayeredModel* m = b->e->lm;
-    const LayerDev& L = m->L[m->runs[r].layer];
-    LayeredBatch* s = b->lb;
-    QIE_TRY(dense(b, s->y, m->a.width, L.w_in, s->proj, L.n_in, T, L.n_in, m->a.width, s->y_bf));
+    QIE_TRY(enq_in(b, r, T));
     QIE_TRY(enq_mingru(b, r, T));
-    return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
+    return enq_out(b, r, T);
+}
+
+// Real-gated linear recurrent unit of layer run r on its projection rows: convolution, gates, recurrence times the gelu
+// branch -> s->ov.  Short entries take gates and recurrence in one launch; entries above kScanLong rows run the recurrence
+// in pieces (as enq_mingru).
+static int enq_rglru(qie_batch* b, int r, int T) {
+    const qie_engine* e = b->e;
+    const LayeredModel* m = e->lm;
+    const LayerDev& L = m->L[m->runs[r].layer];
+    const qie_rglru_desc& c = L.d.rglru;
+    LayeredBatch* s = b->lb;
+    const int n = c.width;
+    lay::CausalConvP cv{};
+    cv.in = s->proj; cv.ld_in = L.n_in; cv.col = n; cv.C = n; cv.taps = c.conv; cv.w = L.lr_conv; cv.bias = L.lr_conv_b; cv.in_bias = L.lr_xb;
+    cv.row_slot = s->row_slot; cv.row_pos = s->row_pos; cv.row_k = s->row_k;
+    cv.state = s->state; cv.slot_stride = s->slot_state; cv.state_off = s->conv_off[r];
+    cv.out = s->pre; cv.ld_out = n;
+    cv.entries = s->d_ent; cv.n_entries = s->n_ent;
+    QIE_TRY(lay::causal_conv_advance(cv, T, e->stream));
+    lay::RgLruP p{};
+    p.u = s->pre; p.ld_u = n; p.w = L.lr_gates; p.w_f32 = m->f32; p.r_b = L.lr_rb; p.i_b = L.lr_ib; p.decay = L.lr_decay;
+    p.blocks = c.blocks; p.bs = n / c.blocks;
+    p.a = s->qabs; p.b = s->olat; p.z = s->aux;
+    p.y = s->proj; p.ld_y = L.n_in; p.y_b = L.lr_yb;
+    p.row_slot = s->row_slot; p.row_pos = s->row_pos; p.row_k = s->row_k;
+    p.entries = s->d_ent; p.n_entries = s->n_ent;
+    p.init = p.end = s->state; p.init_stride = p.end_stride = s->slot_state; p.init_off = p.end_off = s->state_off[r];
+    p.init_if_pos = 1;
+    p.out = ov_out(b, L); p.out_bf = s->ov_bf; p.ld_out = L.n_cat; p.want_out = 1;
+    if (s->max_count <= kLinStep && T <= lay::kRgLruStepRows) return lay::rglru_step(p, T, e->stream);
+    QIE_TRY(lay::rglru_gates(p, T, e->stream));
+    if (s->max_count <= kScanLong || !s->s_loc) return lay::rglru_scan(p, e->stream);
+    lay::RgLruP a = p;
+    a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
+    a.init = nullptr; a.want_out = 0;
+    a.end = s->s_loc; a.decay_out = s->s_decay; a.end_stride = n; a.end_off = 0;
+    QIE_TRY(lay::rglru_scan(a, e->stream));
+    lay::MinGruCarryP k{s->pieces.d_spans, s->n_ent, n, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state, s->state_off[r]};
+    QIE_TRY(lay::mingru_carry(k, e->stream));
+    a.init = s->s_in; a.init_stride = n; a.init_off = 0; a.init_if_pos = 0;
+    a.end = nullptr; a.decay_out = nullptr; a.want_out = 1;
+    return lay::rglru_scan(a, e->stream);
+}
+
+static int enq_rglru_mixer(qie_batch* b, int r, int T) {
+    QIE_TRY(enq_in(b, r, T));
+    QIE_TRY(enq_rglru(b, r, T));
+    return enq_out(b, r, T);
 }
 
 // Latent attention of layer run r on the branch input s->y -> s->mix (pre-norm blocks).
@@ -1452,41 +1723,43 @@ static int enq_latent_mixer(qie_batch* b, int r, int T) {
     return enq_mixer_out(b, i, T);
 }
 
-// Gated delta rule of layer run r: fused projection [q ; k ; v ; b ; a1 ; g1] and the second-stage
-// products, then (enq_delta_scan) the short convolutions with silu, the gates, the scan and the gated head norm.
-static int enq_delta_proj(qie_batch* b, int r, int T) {
+// Gated delta rule of layer run r after its fused projection: the second-stage products (channel decay), then
+// (enq_delta_scan) the short convolutions with silu, the gates, the scan and the gated head norm.
+static int enq_delta_gates(qie_batch* b, int r, int T) {
     const LayeredModel* m = b->e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     const qie_delta_desc& c = L.d.delta;
     LayeredBatch* s = b->lb;
-    const int W = m->a.width;
-    QIE_TRY(dense(b, s->y, W, L.w_in, s->proj, L.n_in, T, L.n_in, W, s->y_bf));
+    if (c.decay == QIE_DELTA_HEAD) return 0;   // decay and gate are columns of the input product
     QIE_TRY(dense(b, s->proj + L.col_a1, L.n_in, L.w_a2, s->qabs, (int64_t)c.heads * c.dim, T, c.heads * c.dim, L.rank_a));
     return dense(b, s->proj + L.col_g1, L.n_in, L.w_g2, s->aux, (int64_t)c.heads * c.vdim, T, c.heads * c.vdim, L.rank_g);
 }
 
-static int enq_delta_scan(qie_batch* b, int r, int T, bool advance) {
+static int enq_delta_scan(qie_batch* b, int r, int T, bool advance, hipStream_t st) {
     const qie_engine* e = b->e;
     const LayeredModel* m = e->lm;
     const LayerDev& L = m->L[m->runs[r].layer];
     const qie_delta_desc& c = L.d.delta;
     LayeredBatch* s = b->lb;
     const int C = 2 * c.kv_heads * c.dim + c.heads * c.vdim;
+    const bool head = c.decay == QIE_DELTA_HEAD;
     lay::CausalConvP cv{};
-    cv.in = s->proj; cv.ld_in = L.n_in; cv.col = 0; cv.C = C; cv.taps = c.conv; cv.w = L.dl_conv;
+    cv.in = s->proj; cv.ld_in = L.n_in; cv.col = L.col_d; cv.C = C; cv.taps = c.conv; cv.w = L.dl_conv;
     cv.row_slot = s->row_slot; cv.row_pos = s->row_pos; cv.row_k = s->row_k;
     cv.state = s->state; cv.slot_stride = s->slot_state; cv.state_off = s->conv_off[r];
     cv.residual = 0; cv.silu = 1;
     cv.out = s->pre; cv.ld_out = C; cv.out_bf = nullptr;
     cv.entries = s->d_ent; cv.n_entries = s->n_ent;
     if (advance)
-        QIE_TRY(lay::causal_conv_advance(cv, T, e->stream));
+        QIE_TRY(lay::causal_conv_advance(cv, T, st));
     else
-        QIE_TRY(lay::causal_conv(cv, T, e->stream));
-    lay::DeltaPrepP pp{s->pre, C, s->proj, L.n_in, L.col_b, s->qabs, L.dl_dt_bias, L.dl_exp_a, c.heads, c.kv_heads, c.dim, c.vdim};
-    QIE_TRY(lay::delta_prep(pp, T, e->stream));
+        QIE_TRY(lay::causal_conv(cv, T, st));
+    lay::DeltaPrepP pp{s->pre, C, s->proj, L.n_in, L.col_b, head ? nullptr : s->qabs, L.dl_dt_bias, L.dl_exp_a, c.heads, c.kv_heads, c.dim,
+                       c.vdim, L.col_a1};
+    QIE_TRY(lay::delta_prep(pp, T, st));
     lay::DeltaScanP sp{};
-    sp.qkv = s->pre; sp.ld_qkv = C; sp.beta = s->proj + L.col_b; sp.ld_beta = L.n_in; sp.g = s->qabs;
+    sp.qkv = s->pre; sp.ld_qkv = C; sp.beta = s->proj + L.col_b; sp.ld_beta = L.n_in; sp.g = head ? s->proj + L.col_a1 : s->qabs;
+    sp.ld_g = head ? L.n_in : 0;
     sp.entries = s->d_ent; sp.n_entries = s->n_ent;
     sp.H = c.heads; sp.G = c.kv_heads; sp.dim = c.dim; sp.vdim = c.vdim;
     sp.state = s->state; sp.slot_stride = s->slot_state; sp.state_off = s->state_off[r];
@@ -1501,26 +1774,25 @@ static int enq_delta_scan(qie_batch* b, int r, int T, bool advance) {
         a.state = s->s_loc; a.slot_stride = n; a.state_off = 0;
         a.read_state = 0; a.write_state = 1;
         a.trans = s->s_decay; a.w_out = s->dw;
-        QIE_TRY(lay::delta_scan(a, e->stream));
+        QIE_TRY(lay::delta_scan(a, st));
         lay::DeltaCarryP k{s->pieces.d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
                            s->state_off[r], advance ? 1 : 0};
-        QIE_TRY(lay::delta_carry(k, e->stream));
+        QIE_TRY(lay::delta_carry(k, st));
         lay::DeltaApplyP ap{s->pieces.d_chunks, s->pieces.n, kScanPiece, c.heads, c.dim, c.vdim, s->s_in, s->dw, s->olat};
-        QIE_TRY(lay::delta_apply(ap, e->stream));
+        QIE_TRY(lay::delta_apply(ap, st));
     } else {
-        QIE_TRY(lay::delta_scan(sp, e->stream));
+        QIE_TRY(lay::delta_scan(sp, st));
     }
-    return lay::head_norm_rows(s->olat, nullptr, L.dl_norm, m->a.norm_eps, 1.0f, c.heads, c.vdim, T, ov_out(b, L), s->ov_bf, L.n_cat, 0,
-                               e->stream, s->aux);
+    const bool beside = L.d.mixer == QIE_MIXER_GQA_RECURRENT;
+    return lay::head_norm_rows(s->olat, nullptr, L.dl_norm, m->a.norm_eps, rec_out_scale(L.d), c.heads, c.vdim, T, ov_out(b, L), s->ov_bf,
+                               L.n_cat, beside ? L.cat_rec : 0, st, head ? s->proj + L.col_g1 : s->aux, head ? L.n_in : 0, head ? 1 : 0);
 }
 
 static int enq_delta_mixer(qie_batch* b, int r, int T) {
-    const LayeredModel* m = b->e->lm;
-    const LayerDev& L = m->L[m->runs[r].layer];
-    LayeredBatch* s = b->lb;
-    QIE_TRY(enq_delta_proj(b, r, T));
-    QIE_TRY(enq_delta_scan(b, r, T, true));
-    return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
+    QIE_TRY(enq_in(b, r, T));
+    QIE_TRY(enq_delta_gates(b, r, T));
+    QIE_TRY(enq_delta_scan(b, r, T, true, b->e->stream));
+    return enq_out(b, r, T);
 }
 
 // Pre-norm blocks: x += mixer(N1(x)); x += ff(N2(x)) with weights norm_offset + w.  One residual row
@@ -1565,6 +1837,7 @@ static int enq_run_prenorm(qie_batch* b, int r, int T, bool h_ready, bool* next_
     }
     switch (L.d.mixer) {
         case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
+        case QIE_MIXER_RGLRU: QIE_TRY(enq_rglru_mixer(b, r, T)); break;
         case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
         case QIE_MIXER_CHANNEL_DELTA: QIE_TRY(enq_delta_mixer(b, r, T)); break;
         case QIE_MIXER_STATE_SPACE: QIE_TRY(enq_state_space_mixer(b, r, T)); break;
@@ -1629,7 +1902,8 @@ static int enq_run_sandwich(qie_batch* b, int r, int T, bool h_ready, bool* next
     return 0;
 }
 
-// Parallel blocks: x += mixer(N1(x)) + ff(N2(x)).  The stream x lives in plane 1 of the stack, the embedding rows stay in
+// Parallel blocks: x += mixer(N1(x)) + ff(N2(x)), or (one norm) x += mixer(N1(x)) + ff(N1(x)) with the feed-forward's first
+// products inside the mixer's input product (enq_in).  The stream x lives in plane 1 of the stack, the embedding rows stay in
 // plane 0 when a group repeats.  Both normed rows come from one kernel, which also takes the residual add before them
 // (and the embedding rows ahead of a repeated pass); gated dense feed-forwards share the mixer's output product.
 static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next_ready) {
@@ -1641,10 +1915,17 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
     const int64_t plane = s->cap * W;
     float* x0 = s->stack;
     float* x = s->stack + plane;
-    auto norms = [&](const float* xin, const float* v, const float* v2, const float* add, const LayerDev* N) -> int {
-        const bool img = image_only(m, W);
-        lay::NormPairP p{x, xin, v, v2, add, N ? N->n1 : nullptr, N ? N->n2 : nullptr, img ? nullptr : s->y,
-                         img && N && N->d.ff_kind != QIE_FF_MOE ? nullptr : s->y2, s->y_bf, s->y2_bf, T, W, m->a.norm_eps};
+    // x = xin + v + v2 + add (J: v and v2 normed with J's branch weights, v3 added as it is), then N's normed rows
+    auto norms = [&](const float* xin, const float* v, const float* v2, const float* add, const LayerDev* N, const LayerDev* J = nullptr,
+                     const float* v3 = nullptr) -> int {
+        const bool img = image_only(m, W), moe = N && N->d.ff_kind == QIE_FF_MOE;
+        lay::NormPairP p{x, xin, v, v2, add, N ? N->n1 : nullptr, N ? N->n2 : nullptr, img && !(m->a.shared_norm && moe) ? nullptr : s->y,
+                         img && N && !moe ? nullptr : s->y2, s->y_bf, s->y2_bf, T, W, m->a.norm_eps};
+        p.v3 = v3;
+        if (J) {
+            p.v_w = J->out_l; p.v2_w = J->out_r;
+            p.v_scale = J->d.gqa_scale; p.v2_scale = J->d.rec_scale;
+        }
         return lay::norm_pair(p, e->stream);
     };
     if (!h_ready) QIE_TRY(norms(r == 0 && m->loops ? x0 : x, nullptr, nullptr, m->runs[r].add_embed ? x0 : nullptr, &L));
@@ -1652,13 +1933,16 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
     // the feed-forward beside the mixer (the experts' products have side streams of their own), started before it: its
     // tiles fill the rounds that the mixer's input product leaves part empty (started after that product: 2.55 -> 2.61 ms
     // for 2,048 rows at the 2k Sefelorn size)
-    // (a mixer whose output product takes the activations waits for them: enq_gqa_mixer, enq_state_space_mixer)
-    const bool waits = L.cat_ff < 0 || L.d.mixer == QIE_MIXER_STATE_SPACE || L.d.mixer == QIE_MIXER_GQA || L.d.mixer == QIE_MIXER_GQA_RECURRENT;
-    s->ff_branch = L.d.ff_kind == QIE_FF_DENSE && T > kBranchRows && waits;
-    if (s->ff_branch) QIE_TRY(branch_fork(b, 0));
-    if (has_ff) QIE_TRY(enq_ff(b, m->runs[r].layer, T, s->ff_branch ? s->side[0] : nullptr));
+    // (an output product that takes the activations waits for them: enq_out)
+    s->ff_branch = false;
+    if (has_ff && L.col_ff < 0) {
+        s->ff_branch = L.d.ff_kind == QIE_FF_DENSE && T > kBranchRows;
+        if (s->ff_branch) QIE_TRY(branch_fork(b, 0));
+        QIE_TRY(enq_ff(b, m->runs[r].layer, T, s->ff_branch ? s->side[0] : nullptr));
+    }
     switch (L.d.mixer) {
         case QIE_MIXER_MINGRU: QIE_TRY(enq_mingru_mixer(b, r, T)); break;
+        case QIE_MIXER_RGLRU: QIE_TRY(enq_rglru_mixer(b, r, T)); break;
         case QIE_MIXER_LATENT_ATTENTION: QIE_TRY(enq_latent_mixer(b, r, T)); break;
         case QIE_MIXER_CHANNEL_DELTA: QIE_TRY(enq_delta_mixer(b, r, T)); break;
         case QIE_MIXER_STATE_SPACE: QIE_TRY(enq_state_space_mixer(b, r, T)); break;
@@ -1668,7 +1952,11 @@ static int enq_run_parallel(qie_batch* b, int r, int T, bool h_ready, bool* next
     s->ff_branch = false;
     const bool last = r + 1 == (int)m->runs.size(), fuse_next = !last && !s->keep_on;
     const LayerDev* N = fuse_next ? &m->L[m->runs[r + 1].layer] : nullptr;
-    QIE_TRY(norms(x, s->mix, has_ff && L.cat_ff < 0 ? s->ffo : nullptr, fuse_next && m->runs[r + 1].add_embed ? x0 : nullptr, N));
+    const float *ffo = has_ff && L.cat_ff < 0 ? s->ffo : nullptr, *again = fuse_next && m->runs[r + 1].add_embed ? x0 : nullptr;
+    if (L.wo_r)
+        QIE_TRY(norms(x, s->mix, s->mix2, again, N, &L, ffo));
+    else
+        QIE_TRY(norms(x, s->mix, ffo, again, N));
     *next_ready = fuse_next;
     if (s->keep_on && s->keep)
         QIE_HIP(hipMemcpyAsync(s->keep + (int64_t)r * plane, x, (size_t)T * W * 4, hipMemcpyDeviceToDevice, e->stream));
@@ -1758,6 +2046,7 @@ static int enq_forward(qie_batch* b, int T, int n_want) {
     if (n_want > 0) {
         QIE_TRY(lay::final_rows(x, s->want, s->xn, s->xn_bf, n_want, W, m->g_final, m->w_final, m->a.norm_eps, e->stream, w_one));
         QIE_TRY(dense(b, s->xn, W, m->head, s->logits, m->a.vocab, n_want, m->a.vocab, W, s->xn_bf));
+        if (m->a.logit_softcap > 0.f) QIE_TRY(lay::softcap(s->logits, (int64_t)n_want * m->a.vocab, m->a.logit_softcap, e->stream));
     }
     return 0;
 }
@@ -1772,14 +2061,14 @@ static void lb_free(LayeredBatch* s) {
     drop_graphs(s);   // captured launches hold these buffers' addresses
     void* ps[] = {s->stack, s->x, s->proj, s->qabs, s->olat, s->ov, s->mix, s->y, s->gu, s->act, s->ffo, s->xg, s->yd, s->score,
                   s->row_slot, s->row_pos, s->tok, s->sel, s->cnt, s->off, s->slot_of, s->keep, s->abf,
-                  s->x_bf, s->y_bf, s->ov_bf, s->act_bf, s->xg_bf, s->pre, s->aux, s->row_k, s->dw, s->y2, s->y2_bf};
+                  s->x_bf, s->y_bf, s->ov_bf, s->act_bf, s->xg_bf, s->pre, s->aux, s->row_k, s->dw, s->y2, s->y2_bf, s->mix2};
     for (void* p : ps)
         if (p) hipFree(p);
     s->stack = s->x = s->proj = s->qabs = s->olat = s->ov = s->mix = s->y = s->gu = s->act = s->ffo = s->xg = s->yd = s->score =
         s->keep = nullptr;
     s->abf = s->x_bf = s->y_bf = s->ov_bf = s->act_bf = s->xg_bf = nullptr;
     s->row_slot = s->row_pos = s->tok = s->sel = s->cnt = s->off = s->slot_of = s->row_k = nullptr;
-    s->pre = s->aux = s->dw = s->y2 = nullptr;
+    s->pre = s->aux = s->dw = s->y2 = s->mix2 = nullptr;
     s->y2_bf = nullptr;
     s->cap = 0;
 }
@@ -1856,6 +2145,8 @@ static int ensure_rows(qie_batch* b, int64_t T) {
         A((void**)&s->mix, cap * W);
         A((void**)&s->y, cap * W);
         if (m->a.block == QIE_BLOCK_PARALLEL) A((void**)&s->y2, cap * W);
+        for (const LayerDev& d : m->L)
+            if (d.wo_r && !s->mix2) A((void**)&s->mix2, cap * W);
         A((void**)&s->gu, cap * std::max<int64_t>(s->m_gu, 1));
         A((void**)&s->act, cap * std::max<int64_t>(s->m_act, 1));
         A((void**)&s->ffo, cap * W);
@@ -2017,6 +2308,20 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
         s->m_state = std::max<int64_t>(s->m_state, heads * dim * vdim);
         s->m_hd = std::max<int64_t>(s->m_hd, heads * dim);
     };
+    auto delta_state = [&](int r, const qie_delta_desc& c) {   // per slot the heads' states and the short convolutions' last inputs
+        const int64_t C = 2 * (int64_t)c.kv_heads * c.dim + (int64_t)c.heads * c.vdim;
+        s->state_off[r] = s->slot_state;
+        s->slot_state += (int64_t)c.heads * c.dim * c.vdim;
+        s->conv_off[r] = s->slot_state;
+        s->slot_state += (int64_t)(c.conv - 1) * C;
+        s->m_pre = std::max<int64_t>(s->m_pre, C);
+        s->m_hr = std::max<int64_t>({s->m_hr, (int64_t)c.heads * c.dim, (int64_t)c.heads * c.vdim});
+        s->m_aux = std::max<int64_t>(s->m_aux, (int64_t)c.heads * c.vdim);
+        s->m_dw = std::max<int64_t>(s->m_dw, (int64_t)c.heads * c.dim);
+        s->m_state = std::max<int64_t>(s->m_state, (int64_t)c.heads * c.dim * c.vdim);
+        s->m_hd = std::max<int64_t>(s->m_hd, (int64_t)c.heads * c.dim * c.dim);
+        s->has_scan = true;
+    };
     for (int r = 0; r < n_runs; r++) {
         const int i = m->runs[r].layer;
         const qie_layer_desc& d = m->L[i].d;
@@ -2025,20 +2330,23 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
             s->slot_state += (int64_t)(m->a.canon_taps - 1) * m->a.width;
         }
         if (d.mixer == QIE_MIXER_CHANNEL_DELTA) {
-            // no cache rows; per slot the heads' states and the short convolutions' last inputs
-            const qie_delta_desc& c = d.delta;
-            const int64_t C = 2 * (int64_t)c.kv_heads * c.dim + (int64_t)c.heads * c.vdim;
-            s->state_off[r] = s->slot_state;
-            s->slot_state += (int64_t)c.heads * c.dim * c.vdim;
-            s->conv_off[r] = s->slot_state;
-            s->slot_state += (int64_t)(c.conv - 1) * C;
+            delta_state(r, d.delta);   // no cache rows
             s->m_in = std::max<int64_t>(s->m_in, m->L[i].n_in);
-            s->m_pre = std::max<int64_t>(s->m_pre, C);
-            s->m_hr = std::max<int64_t>({s->m_hr, (int64_t)c.heads * c.dim, (int64_t)c.heads * c.vdim});
-            s->m_aux = std::max<int64_t>(s->m_aux, (int64_t)c.heads * c.vdim);
-            s->m_dw = std::max<int64_t>(s->m_dw, (int64_t)c.heads * c.dim);
-            s->m_state = std::max<int64_t>(s->m_state, (int64_t)c.heads * c.dim * c.vdim);
-            s->m_hd = std::max<int64_t>(s->m_hd, (int64_t)c.heads * c.dim * c.dim);
+            s->m_hv = std::max<int64_t>(s->m_hv, m->L[i].n_cat);
+            s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)m->L[i].n_cat});
+        } else if (d.mixer == QIE_MIXER_RGLRU) {
+            // no cache rows; per slot a state element per channel and the convolution's last inputs
+            const int64_t n = d.rglru.width;
+            s->state_off[r] = s->slot_state;
+            s->slot_state += n;
+            s->conv_off[r] = s->slot_state;
+            s->slot_state += (d.rglru.conv - 1) * n;
+            s->m_in = std::max<int64_t>(s->m_in, m->L[i].n_in);
+            s->m_pre = std::max<int64_t>(s->m_pre, n);
+            s->m_hr = std::max<int64_t>(s->m_hr, n);
+            s->m_aux = std::max<int64_t>(s->m_aux, 2 * n);
+            s->m_state = std::max<int64_t>(s->m_state, n);
+            s->m_hd = std::max<int64_t>(s->m_hd, n);
             s->m_hv = std::max<int64_t>(s->m_hv, m->L[i].n_cat);
             s->m_abf = std::max<int64_t>({s->m_abf, (int64_t)m->a.width, (int64_t)m->L[i].n_cat});
             s->has_scan = true;
@@ -2070,12 +2378,19 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
         } else if (d.mixer != QIE_MIXER_LATENT_ATTENTION) {
             // K rows, then V rows of this run; one state per slot for the recurrence
             const qie_gqa_desc& a = d.gqa;
-            s->layer_off[r] = off;
-            off += (int64_t)page_tokens * a.kv_heads * a.dim;
-            s->v_off[r] = off;
-            off += (int64_t)page_tokens * a.kv_heads * a.vdim;
-            const int64_t rv = d.mixer == QIE_MIXER_GQA_RECURRENT ? (int64_t)d.rec.heads * d.rec.vdim : 0;
-            if (rv) {
+            if (d.kv_from >= 0) {   // another layer's rows (no repeated groups with these: run == layer)
+                s->layer_off[r] = s->layer_off[d.kv_from];
+                s->v_off[r] = s->v_off[d.kv_from];
+            } else {
+                s->layer_off[r] = off;
+                off += (int64_t)page_tokens * a.kv_heads * a.dim;
+                s->v_off[r] = off;
+                off += (int64_t)page_tokens * a.kv_heads * a.vdim;
+            }
+            const int64_t rv = rec_cols(d);
+            if (rv && d.rec.kind == QIE_REC_DELTA) {
+                delta_state(r, d.delta);
+            } else if (rv) {
                 s->state_off[r] = s->slot_state;
                 s->slot_state += (int64_t)d.rec.heads * d.rec.dim * d.rec.vdim;
                 if (d.rec.kind == QIE_REC_KEY_DECAY) {
@@ -2214,6 +2529,8 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
     QIE_REQUIRE((arch->pos_embed == QIE_POS_NONE && (arch->embed_scale == 0.f || arch->embed_scale == 1.f)) ||
                     arch->block == QIE_BLOCK_PRENORM || arch->block == QIE_BLOCK_PARALLEL,
                 "qie_engine_create_layered: scaled embeddings and position vectors go with the pre-norm and parallel blocks");
+    QIE_REQUIRE(!arch->shared_norm || arch->block == QIE_BLOCK_PARALLEL, "qie_engine_create_layered: one norm for both branches goes with the parallel block");
+    QIE_REQUIRE(arch->logit_softcap >= 0.f, "qie_engine_create_layered: logit cap %g", (double)arch->logit_softcap);
     QIE_REQUIRE(arch->block == QIE_BLOCK_POSTNORM_GAIN || !arch->depth_mix,
                 "qie_engine_create_layered: depth-weighted residuals go with the post-norm block");
     const bool loops = arch->loop_times > 1 && arch->loop_stop > arch->loop_start;
@@ -2235,7 +2552,7 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
         QIE_REQUIRE(d.ff_kind != QIE_FF_MOE || (d.experts > 0 && d.top > 0 && d.top <= d.experts + std::max(d.identity, 0)),
                     "layer %d: %d of %d experts", i, d.top, d.experts + std::max(d.identity, 0));
         QIE_REQUIRE(d.router >= QIE_ROUTER_SIGMOID_IN && d.router <= QIE_ROUTER_SOFTMAX_ALL, "layer %d: router %d", i, d.router);
-        QIE_REQUIRE(d.ff_act >= QIE_ACT_SILU_GATED && d.ff_act <= QIE_ACT_CLAMPED_GATED, "layer %d: activation %d", i, d.ff_act);
+        QIE_REQUIRE(d.ff_act >= QIE_ACT_SILU_GATED && d.ff_act <= QIE_ACT_RELU_GATED, "layer %d: activation %d", i, d.ff_act);
         const bool pre = arch->block == QIE_BLOCK_PRENORM || arch->block == QIE_BLOCK_PARALLEL;
         if (d.ff_kind == QIE_FF_MOE && d.router == QIE_ROUTER_SOFTMAX_ALL) {
             const int n = d.experts + d.identity;
@@ -2245,6 +2562,18 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
                         d.groups_keep, d.top);
         } else {
             QIE_REQUIRE(d.identity == 0, "layer %d: identity experts go with the grouped softmax router", i);
+        }
+        auto delta_ok = [&](const qie_delta_desc& c) {
+            return c.heads > 0 && c.kv_heads > 0 && c.heads % c.kv_heads == 0 && c.dim > 0 && c.dim <= 512 && c.vdim > 0 && c.conv >= 1 &&
+                   c.conv <= 64 && c.rank_a >= 0 && c.rank_g >= 0 && c.decay >= QIE_DELTA_CHANNEL && c.decay <= QIE_DELTA_HEAD;
+        };
+        if (d.mixer == QIE_MIXER_RGLRU) {
+            const qie_rglru_desc& c = d.rglru;
+            QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
+            QIE_REQUIRE(c.width > 0 && c.blocks > 0 && c.width % c.blocks == 0 && c.conv >= 1 && c.conv <= 64 && c.decay > 0.f,
+                        "layer %d: linear recurrent unit of %d channels in %d blocks, %d taps, decay %g", i, c.width, c.blocks, c.conv,
+                        (double)c.decay);
+            continue;
         }
         if (d.mixer == QIE_MIXER_MINGRU) {
             QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
@@ -2263,8 +2592,7 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
         if (d.mixer == QIE_MIXER_CHANNEL_DELTA) {
             const qie_delta_desc& c = d.delta;
             QIE_REQUIRE(pre, "layer %d: this mixer is wired to the pre-norm and parallel blocks", i);
-            QIE_REQUIRE(c.heads > 0 && c.kv_heads > 0 && c.heads % c.kv_heads == 0 && c.dim > 0 && c.dim <= 512 && c.vdim > 0 &&
-                            c.conv >= 1 && c.conv <= 64 && c.rank_a >= 0 && c.rank_g >= 0,
+            QIE_REQUIRE(delta_ok(c),
                         "layer %d: delta rule with %d heads over %d key heads of %d (at most 512) / %d, %d taps", i, c.heads, c.kv_heads,
                         c.dim, c.vdim, c.conv);
             continue;
@@ -2282,7 +2610,7 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
             QIE_REQUIRE(a.q_temp_every >= 0, "layer %d: query temperature every %d", i, a.q_temp_every);
             QIE_REQUIRE(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0 && a.dim > 0 && a.vdim > 0,
                         "layer %d: %d query heads over %d key heads of %d / %d", i, a.heads, a.kv_heads, a.dim, a.vdim);
-            QIE_REQUIRE(a.qk_norm >= QIE_QKNORM_NONE && a.qk_norm <= QIE_QKNORM_PLAIN, "layer %d: q / k norm %d", i, a.qk_norm);
+            QIE_REQUIRE(a.qk_norm >= QIE_QKNORM_NONE && a.qk_norm <= QIE_QKNORM_ROW, "layer %d: q / k norm %d", i, a.qk_norm);
             QIE_REQUIRE(a.rot_dims >= 0 && a.rot_dims % 2 == 0 && a.rot_dims <= a.dim, "layer %d: rotary dims %d of %d", i, a.rot_dims,
                         a.dim);
             QIE_REQUIRE(a.rot_layout == QIE_ROT_HALVES || a.rot_layout == QIE_ROT_INTERLEAVED, "layer %d: rotary layout %d", i,
@@ -2294,10 +2622,28 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
             QIE_REQUIRE(!a.values_are_keys || (a.vdim == a.dim && !a.rot_values), "layer %d: keys as values need vdim == dim", i);
             QIE_REQUIRE(!(a.out_gate && a.head_gate), "layer %d: one output gate, per head or per coordinate", i);
             QIE_REQUIRE(!a.sink || a.weights == QIE_WEIGHTS_SOFTMAX, "layer %d: a sink goes with softmax weights", i);
-            QIE_REQUIRE(a.rot_scaling.factor == 0.f || (a.rot_scaling.factor > 0.f && a.rot_scaling.high > a.rot_scaling.low &&
+            QIE_REQUIRE(a.softcap >= 0.f, "layer %d: score cap %g", i, (double)a.softcap);
+            if (a.rot_scaling.factor != 0.f && a.rot_scaling.kind == QIE_ROT_SCALE_YARN)
+                QIE_REQUIRE(a.rot_scaling.factor > 0.f && a.rot_scaling.high > 0.f && a.rot_scaling.low > 0.f && a.rot_scaling.original > 0.f &&
+                                a.rot_base > 1.f,
+                            "layer %d: rotary scaling", i);
+            else
+                QIE_REQUIRE(a.rot_scaling.factor == 0.f || (a.rot_scaling.factor > 0.f && a.rot_scaling.high > a.rot_scaling.low &&
                                                         a.rot_scaling.low >= 0.f && a.rot_scaling.original > 0.f),
                         "layer %d: rotary scaling", i);
-            if (d.mixer == QIE_MIXER_GQA_RECURRENT)
+            if (d.kv_from >= 0) {
+                QIE_REQUIRE(d.mixer == QIE_MIXER_GQA && d.kv_from < i && !loops && !a.values_are_keys,
+                            "layer %d: kv_from %d must name an earlier layer (attention alone, no repeated group)", i, d.kv_from);
+                const qie_layer_desc& o = arch->layers[d.kv_from];
+                QIE_REQUIRE((o.mixer == QIE_MIXER_GQA || o.mixer == QIE_MIXER_GQA_RECURRENT) && o.kv_from < 0 && o.gqa.kv_heads == a.kv_heads &&
+                                o.gqa.dim == a.dim && o.gqa.vdim == a.vdim,
+                            "layer %d: the layer it reads its keys and values from (%d) must own some of the same sizes", i, d.kv_from);
+            }
+            QIE_REQUIRE(!d.mix_norm || (d.mixer == QIE_MIXER_GQA_RECURRENT && arch->block == QIE_BLOCK_PARALLEL),
+                        "layer %d: normed branches go with an attention beside a recurrence in the parallel block", i);
+            if (d.mixer == QIE_MIXER_GQA_RECURRENT && d.rec.kind == QIE_REC_DELTA)
+                QIE_REQUIRE(delta_ok(d.delta) && d.delta.decay == QIE_DELTA_HEAD, "layer %d: sizes of the delta rule beside an attention (one decay per head)", i);
+            else if (d.mixer == QIE_MIXER_GQA_RECURRENT)
                 QIE_REQUIRE(d.rec.heads > 0 && d.rec.dim > 0 && d.rec.dim <= 512 && d.rec.vdim > 0 &&
                                 (d.rec.kind == QIE_REC_LOWER_BOUND || (d.rec.kind == QIE_REC_KEY_DECAY && d.rec.tau > 0.f && d.rec.rank >= 0)),
                             "layer %d: recurrence sizes", i);
@@ -2589,10 +2935,11 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
     int rc = 0;
     const bool gqa = which != 0 && m->L[layer].d.mixer != QIE_MIXER_LATENT_ATTENTION;
     QIE_REQUIRE(which != 4 || m->L[layer].d.mixer == QIE_MIXER_GQA_RECURRENT || m->L[layer].d.mixer == QIE_MIXER_MINGRU ||
-                    m->L[layer].d.mixer == QIE_MIXER_CHANNEL_DELTA || m->L[layer].d.mixer == QIE_MIXER_STATE_SPACE,
+                    m->L[layer].d.mixer == QIE_MIXER_CHANNEL_DELTA || m->L[layer].d.mixer == QIE_MIXER_STATE_SPACE ||
+                    m->L[layer].d.mixer == QIE_MIXER_RGLRU,
                 "qie_batch_time_stage: layer %d has no recurrence", layer);
     QIE_REQUIRE(which != 1 || (m->L[layer].d.mixer != QIE_MIXER_MINGRU && m->L[layer].d.mixer != QIE_MIXER_CHANNEL_DELTA &&
-                               m->L[layer].d.mixer != QIE_MIXER_STATE_SPACE),
+                               m->L[layer].d.mixer != QIE_MIXER_STATE_SPACE && m->L[layer].d.mixer != QIE_MIXER_RGLRU),
                 "qie_batch_time_stage: layer %d has no attention", layer);
     int run = 0;   // the layer's first run
     while (which != 0 && m->runs[run].layer != layer) run++;
@@ -2602,10 +2949,11 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
             const LayerDev& L = m->L[layer];
             switch (which) {
                 case 2:
-                    QIE_TRY(enq_delta_proj(b, run, T));
+                    QIE_TRY(enq_proj(b, run, T));
+                    QIE_TRY(enq_delta_gates(b, run, T));
                     return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
                 case 3: return enq_ff(b, layer, T);
-                default: return enq_delta_scan(b, run, T, false);
+                default: return enq_delta_scan(b, run, T, false, st);
             }
         }
         if (!gqa && which != 0 && m->a.block != QIE_BLOCK_POSTNORM_GAIN) {   // latent attention on the branch input s->y
@@ -2623,11 +2971,13 @@ int qie_batch_time_stage(qie_batch* b, int32_t which, int32_t layer, int32_t ite
             switch (which) {
                 case 1: return enq_gqa_attention(b, run, T);
                 case 2:
-                    QIE_TRY(enq_gqa_proj(b, run, T));
-                    return dense(b, s->ov, L.n_cat, L.wo, s->mix, m->a.width, T, m->a.width, L.n_cat, s->ov_bf);
+                    QIE_TRY(enq_proj(b, run, T));
+                    return enq_out(b, run, T);
                 case 3: return enq_ff(b, layer, T);
                 default:
+                    if (L.d.mixer == QIE_MIXER_GQA_RECURRENT && L.d.rec.kind == QIE_REC_DELTA) return enq_delta_scan(b, run, T, false, st);
                     return L.d.mixer == QIE_MIXER_MINGRU        ? enq_mingru(b, run, T)
+                           : L.d.mixer == QIE_MIXER_RGLRU       ? enq_rglru(b, run, T)
                            : L.d.mixer == QIE_MIXER_STATE_SPACE ? enq_state_space(b, run, T)
                                                                 : enq_recurrence(b, run, T);
             }

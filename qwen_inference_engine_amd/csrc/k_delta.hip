@@ -55,6 +55,14 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepP p) {
     float* row = p.proj + t * p.ld;
     if (y == 0)
         for (int h = threadIdx.x; h < p.H; h += 256) row[p.b_col + h] = 1.0f / (1.0f + expf(-row[p.b_col + h]));
+    if (!p.a) {   // one decay per head, in place in the projection row
+        if (y == 0)
+            for (int h = threadIdx.x; h < p.H; h += 256) {
+                const float z = row[p.a_col + h] + p.dt_bias[h];
+                row[p.a_col + h] = expf(-p.exp_a[h] * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
+            }
+        return;
+    }
     float* a = p.a + t * (int64_t)p.H * p.dim;
     for (int i = y * 256 + threadIdx.x; i < p.H * p.dim; i += 256 * ny) {
         const float z = a[i] + p.dt_bias[i];
@@ -64,9 +72,9 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrepP p) {
 }
 
 int delta_prep(const DeltaPrepP& p, int T, hipStream_t st) {
-    QIE_REQUIRE(p.qkv && p.proj && p.a && p.dt_bias && p.exp_a && p.H > 0 && p.G > 0 && p.H % p.G == 0 && p.dim > 0,
+    QIE_REQUIRE(p.qkv && p.proj && p.dt_bias && p.exp_a && p.H > 0 && p.G > 0 && p.H % p.G == 0 && p.dim > 0,
                 "delta_prep: bad arguments");
-    const int ny = T <= 64 ? std::min(8, std::max(1, p.H * p.dim / 256)) : 1;
+    const int ny = T <= 64 ? std::min(8, std::max(1, p.a ? p.H * p.dim / 256 : p.G / 2)) : 1;
     hipLaunchKernelGGL(delta_prep_kernel, dim3(T, ny), dim3(256), 0, st, p);
     QIE_LAUNCH_CHECK();
     return 0;
@@ -77,14 +85,15 @@ constexpr int DS_TT = 8;    // rows staged at a time
 constexpr int DS_SEG = DS_RP + 4;   // a lane group's 32 staged values, padded by 16 bytes: the LP groups of a column read
                                     // different banks (unpadded they sit 128 bytes apart, the same banks)
 
-template <int LP>
+// HEAD: one decay per head (g[t * ld_g + h]), staged beside beta
+template <int LP, bool HEAD>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanP p) {
     extern __shared__ float sm[];
     constexpr int dimP = DS_RP * LP, dimS = DS_SEG * LP, CPB = 256 / LP;
     float* sq = sm;
     float* sk = sm + DS_TT * dimS;
     float* sg = sm + 2 * DS_TT * dimS;
-    float* sb = sm + 3 * DS_TT * dimS;
+    float* sb = sm + (HEAD ? 2 : 3) * DS_TT * dimS;   // beta, then (HEAD) the decays
     const int h = blockIdx.x, tid = threadIdx.x, rg = tid % LP, col = blockIdx.z * CPB + tid / LP;
     const int4 en = p.entries[blockIdx.y];   // {first packed row, rows, slot, first position}
     const int dim = p.dim, vdim = p.vdim, G = p.G, H = p.H;
@@ -115,19 +124,23 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanP p) {
             const int d = tt * dimS + (r / DS_RP) * DS_SEG + r % DS_RP;
             sq[d] = in ? qr[gh * dim + r] : 0.f;
             sk[d] = in ? qr[(G + gh) * dim + r] : 0.f;
-            sg[d] = in ? p.g[row * HD + (int64_t)h * dim + r] : 1.f;
+            if (!HEAD) sg[d] = in ? p.g[row * HD + (int64_t)h * dim + r] : 1.f;
         }
-        if (tid < nt) sb[tid] = p.beta[(int64_t)(en.x + t0 + tid) * p.ld_beta + h];
+        if (tid < nt) {
+            sb[tid] = p.beta[(int64_t)(en.x + t0 + tid) * p.ld_beta + h];
+            if (HEAD) sb[DS_TT + tid] = p.g[(int64_t)(en.x + t0 + tid) * p.ld_g + h];
+        }
         __syncthreads();
         for (int tt = 0; tt < nt; tt++) {
             const float* kk = sk + tt * dimS + rg * DS_SEG;
             const float* qq = sq + tt * dimS + rg * DS_SEG;
             const float* gg = sg + tt * dimS + rg * DS_SEG;
+            const float gh1 = HEAD ? sb[DS_TT + tt] : 0.f;
             // four partial sums per inner product: the adds of one sum wait for each other
             float d0 = 0.f, d1 = 0.f, d2 = 0.f, d3 = 0.f;
 #pragma unroll
             for (int i = 0; i < DS_RP; i += 4) {
-                const float4 g4 = *reinterpret_cast<const float4*>(gg + i);
+                const float4 g4 = HEAD ? make_float4(gh1, gh1, gh1, gh1) : *reinterpret_cast<const float4*>(gg + i);
                 const float4 k4 = *reinterpret_cast<const float4*>(kk + i);
                 S[i] *= g4.x; S[i + 1] *= g4.y; S[i + 2] *= g4.z; S[i + 3] *= g4.w;
                 d0 = fmaf(k4.x, S[i], d0);
@@ -187,14 +200,19 @@ int delta_scan(const DeltaScanP& p, hipStream_t st) {
     QIE_REQUIRE(!p.trans || p.w_out, "delta_scan: the transition matrices go with the rows' transformed queries");
     const int cpb = 256 / LP, ncols = p.vdim + (p.trans ? p.dim : 0);
     const dim3 grid((unsigned)p.H, (unsigned)p.n_entries, (unsigned)((ncols + cpb - 1) / cpb));
-    const size_t shm = (size_t)(3 * DS_TT * DS_SEG * LP + DS_TT) * 4;
+    const bool head = p.ld_g > 0;
+    const size_t shm = (size_t)((head ? 2 : 3) * DS_TT * DS_SEG * LP + 2 * DS_TT) * 4;
+#define QIE_DS(N)                                                                                 \
+    if (head) hipLaunchKernelGGL((delta_scan_kernel<N, true>), grid, dim3(256), shm, st, p);      \
+    else hipLaunchKernelGGL((delta_scan_kernel<N, false>), grid, dim3(256), shm, st, p)
     switch (LP) {
-        case 1: hipLaunchKernelGGL(delta_scan_kernel<1>, grid, dim3(256), shm, st, p); break;
-        case 2: hipLaunchKernelGGL(delta_scan_kernel<2>, grid, dim3(256), shm, st, p); break;
-        case 4: hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(256), shm, st, p); break;
-        case 8: hipLaunchKernelGGL(delta_scan_kernel<8>, grid, dim3(256), shm, st, p); break;
-        default: hipLaunchKernelGGL(delta_scan_kernel<16>, grid, dim3(256), shm, st, p); break;
+        case 1: QIE_DS(1); break;
+        case 2: QIE_DS(2); break;
+        case 4: QIE_DS(4); break;
+        case 8: QIE_DS(8); break;
+        default: QIE_DS(16); break;
     }
+#undef QIE_DS
     QIE_LAUNCH_CHECK();
     return 0;
 }

@@ -560,8 +560,9 @@ int depth_mix(const float* stack, int64_t stride, const float* a, int n, float* 
 // ------------------------------------------------------------------ gated activation
 // a[m, j] = silu(gu[m, j]) * gu[m, ff + j]
 // (act 1: the tanh form of gelu instead of silu, gelu(g) = g / 2 (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)));
-// act 2: g sigmoid(1.702 g) (u + 1) with the gate cut at limit and u clamped to +-limit)
+// act 2: g sigmoid(1.702 g) (u + 1) with the gate cut at limit and u clamped to +-limit; act 3: max(g, 0) u)
 __device__ __forceinline__ float gated_act(float g, float u, int act, float limit) {
+    if (act == 3) return fmaxf(g, 0.f) * u;
     if (act == 2) {
         const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit);
         return gc / (1.0f + expf(-1.702f * gc)) * (uc + 1.0f);
@@ -571,11 +572,11 @@ __device__ __forceinline__ float gated_act(float g, float u, int act, float limi
 // V consecutive columns per thread (V = 4: ff and ld_a multiples of 4)
 template <int V>
 __global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a, uint16_t* a_bf, int ff, uint32_t n, int act, float limit,
-                                                       int64_t ld_a) {
+                                                       int64_t ld_a, int64_t ld_gu) {
     const uint32_t i = blockIdx.x * 256u + threadIdx.x;
     if (i >= n) return;
     const uint32_t per = (uint32_t)ff / V, m = i / per, j = (i - m * per) * V;
-    const float* gp = gu + (int64_t)m * 2 * ff + j;
+    const float* gp = gu + (int64_t)m * ld_gu + j;
     float g[V], u[V], o[V];
     if constexpr (V == 4) {
         *reinterpret_cast<float4*>(g) = *reinterpret_cast<const float4*>(gp);
@@ -595,17 +596,30 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(const float* gu, float* a
         if (a_bf) a_bf[oi] = f2bf(o[0]);
     }
 }
-int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act, float limit, int64_t ld_a) {
+int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act, float limit, int64_t ld_a,
+             int64_t ld_gu) {
     if (M * ff == 0) return 0;
     if (!ld_a) ld_a = ff;
+    if (!ld_gu) ld_gu = 2 * (int64_t)ff;
     QIE_REQUIRE(M * ff < ((int64_t)1 << 32), "gated activation: %lld values in one launch", (long long)(M * ff));
-    const bool v4 = ff % 4 == 0 && ld_a % 4 == 0 && ((uintptr_t)gu & 15) == 0 && ((uintptr_t)a & 15) == 0 && ((uintptr_t)a_bf & 7) == 0;
+    const bool v4 = ff % 4 == 0 && ld_a % 4 == 0 && ld_gu % 4 == 0 && ((uintptr_t)gu & 15) == 0 && ((uintptr_t)a & 15) == 0 && ((uintptr_t)a_bf & 7) == 0;
     const int64_t n = v4 ? M * ff / 4 : M * ff;
     const dim3 grid((unsigned)((n + 255) / 256));
     if (v4)
-        hipLaunchKernelGGL(silu_mul_kernel<4>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a);
+        hipLaunchKernelGGL(silu_mul_kernel<4>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a, ld_gu);
     else
-        hipLaunchKernelGGL(silu_mul_kernel<1>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a);
+        hipLaunchKernelGGL(silu_mul_kernel<1>, grid, dim3(256), 0, st, gu, a, a_bf, ff, (uint32_t)n, act, limit, ld_a, ld_gu);
+    QIE_LAUNCH_CHECK();
+    return 0;
+}
+
+__global__ __launch_bounds__(256) void softcap_kernel(float* x, int64_t n, float c) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i < n) x[i] = c * tanhf(x[i] / c);
+}
+int softcap(float* x, int64_t n, float c, hipStream_t st) {
+    QIE_REQUIRE(x && n > 0 && c > 0.f, "softcap: bad arguments");
+    hipLaunchKernelGGL(softcap_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, x, n, c);
     QIE_LAUNCH_CHECK();
     return 0;
 }

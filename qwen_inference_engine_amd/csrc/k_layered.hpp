@@ -105,7 +105,8 @@ int latent_attention_mfma(const LatentAttnMfmaP& p, hipStream_t st);
 // pool, its block table and the page geometry).
 //
 // gqa_post: per row of the fused projection, every query and key head is RMS-normed over dim
-// (qk_norm: 0 no, 1 with the weight qn_w / kn_w, 2 without one), its first rot_dims coordinates
+// (qk_norm: 0 no, 1 with the weight qn_w / kn_w, 2 without one; 3: all query heads of the row are normed as one vector
+// with weights qn_w [heads * dim], all key heads as another with kn_w [kv_heads * dim]), its first rot_dims coordinates
 // are turned by the row's position (layout 0: i with i + rot_dims / 2; 1: 2i with 2i + 1); queries
 // go back in place, keys to the cache.  Values: v_col < 0 caches the key as projected (before its
 // norm) as the value; else W_v's columns, turned over all vdim coordinates when rot_values.
@@ -140,6 +141,7 @@ struct GqaPostP {
     // transposed values of prompt-sized steps are then written 16 tokens at a time
     const int4* groups;
     int n_groups;
+    int q_only;               // the layer reads another layer's keys and values: no key or value columns, nothing cached
 };
 int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st);
 
@@ -178,11 +180,12 @@ struct GqaAttnP {
     int gate_elem;            // with gate_col: one gate per coordinate, proj[t * ld + gate_col + h * vdim + c]
     const float* sink;        // [heads] or null: exp(sink[h]) joins the softmax denominator (no key, no value)
     int mask_keep;            // mask 1 only, else 0
+    float softcap;            // > 0: the scaled score s becomes softcap * tanh(s / softcap) before biases
 };
 int gqa_attention(const GqaAttnP& p, bool cache_f32, int T, hipStream_t st);
 // The matrix-core form for bf16 caches whose V rows are stored transposed (v_transposed: inside a
 // page [kv_heads][vdim][page_tokens], so that 4 keys of one value coordinate are one 8-byte load;
-// page_tokens a multiple of 32), dim a multiple of 32 and vdim of 16, both up to 256.  A wave takes
+// page_tokens a multiple of 32), dim and vdim 32, 64, 96, 128, 192 or 256.  A wave takes
 // up to 16 (token, head) columns of one slot that share a key head: 16 consecutive tokens of one
 // head, or - for groups of few tokens, see pack - the heads of one key head per token.  groups: {first
 // packed row, tokens (<= 16), slot, first position}.  S > 1 splits every wave's keys S ways
@@ -299,7 +302,7 @@ int head_norm_rows(const float* o, const float* o2, const float* w, float eps, f
 // root mean square and multiplied by w[c] (with its bf16 image)
 int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* w, float eps, int n, int parts, int T, float* out,
                      uint16_t* out_bf, int64_t ld_out, hipStream_t st);
-// Rows of W, two norms of one row: x = xin + v (when v) + v2 (when v2) + add (when add); h1 = rms(x) w1, h2 = rms(x) w2
+// Rows of W, two norms of one row: x = xin + v (when v) + v2 (when v2) + v3 (when v3) + add (when add); h1 = rms(x) w1, h2 = rms(x) w2
 // (each fp32, as its bf16 image, or both; null w1: neither norm is made, null w2: only the first)
 struct NormPairP {
     float* x;
@@ -309,6 +312,10 @@ struct NormPairP {
     uint16_t *h1_bf, *h2_bf;
     int T, W;
     float eps;
+    const float* v3;
+    // both set (then v and v2 are too): v and v2 are RMS-normed with these weights and scaled before they are added
+    const float *v_w, *v2_w;
+    float v_scale, v2_scale;
 };
 int norm_pair(const NormPairP& p, hipStream_t st);
 // (head_norm_rows, gated_norm_parts, silu_mul: with a null fp32 output only the bf16 image is written)
@@ -359,6 +366,7 @@ struct CausalConvP {
     const int4* entries;
     int n_entries;
     const float* bias;    // [C] or null
+    const float* in_bias; // [C] or null: added to every input of the sequence (`in` and the state hold inputs without it)
 };
 int causal_conv(const CausalConvP& p, int T, hipStream_t st);
 int causal_conv_state(const CausalConvP& p, hipStream_t st);
@@ -373,6 +381,7 @@ int rms_rows(const float* in, int64_t ld_in, int col, int n, const float* w, flo
 // qkv [T][ld_qkv]: q (G heads of dim), k (G x dim), v (H x vdim) after their convolutions.  delta_prep,
 // in place: q and k heads to unit length (x / sqrt(sum x^2 + 1e-6)), q also times dim^(-1/2);
 // proj[t, b_col + h] = sigmoid of itself; a [T][H * dim] = exp(-exp_a[h] * softplus(a + dt_bias)).
+// a null: one decay per head, proj[t, a_col + h] = exp(-exp_a[h] * softplus(itself + dt_bias[h])).
 struct DeltaPrepP {
     float* qkv;
     int64_t ld_qkv;
@@ -383,6 +392,7 @@ struct DeltaPrepP {
     const float* dt_bias;   // [H * dim]
     const float* exp_a;     // [H]: exp(A_log)
     int H, G, dim, vdim;
+    int a_col;
 };
 int delta_prep(const DeltaPrepP& p, int T, hipStream_t st);
 // Per entry {first packed row, rows, slot, first position} and head h (key head h / (H / G)), the fp32
@@ -394,7 +404,8 @@ struct DeltaScanP {
     int64_t ld_qkv;
     const float* beta;      // beta[t * ld_beta + h]
     int64_t ld_beta;
-    const float* g;         // [T][H * dim]
+    const float* g;         // [T][H * dim]; with ld_g > 0 one decay per head: g[t * ld_g + h]
+    int64_t ld_g;
     const int4* entries;
     int n_entries;
     int H, G, dim, vdim;
@@ -488,6 +499,44 @@ struct LinRecCarryP {
     int64_t slot_stride, state_off;
 };
 int linrec_carry(const LinRecCarryP& p, hipStream_t st);
+// ------------------------------------------------------------------ real-gated linear recurrent unit (k_rglru.hip)
+// u [T][ld_u]: the convolved input, n = blocks * bs channels.  Gates of channel c of block b: r = sigmoid(R_b[c] . u_b +
+// r_b[c]), i likewise; log a = -decay[c] * r, S_t = a S_(t-1) + sqrt(1 - a^2) i u.  w: [blocks][2 bs][bs], a block's R rows
+// then its I rows, bf16 words or fp32 (w_f32).  All products and sums are fp32 (bf16 weights enter exactly, u as the sum
+// of three bf16 parts that hold its 24 bits).
+struct RgLruP {
+    const float* u;
+    int64_t ld_u;
+    const void* w;
+    int w_f32;
+    const float *r_b, *i_b, *decay;   // [n]; decay = the design's constant * softplus(lam)
+    int blocks, bs;
+    float *a, *b;                     // [T][n]: a and sqrt(1 - a^2) i u (rglru_gates writes them, rglru_scan reads them)
+    float* z;                         // rglru_gates: scratch [T][2 n] where the matrix-core form does not take the shape
+    // the recurrence
+    const float* y;                   // [T][ld_y]: the other branch before its bias and gelu
+    int64_t ld_y;
+    const float* y_b;                 // [n]
+    const int32_t *row_slot, *row_pos, *row_k;
+    const int4* entries;              // as in MinGruScanP
+    int n_entries;
+    const float* init;
+    int64_t init_stride, init_off;
+    int init_if_pos;
+    float *end, *decay_out;
+    int64_t end_stride, end_off;
+    float* out;                       // [T][ld_out] S * gelu_tanh(y + y_b); null: only the bf16 image
+    uint16_t* out_bf;
+    int64_t ld_out;
+    int want_out;                     // 0: only end and decay_out
+};
+int rglru_gates(const RgLruP& p, int T, hipStream_t st);
+bool rglru_gates_mfma_fits(int bs, bool w_f32);
+int rglru_scan(const RgLruP& p, hipStream_t st);
+// Steps of few rows: gates and recurrence in one launch (state at init = end), a wave per channel
+constexpr int kRgLruStepRows = 64;
+int rglru_step(const RgLruP& p, int T, hipStream_t st);
+
 // out[t, c] = log(sigmoid(z)) / tau, z = sum_r w[c * rank + r] in[t * ld_in + r] + bias[c]; c < n
 int low_rank_log_sigmoid(const float* in, int64_t ld_in, int rank, const void* w, bool w_f32, const float* bias, float tau, int n, int T,
                          float* out, hipStream_t st);
@@ -513,9 +562,11 @@ int final_rows(const float* x, const int32_t* rows, float* out, uint16_t* out_bf
                float eps, hipStream_t st, float w_one = 1.0f);
 int depth_mix(const float* stack, int64_t stride, const float* a, int n, float* x, uint16_t* x_bf, int64_t count, hipStream_t st);
 // a[m * ld_a + j] = act(gu[m, j]) * gu[m, ff + j]; act 0: silu, 1: the tanh form of gelu, 2: g sigmoid(1.702 g) (u + 1)
-// with g = min(gu[m, j], limit), u = gu[m, ff + j] clamped to +-limit; ld_a 0: ff
+// with g = min(gu[m, j], limit), u = gu[m, ff + j] clamped to +-limit, 3: relu; ld_a 0: ff; ld_gu (rows of gu) 0: 2 ff
 int silu_mul(const float* gu, float* a, uint16_t* a_bf, int64_t M, int ff, hipStream_t st, int act = 0, float limit = 0.f,
-             int64_t ld_a = 0);
+             int64_t ld_a = 0, int64_t ld_gu = 0);
+// x = c tanh(x / c) in place, n elements
+int softcap(float* x, int64_t n, float c, hipStream_t st);
 // a = ap u^2 + u / 2 where u > 0, else aq (exp(u) - 1 - u) + u / 2; n elements
 int xielu(const float* u, float* a, uint16_t* a_bf, int64_t n, float ap, float aq, hipStream_t st);
 // mode 0: score = sigmoid(z) of the `top` largest z = W_r y; mode 1: z = W_r y + bias, score = the

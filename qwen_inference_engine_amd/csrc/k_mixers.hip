@@ -8,12 +8,13 @@
 //                        and / or a linear one with a slope per head; softmax weights (optionally with a
 //                        sink: one more term exp(sink_h) in the denominator, no key, no value), or sigmoid
 //                        weights with a bias per head; an optional sigmoid gate per head or per coordinate;
-//                        bias vectors on q, k and v (gqa_post); a window that keeps the first tokens visible
+//                        bias vectors on q, k and v (gqa_post); a window that keeps the first tokens visible; soft-capped
+//                        scores; q and k normed as whole rows; keys and values of another layer
 //   lay::gated_scan      gated linear recurrence with an fp32 state per slot and head
 //   lay::mingru_scan     minGRU: a recurrence per channel, update gate and candidate from the current input alone
 //   lay::head_norm_rows  per-head RMS norm with a weight
 //   lay::gated_norm_parts   silu gate, then an RMS norm in equal parts
-//   lay::norm_pair       residual add of parallel branches fused with two norms of the result
+//   lay::norm_pair       residual add of parallel branches (optionally normed first) fused with two norms of the result
 //   lay::add_norm        residual add of a normed branch fused with the next branch's input norm
 //
 // Scores, softmax statistics, norms, gates and the recurrent state are fp32; cache rows are
@@ -94,9 +95,12 @@ __device__ __forceinline__ void wave_lds_fence() {
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-template <typename TC>
-__global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p, int values) {
+// NT threads; ROW: the query heads (and the key heads) of a row are normed as one vector, so the row's sums come first
+// and one block takes the whole row.
+template <typename TC, int NT, bool ROW>
+__global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
     extern __shared__ float sm[];
+    constexpr int NW = NT / 64;
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int slot = p.row_slot[t], pos = p.row_pos[t];
     const int mx = max(p.dim, p.vdim);
@@ -114,20 +118,47 @@ __global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p, int values) {
     };
     const float* cs = p.rope_cos + (int64_t)pos * (p.rot_dims / 2);
     const float* sn = p.rope_sin + (int64_t)pos * (p.rot_dims / 2);
-    const int n_task = H + G + (values ? G : 0);
+    const int n_task = p.q_only ? H : H + G + (values ? G : 0);
+    float row_inv[2] = {1.f, 1.f};   // of the queries, of the keys
+    if constexpr (ROW) {
+        __shared__ float red[2 * NW];
+        float sq = 0.f, sk = 0.f;
+        for (int i = threadIdx.x; i < H * dim; i += NT) {
+            const float a = row[p.q_col + i] + (p.q_bias ? p.q_bias[i] : 0.f);
+            sq += a * a;
+        }
+        for (int i = threadIdx.x; i < (p.q_only ? 0 : G * dim); i += NT) {
+            const float a = row[p.k_col + i] + (p.k_bias ? p.k_bias[i] : 0.f);
+            sk += a * a;
+        }
+        sq = wsum(sq);
+        sk = wsum(sk);
+        if (lane == 0) {
+            red[wave] = sq;
+            red[NW + wave] = sk;
+        }
+        __syncthreads();   // also: every query has been read before the first one is written back
+        sq = sk = 0.f;
+        for (int w = 0; w < NW; w++) {
+            sq += red[w];
+            sk += red[NW + w];
+        }
+        row_inv[0] = 1.0f / sqrtf(sq / (float)(H * dim) + p.eps);
+        row_inv[1] = 1.0f / sqrtf(sk / (float)(G * dim) + p.eps);
+    }
     // the next head's coordinates are on their way while this head is turned (up to 64 * NP of them)
     constexpr int NP = 4;
-    const int step = 4 * gridDim.y;
+    const int step = NW * gridDim.y;
     auto head_at = [&](int hh) { return hh < H ? p.q_col + hh * dim : p.k_col + (hh - H) * dim; };
     float nx[NP];
     auto prefetch = [&](int hh) {
-        const bool on = hh < H + G;
+        const bool on = hh < (p.q_only ? H : H + G);
         const float* x = row + (on ? head_at(hh) : 0);
 #pragma unroll
         for (int k = 0; k < NP; k++) nx[k] = on && lane + 64 * k < dim ? x[lane + 64 * k] : 0.f;
     };
-    prefetch(blockIdx.y * 4 + wave);
-    for (int hh = blockIdx.y * 4 + wave; hh < n_task; hh += step) {
+    prefetch(blockIdx.y * NW + wave);
+    for (int hh = blockIdx.y * NW + wave; hh < n_task; hh += step) {
         if (hh >= H + G) {
             const int g = hh - H - G;
             const float* vb = p.v_bias ? p.v_bias + g * vdim : nullptr;
@@ -169,7 +200,11 @@ __global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p, int values) {
         }
         if (!is_q && p.v_col < 0)   // the value is the key as projected
             for (int i = lane; i < dim; i += 64) stc<TC>(vbase, vidx(hh - H, i), buf[i]);
-        if (p.qk_norm) {
+        if (ROW) {
+            const float inv = row_inv[is_q ? 0 : 1];
+            const float* w = is_q ? p.qn_w + hh * dim : p.kn_w + (hh - H) * dim;
+            for (int i = lane; i < dim; i += 64) buf[i] = buf[i] * inv * w[i];
+        } else if (p.qk_norm) {
             ss = wsum(ss);
             const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
             const float* w = p.qk_norm == 1 ? (is_q ? p.qn_w : p.kn_w) : nullptr;
@@ -215,15 +250,28 @@ int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st) {
     QIE_REQUIRE(p.rot_dims % 2 == 0 && p.rot_dims <= p.dim, "gqa_post: rotary dims %d must be even and <= %d", p.rot_dims, p.dim);
     QIE_REQUIRE(!p.rot_values || p.vdim % 2 == 0, "gqa_post: turned values need an even vdim (%d)", p.vdim);
     QIE_REQUIRE(p.v_col >= 0 || p.vdim == p.dim, "gqa_post: keys as values need vdim == dim");
-    const size_t shm = (size_t)4 * std::max(p.dim, p.vdim) * 4;
-    QIE_REQUIRE(shm <= 48 * 1024, "gqa_post: head size %d above the kernel's staging", std::max(p.dim, p.vdim));
-    const bool apart = p.groups && p.v_col >= 0 && p.v_transposed && !p.rot_values && !cache_f32 && T > 64 && p.vdim <= 512;
+    const bool row = p.qk_norm == 3;
+    QIE_REQUIRE(!p.q_only || p.v_col >= 0, "gqa_post: a layer that reads another layer's keys caches nothing");
+    QIE_REQUIRE(!row || (p.qn_w && (p.q_only || p.kn_w)), "gqa_post: the row norm's weights are missing");
+    const int nt = row && T <= 64 ? 1024 : 256;   // few rows: a row's heads over several blocks, or one wide block
+    const size_t shm = (size_t)(nt / 64) * std::max(p.dim, p.vdim) * 4;
+    QIE_REQUIRE((size_t)4 * std::max(p.dim, p.vdim) * 4 <= 48 * 1024, "gqa_post: head size %d above the kernel's staging",
+                std::max(p.dim, p.vdim));
+    const bool wide = nt == 1024 && shm <= 48 * 1024;
+    const bool apart = p.groups && p.v_col >= 0 && p.v_transposed && !p.rot_values && !cache_f32 && T > 64 && p.vdim <= 512 && !p.q_only;
     const int values = p.v_col >= 0 && !apart ? 1 : 0;
-    const int ny = T <= 64 ? std::min(16, (p.heads + (1 + values) * p.kv_heads + 3) / 4) : 1;   // few rows: a row's heads over several blocks
-    if (cache_f32)
-        hipLaunchKernelGGL(gqa_post_kernel<float>, dim3(T, ny), dim3(256), shm, st, p, values);
-    else
-        hipLaunchKernelGGL(gqa_post_kernel<uint16_t>, dim3(T, ny), dim3(256), shm, st, p, values);
+    const int ny = T <= 64 && !row ? std::min(16, (p.heads + (1 + values) * p.kv_heads + 3) / 4) : 1;
+    const size_t shm4 = (size_t)4 * std::max(p.dim, p.vdim) * 4;
+#define QIE_POST(TC)                                                                                             \
+    if (wide) hipLaunchKernelGGL((gqa_post_kernel<TC, 1024, true>), dim3(T), dim3(1024), shm, st, p, values);    \
+    else if (row) hipLaunchKernelGGL((gqa_post_kernel<TC, 256, true>), dim3(T), dim3(256), shm4, st, p, values); \
+    else hipLaunchKernelGGL((gqa_post_kernel<TC, 256, false>), dim3(T, ny), dim3(256), shm4, st, p, values)
+    if (cache_f32) {
+        QIE_POST(float);
+    } else {
+        QIE_POST(uint16_t);
+    }
+#undef QIE_POST
     if (apart)
         hipLaunchKernelGGL(gqa_values_kernel, dim3((unsigned)p.n_groups, (unsigned)p.kv_heads), dim3(256), (size_t)16 * (p.vdim + 1) * 4, st, p,
                            p.groups);
@@ -278,6 +326,7 @@ __global__ __launch_bounds__(256) void gqa_attention_kernel(GqaAttnP p) {
             s = wsum(s);
             if (lane == 0) {
                 s *= p.scale;
+                if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
                 if (p.r1) s -= b1 * log1pf(b2 * (float)(pos - j));
                 if (p.slopes) s -= slope * (float)(pos - j);
                 sc[jj] = sig ? 1.0f / (1.0f + expf(-(s + pbh))) : s;
@@ -514,6 +563,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
     auto block_of = [&](int i) { return i < nk0 ? i : b0 + i - nk0; };
     const float b1 = a.r1 ? a.r1[hh] : 0.f, b2 = a.r1 ? a.r2[hh] : 0.f;
     const float slope = a.slopes ? a.slopes[hh] : 0.f;
+    const float cap2 = a.softcap > 0.f ? 2.0f / a.softcap : 0.f;
     const bool sig = a.pb != nullptr;   // sigmoid weights: final as computed, no running maximum or sum
     const float pbh = sig ? a.pb[hh] : 0.f;
     const int PT = a.cache.page_tokens;
@@ -615,6 +665,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
             const int kj = key0 + 16 * (e >> 2) + 4 * g + (e & 3);
             vis[e] = valid && kj <= qpos && (kj >= lo_q || kj < a.mask_keep);
             float x = sacc[e >> 2][e & 3] * a.scale;
+            if (a.softcap > 0.f) x = a.softcap * (1.0f - 2.0f / (1.0f + __expf(x * cap2)));   // c tanh(x / c)
             if (a.r1) x -= b1 * __logf(1.0f + b2 * (float)max(qpos - kj, 0));
             x -= slope * (float)max(qpos - kj, 0);
             s[e] = vis[e] ? x : -1e30f;
@@ -722,8 +773,8 @@ __global__ __launch_bounds__(256) void gqa_attn_combine_kernel(GqaAttnMfmaP P, i
 }
 
 bool gqa_attention_mfma_fits(int dim, int vdim, int page_tokens) {
-    auto one_of = [](int x, int unit) { return x == unit || x == 2 * unit || x == 4 * unit || x == 8 * unit; };
-    return one_of(dim, 32) && one_of(vdim, 32) && page_tokens % 32 == 0;
+    auto one_of = [](int x) { return x == 32 || x == 64 || x == 96 || x == 128 || x == 192 || x == 256; };
+    return one_of(dim) && one_of(vdim) && page_tokens % 32 == 0;
 }
 
 template <int DK, int DV>
@@ -739,7 +790,9 @@ static int gqa_mfma_launch(const GqaAttnMfmaP& p, dim3 grid, hipStream_t st) {
     switch (p.a.vdim / 32) {
         case 1: gqa_mfma_launch2<DK, 2>(p, grid, st); break;
         case 2: gqa_mfma_launch2<DK, 4>(p, grid, st); break;
+        case 3: gqa_mfma_launch2<DK, 6>(p, grid, st); break;
         case 4: gqa_mfma_launch2<DK, 8>(p, grid, st); break;
+        case 6: gqa_mfma_launch2<DK, 12>(p, grid, st); break;
         default: gqa_mfma_launch2<DK, 16>(p, grid, st); break;
     }
     QIE_LAUNCH_CHECK();
@@ -758,7 +811,9 @@ int gqa_attention_mfma(const GqaAttnMfmaP& p, hipStream_t st) {
     switch (a.dim / 32) {
         case 1: return gqa_mfma_launch<1>(p, grid, st);
         case 2: return gqa_mfma_launch<2>(p, grid, st);
+        case 3: return gqa_mfma_launch<3>(p, grid, st);
         case 4: return gqa_mfma_launch<4>(p, grid, st);
+        case 6: return gqa_mfma_launch<6>(p, grid, st);
         default: return gqa_mfma_launch<8>(p, grid, st);
     }
 }
@@ -1092,11 +1147,15 @@ __device__ __forceinline__ void store_bf4(uint16_t* p, float4 v) {
     *reinterpret_cast<uint2*>(p) = make_uint2(pack2(v.x, v.y), pack2(v.z, v.w));
 }
 
-template <int NV>
+// BN: v and v2 are normed before they are added.
+__device__ __forceinline__ float sq4(float4 v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); }
+
+template <int NV, bool BN>
 __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
     __shared__ float red[4];
     const int64_t r0 = (int64_t)blockIdx.x * p.W;
-    const bool moved = p.v || p.add || p.xin != p.x;
+    const bool moved = p.v || p.v3 || p.add || p.xin != p.x;
+    float f1 = 1.f, f2 = 1.f;   // BN: the branches' factors
     float ss = 0.f;
     if constexpr (NV > 0) {
         const int n4 = p.W >> 2;
@@ -1111,6 +1170,33 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
             a[k] = p.v ? *reinterpret_cast<const float4*>(p.v + o) : zero;
             b[k] = p.v2 ? *reinterpret_cast<const float4*>(p.v2 + o) : zero;
             c[k] = p.add ? *reinterpret_cast<const float4*>(p.add + o) : zero;
+            if (p.v3) {
+                const float4 d = *reinterpret_cast<const float4*>(p.v3 + o);
+                c[k] = make_float4(c[k].x + d.x, c[k].y + d.y, c[k].z + d.z, c[k].w + d.w);
+            }
+        }
+        if constexpr (BN) {
+            float4 u1[NV], u2[NV];
+            float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+            for (int k = 0; k < NV; k++) {
+                const int i = threadIdx.x + 256 * k, j = 4 * (i < n4 ? i : 0);
+                u1[k] = *reinterpret_cast<const float4*>(p.v_w + j);
+                u2[k] = *reinterpret_cast<const float4*>(p.v2_w + j);
+                if (i < n4) {
+                    s1 += sq4(a[k]);
+                    s2 += sq4(b[k]);
+                }
+            }
+            s1 = bsum256(s1, red);
+            s2 = bsum256(s2, red);
+            f1 = p.v_scale / sqrtf(s1 / (float)p.W + p.eps);
+            f2 = p.v2_scale / sqrtf(s2 / (float)p.W + p.eps);
+#pragma unroll
+            for (int k = 0; k < NV; k++) {
+                a[k] = make_float4(a[k].x * f1 * u1[k].x, a[k].y * f1 * u1[k].y, a[k].z * f1 * u1[k].z, a[k].w * f1 * u1[k].w);
+                b[k] = make_float4(b[k].x * f2 * u2[k].x, b[k].y * f2 * u2[k].y, b[k].z * f2 * u2[k].z, b[k].w * f2 * u2[k].w);
+            }
         }
 #pragma unroll
         for (int k = 0; k < NV; k++) {
@@ -1150,9 +1236,24 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
             }
         }
     } else {
+        if constexpr (BN) {
+            float s1 = 0.f, s2 = 0.f;
+            for (int i = threadIdx.x; i < p.W; i += 256) {
+                s1 += p.v[r0 + i] * p.v[r0 + i];
+                s2 += p.v2[r0 + i] * p.v2[r0 + i];
+            }
+            s1 = bsum256(s1, red);
+            s2 = bsum256(s2, red);
+            f1 = p.v_scale / sqrtf(s1 / (float)p.W + p.eps);
+            f2 = p.v2_scale / sqrtf(s2 / (float)p.W + p.eps);
+        }
         for (int i = threadIdx.x; i < p.W; i += 256) {
             float a = p.xin[r0 + i];
-            if (p.v) a += p.v2 ? p.v[r0 + i] + p.v2[r0 + i] : p.v[r0 + i];
+            if constexpr (BN)
+                a += p.v[r0 + i] * f1 * p.v_w[i] + p.v2[r0 + i] * f2 * p.v2_w[i];
+            else if (p.v)
+                a += p.v2 ? p.v[r0 + i] + p.v2[r0 + i] : p.v[r0 + i];
+            if (p.v3) a += p.v3[r0 + i];
             if (p.add) a += p.add[r0 + i];
             if (moved) p.x[r0 + i] = a;
             ss += a * a;
@@ -1174,18 +1275,24 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
     }
 }
 int norm_pair(const NormPairP& p, hipStream_t st) {
-    QIE_REQUIRE(p.x && p.xin && p.T > 0 && p.W > 0 && (!p.w1 || p.h1 || p.h1_bf) && (!p.w2 || (p.w1 && (p.h2 || p.h2_bf))) && (!p.v2 || p.v),
+    QIE_REQUIRE(p.x && p.xin && p.T > 0 && p.W > 0 && (!p.w1 || p.h1 || p.h1_bf) && (!p.w2 || (p.w1 && (p.h2 || p.h2_bf))) && (!p.v2 || p.v) &&
+                    (!p.v_w == !p.v2_w) && (!p.v_w || p.v2),
                 "norm_pair: bad arguments");
-    if (p.W % 4 == 0 && p.W <= 1024)
-        hipLaunchKernelGGL(norm_pair_kernel<1>, dim3((unsigned)p.T), dim3(256), 0, st, p);
-    else if (p.W % 4 == 0 && p.W <= 2048)
-        hipLaunchKernelGGL(norm_pair_kernel<2>, dim3((unsigned)p.T), dim3(256), 0, st, p);
-    else if (p.W % 4 == 0 && p.W <= 4096)
-        hipLaunchKernelGGL(norm_pair_kernel<4>, dim3((unsigned)p.T), dim3(256), 0, st, p);
-    else if (p.W % 4 == 0 && p.W <= 8192)
-        hipLaunchKernelGGL(norm_pair_kernel<8>, dim3((unsigned)p.T), dim3(256), 0, st, p);
-    else
-        hipLaunchKernelGGL(norm_pair_kernel<0>, dim3((unsigned)p.T), dim3(256), 0, st, p);
+#define QIE_NP(NV)                                                                                        \
+    if (p.v_w) hipLaunchKernelGGL((norm_pair_kernel<NV, true>), dim3((unsigned)p.T), dim3(256), 0, st, p); \
+    else hipLaunchKernelGGL((norm_pair_kernel<NV, false>), dim3((unsigned)p.T), dim3(256), 0, st, p)
+    if (p.W % 4 == 0 && p.W <= 1024) {
+        QIE_NP(1);
+    } else if (p.W % 4 == 0 && p.W <= 2048) {
+        QIE_NP(2);
+    } else if (p.W % 4 == 0 && p.W <= 4096) {
+        QIE_NP(4);
+    } else if (p.W % 4 == 0 && p.W <= 8192) {
+        QIE_NP(8);
+    } else {
+        QIE_NP(0);
+    }
+#undef QIE_NP
     QIE_LAUNCH_CHECK();
     return 0;
 }

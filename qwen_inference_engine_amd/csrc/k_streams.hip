@@ -149,7 +149,8 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(CausalConvP p, int T) 
     const int slot = p.row_slot[t], pos = p.row_pos[t], k = p.row_k[t];
     const float* w = p.w + (int64_t)c * p.taps;
     const float* sb = p.state + (int64_t)slot * p.slot_stride + p.state_off;
-    const float cur = p.in[(int64_t)t * p.ld_in + p.col + c];
+    const float ib = p.in_bias ? p.in_bias[c] : 0.f;
+    const float cur = p.in[(int64_t)t * p.ld_in + p.col + c] + ib;
     float a = p.bias ? p.bias[c] : 0.f;
     for (int j = 0; j < p.taps; j++) {
         const int back = p.taps - 1 - j;
@@ -157,9 +158,9 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(CausalConvP p, int T) 
         if (back == 0)
             x = cur;
         else if (back <= k)
-            x = p.in[(int64_t)(t - back) * p.ld_in + p.col + c];
+            x = p.in[(int64_t)(t - back) * p.ld_in + p.col + c] + ib;
         else if (pos - back >= 0)
-            x = sb[(int64_t)(k - back + p.taps - 1) * p.C + c];
+            x = sb[(int64_t)(k - back + p.taps - 1) * p.C + c] + ib;
         else
             x = 0.f;
         a = fmaf(w[j], x, a);
@@ -183,6 +184,11 @@ __global__ __launch_bounds__(256) void causal_conv_rows_kernel(CausalConvP p, in
     for (int j = 0; j < TAPS; j++) w[j] = p.w[(int64_t)c * TAPS + j];
 #pragma unroll
     for (int i = 0; i < CR; i++) in[i] = p.in[(int64_t)min(t0 + i, T - 1) * p.ld_in + p.col + c];
+    if (p.in_bias) {
+        const float ib = p.in_bias[c];
+#pragma unroll
+        for (int i = 0; i < CR; i++) in[i] += ib;
+    }
     const float b = p.bias ? p.bias[c] : 0.f;
 #pragma unroll
     for (int i = 0; i < CR; i++) {
@@ -192,11 +198,12 @@ __global__ __launch_bounds__(256) void causal_conv_rows_kernel(CausalConvP p, in
         if (i == 0 || k == 0) {
             const int slot = p.row_slot[t], pos = p.row_pos[t];
             const float* sb = p.state + (int64_t)slot * p.slot_stride + p.state_off;
+            const float ib = p.in_bias ? p.in_bias[c] : 0.f;
 #pragma unroll
             for (int j = 0; j < TAPS - 1; j++) {
                 const int back = TAPS - 1 - j;
-                x[j] = back <= k ? p.in[(int64_t)(t - back) * p.ld_in + p.col + c]
-                                 : pos - back >= 0 ? sb[(int64_t)(k - back + TAPS - 1) * p.C + c] : 0.f;
+                x[j] = back <= k ? p.in[(int64_t)(t - back) * p.ld_in + p.col + c] + ib
+                                 : pos - back >= 0 ? sb[(int64_t)(k - back + TAPS - 1) * p.C + c] + ib : 0.f;
             }
         } else {
 #pragma unroll
@@ -245,9 +252,10 @@ __global__ __launch_bounds__(256) void causal_conv_fused_kernel(CausalConvP p) {
     const int4 en = p.entries[blockIdx.y];   // {first packed row, rows, slot, first position}
     float* sb = p.state + (int64_t)en.z * p.slot_stride + p.state_off;
     const float* w = p.w + (int64_t)c * p.taps;
+    const float ib = p.in_bias ? p.in_bias[c] : 0.f;
     for (int k = 0; k < en.y; k++) {
         const int t = en.x + k, pos = en.w + k;
-        const float cur = p.in[(int64_t)t * p.ld_in + p.col + c];
+        const float cur = p.in[(int64_t)t * p.ld_in + p.col + c] + ib;
         float a = p.bias ? p.bias[c] : 0.f;
         for (int j = 0; j < p.taps; j++) {
             const int back = p.taps - 1 - j;
@@ -255,9 +263,9 @@ __global__ __launch_bounds__(256) void causal_conv_fused_kernel(CausalConvP p) {
             if (back == 0)
                 x = cur;
             else if (back <= k)
-                x = p.in[(int64_t)(t - back) * p.ld_in + p.col + c];
+                x = p.in[(int64_t)(t - back) * p.ld_in + p.col + c] + ib;
             else if (pos - back >= 0)
-                x = sb[(int64_t)(k - back + p.taps - 1) * p.C + c];
+                x = sb[(int64_t)(k - back + p.taps - 1) * p.C + c] + ib;
             else
                 x = 0.f;
             a = fmaf(w[j], x, a);

@@ -199,7 +199,7 @@ class GqaAttention:
     dim: int
     vdim: int
     scale: float
-    qk_norm: str = "none"        # "none" | "weight" | "plain"
+    qk_norm: str = "none"        # "none" | "weight" | "plain" (per head) | "row" (all heads at once, weights of that size)
     rot_dims: int = 0
     rot_base: float = 10000.0
     rot_layout: str = "halves"   # "halves" (i, i + dims/2) | "interleaved" (2i, 2i + 1)
@@ -216,9 +216,12 @@ class GqaAttention:
     qk_bias: bool = False        # bias vectors on the q and k projections
     sink: bool = False           # exp(a number per head) joins the softmax denominator
     out_gate: bool = False       # the concatenated head outputs times sigmoid(W_g x), element by element
-    rot_scaling: Optional[Tuple[float, float, float, float]] = None   # (factor, low, high, original) wavelengths
+    rot_scaling: Optional[Tuple[float, float, float, float]] = None   # (factor, low, high, original), see rot_scaling_kind
+    rot_scaling_kind: str = "wavelength"   # "wavelength" | "yarn" (blend by pair index; cos and sin scaled as well)
     v_bias: bool = False         # a bias vector on the v projection
     mask_keep: int = 0           # mask "window": the keys j < mask_keep stay visible beyond the window
+    softcap: float = 0.0         # > 0: scores become softcap * tanh(score / softcap)
+    kv_from: Optional[int] = None   # the earlier layer whose cached keys and values this layer reads (no W_k, W_v)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -241,13 +244,48 @@ class KeyDecayRecurrence:
 
 
 @dataclasses.dataclass(frozen=True)
+class GatedDelta:
+    """Gated delta rule with one decay per head and a silu output gate, as a mixer or as the recurrence beside an
+    attention; short convolutions on q, k, v; a [dim, vdim] fp32 state per head and slot plus the convolutions' last
+    inputs."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int         # taps of the short convolutions
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    def tensors(self, p: str, width: int) -> "dict[str, List[int]]":
+        nk, nv = self.kv_heads * self.dim, self.heads * self.vdim
+        return {p + "q": [nk, width], p + "q.conv": [nk, self.conv], p + "k": [nk, width], p + "k.conv": [nk, self.conv],
+                p + "v": [nv, width], p + "v.conv": [nv, self.conv], p + "b": [self.heads, width], p + "A_log": [self.heads],
+                p + "norm": [self.vdim], p + "a": [self.heads, width], p + "dt_bias": [self.heads], p + "g": [nv, width],
+                p + "o": [width, nv]}
+
+
+@dataclasses.dataclass(frozen=True)
 class AttentionWithRecurrence:
-    """Mixer: a GqaAttention and a recurrence (GatedRecurrence or KeyDecayRecurrence) read the same input; their
-    results are added with fixed scales."""
+    """Mixer: a GqaAttention and a recurrence (GatedRecurrence, KeyDecayRecurrence or GatedDelta) read the same input;
+    their results are added with fixed scales (normed: each RMS-normed over the width with a weight vector first)."""
     attn: GqaAttention
     rec: object
     attn_scale: float
     rec_scale: float
+    normed: bool = False
+
+
+@dataclasses.dataclass(frozen=True)
+class RgLru:
+    """Mixer: a real-gated linear recurrent unit per channel behind a short convolution, its gates block-diagonal
+    products of the convolved input, times a gelu branch; `width` fp32 state elements per slot plus the convolution's
+    last inputs."""
+    width: int
+    blocks: int
+    conv: int             # taps of the short convolution
+    decay: float = 8.0    # log a = -decay * r * softplus(lam)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -305,7 +343,7 @@ class FeedForward:
                                  # biased logits, softmax over the chosen ones weights the output;
                                  # "softmax_all": softmax over all router outputs, chosen by score +
                                  # correction inside the best groups, renormalised, times route_scale
-    act: str = "silu_gated"      # dense: "silu_gated" | "gelu_tanh_gated" | "clamped_gated" (gate, up, down) |
+    act: str = "silu_gated"      # dense: "silu_gated" | "gelu_tanh_gated" | "clamped_gated" | "relu_gated" (gate, up, down) |
                                  # "xielu" (up, down, two numbers)
     identity: int = 0            # "softmax_all": identity experts after the `experts` real ones
     groups: int = 1
@@ -316,7 +354,8 @@ class FeedForward:
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-    mixer: object     # LatentAttention | GqaAttention | AttentionWithRecurrence | MinGru | ChannelDelta | StateSpace
+    mixer: object     # LatentAttention | GqaAttention | AttentionWithRecurrence | MinGru | ChannelDelta | GatedDelta |
+                      # StateSpace | RgLru
     mlp: Optional[FeedForward]
 
 
@@ -330,7 +369,8 @@ class LayeredSpec:
     depth_mix: bool = True
     block: str = "postnorm_gain"     # "postnorm_gain" | "sandwich" (weight-vector norms around every branch)
                                      # | "prenorm" (one plain-weight norm before every branch)
-                                     # | "parallel" (both branches of the same row, each behind its own norm)
+                                     # | "parallel" (both branches of the same row, each behind its own norm, or - with
+                                     # shared_norm - behind one)
     tied_head: bool = False
     embed_scale: float = 1.0
     pos_embed: str = "none"          # "none" | "sinusoid" (added to the scaled embedding row)
@@ -341,6 +381,8 @@ class LayeredSpec:
     canon_taps: int = 0              # >= 1: the mixer reads h + causal conv(h) over time ('l<i>.canon1' [width, taps])
     embed_norm: bool = False         # the embedding rows are normed with 'embed.norm'
     logit_scale: float = 1.0
+    shared_norm: bool = False        # "parallel": mixer and feed-forward read the same normed row
+    logit_softcap: float = 0.0       # > 0: logits become logit_softcap * tanh(logits / logit_softcap)
 
     @property
     def n_layers(self) -> int:
@@ -367,7 +409,8 @@ class LayeredSpec:
         arr = (_lib.LayerDescC * len(self.layers))()
         def gqa(g, m):
             g.heads, g.kv_heads, g.dim, g.vdim, g.scale = m.heads, m.kv_heads, m.dim, m.vdim, m.scale
-            g.qk_norm = {"none": _lib.QIE_QKNORM_NONE, "weight": _lib.QIE_QKNORM_WEIGHT, "plain": _lib.QIE_QKNORM_PLAIN}[m.qk_norm]
+            g.qk_norm = {"none": _lib.QIE_QKNORM_NONE, "weight": _lib.QIE_QKNORM_WEIGHT, "plain": _lib.QIE_QKNORM_PLAIN,
+                         "row": _lib.QIE_QKNORM_ROW}[m.qk_norm]
             g.rot_dims, g.rot_base = m.rot_dims, m.rot_base
             g.rot_layout = {"halves": _lib.QIE_ROT_HALVES, "interleaved": _lib.QIE_ROT_INTERLEAVED}[m.rot_layout]
             g.rot_values = int(m.rot_values)
@@ -378,18 +421,29 @@ class LayeredSpec:
             g.q_temp_coef, g.q_temp_every = m.q_temp_coef, m.q_temp_every
             g.qk_bias, g.sink, g.out_gate = int(m.qk_bias), int(m.sink), int(m.out_gate)
             g.v_bias, g.mask_keep = int(m.v_bias), m.mask_keep
+            g.softcap = m.softcap
             if m.rot_scaling:
                 g.rot_scaling.factor, g.rot_scaling.low, g.rot_scaling.high, g.rot_scaling.original = m.rot_scaling
+                g.rot_scaling.kind = {"wavelength": _lib.QIE_ROT_SCALE_WAVELENGTH, "yarn": _lib.QIE_ROT_SCALE_YARN}[m.rot_scaling_kind]
+
+        def delta(x, m):
+            x.heads, x.kv_heads, x.dim, x.vdim, x.conv, x.decay = m.heads, m.kv_heads, m.dim, m.vdim, m.conv, _lib.QIE_DELTA_HEAD
 
         for d, L in zip(arr, self.layers):
             m = L.mixer
+            d.kv_from = -1
             if isinstance(m, GqaAttention):
                 d.mixer = _lib.QIE_MIXER_GQA
                 gqa(d.gqa, m)
+                d.kv_from = -1 if m.kv_from is None else m.kv_from
             elif isinstance(m, AttentionWithRecurrence):
                 d.mixer = _lib.QIE_MIXER_GQA_RECURRENT
                 gqa(d.gqa, m.attn)
                 d.rec.heads, d.rec.dim, d.rec.vdim = m.rec.heads, m.rec.dim, m.rec.vdim
+                d.mix_norm = int(m.normed)
+                if isinstance(m.rec, GatedDelta):
+                    d.rec.kind = _lib.QIE_REC_DELTA
+                    delta(d.delta, m.rec)
                 if isinstance(m.rec, KeyDecayRecurrence):
                     d.rec.kind, d.rec.rank, d.rec.tau = _lib.QIE_REC_KEY_DECAY, m.rec.rank, m.rec.tau
                 d.gqa_scale, d.rec_scale = m.attn_scale, m.rec_scale
@@ -400,6 +454,12 @@ class LayeredSpec:
                 d.mixer = _lib.QIE_MIXER_CHANNEL_DELTA
                 x = d.delta
                 x.heads, x.kv_heads, x.dim, x.vdim, x.conv, x.rank_a, x.rank_g = m.heads, m.kv_heads, m.dim, m.vdim, m.conv, m.rank_a, m.rank_g
+            elif isinstance(m, GatedDelta):
+                d.mixer = _lib.QIE_MIXER_CHANNEL_DELTA
+                delta(d.delta, m)
+            elif isinstance(m, RgLru):
+                d.mixer = _lib.QIE_MIXER_RGLRU
+                d.rglru.width, d.rglru.blocks, d.rglru.conv, d.rglru.decay = m.width, m.blocks, m.conv, m.decay
             elif isinstance(m, StateSpace):
                 d.mixer = _lib.QIE_MIXER_STATE_SPACE
                 x = d.ssm
@@ -418,7 +478,8 @@ class LayeredSpec:
             elif L.mlp.kind == "dense":
                 d.ff_kind, d.ff = _lib.QIE_FF_DENSE, L.mlp.ff
                 d.ff_act = {"silu_gated": _lib.QIE_ACT_SILU_GATED, "xielu": _lib.QIE_ACT_XIELU,
-                            "gelu_tanh_gated": _lib.QIE_ACT_GELU_TANH_GATED, "clamped_gated": _lib.QIE_ACT_CLAMPED_GATED}[L.mlp.act]
+                            "gelu_tanh_gated": _lib.QIE_ACT_GELU_TANH_GATED, "clamped_gated": _lib.QIE_ACT_CLAMPED_GATED,
+                            "relu_gated": _lib.QIE_ACT_RELU_GATED}[L.mlp.act]
                 d.ff_limit = L.mlp.limit
             else:
                 d.ff_kind, d.ff, d.experts, d.top = _lib.QIE_FF_MOE, L.mlp.ff, L.mlp.experts, L.mlp.top
@@ -438,6 +499,7 @@ class LayeredSpec:
         a.layers = arr
         a.streams, a.canon_taps, a.embed_norm, a.norm_offset = self.streams, self.canon_taps, int(self.embed_norm), self.norm_offset
         a.logit_scale = self.logit_scale
+        a.shared_norm, a.logit_softcap = int(self.shared_norm), self.logit_softcap
         return a, arr
 
     def tensor_shapes(self) -> "dict[str, List[int]]":
@@ -447,11 +509,16 @@ class LayeredSpec:
         nshape = [W] if self.block in ("sandwich", "prenorm", "parallel") else []
 
         def gqa(q, m):
-            out[q + "q"], out[q + "k"] = [m.heads * m.dim, W], [m.kv_heads * m.dim, W]
-            if not m.values_are_keys:
-                out[q + "v"] = [m.kv_heads * m.vdim, W]
-            if m.qk_norm == "weight":
-                out[q + "q.norm"], out[q + "k.norm"] = [m.dim], [m.dim]
+            own = m.kv_from is None
+            out[q + "q"] = [m.heads * m.dim, W]
+            if own:
+                out[q + "k"] = [m.kv_heads * m.dim, W]
+                if not m.values_are_keys:
+                    out[q + "v"] = [m.kv_heads * m.vdim, W]
+            if m.qk_norm in ("weight", "row"):
+                out[q + "q.norm"] = [m.dim if m.qk_norm == "weight" else m.heads * m.dim]
+                if own:
+                    out[q + "k.norm"] = [m.dim if m.qk_norm == "weight" else m.kv_heads * m.dim]
             if m.dist_bias:
                 out[q + "r1"], out[q + "r2"] = [m.heads], [m.heads]
             if m.weights == "sigmoid":
@@ -459,8 +526,10 @@ class LayeredSpec:
             if m.head_gate:
                 out[q + "g"] = [m.heads, W]
             if m.qk_bias:
-                out[q + "q.b"], out[q + "k.b"] = [m.heads * m.dim], [m.kv_heads * m.dim]
-            if m.v_bias:
+                out[q + "q.b"] = [m.heads * m.dim]
+                if own:
+                    out[q + "k.b"] = [m.kv_heads * m.dim]
+            if m.v_bias and own:
                 out[q + "v.b"] = [m.kv_heads * m.vdim]
             if m.sink:
                 out[q + "sink"] = [m.heads]
@@ -479,7 +548,7 @@ class LayeredSpec:
             out[p + "norm1"] = nshape
             if sandwich:
                 out[p + "norm1b"] = nshape
-            if L.mlp is not None:
+            if L.mlp is not None and not self.shared_norm:
                 out[p + "norm2"] = nshape
                 if sandwich:
                     out[p + "norm2b"] = nshape
@@ -489,7 +558,11 @@ class LayeredSpec:
                 gqa(p + "mix.left.", m.attn)
                 r, c = p + "mix.right.", m.rec
                 nk, nv = c.heads * c.dim, c.heads * c.vdim
-                if isinstance(c, KeyDecayRecurrence):
+                if m.normed:
+                    out[p + "mix.left.out"], out[r + "out"] = [W], [W]
+                if isinstance(c, GatedDelta):
+                    out.update(c.tensors(r, W))
+                elif isinstance(c, KeyDecayRecurrence):
                     out.update({r + "q": [nk, W], r + "k": [nk, W], r + "v": [nv, W], r + "g": [nv, W], r + "norm": [c.vdim],
                                 r + "a1": [c.rank, W], r + "a2": [nk, c.rank], r + "a2.b": [nk]})
                 else:
@@ -501,6 +574,13 @@ class LayeredSpec:
                 out.update({q + "in": [m.inner + m.conv_channels + m.heads, W], q + "conv": [m.conv_channels, m.conv],
                             q + "conv.b": [m.conv_channels], q + "dt_bias": [m.heads], q + "A_log": [m.heads], q + "D": [m.heads],
                             q + "norm": [m.inner], q + "o": [W, m.inner]})
+            elif isinstance(m, GatedDelta):
+                out.update(m.tensors(p + "mix.", W))
+            elif isinstance(m, RgLru):
+                q, n, nb = p + "mix.", m.width, m.blocks
+                out.update({q + "y": [n, W], q + "y.b": [n], q + "x": [n, W], q + "x.b": [n], q + "conv": [n, m.conv], q + "conv.b": [n],
+                            q + "ra": [nb, n // nb, n // nb], q + "ra.b": [nb, n // nb], q + "ri": [nb, n // nb, n // nb],
+                            q + "ri.b": [nb, n // nb], q + "lam": [n], q + "o": [W, n]})
             elif isinstance(m, MinGru):
                 q = p + "mix."
                 out.update({q + "z": [m.width, W], q + "z.b": [m.width], q + "x": [m.width, W], q + "x.b": [m.width],
@@ -553,11 +633,12 @@ class LayeredSpec:
             m = self.layers[i].mixer
             if isinstance(m, LatentAttention):
                 n += m.kv_rank + m.rot_dim if m.kv_from is None else 0
-            elif isinstance(m, (MinGru, ChannelDelta, StateSpace)):
+            elif isinstance(m, (MinGru, ChannelDelta, GatedDelta, StateSpace, RgLru)):
                 pass
             else:
                 a = m.attn if isinstance(m, AttentionWithRecurrence) else m
-                n += a.kv_heads * (a.dim + a.vdim)
+                if a.kv_from is None:
+                    n += a.kv_heads * (a.dim + a.vdim)
         return n
 
     def state_elems(self) -> int:
@@ -567,9 +648,13 @@ class LayeredSpec:
             m = self.layers[i].mixer
             if isinstance(m, AttentionWithRecurrence):
                 n += m.rec.heads * m.rec.dim * m.rec.vdim
+                if isinstance(m.rec, GatedDelta):
+                    n += (m.rec.conv - 1) * m.rec.conv_channels
             elif isinstance(m, MinGru):
                 n += m.width
-            elif isinstance(m, ChannelDelta):
+            elif isinstance(m, RgLru):
+                n += m.width * m.conv
+            elif isinstance(m, (ChannelDelta, GatedDelta)):
                 n += m.heads * m.dim * m.vdim + (m.conv - 1) * m.conv_channels
             elif isinstance(m, StateSpace):
                 n += m.heads * m.state * m.vdim + (m.conv - 1) * m.conv_channels
@@ -590,6 +675,15 @@ class LayeredSpec:
                 if L.mlp is not None:
                     f += 2.0 * rows * 3 * W * L.mlp.ff
                 continue
+            if isinstance(m, GatedDelta):
+                nv = m.heads * m.vdim
+                f += 2.0 * rows * W * (m.conv_channels + 2 * m.heads + 2 * nv) + 2.0 * rows * m.heads * m.dim * m.vdim * 3
+                f += 2.0 * rows * 3 * W * L.mlp.ff if L.mlp is not None else 0.0
+                continue
+            if isinstance(m, RgLru):
+                f += 2.0 * rows * W * 3 * m.width + 2.0 * rows * 2 * m.width * (m.width // m.blocks)
+                f += 2.0 * rows * 3 * W * L.mlp.ff if L.mlp is not None else 0.0
+                continue
             if isinstance(m, StateSpace):
                 f += 2.0 * rows * W * (2 * m.inner + m.conv_channels + m.heads) + 2.0 * rows * m.heads * m.state * m.vdim * 2
                 f += 2.0 * rows * 3 * W * L.mlp.ff if L.mlp is not None else 0.0
@@ -601,14 +695,18 @@ class LayeredSpec:
                 continue
             if not isinstance(m, LatentAttention):
                 a = m.attn if isinstance(m, AttentionWithRecurrence) else m
-                n_in = a.heads * a.dim + a.kv_heads * (a.dim + (0 if a.values_are_keys else a.vdim)) + (a.heads if a.head_gate else 0) \
+                n_in = a.heads * a.dim + (a.heads if a.head_gate else 0) \
+                    + (a.kv_heads * (a.dim + (0 if a.values_are_keys else a.vdim)) if a.kv_from is None else 0) \
                     + (a.heads * a.vdim if a.out_gate else 0)
                 n_cat = a.heads * a.vdim
                 keys = ctx if a.mask == "causal" else min(ctx, a.mask_size + a.mask_keep if a.mask == "window" else (a.mask_size + 1) // 2)
                 f += 2.0 * rows * a.heads * keys * (a.dim + a.vdim)
                 if isinstance(m, AttentionWithRecurrence):
                     c = m.rec
-                    n_in += c.heads * (2 * c.dim + c.vdim)
+                    n_in += c.conv_channels + 2 * c.heads if isinstance(c, GatedDelta) else c.heads * (2 * c.dim + c.vdim)
+                    if isinstance(c, GatedDelta):
+                        n_in += c.heads * c.vdim
+                        f += 2.0 * rows * c.heads * c.dim * c.vdim
                     if isinstance(c, KeyDecayRecurrence):
                         n_in += c.heads * c.vdim + c.rank
                         f += 2.0 * rows * c.rank * c.heads * c.dim
@@ -838,8 +936,65 @@ def _sefelorn_from_config(cfg: dict, name: str) -> LayeredSpec:
                        logit_scale=float(cfg.get("logit_scale", 1.0)))
 
 
+def _nukizen_from_config(cfg: dict, name: str) -> LayeredSpec:
+    """Nukizen: blocks whose mixer and feed-forward read one normed row; untied head with soft-capped logits.  Mixers: a
+    real-gated linear recurrent unit behind a short convolution; a block-local grouped-query attention (partial
+    rotate-half rotary, soft-capped scores, a sigmoid gate per head), optionally reading an earlier layer's keys and
+    values; a block-local attention (q and k normed as whole rows, YaRN-scaled rotary, a softmax sink) beside a gated
+    delta rule, each normed over the width before the two are averaged.  Feed-forward: dense, gated ReLU, or none."""
+    eps, layers = float(cfg["norm"]["eps"]), []
+
+    def yarn(rot):
+        sc = rot.get("scaling")
+        if not sc:
+            return None
+        t = (float(sc["factor"]), float(sc["slow"]), float(sc["fast"]), float(sc["original"]))
+        if not (min(t) > 0 and float(rot["base"]) > 1):
+            raise ValueError(f"rotary scaling {sc}: factor, slow, fast and original must be positive, the base above 1")
+        return t
+
+    def attention(m, **kw):
+        rot = m.get("rot") or {}
+        return GqaAttention(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                            scale=float(m["scale"]), rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)),
+                            rot_layout="halves", rot_scaling=yarn(rot), rot_scaling_kind="yarn", mask="chunk",
+                            mask_size=int(m["mask"]["size"]), softcap=float(m.get("softcap") or 0.0), **kw)
+
+    for i, L in enumerate(cfg["layers"]):
+        m = L["mixer"]
+        if L["type"] == "rglru":
+            mixer = RgLru(width=int(m["width"]), blocks=int(m["blocks"]), conv=int(m["conv"]))
+            if mixer.blocks < 1 or mixer.width % mixer.blocks:
+                raise ValueError(f"layer {i}: {mixer.width} channels in {mixer.blocks} blocks")
+        elif L["type"] == "attention":
+            src = None if m.get("kv_from") is None else int(m["kv_from"])
+            mixer = attention(m, head_gate=True, kv_from=src)
+            if src is not None:
+                o = layers[src].mixer if 0 <= src < i else None
+                o = o.attn if isinstance(o, AttentionWithRecurrence) else o
+                if not isinstance(o, GqaAttention) or o.kv_from is not None or (o.kv_heads, o.dim, o.vdim) != (mixer.kv_heads, mixer.dim, mixer.vdim):
+                    raise ValueError(f"layer {i}: kv_from {src} names no earlier attention layer with keys and values of the same sizes")
+        elif L["type"] == "parallel":
+            c = m["right"]
+            rec = GatedDelta(heads=int(c["heads"]), kv_heads=int(c["kv_heads"]), dim=int(c["dim"]), vdim=int(c["vdim"]), conv=int(c["conv"]))
+            mixer = AttentionWithRecurrence(attention(m["left"], qk_norm="row", sink=True), rec, 0.5, 0.5, normed=True)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {L['type']!r}")
+        f = L.get("mlp")
+        if f is None:
+            mlp = None
+        elif f["kind"] == "dense":
+            mlp = FeedForward("dense", int(f["ff"]), act="relu_gated")
+        else:
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+        layers.append(LayerSpec(mixer, mlp))
+    return LayeredSpec(name, int(cfg["width"]), int(cfg["vocab"]), eps, tuple(layers), depth_mix=False, block="parallel",
+                       shared_norm=True, logit_softcap=float(cfg.get("logit_softcap") or 0.0))
+
+
 ARCHITECTURES = {"Tivazen": _tivazen_from_config, "Nodutar": _nodutar_from_config, "Lugipel": _lugipel_from_config,
-                 "Verelorn": _verelorn_from_config, "Sefelorn": _sefelorn_from_config}
+                 "Verelorn": _verelorn_from_config, "Sefelorn": _sefelorn_from_config,
+                 "Nukizen": _nukizen_from_config}
 
 
 def spec_from_config(cfg: dict, name: str = "model", numerics: str = "hf"):
