@@ -211,7 +211,8 @@ def forward(cfg, W, tokens, layers_out=None):
             y = attend(m, W, p, h, kept[i if j is None else int(j)], eps, head_gate=True)
         elif L["type"] == "parallel":
             pl, pr = p + "left.", p + "right."
-            left = attend(m["left"], W, pl, h, keys_values(m["left"], W, pl, h, eps, True), eps, row_norm=True, sink=True)
+            kept[i] = keys_values(m["left"], W, pl, h, eps, True)
+            left = attend(m["left"], W, pl, h, kept[i], eps, row_norm=True, sink=True)
             y = joined(left, delta_rule(m["right"], W, pr, h, eps), W[pl + "out"], W[pr + "out"], eps)
         else:
             raise ValueError(L["type"])
@@ -221,3 +222,112 @@ def forward(cfg, W, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return cap(norm(x, W["final.norm"], eps) @ f64(W["head"]).T, cfg.get("logit_softcap"))
+
+
+# ---------------------------------------------------------------- small configurations and random weights
+def dense(ff=40):
+    return {"kind": "dense", "ff": ff}
+
+
+def _mlp(mlp):
+    return dense() if mlp == "dense" else mlp
+
+
+def lru(width=36, blocks=3, conv=4, mlp="dense"):
+    return {"type": "rglru", "mixer": {"width": width, "blocks": blocks, "conv": conv}, "mlp": _mlp(mlp)}
+
+
+def _attention(heads, kv_heads, dim, vdim, size, rot_dims, base, scale, scaling):
+    a = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": size},
+         "scale": scale if scale is not None else dim ** -0.5}
+    if rot_dims:
+        a["rot"] = {"base": base, "dims": rot_dims}
+        if scaling:
+            a["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    return a
+
+
+def att(heads=4, kv_heads=2, dim=16, vdim=12, size=11, rot_dims=8, base=10000.0, scale=None, scaling=None, softcap=9.0, kv_from=None,
+        mlp="dense"):
+    m = _attention(heads, kv_heads, dim, vdim, size, rot_dims, base, scale, scaling)
+    if softcap:
+        m["softcap"] = softcap
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": _mlp(mlp)}
+
+
+YARN = (5.0, 24, 3.0, 0.4)   # factor, original length, fast and slow turns
+
+
+def par(heads=4, kv_heads=2, dim=16, vdim=12, size=13, rot_dims=16, base=500.0, scale=None, scaling=YARN, d_heads=4, d_kv_heads=2, d_dim=10,
+        d_vdim=14, conv=3, mlp="dense"):
+    return {"type": "parallel", "mlp": _mlp(mlp), "mixer": {
+        "left": _attention(heads, kv_heads, dim, vdim, size, rot_dims, base, scale, scaling),
+        "right": {"heads": d_heads, "kv_heads": d_kv_heads, "dim": d_dim, "vdim": d_vdim, "conv": conv}}}
+
+
+def config(layers, vocab=101, width=40, eps=1e-5, logit_softcap=6.0):
+    cfg = {"architecture": "Nukizen", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+    if logit_softcap:
+        cfg["logit_softcap"] = logit_softcap
+    return cfg
+
+
+def to_bf16_exact(a):
+    """float32 values rounded to the nearest bf16 (kept as float32)."""
+    u = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
+    u = (u + 0x7FFF + ((u >> 16) & 1)) & np.uint32(0xFFFF0000)
+    return u.view(np.float32).reshape(np.shape(a))
+
+
+def random_weights(cfg, seed=0, qk_gain=2.0):
+    """{name: float32 array of exact bf16 values}.  The branches' output projections are small beside the residual rows,
+    so that a rounding error shrinks from layer to layer.  qk_gain: how sharp the softmaxes are."""
+    rng = np.random.default_rng(seed)
+    W, V, T = cfg["width"], cfg["vocab"], {}
+
+    def lin(o, i, gain=1.0):
+        return rng.normal(0.0, gain / math.sqrt(i), (o, i))
+
+    def vec(n, sd=0.2, mean=0.0):
+        return mean + rng.normal(0.0, sd, n)
+
+    def attention(x, a, own=True, row_norm=False):
+        H, G, D, Dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+        T[x + "q"], T[x + "o"] = lin(H * D, W, qk_gain), lin(W, H * Dv, 0.5)
+        if own:
+            T[x + "k"], T[x + "v"] = lin(G * D, W, qk_gain), lin(G * Dv, W)
+        if row_norm:
+            T[x + "q.norm"], T[x + "k.norm"] = vec(H * D, 0.4, qk_gain), vec(G * D, 0.4, 1.0)
+            T[x + "sink"], T[x + "out"] = vec(H, 1.0, 1.0), vec(W, 0.2, 0.9)
+
+    T["embed"], T["final.norm"], T["head"] = rng.normal(0, 1.0, (V, W)), vec(W, 0.2, 1.0), lin(V, W, 2.5)
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        T[p + "norm1"] = vec(W, 0.25, 1.0)
+        x = p + "mix."
+        if L["type"] == "rglru":
+            n, nb, bs = m["width"], m["blocks"], m["width"] // m["blocks"]
+            T[x + "y"], T[x + "y.b"], T[x + "x"], T[x + "x.b"] = lin(n, W, 1.5), vec(n, 0.5), lin(n, W), vec(n, 0.5)
+            T[x + "conv"], T[x + "conv.b"] = rng.normal(0, 0.6, (n, m["conv"])), vec(n, 0.3)
+            for g in ("ra", "ri"):
+                T[x + g] = rng.normal(0, 1.5 / math.sqrt(bs), (nb, bs, bs))
+                T[x + g + ".b"] = rng.normal(0, 0.7, (nb, bs))
+            T[x + "lam"], T[x + "o"] = vec(n, 1.0, -2.0), lin(W, n, 0.5)
+        elif L["type"] == "attention":
+            attention(x, m, own=m.get("kv_from") is None)
+            T[x + "g"] = lin(m["heads"], W, 1.5)
+        else:
+            attention(x + "left.", m["left"], row_norm=True)
+            c, x = m["right"], x + "right."
+            nk, nv, H = c["kv_heads"] * c["dim"], c["heads"] * c["vdim"], c["heads"]
+            for n, k in (("q", nk), ("k", nk), ("v", nv)):
+                T[x + n], T[x + n + ".conv"] = lin(k, W, 1.5), rng.normal(0, 0.7, (k, c["conv"]))
+            T[x + "b"], T[x + "a"], T[x + "g"] = lin(H, W, 1.5), lin(H, W), lin(nv, W)
+            T[x + "A_log"], T[x + "dt_bias"], T[x + "norm"] = vec(H, 0.7, -1.0), vec(H, 0.7, -1.0), vec(c["vdim"], 0.2, 1.0)
+            T[x + "o"], T[x + "out"] = lin(W, nv, 0.5), vec(W, 0.2, 0.9)
+        if L.get("mlp") is not None:
+            ff = L["mlp"]["ff"]
+            T[p + "mlp.gate"], T[p + "mlp.up"], T[p + "mlp.down"] = lin(ff, W, 1.5), lin(ff, W), lin(W, ff, 0.4)
+    return {k: to_bf16_exact(v) for k, v in T.items()}
