@@ -93,6 +93,15 @@ SEFELORN_SIZES = {
 }
 
 
+# Sizes of `--nukizen`: (width, attention heads, kv heads, head dim, rotated dims, block of positions, delta heads, delta key
+# heads, delta dim, delta vdim, delta taps, recurrent channels, gate blocks, taps, ff, vocab).  Four layers, each with its
+# feed-forward: linear recurrent unit, attention, attention joined with the delta rule, attention on the second layer's keys.
+NUKIZEN_SIZES = {
+    "1k": (1024, 16, 4, 64, 32, 512, 16, 8, 64, 64, 4, 1024, 4, 4, 2816, 32000),
+    "2k": (2048, 16, 4, 128, 64, 1024, 16, 8, 128, 128, 4, 2048, 8, 4, 5632, 32000),
+}
+
+
 def parse(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -147,6 +156,10 @@ def parse(argv=None):
                          "layers beside it (one JSON line of its own)")
     ap.add_argument("--sefelorn", choices=sorted(SEFELORN_SIZES), default=None,
                     help="instead of the default workload: prefill and decode throughput of a Sefelorn model at this "
+                         "size with random weights, per-stage times, and the Qwen decoder at equal width / heads / "
+                         "layers beside it (one JSON line of its own)")
+    ap.add_argument("--nukizen", choices=sorted(NUKIZEN_SIZES), default=None,
+                    help="instead of the default workload: prefill and decode throughput of a Nukizen model at this "
                          "size with random weights, per-stage times, and the Qwen decoder at equal width / heads / "
                          "layers beside it (one JSON line of its own)")
     ap.add_argument("--dry-run", action="store_true",
@@ -212,6 +225,8 @@ def main(argv=None):
         return run_verelorn(a)
     if a.sefelorn:
         return run_sefelorn(a)
+    if a.nukizen:
+        return run_nukizen(a)
     return run(a)
 
 
@@ -724,6 +739,126 @@ def run_sefelorn(a):
     b.close()
     eng.close()
     out["qwen_equal_size"] = qwen_twin(Q, S, Wt, a.sefelorn, W, H, G, hd, ff, V, P, B, steps, prompts, a.prefill_iters, max_ctx)
+    print(json.dumps(out), flush=True)
+    return 0
+
+
+def nukizen_model(S, size):
+    """(LayeredSpec, {name: bf16 words}) at one of NUKIZEN_SIZES, random weights from one pool."""
+    W, H, G, hd, rot, blk, DH, DG, dd, dv, dconv, LW, LB, lconv, ff, V = NUKIZEN_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff}
+    att = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "mask": {"size": blk}, "scale": hd ** -0.5,
+           "rot": {"base": 10000.0, "dims": rot}}
+    yarn = {"base": 50000.0, "dims": hd, "scaling": {"factor": 8.0, "original": 1024, "fast": 24.0, "slow": 2.0}}
+    layers = [{"type": "rglru", "mlp": mlp, "mixer": {"width": LW, "blocks": LB, "conv": lconv}},
+              {"type": "attention", "mlp": mlp, "mixer": dict(att, softcap=50.0)},
+              {"type": "parallel", "mlp": mlp, "mixer": {
+                  "left": dict(att, rot=yarn), "right": {"heads": DH, "kv_heads": DG, "dim": dd, "vdim": dv, "conv": dconv}}},
+              {"type": "attention", "mlp": mlp, "mixer": dict(att, softcap=50.0, kv_from=1)}]
+    cfg = {"architecture": "Nukizen", "layers": layers, "norm": {"eps": 1e-6}, "vocab": V, "width": W, "logit_softcap": 25.0}
+    spec = S.spec_from_config(cfg, name=f"nukizen-{size}")
+    pool = np.random.default_rng(0).standard_normal(1 << 22).astype(np.float32)
+    tensors = {}
+    for k, (name, shape) in enumerate(spec.tensor_shapes().items()):
+        n = int(np.prod(shape))
+        if name.endswith(("norm", "norm1", ".out")):
+            v = np.ones(shape, np.float32)
+        elif name.endswith((".b", "sink")) and not name.endswith("right.b"):
+            v = np.zeros(shape, np.float32)
+        elif name.endswith(("dt_bias", "lam")):
+            v = np.full(shape, -3.0, np.float32)
+        elif name.endswith("A_log"):
+            v = np.linspace(0.0, 2.5, n, dtype=np.float32).reshape(shape)
+        else:
+            fan = shape[-1] if name != "embed" else 1
+            v = (np.resize(np.roll(pool, 7919 * k), n) * fan ** -0.5).reshape(shape)
+        tensors[name] = (np.ascontiguousarray(v, np.float32).view(np.uint32) >> 16).astype(np.uint16).reshape(shape)
+    return spec, tensors
+
+
+def run_nukizen(a):
+    """Prefill (one step of P tokens) and decode (B single-token entries a step at context ~P) of a Nukizen model,
+    per-stage hipEvent times at both shapes, and the Qwen decoder at equal sizes."""
+    import qwen_inference_engine_amd as Q
+    from qwen_inference_engine_amd import spec as S, weights as Wt
+    W, H, G, hd, rot, blk, DH, DG, dd, dv, dconv, LW, LB, lconv, ff, V = NUKIZEN_SIZES[a.nukizen]
+    P, B, steps = a.prompt, max(a.batch, 8), min(a.steps, 128)
+    max_ctx = P + steps + 80
+    spec, tensors = nukizen_model(S, a.nukizen)
+    names = ("width", "heads", "kv_heads", "head_dim", "rot_dims", "block", "delta_heads", "delta_kv_heads", "delta_dim", "delta_vdim",
+             "delta_taps", "lru_width", "lru_blocks", "lru_taps", "ff", "vocab")
+    out = {"metric": "nukizen_decode_tokens_per_sec", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
+           "data": "synthetic (random weights, random token ids)", "higher_is_better": True,
+           "config": {"model": spec.name, "sizes": dict(zip(names, NUKIZEN_SIZES[a.nukizen])), "layers": 4, "prompt": P,
+                      "decode_batch": B, "decode_steps": steps}}
+    eng = Q.Engine(spec, max_ctx=max_ctx).load_tensors(tensors)
+    del tensors
+    b = eng.batch(B, max_ctx, page_tokens=64)
+    rng = np.random.default_rng(1)
+    prompts = rng.integers(0, V, size=(B, P), dtype=np.int32)
+    ts = []
+    for it in range(1 + a.prefill_iters):
+        t0 = time.perf_counter()
+        b.step([(0, prompts[0])], [P - 1], fetch=False)
+        ts.append(time.perf_counter() - t0)
+        if it < a.prefill_iters:
+            b.release(0)
+    t_pf = float(np.median(ts[1:]))
+    stages = {"prefill": {}, "decode": {}}
+    # stage 2 of a layer: its input product (with the feed-forward's gate and up rows) and its output product (with the
+    # activations' rows; the joined mixer: one product per branch); stage 3: the activation, in the joined layer with W_down
+    att_cols = H * hd + H + 2 * G * hd + 2 * ff + H * hd + ff
+    shared_cols = H * hd + H + 2 * ff + H * hd + ff
+    lru_cols = 2 * LW + 2 * ff + LW + ff
+    join_cols = H * hd + 2 * G * hd + 2 * DG * dd + 2 * DH * dv + 2 * DH + 2 * ff + H * hd + DH * dv
+
+    def stage_times(tag, rows, ctx):
+        st = stages[tag]
+        st["attention_us"] = round(b.time_stage(1, 1, 10), 2)
+        st["joined_attention_us"] = round(b.time_stage(1, 2, 10), 2)
+        for k, (name, cols) in enumerate((("lru", lru_cols), ("attention", att_cols), ("joined", join_cols), ("shared_kv", shared_cols))):
+            t = b.time_stage(2, k, 10)
+            st[f"{name}_products_us"] = round(t, 2)
+            st[f"{name}_products_tflops"] = round(2.0 * rows * W * cols / t / 1e6, 2)
+            if tag == "decode":
+                st[f"{name}_products_GBps"] = round(2.0 * W * cols / t / 1e3, 1)
+        st["activation_us"] = round(b.time_stage(3, 0, 10), 2)
+        st["activation_and_down_us"] = round(b.time_stage(3, 2, 10), 2)
+        st["delta_scan_us"] = round(b.time_stage(4, 2, 10), 2)
+        st["lru_scan_us"] = round(b.time_stage(4, 0, 10), 2)
+        # keys a row sees: half a block on the average of a prompt; the decoded rows sit just behind a block's edge
+        keys = blk / 2.0 if tag == "prefill" else (ctx + 8) % blk + 1
+        st["attention_keys"] = keys
+        for n in ("attention", "joined_attention"):
+            st[f"{n}_tflops"] = round(4.0 * rows * H * keys * hd / st[f"{n}_us"] / 1e6, 2)
+        # per row and head: decay of the state, two inner products and one rank-one update over dim x vdim (fp32)
+        st["delta_scan_tflops_fp32"] = round(rows * DH * dd * dv * 7.0 / st["delta_scan_us"] / 1e6, 3)
+        # the two gate products (fp32 results) and what the recurrence moves: u, a, b, the gelu branch, the bf16 result
+        st["lru_scan_gate_tflops"] = round(4.0 * rows * LW * (LW // LB) / st["lru_scan_us"] / 1e6, 3)
+        if tag == "decode":
+            st["delta_scan_state_GBps"] = round(rows * DH * dd * dv * 4 * 2 / st["delta_scan_us"] / 1e3, 1)
+            st["lru_gate_weights_GBps"] = round(2.0 * LW * (LW // LB) * 2 / st["lru_scan_us"] / 1e3, 1)
+        st["layer_stack_us"] = round(b.time_stage(0, 0, 5), 2)
+    stage_times("prefill", P, P)
+    b.release(0)
+    for s_ in range(B):
+        for c0 in range(0, P, 512):
+            b.step([(s_, prompts[s_][c0:c0 + 512])], [], fetch=False)
+    toks = rng.integers(0, V, size=(steps + 8, B), dtype=np.int32)
+    for i in range(8):
+        b.step([(s_, [toks[i][s_]]) for s_ in range(B)], range(B), fetch=False)
+    t0 = time.perf_counter()
+    for i in range(8, 8 + steps):
+        b.step([(s_, [toks[i][s_]]) for s_ in range(B)], range(B), fetch=False)
+        b.step_sample()
+    dt = time.perf_counter() - t0
+    stage_times("decode", B, P + steps)
+    out.update(value=round(B * steps / dt, 1), steps=steps, warmup=8, ms_per_step=round(dt * 1e3 / steps, 4),
+               prefill_tok_s=round(P / t_pf, 1), prefill_ms=round(t_pf * 1e3, 3),
+               prefill_tflops=round(spec.step_flops(P, P // 2) / t_pf / 1e12, 2), stages=stages, vs_baseline=None)
+    b.close()
+    eng.close()
+    out["qwen_equal_size"] = qwen_twin(Q, S, Wt, a.nukizen, W, H, G, hd, ff, V, P, B, steps, prompts, a.prefill_iters, max_ctx)
     print(json.dumps(out), flush=True)
     return 0
 
