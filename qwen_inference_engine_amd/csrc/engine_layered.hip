@@ -1679,7 +1679,7 @@ static int enq_rglru(qie_batch* b, int r, int T) {
     p.init = p.end = s->state; p.init_stride = p.end_stride = s->slot_state; p.init_off = p.end_off = s->state_off[r];
     p.init_if_pos = 1;
     p.out = ov_out(b, L); p.out_bf = s->ov_bf; p.ld_out = L.n_cat; p.want_out = 1;
-    if (s->max_count <= kLinStep && T <= lay::kRgLruStepRows) return lay::rglru_step(p, T, e->stream);
+    if (s->max_count <= kLinStep && T <= lay::kRgLruStepRows) return lay::rglru_step(p, T, kLinStep, e->stream);
     QIE_TRY(lay::rglru_gates(p, T, e->stream));
     if (s->max_count <= kScanLong || !s->s_loc) return lay::rglru_scan(p, e->stream);
     lay::RgLruP a = p;
@@ -2622,6 +2622,8 @@ int qie_engine_create_layered(const qie_arch_desc* arch, const qie_engine_opts* 
             QIE_REQUIRE(!a.values_are_keys || (a.vdim == a.dim && !a.rot_values), "layer %d: keys as values need vdim == dim", i);
             QIE_REQUIRE(!(a.out_gate && a.head_gate), "layer %d: one output gate, per head or per coordinate", i);
             QIE_REQUIRE(!a.sink || a.weights == QIE_WEIGHTS_SOFTMAX, "layer %d: a sink goes with softmax weights", i);
+            QIE_REQUIRE(a.qk_norm != QIE_QKNORM_ROW || (!a.rot_values && (int64_t)(a.heads + a.kv_heads) * a.dim <= 15 * 1024),
+                        "layer %d: q and k normed as whole rows: at most 15360 coordinates together, no turned values", i);
             QIE_REQUIRE(a.softcap >= 0.f, "layer %d: score cap %g", i, (double)a.softcap);
             if (a.rot_scaling.factor != 0.f && a.rot_scaling.kind == QIE_ROT_SCALE_YARN)
                 QIE_REQUIRE(a.rot_scaling.factor > 0.f && a.rot_scaling.high > 0.f && a.rot_scaling.low > 0.f && a.rot_scaling.original > 0.f &&

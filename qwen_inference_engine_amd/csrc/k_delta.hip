@@ -1,7 +1,8 @@
-// k_delta.hip — the gated delta rule with channel-wise decay (QIE_MIXER_CHANNEL_DELTA; k_layered.hpp):
+// k_delta.hip — the gated delta rule, decay per key channel or per head (QIE_MIXER_CHANNEL_DELTA, QIE_REC_DELTA; k_layered.hpp):
 //
 //   lay::delta_prep   per row: q and k of every key head to unit length (q also times dim^(-1/2)),
-//                     beta = sigmoid, decay g = exp(-exp(A_log) softplus(a + dt_bias)) - all fp32
+//                     beta = sigmoid, decay g = exp(-exp(A_log) softplus(a + dt_bias)), per head and key
+//                     channel or one per head - all fp32
 //   lay::delta_scan   per entry and head the state S [dim][vdim] walks the entry's rows in order:
 //                     S = diag(g) S; u = beta (v - S^T k); S += k u^T; o = S^T q
 //

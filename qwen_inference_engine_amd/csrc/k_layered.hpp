@@ -148,7 +148,7 @@ int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st);
 // Softmax attention of every (row, head) over the keys its mask lets it see (mask 0: all j <= i;
 // 1: the last mask_size and, of the earlier ones, the first mask_keep of the sequence; 2: those with
 // j / mask_size == i / mask_size); score = q.k * scale
-// - r1[h] * ln(1 + r2[h] * (i - j)) when r1 is set.  rot_values: the weighted sum is turned back
+// (soft-capped when softcap > 0) - r1[h] * ln(1 + r2[h] * (i - j)) when r1 is set.  rot_values: the weighted sum is turned back
 // by the row's position.  The result times out_scale goes to out[t * ld_out + out_col + h * vdim
 // ...] (and its bf16 image).
 struct GqaAttnP {
@@ -533,9 +533,10 @@ struct RgLruP {
 int rglru_gates(const RgLruP& p, int T, hipStream_t st);
 bool rglru_gates_mfma_fits(int bs, bool w_f32);
 int rglru_scan(const RgLruP& p, hipStream_t st);
-// Steps of few rows: gates and recurrence in one launch (state at init = end), a wave per channel
+// Steps of few rows: gates and recurrence in one launch (state at init = end), a wave per channel, a lane per row.
+// chain: no entry has more rows
 constexpr int kRgLruStepRows = 64;
-int rglru_step(const RgLruP& p, int T, hipStream_t st);
+int rglru_step(const RgLruP& p, int T, int chain, hipStream_t st);
 
 // out[t, c] = log(sigmoid(z)) / tau, z = sum_r w[c * rank + r] in[t * ld_in + r] + bias[c]; c < n
 int low_rank_log_sigmoid(const float* in, int64_t ld_in, int rank, const void* w, bool w_f32, const float* bias, float tau, int n, int T,

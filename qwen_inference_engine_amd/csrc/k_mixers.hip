@@ -95,12 +95,9 @@ __device__ __forceinline__ void wave_lds_fence() {
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-// NT threads; ROW: the query heads (and the key heads) of a row are normed as one vector, so the row's sums come first
-// and one block takes the whole row.
-template <typename TC, int NT, bool ROW>
-__global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
+template <typename TC>
+__global__ __launch_bounds__(256) void gqa_post_kernel(GqaPostP p, int values) {
     extern __shared__ float sm[];
-    constexpr int NW = NT / 64;
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int slot = p.row_slot[t], pos = p.row_pos[t];
     const int mx = max(p.dim, p.vdim);
@@ -119,36 +116,9 @@ __global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
     const float* cs = p.rope_cos + (int64_t)pos * (p.rot_dims / 2);
     const float* sn = p.rope_sin + (int64_t)pos * (p.rot_dims / 2);
     const int n_task = p.q_only ? H : H + G + (values ? G : 0);
-    float row_inv[2] = {1.f, 1.f};   // of the queries, of the keys
-    if constexpr (ROW) {
-        __shared__ float red[2 * NW];
-        float sq = 0.f, sk = 0.f;
-        for (int i = threadIdx.x; i < H * dim; i += NT) {
-            const float a = row[p.q_col + i] + (p.q_bias ? p.q_bias[i] : 0.f);
-            sq += a * a;
-        }
-        for (int i = threadIdx.x; i < (p.q_only ? 0 : G * dim); i += NT) {
-            const float a = row[p.k_col + i] + (p.k_bias ? p.k_bias[i] : 0.f);
-            sk += a * a;
-        }
-        sq = wsum(sq);
-        sk = wsum(sk);
-        if (lane == 0) {
-            red[wave] = sq;
-            red[NW + wave] = sk;
-        }
-        __syncthreads();   // also: every query has been read before the first one is written back
-        sq = sk = 0.f;
-        for (int w = 0; w < NW; w++) {
-            sq += red[w];
-            sk += red[NW + w];
-        }
-        row_inv[0] = 1.0f / sqrtf(sq / (float)(H * dim) + p.eps);
-        row_inv[1] = 1.0f / sqrtf(sk / (float)(G * dim) + p.eps);
-    }
     // the next head's coordinates are on their way while this head is turned (up to 64 * NP of them)
     constexpr int NP = 4;
-    const int step = NW * gridDim.y;
+    const int step = 4 * gridDim.y;
     auto head_at = [&](int hh) { return hh < H ? p.q_col + hh * dim : p.k_col + (hh - H) * dim; };
     float nx[NP];
     auto prefetch = [&](int hh) {
@@ -157,8 +127,8 @@ __global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
 #pragma unroll
         for (int k = 0; k < NP; k++) nx[k] = on && lane + 64 * k < dim ? x[lane + 64 * k] : 0.f;
     };
-    prefetch(blockIdx.y * NW + wave);
-    for (int hh = blockIdx.y * NW + wave; hh < n_task; hh += step) {
+    prefetch(blockIdx.y * 4 + wave);
+    for (int hh = blockIdx.y * 4 + wave; hh < n_task; hh += step) {
         if (hh >= H + G) {
             const int g = hh - H - G;
             const float* vb = p.v_bias ? p.v_bias + g * vdim : nullptr;
@@ -200,11 +170,7 @@ __global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
         }
         if (!is_q && p.v_col < 0)   // the value is the key as projected
             for (int i = lane; i < dim; i += 64) stc<TC>(vbase, vidx(hh - H, i), buf[i]);
-        if (ROW) {
-            const float inv = row_inv[is_q ? 0 : 1];
-            const float* w = is_q ? p.qn_w + hh * dim : p.kn_w + (hh - H) * dim;
-            for (int i = lane; i < dim; i += 64) buf[i] = buf[i] * inv * w[i];
-        } else if (p.qk_norm) {
+        if (p.qk_norm) {
             ss = wsum(ss);
             const float inv = 1.0f / sqrtf(ss / (float)dim + p.eps);
             const float* w = p.qk_norm == 1 ? (is_q ? p.qn_w : p.kn_w) : nullptr;
@@ -221,6 +187,92 @@ __global__ __launch_bounds__(NT) void gqa_post_kernel(GqaPostP p, int values) {
                 x[i] = o;
             else
                 stc<TC>(krow, (int64_t)(hh - H) * dim + i, o);
+        }
+    }
+}
+
+// Query heads (and key heads) of a row normed as one vector: a block takes the row.  Its coordinates are staged in LDS while
+// their squares are summed; after one barrier every thread norms and turns its own coordinates (a pair's partner is normed
+// again rather than exchanged).
+template <typename TC, int NT>
+__global__ __launch_bounds__(NT) void gqa_post_row_kernel(GqaPostP p, int values) {
+    extern __shared__ float sm[];
+    constexpr int NW = NT / 64, U = 8;
+    __shared__ float red[2 * NW];
+    const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int slot = p.row_slot[t], pos = p.row_pos[t];
+    const int dim = p.dim, vdim = p.vdim, G = p.kv_heads, nq = p.heads * dim, nk = p.q_only ? 0 : G * dim, PT = p.cache.page_tokens;
+    float* row = p.proj + (int64_t)t * p.ld;
+    const int64_t pb = page_base(p.cache, slot, pos);
+    const int pt = pos % PT;
+    TC* krow = (TC*)p.cache.pool + pb + p.k_off + (int64_t)pt * G * dim;
+    TC* vbase = (TC*)p.cache.pool + pb + p.v_off;
+    auto vidx = [&](int g, int i) -> int64_t {
+        return p.v_transposed ? ((int64_t)g * vdim + i) * PT + pt : ((int64_t)pt * G + g) * vdim + i;
+    };
+    float sq = 0.f, sk = 0.f;
+    for (int i0 = tid; i0 < nq + nk; i0 += NT * U) {
+        float a[U];
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const int i = i0 + u * NT;
+            a[u] = i < nq ? row[p.q_col + i] : i < nq + nk ? row[p.k_col + i - nq] : 0.f;
+        }
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const int i = i0 + u * NT;
+            if (i >= nq + nk) break;
+            const float* b = i < nq ? p.q_bias : p.k_bias;
+            const float x = b ? a[u] + b[i < nq ? i : i - nq] : a[u];
+            sm[i] = x;
+            if (i < nq) sq += x * x;
+            else sk += x * x;
+        }
+    }
+    if (values && !p.q_only) {   // as they are
+        for (int i = tid; i < G * vdim; i += NT) {
+            const float x = row[p.v_col + i];
+            stc<TC>(vbase, vidx(i / vdim, i % vdim), p.v_bias ? x + p.v_bias[i] : x);
+        }
+    }
+    sq = wsum(sq);
+    sk = wsum(sk);
+    if (lane == 0) {
+        red[wave] = sq;
+        red[NW + wave] = sk;
+    }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; w++) {
+        sq += red[w];
+        sk += red[NW + w];
+    }
+    float iq = 1.0f / sqrtf(sq / (float)nq + p.eps);
+    const float ik = nk ? 1.0f / sqrtf(sk / (float)nk + p.eps) : 0.f;
+    if (p.q_temp_every > 0) iq *= 1.0f + p.q_temp_coef * logf((float)((pos + 1) / p.q_temp_every + 1));
+    const int half = p.rot_dims >> 1;
+    const float* cs = p.rope_cos + (int64_t)pos * half;
+    const float* sn = p.rope_sin + (int64_t)pos * half;
+    for (int i = tid; i < nq + nk; i += NT) {
+        const bool is_q = i < nq;
+        const int ii = is_q ? i : i - nq, c = ii % dim;
+        const float inv = is_q ? iq : ik;
+        const float* w = is_q ? p.qn_w : p.kn_w;
+        const float raw = sm[i];
+        float o = raw * inv * w[ii];
+        if (c < p.rot_dims) {
+            const bool second = p.rot_layout == 1 ? (c & 1) != 0 : c >= half;
+            const int j = p.rot_layout == 1 ? c >> 1 : second ? c - half : c;
+            const int d = p.rot_layout == 1 ? (second ? -1 : 1) : (second ? -half : half);   // to the pair's partner
+            const float other = sm[i + d] * inv * w[ii + d];
+            o = o * cs[j] + (second ? other : -other) * sn[j];
+        }
+        if (is_q) {
+            row[p.q_col + i] = o;
+        } else {
+            if (p.v_col < 0) stc<TC>(vbase, vidx(ii / dim, c), raw);   // the value is the key as projected
+            stc<TC>(krow, ii, o);
         }
     }
 }
@@ -250,28 +302,29 @@ int gqa_post(const GqaPostP& p, bool cache_f32, int T, hipStream_t st) {
     QIE_REQUIRE(p.rot_dims % 2 == 0 && p.rot_dims <= p.dim, "gqa_post: rotary dims %d must be even and <= %d", p.rot_dims, p.dim);
     QIE_REQUIRE(!p.rot_values || p.vdim % 2 == 0, "gqa_post: turned values need an even vdim (%d)", p.vdim);
     QIE_REQUIRE(p.v_col >= 0 || p.vdim == p.dim, "gqa_post: keys as values need vdim == dim");
-    const bool row = p.qk_norm == 3;
     QIE_REQUIRE(!p.q_only || p.v_col >= 0, "gqa_post: a layer that reads another layer's keys caches nothing");
-    QIE_REQUIRE(!row || (p.qn_w && (p.q_only || p.kn_w)), "gqa_post: the row norm's weights are missing");
-    const int nt = row && T <= 64 ? 1024 : 256;   // few rows: a row's heads over several blocks, or one wide block
-    const size_t shm = (size_t)(nt / 64) * std::max(p.dim, p.vdim) * 4;
-    QIE_REQUIRE((size_t)4 * std::max(p.dim, p.vdim) * 4 <= 48 * 1024, "gqa_post: head size %d above the kernel's staging",
-                std::max(p.dim, p.vdim));
-    const bool wide = nt == 1024 && shm <= 48 * 1024;
+    const size_t shm = (size_t)4 * std::max(p.dim, p.vdim) * 4;
+    QIE_REQUIRE(shm <= 48 * 1024, "gqa_post: head size %d above the kernel's staging", std::max(p.dim, p.vdim));
     const bool apart = p.groups && p.v_col >= 0 && p.v_transposed && !p.rot_values && !cache_f32 && T > 64 && p.vdim <= 512 && !p.q_only;
     const int values = p.v_col >= 0 && !apart ? 1 : 0;
-    const int ny = T <= 64 && !row ? std::min(16, (p.heads + (1 + values) * p.kv_heads + 3) / 4) : 1;
-    const size_t shm4 = (size_t)4 * std::max(p.dim, p.vdim) * 4;
-#define QIE_POST(TC)                                                                                             \
-    if (wide) hipLaunchKernelGGL((gqa_post_kernel<TC, 1024, true>), dim3(T), dim3(1024), shm, st, p, values);    \
-    else if (row) hipLaunchKernelGGL((gqa_post_kernel<TC, 256, true>), dim3(T), dim3(256), shm4, st, p, values); \
-    else hipLaunchKernelGGL((gqa_post_kernel<TC, 256, false>), dim3(T, ny), dim3(256), shm4, st, p, values)
-    if (cache_f32) {
-        QIE_POST(float);
+    const int ny = T <= 64 ? std::min(16, (p.heads + (1 + values) * p.kv_heads + 3) / 4) : 1;   // few rows: a row's heads over several blocks
+    if (p.qk_norm == 3) {
+        const size_t rows = (size_t)(p.heads + (p.q_only ? 0 : p.kv_heads)) * p.dim * 4;
+        QIE_REQUIRE(p.qn_w && (p.q_only || p.kn_w) && !p.rot_values, "gqa_post: the row norm's weights are missing (or turned values, not wired to it)");
+        QIE_REQUIRE(rows <= 60 * 1024, "gqa_post: %d + %d heads of %d above the row norm's staging", p.heads, p.kv_heads, p.dim);
+        if (T <= 64 && cache_f32)
+            hipLaunchKernelGGL((gqa_post_row_kernel<float, 1024>), dim3(T), dim3(1024), rows, st, p, values);
+        else if (T <= 64)
+            hipLaunchKernelGGL((gqa_post_row_kernel<uint16_t, 1024>), dim3(T), dim3(1024), rows, st, p, values);
+        else if (cache_f32)
+            hipLaunchKernelGGL((gqa_post_row_kernel<float, 256>), dim3(T), dim3(256), rows, st, p, values);
+        else
+            hipLaunchKernelGGL((gqa_post_row_kernel<uint16_t, 256>), dim3(T), dim3(256), rows, st, p, values);
+    } else if (cache_f32) {
+        hipLaunchKernelGGL(gqa_post_kernel<float>, dim3(T, ny), dim3(256), shm, st, p, values);
     } else {
-        QIE_POST(uint16_t);
+        hipLaunchKernelGGL(gqa_post_kernel<uint16_t>, dim3(T, ny), dim3(256), shm, st, p, values);
     }
-#undef QIE_POST
     if (apart)
         hipLaunchKernelGGL(gqa_values_kernel, dim3((unsigned)p.n_groups, (unsigned)p.kv_heads), dim3(256), (size_t)16 * (p.vdim + 1) * 4, st, p,
                            p.groups);

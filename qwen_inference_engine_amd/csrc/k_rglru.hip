@@ -8,8 +8,8 @@
 // Everything here is fp32.  The gate products of many rows run on the bf16 matrix cores without losing bits: the
 // weights are bf16 already, and u is split into three bf16 parts (8 + 8 + 8 bits, each the truncated rest of the one
 // before) whose products with a weight are exact in the fp32 accumulator's inputs; the sum of the three products is the
-// fp32 product up to the rounding of its additions.  At a sixteenth of the fp32 matrix rate per product the three still
-// cost a fifth of one fp32 product.
+// fp32 product up to the rounding of its additions.  The bf16 matrix rate is sixteen times the fp32 one, so the three cost
+// about a fifth of the one.
 #include "k_layered.hpp"
 
 namespace qie {
@@ -209,94 +209,96 @@ int rglru_scan(const RgLruP& p, hipStream_t st) {
 }
 
 // ------------------------------------------------------------------ steps of few rows
-// A wave per channel: its two weight rows against every row's block of u, four rows at a time; then the rows' recurrence in
-// order (rows of an entry are neighbours, its first one loads the slot's state, its last one stores it).  V inputs a lane.
-template <typename TW> __device__ __forceinline__ float ldw_r(const TW* p, int64_t i);
-template <> __device__ __forceinline__ float ldw_r<float>(const float* p, int64_t i) { return p[i]; }
-template <> __device__ __forceinline__ float ldw_r<uint16_t>(const uint16_t* p, int64_t i) { return bf2f(p[i]); }
+// A wave per channel: its two weight rows against every row's block of u, eight rows a turn; lane t then owns row t (gates,
+// the other branch, the slot's state: all rows' loads and exponentials at once), and rows of one entry, neighbours at most
+// `chain` long, hand their state to the next lane.  V inputs per lane and load.
+template <typename TW, int V> __device__ __forceinline__ void ldw_r(const TW* p, float* o) {
+    if constexpr (V == 1) {
+        if constexpr (sizeof(TW) == 4) o[0] = p[0];
+        else o[0] = bf2f(p[0]);
+    } else if constexpr (sizeof(TW) == 4) {
+        *reinterpret_cast<float4*>(o) = *reinterpret_cast<const float4*>(p);
+    } else {
+        const uint2 u = *reinterpret_cast<const uint2*>(p);
+        o[0] = bf2f(u.x & 0xffffu); o[1] = bf2f(u.x >> 16); o[2] = bf2f(u.y & 0xffffu); o[3] = bf2f(u.y >> 16);
+    }
+}
 
-template <typename TW>
-__global__ __launch_bounds__(256) void rglru_step_kernel(RgLruP p, int T) {
+template <typename TW, int V>
+__global__ __launch_bounds__(256) void rglru_step_kernel(RgLruP p, int T, int chain) {
     const int n = p.blocks * p.bs, bs = p.bs, lane = threadIdx.x & 63, c = blockIdx.x * 4 + (threadIdx.x >> 6);
     if (c >= n) return;
     const int blk = c / bs, j = c % bs;
     const TW* wr = (const TW*)p.w + ((int64_t)blk * 2 * bs + j) * bs;
     const TW* wi = wr + (int64_t)bs * bs;
-    const float rb = p.r_b[c], ib = p.i_b[c], dc = p.decay[c], yb = p.y_b[c];
-    constexpr int R = 4, NP = 4;   // rows a turn; 64 NP weight pairs stay in registers
-    float kr[NP], ki[NP];
-#pragma unroll
-    for (int q = 0; q < NP; q++) {
-        const int k = lane + 64 * q;
-        kr[q] = k < bs ? ldw_r<TW>(wr, k) : 0.f;
-        ki[q] = k < bs ? ldw_r<TW>(wi, k) : 0.f;
-    }
-    float S = 0.f;
+    // this lane's row
+    const int row = min(lane, T - 1);
+    const int64_t so = (int64_t)p.row_slot[row] * p.init_stride + p.init_off + c;
+    const int k = p.row_k[row];
+    const bool last = row + 1 == T || p.row_k[min(row + 1, T - 1)] == 0;
+    float S = k == 0 && p.row_pos[row] > 0 ? p.init[so] : 0.f;
+    const float uc = p.u[row * p.ld_u + c], yc = p.y[row * p.ld_y + c] + p.y_b[c];
+    float zr = p.r_b[c], zi = p.i_b[c];
+    constexpr int R = 8;
     for (int t0 = 0; t0 < T; t0 += R) {
-        float zr[R], zi[R], uc[R], yc[R];
+        float ar[R], ai[R];
         const float* ub[R];
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            const int64_t t = min(t0 + r, T - 1);
-            ub[r] = p.u + t * p.ld_u + blk * bs;
-            uc[r] = ub[r][j];
-            yc[r] = p.y[t * p.ld_y + c];
-            zr[r] = zi[r] = 0.f;
+            ub[r] = p.u + (int64_t)min(t0 + r, T - 1) * p.ld_u + blk * bs;
+            ar[r] = ai[r] = 0.f;
         }
+        for (int q = lane * V; q < bs; q += 64 * V) {
+            float a[V], b[V], x[R][V];
+            ldw_r<TW, V>(wr + q, a);
+            ldw_r<TW, V>(wi + q, b);
 #pragma unroll
-        for (int q = 0; q < NP; q++) {
-            const int k = lane + 64 * q;
-            if (k < bs) {
+            for (int r = 0; r < R; r++) ldw_r<float, V>(ub[r] + q, x[r]);
 #pragma unroll
-                for (int r = 0; r < R; r++) {
-                    const float x = ub[r][k];
-                    zr[r] = fmaf(kr[q], x, zr[r]);
-                    zi[r] = fmaf(ki[q], x, zi[r]);
+            for (int r = 0; r < R; r++)
+#pragma unroll
+                for (int v = 0; v < V; v++) {
+                    ar[r] = fmaf(a[v], x[r][v], ar[r]);
+                    ai[r] = fmaf(b[v], x[r][v], ai[r]);
                 }
-            }
-        }
-        for (int k = lane + 64 * NP; k < bs; k += 64) {
-            const float a = ldw_r<TW>(wr, k), b = ldw_r<TW>(wi, k);
-#pragma unroll
-            for (int r = 0; r < R; r++) {
-                const float x = ub[r][k];
-                zr[r] = fmaf(a, x, zr[r]);
-                zi[r] = fmaf(b, x, zi[r]);
-            }
         }
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            zr[r] = wsum_r(zr[r]);
-            zi[r] = wsum_r(zi[r]);
-        }
-#pragma unroll
-        for (int r = 0; r < R; r++) {
-            const int t = t0 + r;
-            if (t >= T) break;
-            const int64_t so = (int64_t)p.row_slot[t] * p.init_stride + p.init_off + c;
-            if (p.row_k[t] == 0) S = p.row_pos[t] > 0 ? p.init[so] : 0.f;
-            float a, b;
-            lru_terms(zr[r] + rb, zi[r] + ib, dc, uc[r], &a, &b);
-            S = fmaf(a, S, b);
-            if (lane == 0) {
-                const float o = S * gelu_t(yc[r] + yb);
-                if (p.out) p.out[(int64_t)t * p.ld_out + c] = o;
-                if (p.out_bf) p.out_bf[(int64_t)t * p.ld_out + c] = f2bf(o);
-                if (t + 1 == T || p.row_k[t + 1] == 0) p.end[so] = S;
+            const float sr = wsum_r(ar[r]), si = wsum_r(ai[r]);
+            if (lane == t0 + r) {
+                zr += sr;
+                zi += si;
             }
         }
     }
+    float a, b;
+    lru_terms(zr, zi, p.decay[c], uc, &a, &b);
+    if (k == 0) S = fmaf(a, S, b);
+    for (int s = 1; s < chain; s++) {
+        const float prev = __shfl_up(S, 1, 64);
+        if (k == s) S = fmaf(a, prev, b);
+    }
+    if (lane >= T) return;
+    const float o = S * gelu_t(yc);
+    if (p.out) p.out[(int64_t)row * p.ld_out + c] = o;
+    if (p.out_bf) p.out_bf[(int64_t)row * p.ld_out + c] = f2bf(o);
+    if (last) p.end[so] = S;
 }
 
-int rglru_step(const RgLruP& p, int T, hipStream_t st) {
+int rglru_step(const RgLruP& p, int T, int chain, hipStream_t st) {
     QIE_REQUIRE(p.u && p.w && p.y && p.y_b && p.row_slot && p.row_pos && p.row_k && p.init && p.end && (p.out || p.out_bf) && T > 0 &&
-                    T <= kRgLruStepRows && p.init == p.end && p.init_stride == p.end_stride && p.init_off == p.end_off,
+                    T <= kRgLruStepRows && chain >= 1 && p.init == p.end && p.init_stride == p.end_stride && p.init_off == p.end_off,
                 "rglru step: bad arguments");
     const dim3 grid((unsigned)((p.blocks * p.bs + 3) / 4));
-    if (p.w_f32)
-        hipLaunchKernelGGL(rglru_step_kernel<float>, grid, dim3(256), 0, st, p, T);
+    const bool v4 = p.bs % 4 == 0 && p.ld_u % 4 == 0 && (((uintptr_t)p.u | (uintptr_t)p.w) & 15) == 0;
+    if (p.w_f32 && v4)
+        hipLaunchKernelGGL((rglru_step_kernel<float, 4>), grid, dim3(256), 0, st, p, T, chain);
+    else if (p.w_f32)
+        hipLaunchKernelGGL((rglru_step_kernel<float, 1>), grid, dim3(256), 0, st, p, T, chain);
+    else if (v4)
+        hipLaunchKernelGGL((rglru_step_kernel<uint16_t, 4>), grid, dim3(256), 0, st, p, T, chain);
     else
-        hipLaunchKernelGGL(rglru_step_kernel<uint16_t>, grid, dim3(256), 0, st, p, T);
+        hipLaunchKernelGGL((rglru_step_kernel<uint16_t, 1>), grid, dim3(256), 0, st, p, T, chain);
     QIE_LAUNCH_CHECK();
     return 0;
 }
