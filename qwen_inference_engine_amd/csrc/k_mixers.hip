@@ -484,6 +484,7 @@ int gqa_attention(const GqaAttnP& p, bool cache_f32, int T, hipStream_t st) {
 // No LDS, no barrier: waves of a workgroup are independent (they share key heads through the L1).
 typedef __bf16 gbf16x8_t __attribute__((ext_vector_type(8)));
 typedef float gf32x4_t __attribute__((ext_vector_type(4)));
+typedef uint32_t gu32x4_t __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ float xg_max(float v) {   // over the 4 lanes n, n + 16, n + 32, n + 48
     v = fmaxf(v, __shfl_xor(v, 16, 64));
@@ -642,7 +643,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
     };
     // SHARE: a thread's 16-byte pieces of the workgroup's tiles (K: 32 keys x dim, V^T: vdim x 32 keys)
     constexpr int NKP = (32 * dim / 8 + 255) / 256, NVP = (vdim * 4 + 255) / 256;
-    uint4 gk[NKP], gv[NVP];
+    gu32x4_t gk[NKP], gv[NVP];   // (native vectors: arrays of the struct type end up in scratch memory)
     auto fetch_tiles = [&](int kb) {
         const int key0 = kb << 5;
         const int64_t pb = (int64_t)tab[key0 / PT] * a.cache.page_stride;
@@ -650,24 +651,24 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(GqaAttnMfmaP P) {
 #pragma unroll
         for (int k = 0; k < NKP; k++) {
             const int c = (int)threadIdx.x + 256 * k, key = c / (dim / 8), part = c % (dim / 8);
-            if (c < 32 * dim / 8) gk[k] = *reinterpret_cast<const uint4*>(pool + pb + a.k_off + ((int64_t)(tok0 + key) * G + kvh) * dim + part * 8);
+            if (c < 32 * dim / 8) gk[k] = *reinterpret_cast<const gu32x4_t*>(pool + pb + a.k_off + ((int64_t)(tok0 + key) * G + kvh) * dim + part * 8);
         }
 #pragma unroll
         for (int k = 0; k < NVP; k++) {
             const int c = (int)threadIdx.x + 256 * k, r = c >> 2, part = c & 3;
-            if (c < vdim * 4) gv[k] = *reinterpret_cast<const uint4*>(pool + pb + a.v_off + ((int64_t)kvh * vdim + r) * PT + tok0 + part * 8);
+            if (c < vdim * 4) gv[k] = *reinterpret_cast<const gu32x4_t*>(pool + pb + a.v_off + ((int64_t)kvh * vdim + r) * PT + tok0 + part * 8);
         }
     };
     auto store_tiles = [&]() {
 #pragma unroll
         for (int k = 0; k < NKP; k++) {
             const int c = (int)threadIdx.x + 256 * k, key = c / (dim / 8), part = c % (dim / 8);
-            if (c < 32 * dim / 8) *reinterpret_cast<uint4*>(lk + key * KROW + part * 8) = gk[k];
+            if (c < 32 * dim / 8) *reinterpret_cast<gu32x4_t*>(lk + key * KROW + part * 8) = gk[k];
         }
 #pragma unroll
         for (int k = 0; k < NVP; k++) {
             const int c = (int)threadIdx.x + 256 * k, r = c >> 2, part = c & 3;
-            if (c < vdim * 4) *reinterpret_cast<uint4*>(lv + r * VROW + part * 8) = gv[k];
+            if (c < vdim * 4) *reinterpret_cast<gu32x4_t*>(lv + r * VROW + part * 8) = gv[k];
         }
     };
     if (bs < be) {
@@ -1196,13 +1197,13 @@ int gated_norm_parts(const float* y, const float* z, int64_t ld_z, const float* 
 // ------------------------------------------------------------------ two norms of one row
 // One block per row.  Rows of whole float4s (NV > 0): a thread's NV vectors stay in registers between the sum and the
 // two scaled copies, every load issued before the first use; NV = 0: any width, the row re-read.
-__device__ __forceinline__ void store_bf4(uint16_t* p, float4 v) {
-    *reinterpret_cast<uint2*>(p) = make_uint2(pack2(v.x, v.y), pack2(v.z, v.w));
+__device__ __forceinline__ void store_bf4(uint16_t* p, gf32x4_t v) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack2(v[0], v[1]), pack2(v[2], v[3]));
 }
+__device__ __forceinline__ gf32x4_t ld4(const float* p) { return *reinterpret_cast<const gf32x4_t*>(p); }
+__device__ __forceinline__ float sq4(gf32x4_t v) { return (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
 
 // BN: v and v2 are normed before they are added.
-__device__ __forceinline__ float sq4(float4 v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); }
-
 template <int NV, bool BN>
 __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
     __shared__ float red[4];
@@ -1211,31 +1212,29 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
     float f1 = 1.f, f2 = 1.f;   // BN: the branches' factors
     float ss = 0.f;
     if constexpr (NV > 0) {
+        // (native vectors: arrays of the struct type end up in scratch memory)
         const int n4 = p.W >> 2;
-        float4 x[NV], a[NV], b[NV], c[NV];
-        const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+        gf32x4_t x[NV], a[NV], b[NV], c[NV];
+        const gf32x4_t zero = gf32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int k = 0; k < NV; k++) {
             const int i = threadIdx.x + 256 * k;
             const bool on = i < n4;
             const int64_t o = r0 + 4 * (on ? i : 0);
-            x[k] = *reinterpret_cast<const float4*>(p.xin + o);
-            a[k] = p.v ? *reinterpret_cast<const float4*>(p.v + o) : zero;
-            b[k] = p.v2 ? *reinterpret_cast<const float4*>(p.v2 + o) : zero;
-            c[k] = p.add ? *reinterpret_cast<const float4*>(p.add + o) : zero;
-            if (p.v3) {
-                const float4 d = *reinterpret_cast<const float4*>(p.v3 + o);
-                c[k] = make_float4(c[k].x + d.x, c[k].y + d.y, c[k].z + d.z, c[k].w + d.w);
-            }
+            x[k] = ld4(p.xin + o);
+            a[k] = p.v ? ld4(p.v + o) : zero;
+            b[k] = p.v2 ? ld4(p.v2 + o) : zero;
+            c[k] = p.add ? ld4(p.add + o) : zero;
+            if (p.v3) c[k] += ld4(p.v3 + o);
         }
         if constexpr (BN) {
-            float4 u1[NV], u2[NV];
+            gf32x4_t u1[NV], u2[NV];
             float s1 = 0.f, s2 = 0.f;
 #pragma unroll
             for (int k = 0; k < NV; k++) {
                 const int i = threadIdx.x + 256 * k, j = 4 * (i < n4 ? i : 0);
-                u1[k] = *reinterpret_cast<const float4*>(p.v_w + j);
-                u2[k] = *reinterpret_cast<const float4*>(p.v2_w + j);
+                u1[k] = ld4(p.v_w + j);
+                u2[k] = ld4(p.v2_w + j);
                 if (i < n4) {
                     s1 += sq4(a[k]);
                     s2 += sq4(b[k]);
@@ -1247,29 +1246,26 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
             f2 = p.v2_scale / sqrtf(s2 / (float)p.W + p.eps);
 #pragma unroll
             for (int k = 0; k < NV; k++) {
-                a[k] = make_float4(a[k].x * f1 * u1[k].x, a[k].y * f1 * u1[k].y, a[k].z * f1 * u1[k].z, a[k].w * f1 * u1[k].w);
-                b[k] = make_float4(b[k].x * f2 * u2[k].x, b[k].y * f2 * u2[k].y, b[k].z * f2 * u2[k].z, b[k].w * f2 * u2[k].w);
+                a[k] = a[k] * f1 * u1[k];
+                b[k] = b[k] * f2 * u2[k];
             }
         }
 #pragma unroll
         for (int k = 0; k < NV; k++) {
             const int i = threadIdx.x + 256 * k;
-            x[k].x += (a[k].x + b[k].x) + c[k].x;
-            x[k].y += (a[k].y + b[k].y) + c[k].y;
-            x[k].z += (a[k].z + b[k].z) + c[k].z;
-            x[k].w += (a[k].w + b[k].w) + c[k].w;
+            x[k] += (a[k] + b[k]) + c[k];
             if (i < n4) {
-                if (moved) *reinterpret_cast<float4*>(p.x + r0 + 4 * i) = x[k];
-                ss += (x[k].x * x[k].x + x[k].y * x[k].y) + (x[k].z * x[k].z + x[k].w * x[k].w);
+                if (moved) *reinterpret_cast<gf32x4_t*>(p.x + r0 + 4 * i) = x[k];
+                ss += sq4(x[k]);
             }
         }
         if (!p.w1) return;
-        float4 w1[NV], w2[NV];
+        gf32x4_t w1[NV], w2[NV];
 #pragma unroll
         for (int k = 0; k < NV; k++) {
             const int i = threadIdx.x + 256 * k, j = 4 * (i < n4 ? i : 0);
-            w1[k] = *reinterpret_cast<const float4*>(p.w1 + j);
-            w2[k] = p.w2 ? *reinterpret_cast<const float4*>(p.w2 + j) : zero;
+            w1[k] = ld4(p.w1 + j);
+            w2[k] = p.w2 ? ld4(p.w2 + j) : zero;
         }
         ss = bsum256(ss, red);
         const float inv = 1.0f / sqrtf(ss / (float)p.W + p.eps);
@@ -1278,13 +1274,12 @@ __global__ __launch_bounds__(256) void norm_pair_kernel(NormPairP p) {
             const int i = threadIdx.x + 256 * k;
             if (i >= n4) break;
             const int64_t o = r0 + 4 * i;
-            const float4 y = make_float4(x[k].x * inv, x[k].y * inv, x[k].z * inv, x[k].w * inv);
-            const float4 y1 = make_float4(y.x * w1[k].x, y.y * w1[k].y, y.z * w1[k].z, y.w * w1[k].w);
-            if (p.h1) *reinterpret_cast<float4*>(p.h1 + o) = y1;
+            const gf32x4_t y = x[k] * inv, y1 = y * w1[k];
+            if (p.h1) *reinterpret_cast<gf32x4_t*>(p.h1 + o) = y1;
             if (p.h1_bf) store_bf4(p.h1_bf + o, y1);
             if (p.w2) {
-                const float4 y2 = make_float4(y.x * w2[k].x, y.y * w2[k].y, y.z * w2[k].z, y.w * w2[k].w);
-                if (p.h2) *reinterpret_cast<float4*>(p.h2 + o) = y2;
+                const gf32x4_t y2 = y * w2[k];
+                if (p.h2) *reinterpret_cast<gf32x4_t*>(p.h2 + o) = y2;
                 if (p.h2_bf) store_bf4(p.h2_bf + o, y2);
             }
         }
