@@ -184,6 +184,8 @@ struct LayeredBatch {
     // recurrent mixers, long entries: pieces of kScanPiece rows scanned side by side (lay::gated_carry); pieces of
     // lin_rows rows for the mixers of lay::linrec_walk
     PieceList pieces, lin[3];         // lin: pieces of 128, 256, 512 rows
+    PieceList del[2];                 // delta rule: pieces of 128, 256 rows (64: pieces)
+    std::vector<int> del_units;       // (head, column tile) blocks of the model's delta rules, transition columns included
     int max_count = 0;
     int64_t step_T = 0;               // rows of the step being built
     bool ff_branch = false;           // parallel blocks: the layer's feed-forward is running on side[0]
@@ -950,6 +952,20 @@ static int lin_units(int heads, int vdim) { return heads * ((vdim + 63) / 64); }
 static int lin_list_of(int64_t T, int units) {
     const int64_t want = T * units / 512;
     return want >= 512 ? 2 : want >= 256 ? 1 : 0;
+}
+
+// Pieces of 64, 128 or 256 rows for a delta rule: the longest (the carry walks the pieces one after the other) that leaves
+// four blocks a CU to the scan and an entry at least two pieces.  0: 64, 1: 128, 2: 256.
+static int delta_units(const qie_delta_desc& c) {
+    int lp = 1;
+    while (lp * 32 < c.dim) lp *= 2;
+    const int cols = 256 / lp;
+    return c.heads * ((c.vdim + c.dim + cols - 1) / cols);
+}
+static int delta_list_of(int64_t T, int max_count, int units) {
+    int k = 0;
+    while (k < 2 && (128 << k) * 2 <= max_count && T * units / (128 << k) >= 1024) k++;
+    return k;
 }
 
 // Rows above which independent branches of a layer run on streams of their own (below, a step is a chain of launches of a
@@ -1769,16 +1785,18 @@ static int enq_delta_scan(qie_batch* b, int r, int T, bool advance, hipStream_t 
         // long entries: pieces from zero states side by side (end states, transition matrices, transformed
         // queries), a carry over each entry's pieces, then the incoming states' share of every row
         const int64_t n = (int64_t)c.heads * c.dim * c.vdim;
+        const int list = delta_list_of(s->step_T, s->max_count, delta_units(c));
+        const PieceList& pl = list ? s->del[list - 1] : s->pieces;
         lay::DeltaScanP a = sp;
-        a.entries = s->pieces.d_chunks; a.n_entries = s->pieces.n;
+        a.entries = pl.d_chunks; a.n_entries = pl.n;
         a.state = s->s_loc; a.slot_stride = n; a.state_off = 0;
         a.read_state = 0; a.write_state = 1;
         a.trans = s->s_decay; a.w_out = s->dw;
         QIE_TRY(lay::delta_scan(a, st));
-        lay::DeltaCarryP k{s->pieces.d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
+        lay::DeltaCarryP k{pl.d_spans, s->n_ent, c.heads, c.dim, c.vdim, s->s_loc, s->s_decay, s->s_in, s->state, s->slot_state,
                            s->state_off[r], advance ? 1 : 0};
         QIE_TRY(lay::delta_carry(k, st));
-        lay::DeltaApplyP ap{s->pieces.d_chunks, s->pieces.n, kScanPiece, c.heads, c.dim, c.vdim, s->s_in, s->dw, s->olat};
+        lay::DeltaApplyP ap{pl.d_chunks, pl.n, pl.rows, c.heads, c.dim, c.vdim, s->s_in, s->dw, s->olat};
         QIE_TRY(lay::delta_apply(ap, st));
     } else {
         QIE_TRY(lay::delta_scan(sp, st));
@@ -2308,7 +2326,9 @@ int layered_batch_create(qie_engine* e, int32_t batch, int32_t max_ctx, int32_t 
         s->m_state = std::max<int64_t>(s->m_state, heads * dim * vdim);
         s->m_hd = std::max<int64_t>(s->m_hd, heads * dim);
     };
-    auto delta_state = [&](int r, const qie_delta_desc& c) {   // per slot the heads' states and the short convolutions' last inputs
+    auto delta_state = [&](int r, const qie_delta_desc& c) {
+        s->del_units.push_back(delta_units(c));
+        // per slot the heads' states and the short convolutions' last inputs
         const int64_t C = 2 * (int64_t)c.kv_heads * c.dim + (int64_t)c.heads * c.vdim;
         s->state_off[r] = s->slot_state;
         s->slot_state += (int64_t)c.heads * c.dim * c.vdim;
@@ -2491,7 +2511,8 @@ void layered_batch_destroy(qie_batch* b) {
                   s->state, s->d_ent, s->d_qgroups, s->gpart_o, s->gpart_ml, s->pieces.d_chunks, s->pieces.d_spans, s->s_loc, s->s_in, s->s_decay};
     for (void* p : ps)
         if (p) hipFree(p);
-    for (PieceList& l : s->lin) {
+    for (PieceList* q : {&s->lin[0], &s->lin[1], &s->lin[2], &s->del[0], &s->del[1]}) {
+        PieceList& l = *q;
         if (l.d_chunks) hipFree(l.d_chunks);
         if (l.d_spans) hipFree(l.d_spans);
     }
@@ -2846,6 +2867,11 @@ int qie_batch_step(qie_batch* b, int32_t n_entries, const int32_t* slots, const 
         s->max_count = 0;
         for (int i = 0; i < n_entries; i++) s->max_count = std::max(s->max_count, (int)counts[i]);
         if (s->has_scan && s->max_count > kScanLong) QIE_TRY(build_pieces(b, s->pieces, kScanPiece));
+        for (int k = 0; k < 2 && s->max_count > kScanLong; k++) {
+            bool used = false;
+            for (int u : s->del_units) used = used || delta_list_of(T, s->max_count, u) == k + 1;
+            if (used) QIE_TRY(build_pieces(b, s->del[k], 128 << k));
+        }
         for (int k = 0; k < 3 && s->has_lin; k++) {
             s->lin[k].rows = 128 << k;
             bool used = false;

@@ -302,12 +302,15 @@ int delta_carry(const DeltaCarryP& p, hipStream_t st) {
     return 0;
 }
 
-// out[t, h, col] += sum_j s_in[piece][h][j][col] w[t, h, j]: one block per (piece, head, 64 columns), j in tiles of 64
-// through LDS; thread (rq, col) owns rows rq, rq + 4, ... of the piece (at most 64).
-__global__ __launch_bounds__(256) void delta_apply_kernel(DeltaApplyP p) {
+// out[t, h, col] += sum_j s_in[piece][h][j][col] w[t, h, j]: one block per (64 rows of a piece, head, 64 columns), j in tiles
+// of 64 through LDS; thread (rq, col) owns rows rq, rq + 4, ...
+__global__ __launch_bounds__(256) void delta_apply_kernel(DeltaApplyP p, int per) {
     __shared__ float sw[64 * 64];   // [row][j]
     __shared__ float st[64 * 64];   // [j][col]
-    const int4 en = p.chunks[blockIdx.x];   // {first packed row, rows, piece index, 0}
+    int4 en = p.chunks[blockIdx.x / per];   // {first packed row, rows, piece index, 0}: 64 of its rows
+    en.x += blockIdx.x % per * 64;
+    en.y = min(64, en.y - (int)(blockIdx.x % per) * 64);
+    if (en.y <= 0) return;
     const int h = blockIdx.y, lc = threadIdx.x & 63, rq = threadIdx.x >> 6, col = blockIdx.z * 64 + lc;
     const int dim = p.dim, vdim = p.vdim, H = p.H;
     const float* sin = p.s_in + ((int64_t)en.z * H + h) * dim * vdim;
@@ -337,9 +340,10 @@ __global__ __launch_bounds__(256) void delta_apply_kernel(DeltaApplyP p) {
 }
 
 int delta_apply(const DeltaApplyP& p, hipStream_t st) {
-    QIE_REQUIRE(p.chunks && p.n_chunks > 0 && p.s_in && p.w && p.out && p.max_rows <= 64, "delta_apply: bad arguments (pieces of at most 64 rows)");
-    const dim3 grid((unsigned)p.n_chunks, (unsigned)p.H, (unsigned)((p.vdim + 63) / 64));
-    hipLaunchKernelGGL(delta_apply_kernel, grid, dim3(256), 0, st, p);
+    QIE_REQUIRE(p.chunks && p.n_chunks > 0 && p.s_in && p.w && p.out && p.max_rows > 0, "delta_apply: bad arguments");
+    const int per = (p.max_rows + 63) / 64;
+    const dim3 grid((unsigned)(p.n_chunks * per), (unsigned)p.H, (unsigned)((p.vdim + 63) / 64));
+    hipLaunchKernelGGL(delta_apply_kernel, grid, dim3(256), 0, st, p, per);
     QIE_LAUNCH_CHECK();
     return 0;
 }

@@ -436,7 +436,7 @@ struct DeltaCarryP {
     int write_state;
 };
 int delta_carry(const DeltaCarryP& p, hipStream_t st);
-// out[t, h, :] += s_in[piece of t][h]^T w[t, h, :] over the pieces {first packed row, rows (<= 64), piece index, 0}
+// out[t, h, :] += s_in[piece of t][h]^T w[t, h, :] over the pieces {first packed row, rows (<= max_rows), piece index, 0}
 struct DeltaApplyP {
     const int4* chunks;
     int n_chunks, max_rows;

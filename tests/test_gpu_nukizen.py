@@ -431,6 +431,22 @@ def test_long_prompts_beside_decoding(model):
     assert rel(np.concatenate([r1[600:], r2[:7]]), wb) < m.tol
 
 
+@pytest.mark.parametrize("n,last", [(1000, 700), (2200, 1900)])
+def test_delta_rule_in_pieces_of_128_and_256_rows(model, n, last):
+    """Many state columns and a long prompt: the delta rule takes longer pieces (whole ones and ragged ends), from a fresh
+    and from a kept state, beside a short entry."""
+    m = model([par(heads=1, kv_heads=1, size=20, d_heads=4, d_kv_heads=2, d_dim=512, d_vdim=16, mlp=None)], seed=23, slots=2, page_tokens=64,
+              max_ctx=2304, tweak=slow_decay)
+    a, b = m.tokens(n), m.tokens(6)
+    wa, wb = m.ref(a), m.ref(b)
+    assert rel(m.batch.step([(0, a)], range(n)), wa) < m.tol
+    m.batch.release(0)
+    r1 = m.batch.step([(0, a[:n - last]), (1, b[:4])], range(n - last + 4))
+    r2 = m.batch.step([(1, b[4:]), (0, a[n - last:])], range(last + 2))
+    assert rel(np.concatenate([r1[:n - last], r2[2:]]), wa) < m.tol
+    assert rel(np.concatenate([r1[n - last:], r2[:2]]), wb) < m.tol
+
+
 def test_bf16_sizes_of_the_matrix_core_kernels(model):
     """Head sizes that are multiples of 32, gate blocks of 32 and 64, a width that is a multiple of 8: the shapes the bf16
     engine's matrix-core products, gates and attention kernels take."""
